@@ -1,6 +1,7 @@
 from .base import ConfigError, ModelConfig, read_config_json
 from .dizizen import DizizenConfig
 from .gimozen import GimozenConfig
+from .goletar import GoletarConfig
 from .gpt2 import GPT2Config
 from .ketolix import KetolixConfig
 from .perezen import PerezenConfig
@@ -19,6 +20,7 @@ __all__ = [
     "ConfigError",
     "DizizenConfig",
     "GimozenConfig",
+    "GoletarConfig",
     "GPT2Config",
     "KetolixConfig",
     "ModelConfig",

@@ -2,6 +2,21 @@
 // add for parts that do not fuse it into a matrix product.
 #include "common.h"
 
+// A second table whose row a token picks together with the token before it in its sequence: (previous * mul_previous + token *
+// mul_current) mod buckets, in 64-bit, and row `buckets` for a sequence's first token. Inside a portion the previous token is the row
+// above; for a portion's first row it lies in the request's state slot. The block of that first row, which reads the slot, also
+// moves it on to the portion's last token, so that no other block touches it. (Only portions of one token take their token from the
+// device, so a token read from a neighbouring row is always as the host gave it.) table null: no second table.
+struct TokenPairs {
+    const void* table;
+    long long mul_previous, mul_current;
+    int buckets;
+    const int* token_request;
+    const int* q_starts;
+    const int* state_slots;
+    int* previous;
+};
+
 // out[t, :] = wte[token[t], :] + wpe[position[t], :]   (reference: engine/src/embedding.cu:7-27,
 // per-row positions as in embed_batch_kernel :89-104). One block per row; a negative token marks
 // a padding row, which is filled with zeros. With `sources`, the token of a row whose source is
@@ -11,7 +26,7 @@ template <typename T>
 __global__ void embed_kernel(int* __restrict__ tokens, const int* __restrict__ positions,
                              const int* __restrict__ sources, const int* __restrict__ token_slots,
                              const T* __restrict__ wte, const T* __restrict__ wpe,
-                             float* __restrict__ out, int width, float scale) {
+                             float* __restrict__ out, int width, float scale, TokenPairs pairs) {
     int row = blockIdx.x;
     int token = tokens[row];
     if (sources) {
@@ -27,6 +42,22 @@ __global__ void embed_kernel(int* __restrict__ tokens, const int* __restrict__ p
         return;
     }
     const T* token_row = wte + (size_t)token * width;
+    if (pairs.table) {
+        const int request = pairs.token_request[row];
+        const int slot = request >= 0 ? pairs.state_slots[request] : -1;
+        const int first = request >= 0 ? pairs.q_starts[request] : row;
+        int before = row > first ? tokens[row - 1] : (slot >= 0 && positions[row] > 0 ? pairs.previous[slot] : -1);
+        if (row == first && slot >= 0) {   // (uniform over the block)
+            __syncthreads();   // everyone has read the slot
+            const int last = pairs.q_starts[request + 1] - 1;
+            if (threadIdx.x == 0) pairs.previous[slot] = last > row ? tokens[last] : token;
+        }
+        const long long hashed = before < 0 || positions[row] == 0 ? pairs.buckets
+                                                                   : ((long long)before * pairs.mul_previous + (long long)token * pairs.mul_current) % pairs.buckets;
+        const T* pair_row = reinterpret_cast<const T*>(pairs.table) + (size_t)hashed * width;
+        for (int i = threadIdx.x; i < width; i += blockDim.x) out_row[i] = to_float(token_row[i]) * scale + to_float(pair_row[i]);
+        return;
+    }
     if (wpe == nullptr) {  // positions enter the model elsewhere (or nowhere)
         for (int i = threadIdx.x; i < width; i += blockDim.x) out_row[i] = to_float(token_row[i]) * scale;
         return;
@@ -38,7 +69,12 @@ __global__ void embed_kernel(int* __restrict__ tokens, const int* __restrict__ p
 
 MLLM_API int mllm_embed(int* tokens, const int* positions, const int* sources, const int* token_slots,
                         const void* wte, const void* wpe, float* out, int n_rows, int width, int table_dtype,
-                        float scale, hipStream_t stream) {
+                        float scale, const void* pair_table, long long mul_previous, long long mul_current, int buckets,
+                        const int* token_request, const int* q_starts, const int* state_slots, int* previous, hipStream_t stream) {
+    MLLM_REQUIRE(pair_table == nullptr || (wpe == nullptr && buckets > 0 && mul_previous >= 0 && mul_current >= 0 && mul_previous < (1LL << 31) &&
+                                           mul_current < (1LL << 31) && token_request && q_starts && state_slots && previous),
+                 "embed: a table of token pairs needs its numbers, the batch's requests and their state, and takes no position rows");
+    const TokenPairs pairs{pair_table, mul_previous, mul_current, buckets, token_request, q_starts, state_slots, previous};
     MLLM_REQUIRE(n_rows >= 0 && width > 0, "embed: bad sizes rows=%d width=%d", n_rows, width);
     MLLM_REQUIRE(sources == nullptr || token_slots != nullptr, "embed: sources without token slots");
     if (n_rows == 0) return 0;
@@ -46,10 +82,10 @@ MLLM_API int mllm_embed(int* tokens, const int* positions, const int* sources, c
     mllm_count_kernel(MLLM_K_EMBED);
     if (table_dtype == MLLM_F32)
         embed_kernel<float><<<n_rows, threads, 0, stream>>>(tokens, positions, sources, token_slots, (const float*)wte,
-                                                            (const float*)wpe, out, width, scale);
+                                                            (const float*)wpe, out, width, scale, pairs);
     else if (table_dtype == MLLM_BF16)
         embed_kernel<bf16_t><<<n_rows, threads, 0, stream>>>(tokens, positions, sources, token_slots, (const bf16_t*)wte,
-                                                             (const bf16_t*)wpe, out, width, scale);
+                                                             (const bf16_t*)wpe, out, width, scale, pairs);
     else
         MLLM_REQUIRE(false, "embed: unknown table dtype %d", table_dtype);
     return mllm_check_launch("embed");

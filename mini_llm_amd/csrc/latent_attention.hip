@@ -19,15 +19,15 @@ __device__ __forceinline__ void store_from_float(void* base, size_t index, int c
     else reinterpret_cast<bf16_t*>(base)[index] = static_cast<bf16_t>(value);
 }
 
-// out[row, head, n] = sum_k x[row, head, k] * w[head, n, k] (* sigmoid(gate[row, head * N + n]), the gate's rows gate_row_stride apart):
-// one small product per head.
+// out[row, head, n] = sum_k x[row, head, k] * w[head, n, k] (* sigmoid(gate[row, head * N + n]), or with gate_per_head gate[row, head],
+// the gate's rows gate_row_stride apart): one small product per head.
 // A block takes HEADS_ROWS rows of one head: their x in LDS (32-bit), a thread an output column at a time, its W row read in
 // 16-byte pieces where K allows; with fewer columns than threads the threads cut K among themselves and add up through LDS.
 constexpr int HEADS_ROWS = 16;
 
 template <typename WT>
 __global__ __launch_bounds__(256) void heads_linear_kernel(const void* __restrict__ x, int x_code, int x_row_stride, int x_head_stride,
-                                                           const WT* __restrict__ w, const void* __restrict__ gate, int gate_code, int gate_row_stride,
+                                                           const WT* __restrict__ w, const void* __restrict__ gate, int gate_code, int gate_row_stride, int gate_per_head,
                                                            void* __restrict__ out, int out_code, int out_row_stride, int out_head_stride,
                                                            int n_rows, int N, int K, int cols) {
     extern __shared__ float heads_lds[];   // x_tile [HEADS_ROWS][K], then the partial sums [slices - 1][cols][HEADS_ROWS]
@@ -87,7 +87,7 @@ __global__ __launch_bounds__(256) void heads_linear_kernel(const void* __restric
             for (int r = 0; r < rows; r++) {
                 float value = acc[r];
                 if (gate) {
-                    const float g = load_as_float(gate, (size_t)(row0 + r) * gate_row_stride + (size_t)head * N + n, gate_code);
+                    const float g = load_as_float(gate, (size_t)(row0 + r) * gate_row_stride + (gate_per_head ? (size_t)head : (size_t)head * N + n), gate_code);
                     value *= 1.0f / (1.0f + expf(-g));
                 }
                 store_from_float(out, (size_t)(row0 + r) * out_row_stride + (size_t)head * out_head_stride + n, out_code, value);
@@ -103,7 +103,7 @@ __global__ __launch_bounds__(256) void heads_linear_kernel(const void* __restric
 template <typename XT>
 __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(const XT* __restrict__ x, int x_row_stride, int x_head_stride,
                                                                 const bf16_t* __restrict__ w, const void* __restrict__ gate, int gate_code,
-                                                                int gate_row_stride, void* __restrict__ out, int out_code, int out_row_stride,
+                                                                int gate_row_stride, int gate_per_head, void* __restrict__ out, int out_code, int out_row_stride,
                                                                 int out_head_stride, int n_rows, int N, int K) {
     const int lane = threadIdx.x % WAVE, lane32 = lane % 32, half = lane / 32;
     const int head = blockIdx.y, row0 = blockIdx.x * 32;
@@ -138,7 +138,7 @@ __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(const XT* __rest
         if (n >= N) continue;
         float value = acc[v];
         if (gate) {
-            const float g = load_as_float(gate, (size_t)row * gate_row_stride + (size_t)head * N + n, gate_code);
+            const float g = load_as_float(gate, (size_t)row * gate_row_stride + (gate_per_head ? (size_t)head : (size_t)head * N + n), gate_code);
             value *= 1.0f / (1.0f + expf(-g));
         }
         store_from_float(out, (size_t)row * out_row_stride + (size_t)head * out_head_stride + n, out_code, value);
@@ -582,14 +582,14 @@ void launch_latent_hg(const LatentArgs& a) {
 }  // namespace
 
 MLLM_API int mllm_heads_linear(const void* x, int x_dtype, int x_row_stride, int x_head_stride, const void* w, int w_dtype, const void* gate,
-                               int gate_dtype, int gate_row_stride, void* out, int out_dtype, int out_row_stride, int out_head_stride, int n_rows, int n_heads,
+                               int gate_dtype, int gate_row_stride, int gate_per_head, void* out, int out_dtype, int out_row_stride, int out_head_stride, int n_rows, int n_heads,
                                int N, int K, hipStream_t stream) {
     MLLM_REQUIRE(n_rows >= 0 && n_heads > 0 && N > 0 && K > 0, "heads_linear: bad sizes");
     MLLM_REQUIRE(x_head_stride >= 0 && out_head_stride >= N, "heads_linear: heads overlap");
     MLLM_REQUIRE(x_row_stride >= (n_heads - 1) * x_head_stride + K && out_row_stride >= (n_heads - 1) * out_head_stride + N,
                  "heads_linear: rows are too short for the heads");
     for (int code : {x_dtype, w_dtype, out_dtype}) MLLM_REQUIRE(code == MLLM_F32 || code == MLLM_BF16, "heads_linear: unknown dtype %d", code);
-    MLLM_REQUIRE(gate == nullptr || ((gate_dtype == MLLM_F32 || gate_dtype == MLLM_BF16) && gate_row_stride >= n_heads * N), "heads_linear: a gate of unknown element type or with rows too short");
+    MLLM_REQUIRE(gate == nullptr || ((gate_dtype == MLLM_F32 || gate_dtype == MLLM_BF16) && gate_row_stride >= (gate_per_head ? n_heads : n_heads * N)), "heads_linear: a gate of unknown element type or with rows too short");
     const int threads = 256, cols = N > 128 ? 256 : (N > 64 ? 128 : 64);
     const size_t lds = ((size_t)HEADS_ROWS * K + (size_t)(threads / cols - 1) * cols * HEADS_ROWS) * sizeof(float);
     MLLM_REQUIRE(lds <= 64 * 1024, "heads_linear: K = %d is more than a block holds in LDS", K);
@@ -601,20 +601,20 @@ MLLM_API int mllm_heads_linear(const void* x, int x_dtype, int x_row_stride, int
         dim3 tiles(ceil_div(n_rows, 32), n_heads, ceil_div(N, 128));
         if (x_dtype == MLLM_F32)
             heads_linear_mfma_kernel<float><<<tiles, 256, 0, stream>>>((const float*)x, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype,
-                                                                       gate_row_stride, out, out_dtype, out_row_stride, out_head_stride, n_rows, N, K);
+                                                                       gate_row_stride, gate_per_head, out, out_dtype, out_row_stride, out_head_stride, n_rows, N, K);
         else
             heads_linear_mfma_kernel<bf16_t><<<tiles, 256, 0, stream>>>((const bf16_t*)x, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype,
-                                                                        gate_row_stride, out, out_dtype, out_row_stride, out_head_stride, n_rows, N, K);
+                                                                        gate_row_stride, gate_per_head, out, out_dtype, out_row_stride, out_head_stride, n_rows, N, K);
         return mllm_check_launch("heads_linear");
     }
     dim3 grid(ceil_div(n_rows, HEADS_ROWS), n_heads);
     if (w_dtype == MLLM_F32) {
         if (allow_lds(heads_linear_kernel<float>, lds, "heads_linear")) return 1;
-        heads_linear_kernel<float><<<grid, threads, lds, stream>>>(x, x_dtype, x_row_stride, x_head_stride, (const float*)w, gate, gate_dtype, gate_row_stride, out, out_dtype,
+        heads_linear_kernel<float><<<grid, threads, lds, stream>>>(x, x_dtype, x_row_stride, x_head_stride, (const float*)w, gate, gate_dtype, gate_row_stride, gate_per_head, out, out_dtype,
                                                                    out_row_stride, out_head_stride, n_rows, N, K, cols);
     } else {
         if (allow_lds(heads_linear_kernel<bf16_t>, lds, "heads_linear")) return 1;
-        heads_linear_kernel<bf16_t><<<grid, threads, lds, stream>>>(x, x_dtype, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype, gate_row_stride, out, out_dtype,
+        heads_linear_kernel<bf16_t><<<grid, threads, lds, stream>>>(x, x_dtype, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype, gate_row_stride, gate_per_head, out, out_dtype,
                                                                     out_row_stride, out_head_stride, n_rows, N, K, cols);
     }
     return mllm_check_launch("heads_linear");

@@ -238,11 +238,16 @@ __global__ __launch_bounds__(256) void head_norm_pieces_kernel(const T* __restri
     *reinterpret_cast<Vec16*>(out + at) = result;
 }
 
-// Rotation of `dims` elements in the "rotate half" pairing: element i pairs with i + dims / 2, and the pair (u, v) at
-// position p becomes (u c - v s, v c + u s) with c = cos(p f_i) m, s = sin(p f_i) m. The angle is a 32-bit product.
-__device__ __forceinline__ void rotated_pair(float u, float v, int position, float frequency, float magnitude, float& a, float& b) {
-    const float angle = (float)position * frequency;
-    const float c = cosf(angle) * magnitude, s = sinf(angle) * magnitude;
+// Rotation of the pair (u, v) at position p: (u c - v s, v c + u s) with c = cos(p f) m, s = sin(p f) m. The angle is taken in 64-bit
+// (a 32-bit product of a position in the thousands is good to 1e-4 only) and brought into -pi .. pi, where its sine and cosine are
+// taken in 32-bit.
+__device__ __forceinline__ void rotated_pair(float u, float v, int position, double frequency, float magnitude, float& a, float& b) {
+    const double angle = (double)position * frequency;
+    const double turns = rint(angle * 0.15915494309189535);
+    float s, c;
+    sincosf((float)(angle - turns * 6.283185307179586), &s, &c);
+    c *= magnitude;
+    s *= magnitude;
     a = u * c - v * s;
     b = v * c + u * s;
 }
@@ -253,11 +258,12 @@ __device__ __forceinline__ void rotated_pair(float u, float v, int position, flo
 //    query, what lies beyond rank + rot up to `row_size` is zero);
 //  - the row of dkv [rows, rank + rot]: its first `rank` elements RMS-normed with `gain`, its last `rot` rotated, stored as
 //    the row's cache line [rank | rot | zeros up to row_size] in pages [num_pages, page_size, row_size].
-// The first `rot_dims` of the rot elements are rotated, the rest pass unchanged.
+// The first `rot_dims` of the rot elements are rotated, the rest pass unchanged; pair i is elements (i, i + rot_dims / 2) or, with
+// `neighbours`, (2i, 2i + 1).
 template <typename T>
 __global__ __launch_bounds__(256) void latent_rows_kernel(const T* __restrict__ q, int q_stride, const T* __restrict__ dkv, int dkv_stride,
-                                                          const float* __restrict__ gain, float eps, const float* __restrict__ frequencies,
-                                                          float magnitude, int rot_dims, const int* __restrict__ positions,
+                                                          const float* __restrict__ gain, float eps, const double* __restrict__ frequencies,
+                                                          float magnitude, int rot_dims, int neighbours, const int* __restrict__ positions,
                                                           const int* __restrict__ slots, float* __restrict__ q_full, T* __restrict__ pages,
                                                           int n_rows, int n_heads, int dim, int rot, int rank, int row_size, int page_size) {
     const int lane = threadIdx.x % WAVE;
@@ -267,14 +273,16 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const T* __restrict__ 
     const int row = (int)(item / per_row), head = (int)(item % per_row);
     const int position = positions[row];
     const int half = rot_dims / 2;
+    const int step = neighbours ? 2 : 1, apart = neighbours ? 1 : half;   // pair i: elements i * step and i * step + apart
     if (head < n_heads) {
         const T* in = q + (size_t)row * q_stride + (size_t)head * (dim + rot) + dim;
         float* out = q_full + ((size_t)row * n_heads + head) * row_size + rank;
         for (int i = lane; i < half; i += WAVE) {
             float a, b;
-            rotated_pair(to_float(in[i]), to_float(in[i + half]), position, frequencies[i], magnitude, a, b);
-            out[i] = a;
-            out[i + half] = b;
+            const int at = i * step;
+            rotated_pair(to_float(in[at]), to_float(in[at + apart]), position, frequencies[i], magnitude, a, b);
+            out[at] = a;
+            out[at + apart] = b;
         }
         for (int i = 2 * half + lane; i < row_size - rank; i += WAVE) out[i] = i < rot ? to_float(in[i]) : 0.0f;
         return;
@@ -293,9 +301,10 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const T* __restrict__ 
     for (int d = lane; d < rank; d += WAVE) out[d] = from_float<T>(to_float(in[d]) * inverse * gain[d]);
     for (int i = lane; i < half; i += WAVE) {
         float a, b;
-        rotated_pair(to_float(in[rank + i]), to_float(in[rank + i + half]), position, frequencies[i], magnitude, a, b);
-        out[rank + i] = from_float<T>(a);
-        out[rank + i + half] = from_float<T>(b);
+        const int at = rank + i * step;
+        rotated_pair(to_float(in[at]), to_float(in[at + apart]), position, frequencies[i], magnitude, a, b);
+        out[at] = from_float<T>(a);
+        out[at + apart] = from_float<T>(b);
     }
     for (int i = 2 * half + lane; i < row_size - rank; i += WAVE) out[rank + i] = i < rot ? in[rank + i] : from_float<T>(0.0f);
 }
@@ -398,8 +407,8 @@ MLLM_API int mllm_head_norm(const void* qkv, int qkv_stride, const float* q_gain
     return mllm_check_launch("head_norm");
 }
 
-MLLM_API int mllm_latent_rows(const void* q, int q_stride, const void* dkv, int dkv_stride, const float* gain, float eps, const float* frequencies,
-                              float magnitude, int rot_dims, const int* positions, const int* slots, float* q_full, void* pages, int n_rows,
+MLLM_API int mllm_latent_rows(const void* q, int q_stride, const void* dkv, int dkv_stride, const float* gain, float eps, const double* frequencies,
+                              float magnitude, int rot_dims, int neighbours, const int* positions, const int* slots, float* q_full, void* pages, int n_rows,
                               int n_heads, int dim, int rot, int rank, int row_size, int page_size, int dtype, hipStream_t stream) {
     MLLM_REQUIRE(n_rows >= 0 && n_heads > 0 && dim > 0 && rot >= 0 && rank > 0 && page_size > 0, "latent_rows: bad sizes");
     MLLM_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= rot, "latent_rows: %d rotated elements of %d", rot_dims, rot);
@@ -414,11 +423,11 @@ MLLM_API int mllm_latent_rows(const void* q, int q_stride, const void* dkv, int 
     mllm_count_kernel(MLLM_K_LATENT_ROWS);
     if (dtype == MLLM_F32)
         latent_rows_kernel<float><<<blocks, 256, 0, stream>>>((const float*)q, q_stride, (const float*)dkv, dkv_stride, gain, eps, frequencies, magnitude,
-                                                              rot_dims, positions, slots, q_full, (float*)pages, n_rows, n_heads, dim, rot, rank,
+                                                              rot_dims, neighbours, positions, slots, q_full, (float*)pages, n_rows, n_heads, dim, rot, rank,
                                                               row_size, page_size);
     else if (dtype == MLLM_BF16)
         latent_rows_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)q, q_stride, (const bf16_t*)dkv, dkv_stride, gain, eps, frequencies,
-                                                               magnitude, rot_dims, positions, slots, q_full, (bf16_t*)pages, n_rows, n_heads, dim, rot,
+                                                               magnitude, rot_dims, neighbours, positions, slots, q_full, (bf16_t*)pages, n_rows, n_heads, dim, rot,
                                                                rank, row_size, page_size);
     else
         MLLM_REQUIRE(false, "latent_rows: unknown dtype %d", dtype);

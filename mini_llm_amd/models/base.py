@@ -13,6 +13,9 @@ from ..parts.base import Norm, Part, PositionEncoding
 from ..parts.embedding import TokenEmbedding
 
 
+EMBEDDING_STATE = "embedding"   # the state layer of an embedding that keeps state (mixers' are named by their cache layer)
+
+
 @dataclass(frozen=True)
 class LayerCall:
     block: int               # index into Model.blocks
@@ -134,12 +137,15 @@ class Model(Part):
         ]
 
     def state_needs(self) -> dict:
-        """state layer id -> StateNeed, for the mixers that keep state of fixed size."""
+        """state layer id -> StateNeed, for the mixers that keep state of fixed size, and for an embedding that does."""
         out = {}
         for call in self.schedule:
             need = self.blocks[call.block].mixer_part().state_need()
             if need is not None and call.write_cache:
                 out[call.cache] = need
+        need = self.embedding.state_need()
+        if need is not None:
+            out[EMBEDDING_STATE] = need
         return out
 
     def _layers(self, hidden, batch, cache, observer=None):
@@ -192,7 +198,8 @@ class Model(Part):
         where a difference starts (engine/include/gpt2_gpu.h:21-25). The step itself runs as without."""
         hidden = self.embedding.forward(batch.tokens, batch.positions, self.position_encoding,
                                         token_sources=batch.token_sources if resolve_tokens else None,
-                                        token_slots=cache.last_token if resolve_tokens else None)
+                                        token_slots=cache.last_token if resolve_tokens else None, batch=batch,
+                                        state=cache.state.get(EMBEDDING_STATE))
         if observer is not None:
             observer("embedding", kernels.settle(hidden))
         if lanes is not None:

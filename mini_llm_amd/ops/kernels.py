@@ -62,11 +62,29 @@ def _stream():
     return torch.cuda.current_stream().cuda_stream
 
 
-def embed(tokens, positions, wte, wpe, out=None, token_sources=None, token_slots=None, scale: float = 1.0):
+@dataclass
+class TokenPairs:
+    """A second table of an embedding, [buckets + 1, width], whose row a token picks together with the one before it in its sequence: row
+    (before * mul_previous + token * mul_current) mod buckets, and the last row for a sequence's first token (position 0).
+    ``token_request``, ``q_starts``, ``state_slots``: the batch's; ``previous``: int32, one number a state slot, the last token of the
+    sequence's portions so far."""
+
+    table: torch.Tensor
+    mul_previous: int
+    mul_current: int
+    token_request: torch.Tensor
+    q_starts: torch.Tensor
+    state_slots: torch.Tensor
+    previous: torch.Tensor
+
+
+def embed(tokens, positions, wte, wpe, out=None, token_sources=None, token_slots=None, scale: float = 1.0, pairs: TokenPairs | None = None):
     """out[t] = scale * wte[tokens[t]] + wpe[positions[t]] in float32 (``wpe`` None: the token row alone). A
     negative token gives a zero row.
     With ``token_sources`` and ``token_slots`` the token of a row whose source is not negative is
-    token_slots[source]; it is also written into ``tokens``."""
+    token_slots[source]; it is also written into ``tokens``.
+    ``pairs`` (without ``wpe``): the row of the pairs' table that a token and the one before it pick is added (TokenPairs); what it keeps
+    of every request moves on to the last token of the request's portion."""
     _device_tensor(tokens, "tokens", torch.int32, 1)
     _device_tensor(positions, "positions", torch.int32, 1)
     _device_tensor(wte, "wte", dim=2)
@@ -79,12 +97,22 @@ def embed(tokens, positions, wte, wpe, out=None, token_sources=None, token_slots
         _device_tensor(token_sources, "token_sources", torch.int32, 1)
         _device_tensor(token_slots, "token_slots", torch.int32, 1)
         _require(token_sources.shape[0] >= n, "fewer sources than tokens")
+    more = (None, 0, 0, 0, None, None, None, None)
+    if pairs is not None:
+        _require(wpe is None, "no position rows are added to token pairs")
+        _device_tensor(pairs.table, "the pairs' table", wte.dtype, 2)
+        _require(pairs.table.shape[1] == width and pairs.table.shape[0] >= 2, "the pairs' table does not match the width")
+        for t, name in ((pairs.token_request, "token_request"), (pairs.q_starts, "q_starts"), (pairs.state_slots, "state_slots"), (pairs.previous, "previous")):
+            _device_tensor(t, name, torch.int32, 1)
+        _require(pairs.token_request.shape[0] >= n and pairs.q_starts.shape[0] >= pairs.state_slots.shape[0] + 1, "the batch's arrays are too short")
+        more = (_ptr(pairs.table), int(pairs.mul_previous), int(pairs.mul_current), pairs.table.shape[0] - 1, _ptr(pairs.token_request), _ptr(pairs.q_starts),
+                _ptr(pairs.state_slots), _ptr(pairs.previous))
     if out is None:
         out = torch.empty((n, width), dtype=torch.float32, device=tokens.device)
     _device_tensor(out, "out", torch.float32, 2)
     _require(tuple(out.shape) == (n, width), "out has the wrong shape")
     check(library().mllm_embed(_ptr(tokens), _ptr(positions), _ptr(token_sources), _ptr(token_slots if token_sources is not None else None),
-                               _ptr(wte), _ptr(wpe), _ptr(out), n, width, _code(wte.dtype), float(scale), _stream()))
+                               _ptr(wte), _ptr(wpe), _ptr(out), n, width, _code(wte.dtype), float(scale), *more, _stream()))
     return out
 
 
@@ -943,12 +971,14 @@ def silu_mul(both):
     return out
 
 
-def latent_rows(q, dkv, gain, eps, frequencies, magnitude, rot_dims, positions, slots, pages, n_heads, dim, rot, rank):
+def latent_rows(q, dkv, gain, eps, frequencies, magnitude, rot_dims, positions, slots, pages, n_heads, dim, rot, rank, *, pairing: str = "half"):
     """A latent-attention layer's row-wise work. q: [rows, n_heads * (dim + rot)]; dkv: [rows, rank + rot] or None (the layer
     reads rows another layer keeps). Returns q_full, float32 [rows, n_heads, row_size] with the rotated query part at
     [rank, rank + rot) and zeros behind (the first ``rank`` elements are left for ``heads_linear``); stores, with dkv, the
     RMS-normed latent (gain [rank]) and the rotated key part at slots[row] of pages [num_pages, 1, page_size, row_size].
-    ``frequencies``: float32 [rot_dims / 2], the angle per position of each rotated pair; ``magnitude`` multiplies cos and sin."""
+    ``frequencies``: float64 [rot_dims / 2], the angle per position of each rotated pair (the angle is taken in 64-bit); ``magnitude``
+    multiplies cos and sin. ``pairing``: pair i is elements (i, i + rot_dims / 2), "half", or (2i, 2i + 1), "neighbours"."""
+    _require(pairing in ("half", "neighbours"), "pairs go by halves or by neighbours")
     _require(q.is_cuda and q.dim() == 2 and q.stride(1) == 1, "q must be a 2-D GPU tensor with contiguous columns")
     _device_tensor(pages, "pages", q.dtype, 4)
     _require(pages.shape[1] == 1, "a latent cache has one row per token")
@@ -959,14 +989,14 @@ def latent_rows(q, dkv, gain, eps, frequencies, magnitude, rot_dims, positions, 
         _require(dkv.is_cuda and dkv.dim() == 2 and dkv.stride(1) == 1 and dkv.dtype == q.dtype and tuple(dkv.shape) == (n, rank + rot), "dkv does not match the latent")
         _device_tensor(gain, "gain", torch.float32, 1)
         _require(gain.shape[0] == rank, "the gain vector does not match the latent")
-    _device_tensor(frequencies, "frequencies", torch.float32, 1)
+    _device_tensor(frequencies, "frequencies", torch.float64, 1)
     _require(rot_dims % 2 == 0 and rot_dims <= rot and frequencies.shape[0] >= rot_dims // 2, "the rotation does not fit the rotated part")
     _device_tensor(positions, "positions", torch.int32, 1)
     _device_tensor(slots, "slots", torch.int32, 1)
     _require(positions.shape[0] >= n and slots.shape[0] >= n, "fewer positions or slots than rows")
     q_full = torch.empty((n, n_heads, row_size), dtype=torch.float32, device=q.device)
     check(library().mllm_latent_rows(_ptr(q), q.stride(0), _ptr(dkv), 0 if dkv is None else dkv.stride(0), _ptr(gain if dkv is not None else None), float(eps),
-                                     _ptr(frequencies), float(magnitude), int(rot_dims), _ptr(positions), _ptr(slots), _ptr(q_full), _ptr(pages), n, n_heads,
+                                     _ptr(frequencies), float(magnitude), int(rot_dims), int(pairing == "neighbours"), _ptr(positions), _ptr(slots), _ptr(q_full), _ptr(pages), n, n_heads,
                                      dim, rot, rank, row_size, page_size, _code(q.dtype), _stream()))
     return q_full
 
@@ -974,7 +1004,7 @@ def latent_rows(q, dkv, gain, eps, frequencies, magnitude, rot_dims, positions, 
 def heads_linear(x, weight, out, *, n_heads, k, x_head_stride, n_out=None, gate=None):
     """out[row, h, :n] = x[row, h, :k] @ weight[h].T (* sigmoid(gate[row, h, :n])): one small product per head. x: 2-D or 3-D,
     its rows ``x.stride(0)`` apart and its heads ``x_head_stride``; weight: [n_heads, n, k]; out: [rows, n_heads, >= n] (a view
-    whose last elements may belong to someone else); gate: [rows, n_heads * n]."""
+    whose last elements may belong to someone else); gate: [rows, n_heads * n], or [rows, n_heads], one number a head."""
     _require(x.is_cuda and x.stride(-1) == 1, "x must be on the GPU with contiguous elements")
     _device_tensor(weight, "weight", dim=3)
     _require(weight.shape[0] == n_heads and weight.shape[2] == k, "weight does not match the heads")
@@ -984,9 +1014,11 @@ def heads_linear(x, weight, out, *, n_heads, k, x_head_stride, n_out=None, gate=
     _require(out.shape[0] == rows, "x and out differ in rows")
     _require(x.stride(0) >= (n_heads - 1) * x_head_stride + k, "x's rows are too short for the heads")
     if gate is not None:
-        _require(gate.is_cuda and gate.dim() == 2 and gate.stride(1) == 1 and tuple(gate.shape) == (rows, n_heads * n), "the gate does not match the output")
+        _require(gate.is_cuda and gate.dim() == 2 and gate.stride(1) == 1 and tuple(gate.shape) in ((rows, n_heads * n), (rows, n_heads)),
+                 "the gate does not match the output")
     check(library().mllm_heads_linear(_ptr(x), _code(x.dtype), x.stride(0), int(x_head_stride), _ptr(weight), _code(weight.dtype), _ptr(gate),
-                                      0 if gate is None else _code(gate.dtype), 0 if gate is None else gate.stride(0), _ptr(out), _code(out.dtype), out.stride(0), out.stride(1), rows, n_heads,
+                                      0 if gate is None else _code(gate.dtype), 0 if gate is None else gate.stride(0),
+                                      int(gate is not None and gate.shape[1] == n_heads), _ptr(out), _code(out.dtype), out.stride(0), out.stride(1), rows, n_heads,
                                       n, k, _stream()))
     return out
 
@@ -1300,11 +1332,14 @@ def gate_unit(both, limit: float | None = None, alpha: float = 1.0, shift: float
 ROUTE_MAX_EXPERTS = 1024
 
 
-def route(logits, n_experts: int, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0):
+def route(logits, n_experts: int, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0, score: str = "softmax",
+          renormalise: bool = True):
     """A router's choice, row by row. ``logits``: float32 rows whose first ``n_experts`` columns are the router's sums (rows may be
-    strided). Scores are their softmax over all experts; the choice goes by score + correction (float32 [n_experts]; None: by the score)
+    strided). Scores are their softmax over all experts or, with ``score`` "sigmoid", each one's own sigmoid; the choice goes by score + correction (float32 [n_experts]; None: by the score)
     among the experts of the ``keep`` best of ``n_groups`` equal groups of neighbours (a group counts by its best choice score); the ``top``
-    best are picked. Returns float32 [rows, n_experts]: a picked expert's score over (the sum of the picked scores + floor), zero for the rest."""
+    best are picked. Returns float32 [rows, n_experts]: a picked expert's score over (the sum of the picked scores + floor), without
+    ``renormalise`` its score itself, zero for the rest."""
+    _require(score in ("softmax", "sigmoid"), "scores are a softmax or sigmoids")
     _require(isinstance(logits, torch.Tensor) and logits.is_cuda and logits.dim() == 2 and logits.dtype == torch.float32 and logits.stride(1) == 1
              and logits.shape[1] >= n_experts, "the router's sums must be float32 GPU rows with contiguous columns")
     _require(1 <= n_experts <= ROUTE_MAX_EXPERTS, f"the router kernel takes up to {ROUTE_MAX_EXPERTS} experts")
@@ -1316,7 +1351,7 @@ def route(logits, n_experts: int, top: int, *, correction=None, n_groups: int = 
     n = logits.shape[0]
     weights = torch.empty((n, n_experts), dtype=torch.float32, device=logits.device)
     check(library().mllm_route(_ptr(logits), logits.stride(0), _ptr(correction), _ptr(weights), n_experts, n, n_experts, int(top), int(n_groups), int(keep),
-                               float(floor), _stream()))
+                               float(floor), int(score == "sigmoid"), int(bool(renormalise)), _stream()))
     return weights
 
 
@@ -1343,6 +1378,51 @@ def expert_unit(up, weights, n_routed: int, ff: int, shared: int = 0, *, h=None,
     check(library().mllm_expert_unit(_ptr(up), _ptr(out), _ptr(weights), weights.stride(0), n, int(n_routed), int(ff), int(shared), _ptr(h if n_identity else None),
                                      _ptr(carried), int(n_identity), int(width), _code(up.dtype), _stream()))
     return out, carried
+
+
+def gated_expert_unit(both, weights, n_experts: int, ff: int, *, limit: float | None = None, alpha: float = 1.0, shift: float = 0.0, weigh_input: bool = False):
+    """``expert_unit`` for experts with a gate unit (``gate_unit``): ``both`` [rows, n_experts * 2 * ff], per expert the sums of its gate and
+    of its up matrix -> [rows, n_experts * ff], the unit times the row's weight for the expert, or with ``weigh_input`` the unit of the
+    sums times that weight (the experts of weight * h instead of weight * the experts of h). Experts of weight zero give zeros."""
+    _device_tensor(both, "both", dim=2)
+    n = both.shape[0]
+    _require(both.shape[1] == 2 * n_experts * ff, "the hidden units do not match the experts")
+    _require(limit is None or limit > 0, "the limit must be positive")
+    _require(isinstance(weights, torch.Tensor) and weights.is_cuda and weights.dim() == 2 and weights.dtype == torch.float32 and weights.stride(1) == 1
+             and weights.shape[0] == n and weights.shape[1] >= n_experts, "the weights must be float32 GPU rows, one column an expert")
+    out = torch.empty((n, n_experts * ff), dtype=both.dtype, device=both.device)
+    check(library().mllm_gated_expert_unit(_ptr(both), _ptr(out), _ptr(weights), weights.stride(0), n, int(n_experts), int(ff),
+                                           float("inf") if limit is None else float(limit), float(alpha), float(shift), int(bool(weigh_input)), _code(both.dtype),
+                                           _stream()))
+    return out
+
+
+def gated_scan(rows, z_at: int, x_at: int, g_at: int, width: int, state, q_starts, state_slots, out_dtype, *, shift: float, max_q_len: int | None = None):
+    """A gated recurrence whose gates read the current row alone (minGRU). ``rows``: the float32 sums of a fused product (rows may be
+    strided) holding ``width`` columns each of the update gate's sums p (at ``z_at``), the candidate's u (``x_at``) and the output gate's g
+    (``g_at``), biases inside. With z = sigmoid(p), c = u + shift where u >= 0 and sigmoid(u) where u < 0: S <- (1 - z) S + z c, and the
+    result S * silu(g), [rows, width] of ``out_dtype``. ``state``: float32 [slots, width] (rows may be strided), moved on in place;
+    request r's rows are q_starts[r] .. q_starts[r + 1], its slot state_slots[r] (negative: passed by, its rows of the result are undefined).
+    ``max_q_len``: the longest portion of the batch, or a bound on it: long portions run as chunks side by side."""
+    _require(isinstance(rows, torch.Tensor) and rows.is_cuda and rows.dim() == 2 and rows.dtype == torch.float32 and rows.stride(1) == 1,
+             "the rows must be float32 GPU rows with contiguous columns")
+    _require(all(0 <= at and at + width <= rows.shape[1] for at in (z_at, x_at, g_at)), "the columns lie beyond the rows")
+    _require(state.is_cuda and state.dim() == 2 and state.dtype == torch.float32 and state.stride(1) == 1 and state.shape[1] >= width,
+             "the state must be float32 rows on the GPU")
+    _device_tensor(q_starts, "q_starts", torch.int32, 1)
+    _device_tensor(state_slots, "state_slots", torch.int32, 1)
+    n, n_requests = rows.shape[0], state_slots.shape[0]
+    _require(q_starts.shape[0] >= n_requests + 1, "q_starts must have one entry more than there are requests")
+    longest = n if max_q_len is None else max(1, min(int(max_q_len), n))
+    out = torch.empty((n, width), dtype=out_dtype, device=rows.device)
+    chunk = int(library().mllm_gated_scan_chunk_rows())
+    records = None
+    if longest > chunk:
+        records = torch.empty(((n // chunk + n_requests + 1) * 2 * width,), dtype=torch.float32, device=rows.device)
+    check(library().mllm_gated_scan(_ptr(rows), rows.stride(0), int(z_at), int(x_at), int(g_at), _ptr(state), state.stride(0), _ptr(q_starts), _ptr(state_slots),
+                                    _ptr(out), out.stride(0), n, n_requests, int(width), float(shift), longest, _ptr(records),
+                                    0 if records is None else records.numel(), _code(out_dtype), _stream()))
+    return out
 
 
 def branch_join(stream, a, b=None, *, a_bias=None, b_bias=None, scale_a=None, scale_b=None, gates=None, gate_a_at: int = 0, gate_b_at: int = 0,

@@ -15,7 +15,7 @@ _library: ctypes.CDLL | None = None
 
 P = c_void_p
 _SIGNATURES = {
-    "mllm_embed": [P, P, P, P, P, P, P, c_int, c_int, c_int, c_float, P],
+    "mllm_embed": [P, P, P, P, P, P, P, c_int, c_int, c_int, c_float, P, c_longlong, c_longlong, c_int, P, P, P, P, P],
     "mllm_layernorm": [P, P, P, P, P, c_int, c_int, c_float, c_int, c_int, P],
     "mllm_add": [P, P, P, c_longlong, c_int, P],
     "mllm_gemm": [P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
@@ -49,18 +49,21 @@ _SIGNATURES = {
     "mllm_pending_layernorm": [P, P, P, c_int, c_int, P, P, P, P, P, c_int, c_int, c_float, c_int, c_int, P],
     "mllm_rms_norm": [P, P, c_int, c_float, P, P, c_int, c_float, P, P, c_int, c_int, c_int, c_int, c_longlong, P, P, P],
     "mllm_head_norm": [P, c_int, P, P, c_float, c_float, c_int, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_latent_rows": [P, c_int, P, c_int, P, c_float, P, c_float, c_int, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
+    "mllm_latent_rows": [P, c_int, P, c_int, P, c_float, P, c_float, c_int, c_int, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_silu_mul": [P, P, c_int, c_int, c_int, P],
     "mllm_map_rows": [P, c_int, c_int, c_int, c_int, P, P, c_float, P, c_int, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                       c_int, P, c_int, c_int, P],
     "mllm_turn_heads": [P, c_int, P, c_int, P, c_int, c_int, c_float, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_route": [P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, P],
+    "mllm_route": [P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, P],
     "mllm_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P],
+    "mllm_gated_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_int, P],
+    "mllm_gated_scan": [P, c_int, c_int, c_int, c_int, P, c_longlong, P, P, P, c_int, c_int, c_int, c_int, c_float, c_int, P, c_longlong, P],
+    "mllm_gated_scan_chunk_rows": [],
     "mllm_gate_unit": [P, P, c_int, c_int, c_float, c_float, c_float, c_int, P],
     "mllm_branch_join": [P, P, c_int, c_longlong, P, P, c_int, c_longlong, P, P, P, P, c_int, c_int, c_int, c_float, P, P, c_int, c_float, P, c_int,
                          c_int, c_int, P],
     "mllm_map_difference": [P, c_int, P, c_int, P, c_int, c_float, c_float, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_heads_linear": [P, c_int, c_int, c_int, P, c_int, P, c_int, c_int, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
+    "mllm_heads_linear": [P, c_int, c_int, c_int, P, c_int, P, c_int, c_int, c_int, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_latent_attention_supported": [c_int, c_int, c_int],
     "mllm_latent_attention_head_group": [c_int],
     "mllm_latent_mfma_row_size": [c_int],

@@ -4,7 +4,7 @@ from __future__ import annotations
 
 from ..ops import kernels
 from ..weights.spec import MATRIX, TABLE, Normal, TensorSpec
-from .base import Part, PositionEncoding
+from .base import Part, PositionEncoding, StateNeed
 
 
 class TokenEmbedding(Part):
@@ -22,14 +22,50 @@ class TokenEmbedding(Part):
     def bind(self, tensors):
         self.weight = tensors[self._tensor_name]
 
-    def forward(self, tokens, positions, position_encoding: PositionEncoding | None, token_sources=None, token_slots=None):
+    def state_need(self) -> StateNeed | None:
+        """What the embedding keeps of a sequence from step to step (nothing: a row is a function of its token and position)."""
+        return None
+
+    def forward(self, tokens, positions, position_encoding: PositionEncoding | None, token_sources=None, token_slots=None, batch=None, state=None):
         """[rows, width] float32: token rows, with the position rows added when the encoding
         is one that enters at the embedding (a table ``weight`` [positions, width]); an encoding
         of stage "mixer", or none, leaves the token rows as they are. ``token_sources`` /
         ``token_slots``: rows whose token is still on the device, in the slot the sampler left it
-        in (kernels.embed)."""
+        in (kernels.embed). ``batch`` / ``state``: the step's batch and the slots of ``state_need``, for an embedding that keeps state."""
         table = position_encoding.weight if position_encoding is not None and position_encoding.stage == "embedding" else None
         return kernels.embed(tokens, positions, self.weight, table, token_sources=token_sources, token_slots=token_slots, scale=self.scale)
+
+
+class PairEmbedding(TokenEmbedding):
+    """A token's row plus a row of a second table [buckets + 1, width] picked by the token and the one before it in its sequence: row
+    (previous * mul_previous + token * mul_current) mod buckets, and the last row for a sequence's first token. The previous token of
+    a portion's first row is part of the sequence's state: one integer a state slot, read and moved on to the portion's last token
+    inside the gather, also where that token is still on the device. ``pair_name``: the second table's name behind the part's prefix."""
+
+    def __init__(self, vocab_size: int, width: int, *, buckets: int, mul_previous: int, mul_current: int, scale: float = 1.0,
+                 tensor_name: str = "weight", pair_name: str = "pairs", std: float = 0.02):
+        super().__init__(vocab_size, width, scale=scale, tensor_name=tensor_name, std=std)
+        self.buckets, self.mul_previous, self.mul_current = buckets, mul_previous, mul_current
+        self._pair_name = pair_name
+        self.pairs = None
+
+    def tensor_specs(self):
+        return {**super().tensor_specs(), self._pair_name: TensorSpec((self.buckets + 1, self.width), TABLE, Normal(self._std))}
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        self.pairs = tensors[self._pair_name]
+
+    def state_need(self):
+        import torch
+
+        return StateNeed((), torch.int32)
+
+    def forward(self, tokens, positions, position_encoding: PositionEncoding | None, token_sources=None, token_slots=None, batch=None, state=None):
+        if position_encoding is not None and position_encoding.stage == "embedding":
+            raise ValueError("no position rows are added to token pairs")
+        pairs = kernels.TokenPairs(self.pairs, self.mul_previous, self.mul_current, batch.token_request, batch.q_starts, batch.state_slots, state)
+        return kernels.embed(tokens, positions, self.weight, None, token_sources=token_sources, token_slots=token_slots, scale=self.scale, pairs=pairs)
 
 
 class TiedHead(Part):

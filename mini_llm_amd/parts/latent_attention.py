@@ -4,7 +4,8 @@ part of ``rot_dim`` elements, shared by all heads, instead of keys and values pe
 In formulas (h the layer's input, H heads): q = W_q h, per head [dim plain | rot_dim rotated]; [c' | k_r'] = W_dkv h, c =
 rmsnorm(c') * g, k_r = rotate(k_r'); head i's key is [W_uk,i c | k_r] and its value W_uv,i c; score = scale * (q_plain . k_plain
 + rotate(q_rot) . k_r); causal softmax whose denominator also holds exp(sink_i); the heads' outputs, laid behind each other,
-are multiplied by sigmoid(W_g h) and go through W_o. A layer built with ``own_latent=False`` has no W_dkv: it reads the rows that
+are multiplied by sigmoid(W_g h) and go through W_o (``gate`` "elements": W_g has a row for every element of every head; "heads": a
+row a head, one number for all its elements; None: no gate). A layer built with ``own_latent=False`` has no W_dkv: it reads the rows that
 the layer whose cache it is given has stored, with its own W_uk, W_uv and queries.
 
 Keys and values are never expanded: W_uk is folded into the query (q'_i = W_uk,i^T q_plain,i, so that a score is a dot product
@@ -17,7 +18,7 @@ import torch
 from ..ops import kernels
 from ..weights.spec import TABLE, VECTOR, Normal, TensorSpec
 from .base import KVNeed, LayerContext, Mixer, register_part
-from .linear import BranchProduct
+from .linear import BranchProduct, fuse_rows
 from .positions import RotaryEncoding
 
 
@@ -25,12 +26,15 @@ class LatentAttention(Mixer):
     graph_safe = True
 
     def __init__(self, width: int, n_heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, scale: float, eps: float,
-                 rotary: RotaryEncoding, sink: bool = True, gated: bool = True, own_latent: bool = True):
+                 rotary: RotaryEncoding, sink: bool = True, gate: str | None = "elements", own_latent: bool = True):
+        if gate not in (None, "elements", "heads"):
+            raise ValueError(f"unknown gate {gate!r}: elements, heads or None")
         if rotary.dims > rot_dim:
             raise ValueError(f"{rotary.dims} rotated elements do not fit a rotated part of {rot_dim}")
         self.width, self.n_heads, self.dim, self.rot_dim, self.vdim, self.kv_rank = width, n_heads, dim, rot_dim, vdim, kv_rank
         self.scale, self.eps, self.rotary = float(scale), float(eps), rotary
-        self.has_sink, self.gated, self.own_latent = sink, gated, own_latent
+        self.has_sink, self.own_latent = sink, own_latent
+        self.gate_rows = {None: 0, "elements": n_heads * vdim, "heads": n_heads}[gate]
         # a cached row: [latent | rotated key part | zeros up to a size the attention kernels take]
         self.row_size = kernels.latent_row_size(kv_rank + rot_dim)
         self.w_in = self.uk_t = self.uv = self.o = self.sink = self.dkv_norm = None
@@ -47,14 +51,14 @@ class LatentAttention(Mixer):
             specs["dkv.norm"] = TensorSpec((self.kv_rank,), VECTOR, Normal(0.1, mean=1.0))
         if self.has_sink:
             specs["sink"] = TensorSpec((H,), VECTOR, Normal(1.0))
-        if self.gated:
-            specs["g"] = TensorSpec((H * self.vdim, self.width), TABLE, Normal(std))
+        if self.gate_rows:
+            specs["g"] = TensorSpec((self.gate_rows, self.width), TABLE, Normal(std))
         return specs
 
     def bind(self, tensors):
         H = self.n_heads
         # one product for everything that reads the layer's input: [q | dkv | g]
-        fused = torch.cat([tensors[name] for name in ("q", "dkv", "g") if name in tensors], dim=0).contiguous()
+        fused = fuse_rows([tensors[name] for name in ("q", "dkv", "g") if name in tensors])
         on_gpu = fused.is_cuda
         self.w_in = kernels.pack_matrix(fused) if on_gpu else fused
         self.uk_t = tensors["uk"].view(H, self.dim, self.kv_rank).transpose(1, 2).contiguous()   # [H, rank, dim]: q' = uk_t q
@@ -77,9 +81,9 @@ class LatentAttention(Mixer):
         dkv = None
         if self.own_latent:
             dkv, at = fused[:, at : at + kept], at + kept
-        gate = fused[:, at:] if self.gated else None
-        q_full = kernels.latent_rows(q, dkv, self.dkv_norm, self.eps, self.rotary.frequencies(x.device), self.rotary.magnitude, self.rotary.dims,
-                                     batch.positions, ctx.group.slots, ctx.k_pages, H, self.dim, self.rot_dim, self.kv_rank)
+        gate = fused[:, at : at + self.gate_rows] if self.gate_rows else None
+        q_full = kernels.latent_rows(q, dkv, self.dkv_norm, self.eps, self.rotary.frequencies64(x.device), self.rotary.magnitude, self.rotary.dims,
+                                     batch.positions, ctx.group.slots, ctx.k_pages, H, self.dim, self.rot_dim, self.kv_rank, pairing=self.rotary.pairing)
         kernels.heads_linear(q, self.uk_t, q_full, n_heads=H, k=self.dim, x_head_stride=self.dim + self.rot_dim)
         whole = getattr(batch, "first_row", 0) == 0   # a part of a batch numbers its rows from the whole batch's top
         summed = kernels.latent_attention(q_full, ctx.k_pages, self.sink, batch.token_request, batch.positions, ctx.group.block_tables,

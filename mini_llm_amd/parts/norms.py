@@ -36,22 +36,26 @@ class RMSNorm(Norm):
     """x / sqrt(mean(x^2) + eps) * g, in 32-bit. ``one_plus``: the stored vector lies around zero and g = 1 + weight.
     ``tensor_name``: the vector's name behind the part's prefix ("" where the part's own name is the tensor's). ``out_scale``: a
     constant that multiplies the normed rows, folded into the 32-bit gain when the weights are bound (a model whose logits are scaled
-    gives its final norm the scale: the head's product is linear)."""
+    gives its final norm the scale: the head's product is linear). ``one_gain``: the file holds one number, the gain of every element;
+    it is laid out as a vector when it is bound, so that the kernels know one kind of gain."""
 
-    def __init__(self, width: int, eps: float, one_plus: bool = False, tensor_name: str = "weight", out_scale: float = 1.0):
+    def __init__(self, width: int, eps: float, one_plus: bool = False, tensor_name: str = "weight", out_scale: float = 1.0,
+                 one_gain: bool = False):
         if not eps > 0:
             raise ValueError(f"eps must be positive, not {eps}")
         if out_scale != 1.0 and one_plus:
             raise ValueError("a scale is folded into a plain gain vector, not into one stored around zero")
-        self.width, self.eps, self.one_plus, self.out_scale = width, float(eps), bool(one_plus), float(out_scale)
+        self.width, self.eps, self.one_plus, self.out_scale, self.one_gain = width, float(eps), bool(one_plus), float(out_scale), bool(one_gain)
         self._tensor_name = tensor_name
         self.weight = None
 
     def tensor_specs(self):
-        return {self._tensor_name: TensorSpec((self.width,), VECTOR, Normal(0.05, mean=0.0 if self.one_plus else 1.0))}
+        return {self._tensor_name: TensorSpec(() if self.one_gain else (self.width,), VECTOR, Normal(0.05, mean=0.0 if self.one_plus else 1.0))}
 
     def bind(self, tensors):
         self.weight = tensors[self._tensor_name]
+        if self.one_gain:
+            self.weight = self.weight.reshape(1).expand(self.width).contiguous()
         if self.out_scale != 1.0:
             self.weight = (self.weight.double() * self.out_scale).float()
 

@@ -14,6 +14,10 @@ Both: one product makes everything that reads h (32-bit sums), ``kernels.recurre
 the state its slot holds (zero at admission), ``kernels.gated_norm`` norms and gates. State, gates and sums are 32-bit in every
 precision.
 
+``MinGRUMixer``: a vector per request; z = sigmoid(W_z h + b_z), u = W_x h + b_x, candidate c = u + shift where u >= 0 and sigmoid(u) where u
+< 0; S_t = (1 - z) S_(t-1) + z c element by element, and W_o (S_t * silu(W_g h)). The gates read the current row alone, so a portion is
+a scan (``kernels.gated_scan``).
+
 ``ParallelMixer``: left_scale * left(h) + right_scale * right(h), two mixers of the framework reading the same rows. Each folds
 its scale into its last elementwise kernel, and the second one's output product adds the first one's result, so the sum costs no
 kernel of its own."""
@@ -137,6 +141,46 @@ class DecayedLinearAttention(Mixer):
         return self._out_product(mixed, self.o, residual)
 
 
+class MinGRUMixer(Mixer):
+    graph_safe = True
+
+    def __init__(self, width: int, state_width: int, candidate_shift: float):
+        self.width, self.state_width, self.candidate_shift = width, state_width, float(candidate_shift)
+        self.w_in = self.b_in = self.o = None
+        self._out_product = BranchProduct()
+
+    def tensor_specs(self):
+        S, std = self.state_width, self.width ** -0.5
+        return {"z": TensorSpec((S, self.width), TABLE, Normal(std)),
+                "z.b": TensorSpec((S,), VECTOR, Normal(1.0, mean=-2.0)),
+                "x": TensorSpec((S, self.width), TABLE, Normal(std)),
+                "x.b": TensorSpec((S,), VECTOR, Normal(0.4)),
+                "g": TensorSpec((S, self.width), TABLE, Normal(std)),
+                "o": TensorSpec((self.width, S), TABLE, Normal(S ** -0.5))}
+
+    def bind(self, tensors):
+        S = self.state_width
+        fused = fuse_rows([tensors[name] for name in ("z", "x", "g")])
+        on_gpu = fused.is_cuda
+        self.w_in = kernels.pack_matrix(fused) if on_gpu else fused
+        self.b_in = torch.zeros((fused.shape[0],), dtype=torch.float32, device=fused.device)
+        self.b_in[:S] = tensors["z.b"]
+        self.b_in[S : 2 * S] = tensors["x.b"]
+        self.o = kernels.pack_matrix(tensors["o"].contiguous()) if on_gpu else tensors["o"]
+
+    def state_need(self):
+        return StateNeed((self.state_width,), torch.float32)
+
+    def forward(self, x, residual, ctx: LayerContext):
+        """The branch alone (float32) when ``residual`` is None, else residual + branch."""
+        batch, S = ctx.batch, self.state_width
+        _whole_batch(batch)
+        fused = kernels.linear(x, self.w_in, self.b_in, out_dtype=torch.float32)
+        mixed = kernels.gated_scan(fused, 0, S, 2 * S, S, ctx.state, batch.q_starts, batch.state_slots, x.dtype, shift=self.candidate_shift,
+                                   max_q_len=batch.max_q_len)
+        return self._out_product(mixed, self.o, residual)
+
+
 class ParallelMixer(Mixer):
     """``left`` and ``right`` are built with their share of the sum as their ``out_scale``. At most one of them keeps keys and
     values in pages; the state slots of both lie behind each other in one slot."""
@@ -182,4 +226,5 @@ class ParallelMixer(Mixer):
 
 register_part("mixer", "matrix_memory", MatrixMemoryMixer)
 register_part("mixer", "decayed_linear_attention", DecayedLinearAttention)
+register_part("mixer", "mingru", MinGRUMixer)
 register_part("mixer", "parallel", ParallelMixer)

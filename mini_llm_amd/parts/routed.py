@@ -1,12 +1,18 @@
 """A feed-forward of routed experts: many small feed-forwards of which a router picks a few for every row.
 
-With h the layer's input and E = ``n_experts`` + ``n_identity`` router outputs: z = W_router h in 32-bit, scores s = softmax(z) over all E.
+The plain form first. With h the layer's input and E = ``n_experts`` + ``n_identity`` router outputs: z = W_router h in 32-bit, scores s = softmax(z) over all E.
 The choice goes by s + ``correction`` (a stored vector; the weights do not see it): the experts form ``n_groups`` equal groups of
 neighbours, a group counts by the largest choice score in it, only experts of the best ``keep`` groups can be picked, and the ``top``
 largest choice scores among those are. The picked experts' weights are their scores s over (their sum + ``floor``). Expert e is W_down,e
 act(W_up,e h) with act the square of relu, no biases; the last ``n_identity`` router outputs are experts without tensors whose result is
 h itself. The result is the weighted sum over the picked experts, plus (``shared_ff``) one more expert of the same form that every row
 uses with weight 1.
+
+Other designs' forms: ``score`` "sigmoid" takes s = sigmoid(z), each expert's own; ``renormalise`` False keeps the picked scores as they are;
+``correction`` False picks by the scores; ``unit`` "clamped_gate" gives an expert a gate matrix beside its up matrix (stored ``gate``, ``up``,
+``down``) and the unit g * sigmoid(alpha g) * (u + shift), g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit), in place of the squared
+relu; ``weigh`` "input" multiplies an expert's input by its weight instead of its output (the same thing only for linear experts): the
+gate unit then takes the weight times the sums.
 
 All experts run as ONE up product over their matrices laid behind each other (the shared expert's last) and ONE down product over their
 down matrices laid side by side: ``kernels.expert_unit`` between the two multiplies every hidden unit by its expert's weight for the
@@ -27,7 +33,16 @@ from .linear import BranchProduct, fuse_rows
 
 class RoutedExperts(FeedForward):
     def __init__(self, width: int, n_experts: int, ff: int, top: int, *, n_identity: int = 0, n_groups: int = 1, keep: int = 1,
-                 correction: bool = True, shared_ff: int | None = None, floor: float = 0.0):
+                 correction: bool = True, shared_ff: int | None = None, floor: float = 0.0, score: str = "softmax", renormalise: bool = True,
+                 unit: str = "squared_relu", limit: float | None = None, alpha: float = 1.0, shift: float = 0.0, weigh: str = "output"):
+        if score not in ("softmax", "sigmoid") or unit not in ("squared_relu", "clamped_gate") or weigh not in ("output", "input"):
+            raise ValueError(f"unknown score {score!r}, unit {unit!r} or weigh {weigh!r}")
+        if unit == "clamped_gate" and (n_identity or shared_ff or n_experts < 1):
+            raise ValueError("experts with a gate unit go without shared experts and without experts that hand their input on")
+        if unit != "clamped_gate" and (limit is not None or weigh == "input"):
+            raise ValueError("a limit and weights on the input go with experts that have a gate unit")
+        if limit is not None and not limit > 0:
+            raise ValueError(f"the limit must be positive, not {limit}")
         total = n_experts + n_identity
         if n_experts < 0 or n_identity < 0 or total < 1 or total > kernels.ROUTE_MAX_EXPERTS:
             raise ValueError(f"{n_experts} experts and {n_identity} that hand their input on: the router takes 1 to {kernels.ROUTE_MAX_EXPERTS} outputs")
@@ -38,6 +53,8 @@ class RoutedExperts(FeedForward):
         self.width, self.n_experts, self.ff, self.top, self.n_identity = width, n_experts, ff, top, n_identity
         self.n_groups, self.keep, self.has_correction, self.shared_ff, self.floor = n_groups, keep, bool(correction), shared_ff or 0, float(floor)
         self.n_outputs = total
+        self.score, self.renormalise, self.weigh_input = score, bool(renormalise), weigh == "input"
+        self.gated, self.limit, self.alpha, self.shift = unit == "clamped_gate", limit, float(alpha), float(shift)
         self.router = self.correction = self.up = self.down = self._router_rows = None
         self.shared_units = 0   # the shared expert's hidden units and the zeros that fill the up matrix to whole blocks
         self._down_product = BranchProduct()
@@ -53,6 +70,8 @@ class RoutedExperts(FeedForward):
             names.append("shared.")
             sizes.append(self.shared_ff)
         for name, size in zip(names, sizes):
+            if self.gated:
+                specs[name + "gate"] = TensorSpec((size, self.width), TABLE, Normal(self.width ** -0.5))
             specs[name + "up"] = TensorSpec((size, self.width), TABLE, Normal(self.width ** -0.5))
             specs[name + "down"] = TensorSpec((self.width, size), TABLE, Normal(size ** -0.5))
         return specs
@@ -63,6 +82,9 @@ class RoutedExperts(FeedForward):
         self._router_rows = router
         self.router = kernels.pack_matrix(router) if router.is_cuda else router
         self.correction = tensors.get("correction")
+        if self.gated:
+            self._bind_gated(tensors, names)
+            return
         up = fuse_rows([tensors[name + "up"] for name in names]) if names else None
         if up is None:
             return
@@ -74,6 +96,18 @@ class RoutedExperts(FeedForward):
         down = down.contiguous()
         self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
 
+    def _bind_gated(self, tensors, names):
+        up = torch.cat([tensors[name + part] for name in names for part in ("gate", "up")], dim=0).contiguous()
+        down = torch.cat([tensors[name + "down"] for name in names], dim=1).contiguous()
+        self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
+
+    def _forward_gated(self, x, weights, residual):
+        units = kernels.gated_expert_unit(kernels.linear(x, self.up), weights, self.n_experts, self.ff, limit=self.limit, alpha=self.alpha, shift=self.shift,
+                                          weigh_input=self.weigh_input)
+        if residual is None and self.sums_later:
+            return self._down_product.later(units, self.down)
+        return self._down_product(units, self.down, residual)
+
     def rows_to_carry(self):
         """The router's matrix (and no bias), for a block that lets another product over the same input rows carry it along; ``forward`` is
         then given the router's sums as ``carried``."""
@@ -81,7 +115,10 @@ class RoutedExperts(FeedForward):
 
     def forward(self, x, residual, carried=None):
         logits = carried if carried is not None else kernels.linear(x, self.router, out_dtype=torch.float32)
-        weights = kernels.route(logits, self.n_outputs, self.top, correction=self.correction, n_groups=self.n_groups, keep=self.keep, floor=self.floor)
+        weights = kernels.route(logits, self.n_outputs, self.top, correction=self.correction, n_groups=self.n_groups, keep=self.keep, floor=self.floor,
+                                score=self.score, renormalise=self.renormalise)
+        if self.gated:
+            return self._forward_gated(x, weights, residual)
         if self.up is None:   # nothing but experts that hand their input on
             raise ValueError("a routed feed-forward needs at least one expert with matrices")
         if residual is None and self.sums_later:

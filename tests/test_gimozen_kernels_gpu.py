@@ -140,7 +140,7 @@ def test_latent_rows_rotate_and_keep(dtype, heads, dim, rot, rot_dims, rank):
     dkv = rounded(rng.normal(0, 1, (rows, rank + rot)), dtype)
     gain = rng.normal(1, 0.2, rank)
     pages = torch.full((n_pages, 1, page_size, row_size), 7.0, dtype=dtype).cuda()
-    q_full = k.latent_rows(gpu(q, dtype), gpu(dkv, dtype), gpu(gain), eps, part.frequencies("cuda"), part.magnitude, rot_dims,
+    q_full = k.latent_rows(gpu(q, dtype), gpu(dkv, dtype), gpu(gain), eps, part.frequencies64("cuda"), part.magnitude, rot_dims,
                            torch.tensor(positions, dtype=torch.int32).cuda(), torch.tensor(slots, dtype=torch.int32).cuda(), pages, heads, dim, rot, rank)
     rotate = (lambda x: plain.rotate_half(x, positions, rot_config)) if rot_dims else (lambda x: x)
     want_q = rotate(q.reshape(rows, heads, dim + rot)[:, :, dim:])
@@ -159,7 +159,7 @@ def test_latent_rows_rotate_and_keep(dtype, heads, dim, rot, rot_dims, rank):
     assert (np.delete(kept, [s for s in slots if s >= 0], axis=0) == 7).all()
     # a layer that borrows another's rows stores nothing
     before = pages.clone()
-    k.latent_rows(gpu(q, dtype), None, None, eps, part.frequencies("cuda"), part.magnitude, rot_dims, torch.tensor(positions, dtype=torch.int32).cuda(),
+    k.latent_rows(gpu(q, dtype), None, None, eps, part.frequencies64("cuda"), part.magnitude, rot_dims, torch.tensor(positions, dtype=torch.int32).cuda(),
                   torch.tensor(slots, dtype=torch.int32).cuda(), pages, heads, dim, rot, rank)
     assert torch.equal(before, pages)
 

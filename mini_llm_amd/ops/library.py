@@ -57,7 +57,7 @@ _SIGNATURES = {
     "mllm_route": [P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, P],
     "mllm_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P],
     "mllm_gated_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_int, P],
-    "mllm_gated_scan": [P, c_int, c_int, c_int, c_int, P, c_longlong, P, P, P, c_int, c_int, c_int, c_int, c_float, c_int, P, c_longlong, P],
+    "mllm_gated_scan": [P, c_int, c_int, c_int, c_int, P, c_longlong, P, P, P, c_int, c_int, c_int, c_int, c_float, c_int, P, c_longlong, c_int, P],
     "mllm_gated_scan_chunk_rows": [],
     "mllm_gate_unit": [P, P, c_int, c_int, c_float, c_float, c_float, c_int, P],
     "mllm_branch_join": [P, P, c_int, c_longlong, P, P, c_int, c_longlong, P, P, P, P, c_int, c_int, c_int, c_float, P, P, c_int, c_float, P, c_int,

@@ -340,9 +340,9 @@ _KERNEL_CLASSES = {
     "products": ("gemm", "gemm_split", "gemm_qkv_cache", "gemm_best", "heads_linear"),
     "attention": ("attention", "attention_decode", "attention_prefill", "latent_attention"),
     "row-wise": ("layernorm", "pending_layernorm", "rms_norm", "head_norm", "latent_rows", "silu_mul", "pending_sum", "add", "cache_write", "embed",
-                 "projection_rows", "head_gate", "gated_norm", "short_conv", "map_rows", "map_difference", "turn_heads", "gate_unit", "route", "expert_unit",
+                 "projection_rows", "head_gate", "gated_norm", "short_conv", "map_rows", "map_difference", "turn_heads", "gate_unit", "route", "expert_unit", "gated_expert_unit",
                  "branch_join"),
-    "recurrence": ("recurrence",),
+    "recurrence": ("recurrence", "gated_scan"),
     "layer kernels": ("decode_attention_half", "decode_mlp_half"),
     "choice": ("choose", "sample"),
 }
@@ -429,9 +429,22 @@ def dizizen_shape(width: int, layers: int, vocab: int = 50257) -> dict:
             "layers": out}
 
 
+def goletar_shape(width: int, layers: int, vocab: int = 50257) -> dict:
+    """Layers in turn: a gated recurrence of 5/4 x width elements, and attention over a latent of 256 and a rotated part of 32 (heads of 64 +
+    32, values of 64: Gimozen's latent layers with a gate a head); feed-forwards of eight routed experts of 4/3 x width, two picked (as
+    many multiply-adds a token as a dense gated feed-forward of 8/3 x width, for the picked experts)."""
+    heads = width // 64
+    mlp = {"kind": "moe", "expert": {"ff": -(-(4 * width // 3) // 64) * 64, "limit": 7.0}, "router": {"experts": 8, "top": 2}}
+    latent = {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": 256, "rot": {"dims": 32, "base": 10000.0}, "scale": 96 ** -0.5}
+    return {"architecture": "Goletar", "vocab": vocab, "width": width, "embedding": {"bigram": {"buckets": 65521, "mul_prev": 7919, "mul_cur": 104729}},
+            "norm": {"eps": 1e-5},
+            "layers": [{"type": "latent_attention", "mixer": latent, "mlp": mlp} if index % 2 else {"type": "mingru", "mixer": {"width": 5 * width // 4}, "mlp": mlp}
+                       for index in range(layers)]}
+
+
 def measure_design(args) -> dict:
     """Prefill and decode throughput of a design and of the framework's closest older model with as many layers of the same width
-    (random weights): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen; and where each model's step spends its time, by class of
+    (random weights): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen, Goletar beside Dizizen (routed experts) and Gimozen (latent attention); and where each model's step spends its time, by class of
     kernel, inside a prompt step and a decode step."""
     import numpy as np
     import torch
@@ -441,7 +454,9 @@ def measure_design(args) -> dict:
     from mini_llm_amd.engine.engine import Engine, EngineOptions
 
     width, layers = DESIGN_SIZES[args.shape]
-    if args.design == "dizizen":
+    if args.design == "goletar":
+        raws = {"goletar": goletar_shape(width, layers), "dizizen": dizizen_shape(width, layers), "gimozen": gimozen_shape(width, layers)}
+    elif args.design == "dizizen":
         raws = {"dizizen": dizizen_shape(width, layers), "gimozen": gimozen_shape(width, layers)}
     elif args.design == "perezen":
         raws = {"perezen": perezen_shape(width, layers), "ketolix": ketolix_shape(width, layers)}
@@ -710,8 +725,8 @@ def main() -> int:
     parser.add_argument("--serving", action="store_true", help="continuous batching of 64 requests on the GPT-2 medium shape through the scheduler")
     parser.add_argument("--temperature", type=float, default=0.0, help="sampling temperature of --serving (0: greedy)")
     parser.add_argument("--step-by-step", action="store_true", help="--serving reads every step's tokens before it launches the next")
-    parser.add_argument("--design", default=None, choices=("gimozen", "ketolix", "perezen", "dizizen"), help="a design beside the closest older model with as many layers of the same width "
-                        "(--shape small|medium): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen; prefill and decode throughput of both, and where their steps spend the time")
+    parser.add_argument("--design", default=None, choices=("gimozen", "ketolix", "perezen", "dizizen", "goletar"), help="a design beside the closest older model with as many layers of the same width "
+                        "(--shape small|medium): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen, Goletar beside Dizizen and Gimozen; prefill and decode throughput of both, and where their steps spend the time")
     parser.add_argument("--peaks", action="store_true", help="measure this machine's read bandwidth and matrix-core rate with the library's probes")
     args = parser.parse_args()
     if args.gpus != 1:

@@ -70,7 +70,7 @@ enum MllmKernel : int {
     MLLM_K_LATENT_ROWS, MLLM_K_SILU_MUL, MLLM_K_HEADS_LINEAR, MLLM_K_LATENT_ATTENTION, MLLM_K_LATENT_MERGE, MLLM_K_PROJECTION_ROWS,
     MLLM_K_HEAD_GATE, MLLM_K_GATED_NORM, MLLM_K_SHORT_CONV, MLLM_K_RECURRENCE, MLLM_K_MAP_ROWS,
     MLLM_K_MAP_DIFFERENCE, MLLM_K_TURN_HEADS, MLLM_K_GATE_UNIT, MLLM_K_ROUTE, MLLM_K_EXPERT_UNIT, MLLM_K_BRANCH_JOIN,
-    MLLM_K_GATED_SCAN, MLLM_K_KINDS
+    MLLM_K_GATED_SCAN, MLLM_K_EXPERT_LISTS, MLLM_K_EXPERTS_FEW, MLLM_K_KINDS
 };
 void mllm_count_kernel(MllmKernel kind);
 

@@ -1,0 +1,268 @@
+// Routed experts that run for the rows that picked them, and for no others: the lists of rows by expert that the grouped products of
+// many rows walk (gemm_stream.h), and the two products of few rows (decoding), which find their rows themselves.
+//
+// A router leaves picks [rows, top] (expert ids, -1 for none) and their weights. Entry p = row * top + k is row `row` with its k-th
+// pick. An expert's matrices: the gate and up rows of the up matrix in turns of 32, [2 * units, width], and the down matrix [width,
+// units], both packed, one expert behind the other; units a multiple of 64 (zero rows and columns fill it up). The down product of a
+// row's k-th pick goes to plane k of out [top, rows, width]: whoever reads the branch adds the planes up, in that order.
+#include "common.h"
+#include "gate_unit.h"
+
+namespace {
+
+constexpr int MAX_EXPERTS = 1024;
+
+// The lists, a block an expert, without an atomic that could order them: entries of an expert in the order of their rows, experts behind
+// each other. Every block counts all experts' entries (so that it knows where its own begin) and places its own.
+__global__ __launch_bounds__(256) void expert_lists_kernel(const int* __restrict__ picks, const float* __restrict__ pick_weights, int n_rows, int top, int n_experts,
+                                                           int tile_rows, int* __restrict__ a_row, int* __restrict__ out_row, float* __restrict__ weight,
+                                                           int4* __restrict__ tiles, int* __restrict__ n_tiles) {
+    __shared__ int counts[MAX_EXPERTS];
+    __shared__ int wave_counts[4], start, first_tile;
+    const int expert = blockIdx.x, tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
+    const int entries = n_rows * top;
+    for (int e = tid; e < n_experts; e += 256) counts[e] = 0;
+    __syncthreads();
+    for (int p = tid; p < entries; p += 256) {
+        const int e = picks[p];
+        if (e >= 0 && e < n_experts) atomicAdd(&counts[e], 1);
+    }
+    __syncthreads();
+    if (wave == 0) {
+        int before = 0, tiles_before = 0;
+        for (int e = lane; e < expert; e += WAVE) {
+            before += counts[e];
+            tiles_before += (counts[e] + tile_rows - 1) / tile_rows;
+        }
+#pragma unroll
+        for (int offset = WAVE / 2; offset > 0; offset >>= 1) {
+            before += __shfl_xor(before, offset, WAVE);
+            tiles_before += __shfl_xor(tiles_before, offset, WAVE);
+        }
+        if (lane == 0) {
+            start = before;
+            first_tile = tiles_before;
+        }
+    }
+    __syncthreads();
+    const int mine = counts[expert], my_tiles = (mine + tile_rows - 1) / tile_rows, first = start;
+    for (int t = tid; t < my_tiles; t += 256) tiles[first_tile + t] = make_int4(expert, first + t * tile_rows, first + mine, 0);
+    if (expert == n_experts - 1 && tid == 0) *n_tiles = first_tile + my_tiles;
+    int placed = first;
+    for (int p0 = 0; p0 < entries; p0 += 256) {   // (the same number of turns for every thread)
+        const int p = p0 + tid;
+        const bool here = p < entries && picks[p] == expert;
+        const unsigned long long ballot = __ballot(here);
+        if (lane == 0) wave_counts[wave] = __popcll(ballot);
+        __syncthreads();
+        int at = placed + __popcll(ballot & ((1ull << lane) - 1));
+        for (int w = 0; w < wave; w++) at += wave_counts[w];
+        placed += wave_counts[0] + wave_counts[1] + wave_counts[2] + wave_counts[3];
+        __syncthreads();
+        if (here) {
+            const int row = p / top;
+            a_row[at] = row;
+            out_row[at] = (p - row * top) * n_rows + row;
+            weight[at] = pick_weights[p];
+        }
+    }
+}
+
+constexpr int FEW_ROWS = 64;
+
+// This block's expert: the entries that picked it, in LDS (a row picks an expert at most once, so there are at most FEW_ROWS). Returns
+// how many; called by all threads.
+__device__ __forceinline__ int gather_entries(const int* __restrict__ picks, int entries, int expert, int* list, int* count) {
+    if (threadIdx.x < WAVE) {
+        int found = 0;
+        for (int p0 = 0; p0 < entries; p0 += WAVE) {
+            const int p = p0 + threadIdx.x;
+            const bool here = p < entries && picks[p] == expert;
+            const unsigned long long ballot = __ballot(here);
+            const int at = found + __popcll(ballot & ((1ull << threadIdx.x) - 1));
+            if (here && at < FEW_ROWS) list[at] = p;
+            found += __popcll(ballot);
+        }
+        if (threadIdx.x == 0) *count = min(found, FEW_ROWS);
+    }
+    __syncthreads();
+    return *count;
+}
+
+// hidden[p, units] = the gate unit of entry p's row with its expert's matrices. A block takes 16 units of an expert: its gate and up rows
+// stream from memory once, straight into matrix-core operands (out^T = W . x^T, W the 16-row operand), for up to MT times 16 rows at a
+// time; the waves take the steps of 32 along the width in turns and their sums meet in LDS, where the gate unit is.
+template <int MT, int KSPLIT>
+__global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ W, bf16_t* __restrict__ hidden,
+                                                                     const int* __restrict__ picks, const float* __restrict__ pick_weights, int n_rows, int top,
+                                                                     int units, int width, GateUnit unit, int weigh_input) {
+    constexpr int UNROLL = MT == 4 ? 4 : 8;
+    __shared__ float sums[KSPLIT][2 * MT * 4][WAVE];
+    __shared__ int list[FEW_ROWS], count;
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, row16 = lane % 16, quad = lane / 16;
+    const int expert = blockIdx.y, u0 = blockIdx.x * 16;
+    const int n = gather_entries(picks, n_rows * top, expert, list, &count);
+    if (n == 0) return;   // nobody picked this expert (uniform over the block)
+    const int steps = width / 32;   // a multiple of two: the width is one of 64
+    const int gate_tile = expert * (2 * units / 16) + u0 / 32 * 4 + u0 / 16 % 2;   // 32 gate rows, 32 up rows in turn
+    const bf16_t* x_row[MT];
+#pragma unroll
+    for (int i = 0; i < MT; i++) x_row[i] = x + (size_t)(list[min(i * 16 + row16, n - 1)] / top) * width + quad * 8;   // beyond the last: never stored
+    f32x4 gate[MT], up[MT];
+#pragma unroll
+    for (int i = 0; i < MT; i++) gate[i] = up[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    for (int step0 = wave * UNROLL; step0 < steps; step0 += KSPLIT * UNROLL) {
+        bf16x8 g_op[UNROLL], u_op[UNROLL], x_op[UNROLL][MT];
+#pragma unroll
+        for (int u = 0; u < UNROLL; u++) {
+            const int step = min(step0 + u, steps - 1);   // beyond the end: the last step again, not used
+            g_op[u] = *reinterpret_cast<const bf16x8*>(W + packed_offset<bf16_t>(gate_tile, step, steps, lane));
+            u_op[u] = *reinterpret_cast<const bf16x8*>(W + packed_offset<bf16_t>(gate_tile + 2, step, steps, lane));
+#pragma unroll
+            for (int i = 0; i < MT; i++) x_op[u][i] = *reinterpret_cast<const bf16x8*>(x_row[i] + step * 32);
+        }
+#pragma unroll
+        for (int u = 0; u < UNROLL; u++) {
+            if (step0 + u >= steps) break;
+#pragma unroll
+            for (int i = 0; i < MT; i++) {
+                gate[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(g_op[u], x_op[u][i], gate[i], 0, 0, 0);
+                up[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u_op[u], x_op[u][i], up[i], 0, 0, 0);
+            }
+        }
+    }
+    // gate[i][r] belongs to entry i * 16 + lane % 16, unit u0 + 4 * (lane / 16) + r
+#pragma unroll
+    for (int i = 0; i < MT; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            sums[wave][i * 4 + r][lane] = gate[i][r];
+            sums[wave][(MT + i) * 4 + r][lane] = up[i][r];
+        }
+    __syncthreads();
+    // a thread finishes whole units: entry index / 16, unit index % 16
+    for (int index = threadIdx.x; index < n * 16; index += 64 * KSPLIT) {
+        const int entry = index / 16, unit_at = index % 16, i = entry / 16;
+        const int l = (unit_at / 4) * 16 + entry % 16, r = unit_at % 4;
+        float g = 0.0f, u = 0.0f;
+#pragma unroll
+        for (int w = 0; w < KSPLIT; w++) {   // the same order for every element
+            g += sums[w][i * 4 + r][l];
+            u += sums[w][(MT + i) * 4 + r][l];
+        }
+        const int p = list[entry];
+        const float weight = pick_weights[p];
+        const float value = weigh_input ? gated(g * weight, u * weight, unit) : gated(g, u, unit) * weight;
+        hidden[(size_t)p * units + u0 + unit_at] = static_cast<bf16_t>(value);
+    }
+}
+
+// out[k, row, :] = hidden[row * top + k, units] . its expert's down matrix^T, 32-bit; a block takes 16 columns of an expert.
+template <int MT, int KSPLIT>
+__global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const bf16_t* __restrict__ hidden, const bf16_t* __restrict__ W, float* __restrict__ out,
+                                                                       const int* __restrict__ picks, int n_rows, int top, int units, int width) {
+    constexpr int UNROLL = MT == 4 ? 4 : 8;
+    __shared__ float sums[KSPLIT][MT * 4][WAVE];
+    __shared__ int list[FEW_ROWS], count;
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, row16 = lane % 16, quad = lane / 16;
+    const int expert = blockIdx.y, n0 = blockIdx.x * 16;
+    const int n = gather_entries(picks, n_rows * top, expert, list, &count);
+    if (n == 0) return;
+    const int steps = units / 32, tile = expert * (width / 16) + blockIdx.x;
+    const bf16_t* h_row[MT];
+#pragma unroll
+    for (int i = 0; i < MT; i++) h_row[i] = hidden + (size_t)list[min(i * 16 + row16, n - 1)] * units + quad * 8;
+    f32x4 acc[MT];
+#pragma unroll
+    for (int i = 0; i < MT; i++) acc[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    for (int step0 = wave * UNROLL; step0 < steps; step0 += KSPLIT * UNROLL) {
+        bf16x8 w_op[UNROLL], h_op[UNROLL][MT];
+#pragma unroll
+        for (int u = 0; u < UNROLL; u++) {
+            const int step = min(step0 + u, steps - 1);
+            w_op[u] = *reinterpret_cast<const bf16x8*>(W + packed_offset<bf16_t>(tile, step, steps, lane));
+#pragma unroll
+            for (int i = 0; i < MT; i++) h_op[u][i] = *reinterpret_cast<const bf16x8*>(h_row[i] + step * 32);
+        }
+#pragma unroll
+        for (int u = 0; u < UNROLL; u++) {
+            if (step0 + u >= steps) break;
+#pragma unroll
+            for (int i = 0; i < MT; i++) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w_op[u], h_op[u][i], acc[i], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < MT; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) sums[wave][i * 4 + r][lane] = acc[i][r];
+    __syncthreads();
+    for (int index = threadIdx.x; index < n * 16; index += 64 * KSPLIT) {
+        const int entry = index / 16, column = index % 16, i = entry / 16;
+        const int l = (column / 4) * 16 + entry % 16, r = column % 4;
+        float value = 0.0f;
+#pragma unroll
+        for (int w = 0; w < KSPLIT; w++) value += sums[w][i * 4 + r][l];
+        const int p = list[entry], row = p / top;
+        out[((size_t)(p - row * top) * n_rows + row) * width + n0 + column] = value;
+    }
+}
+
+bool few_sizes(int n_rows, int top, int n_experts, int units, int width) {
+    return n_rows >= 0 && n_rows <= FEW_ROWS && top >= 1 && n_experts >= 1 && n_experts <= MAX_EXPERTS && top <= n_experts && units >= 64 && units % 64 == 0 &&
+           width >= 64 && width % 64 == 0;
+}
+
+}  // namespace
+
+// Rows up to which the products of few rows take the experts.
+MLLM_API int mllm_experts_few_rows() { return FEW_ROWS; }
+
+// picks, pick_weights [n_rows, top] -> the lists: a_row, out_row, weight [n_rows * top] (as many entries as picks that name an expert), tiles [up to
+// n_rows * top / tile_rows + min(n_experts, n_rows * top)] of four integers each, n_tiles [1].
+MLLM_API int mllm_expert_lists(const int* picks, const float* pick_weights, int n_rows, int top, int n_experts, int tile_rows, int* a_row, int* out_row, float* weight,
+                               int* tiles, int* n_tiles, hipStream_t stream) {
+    MLLM_REQUIRE(n_rows >= 0 && top >= 1 && n_experts >= 1 && n_experts <= MAX_EXPERTS && tile_rows >= 1 && (long long)n_rows * top < (1LL << 30), "expert_lists: bad sizes");
+    MLLM_REQUIRE(picks && pick_weights && a_row && out_row && weight && tiles && n_tiles && ((uintptr_t)tiles & 15) == 0, "expert_lists: a missing operand");
+    mllm_count_kernel(MLLM_K_EXPERT_LISTS);
+    expert_lists_kernel<<<n_experts, 256, 0, stream>>>(picks, pick_weights, n_rows, top, n_experts, tile_rows, a_row, out_row, weight, (int4*)tiles, n_tiles);
+    return mllm_check_launch("expert_lists");
+}
+
+#define MLLM_FEW_CASES(KERNEL, GRID, STEPS, ...)                                                       \
+    do {                                                                                               \
+        if ((STEPS) <= 32) {                                                                           \
+            if (n_rows <= 16) KERNEL<1, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                     \
+            else if (n_rows <= 32) KERNEL<2, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                \
+            else KERNEL<4, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                                  \
+        } else {                                                                                       \
+            if (n_rows <= 16) KERNEL<1, 8><<<GRID, 512, 0, stream>>>(__VA_ARGS__);                     \
+            else if (n_rows <= 32) KERNEL<2, 8><<<GRID, 512, 0, stream>>>(__VA_ARGS__);                \
+            else KERNEL<4, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);   /* (its sums take 32 KB of LDS as it is) */ \
+        }                                                                                              \
+    } while (0)
+
+// x [n_rows, width], hidden [n_rows * top, units] (rows of picks that name no expert are left alone), W packed [n_experts * 2 * units, width].
+MLLM_API int mllm_experts_few_up(const void* x, const void* W, void* hidden, const int* picks, const float* pick_weights, int n_rows, int top, int n_experts, int units,
+                                 int width, float limit, float alpha, float shift, int weigh_input, hipStream_t stream) {
+    MLLM_REQUIRE(few_sizes(n_rows, top, n_experts, units, width), "experts_few_up: no kernel for %d rows, %d of %d experts, %d units, width %d", n_rows, top, n_experts, units, width);
+    MLLM_REQUIRE(x && W && hidden && picks && pick_weights && limit > 0.0f && ((uintptr_t)x & 15) == 0, "experts_few_up: a missing operand");
+    if (n_rows == 0) return 0;
+    mllm_count_kernel(MLLM_K_EXPERTS_FEW);
+    const dim3 grid(units / 16, n_experts);
+    const GateUnit unit{limit, alpha, shift};
+    MLLM_FEW_CASES(experts_few_up_kernel, grid, width / 32, (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)hidden, picks, pick_weights, n_rows, top, units, width, unit,
+                   weigh_input);
+    return mllm_check_launch("experts_few_up");
+}
+
+// out [top, n_rows, width] (rows of picks that name no expert are left alone), W packed [n_experts * width, units].
+MLLM_API int mllm_experts_few_down(const void* hidden, const void* W, float* out, const int* picks, int n_rows, int top, int n_experts, int units, int width,
+                                   hipStream_t stream) {
+    MLLM_REQUIRE(few_sizes(n_rows, top, n_experts, units, width), "experts_few_down: no kernel for %d rows, %d of %d experts, %d units, width %d", n_rows, top, n_experts, units, width);
+    MLLM_REQUIRE(hidden && W && out && picks && ((uintptr_t)hidden & 15) == 0, "experts_few_down: a missing operand");
+    if (n_rows == 0) return 0;
+    mllm_count_kernel(MLLM_K_EXPERTS_FEW);
+    const dim3 grid(width / 16, n_experts);
+    MLLM_FEW_CASES(experts_few_down_kernel, grid, units / 32, (const bf16_t*)hidden, (const bf16_t*)W, out, picks, n_rows, top, units, width);
+    return mllm_check_launch("experts_few_down");
+}

@@ -799,6 +799,53 @@ MLLM_API int mllm_gemm_qkv_cache(const void* A, const void* W, int w_packed, con
 }
 
 // ------------------------------------------------------------------------------------------------
+// Products over rows grouped by expert (many rows): gemm_stream.h's ExpertTiles.
+// ------------------------------------------------------------------------------------------------
+namespace {
+constexpr int EXPERT_TILE = 128;   // entries a tile of the lists holds
+}
+
+MLLM_API int mllm_expert_tile_rows() { return EXPERT_TILE; }
+
+// Whether the two products of experts run grouped: bfloat16, whole tiles of K in both (the width and an expert's padded units).
+MLLM_API int mllm_experts_supported(int width, int units, int dtype) {
+    return dtype == MLLM_BF16 && width >= 64 && width % 64 == 0 && units >= 64 && units % 64 == 0;
+}
+
+// hidden [entries, units]: the gate unit of row a_row[i] of x [.., width] with its expert's matrices, W [n_experts * 2 * units, width] packed, an
+// expert's rows 32 gate rows and 32 up rows in turn. tiles / n_tiles / max_tiles: see ExpertTiles.
+MLLM_API int mllm_experts_up(const void* x, const void* W, void* hidden, const int* tiles, const int* n_tiles, const int* a_row, const float* weight, int entries,
+                             int max_tiles, int units, int width, float limit, float alpha, float shift, int weigh_input, hipStream_t stream) {
+    MLLM_REQUIRE(mllm_experts_supported(width, units, MLLM_BF16), "experts_up: no kernel for width %d with %d units", width, units);
+    MLLM_REQUIRE(x && W && hidden && tiles && n_tiles && a_row && weight && limit > 0.0f && ((uintptr_t)tiles & 15) == 0, "experts_up: a missing operand");
+    MLLM_REQUIRE(entries >= 0 && max_tiles >= 0 && (long long)max_tiles * ceil_div(2 * units, 128) < (1LL << 30) && (long long)entries * width * 2 < (1LL << 32),
+                 "experts_up: bad sizes");
+    if (entries == 0) return 0;
+    const stream::ExpertTiles<true> group{(const int4*)tiles, n_tiles, a_row, nullptr, weight, GateUnit{limit, alpha, shift}, weigh_input};
+    stream::launch_grouped<bf16_t, EXPERT_TILE, 128, 2, 2, 3>((const bf16_t*)x, (const bf16_t*)W, (bf16_t*)hidden, entries, max_tiles, 2 * units, width, group, stream);
+    return mllm_check_launch("experts_up");
+}
+
+// out row out_row[i] = hidden row i . its expert's down matrix^T, 32-bit; W [n_experts * width, units] packed.
+MLLM_API int mllm_experts_down(const void* hidden, const void* W, float* out, const int* tiles, const int* n_tiles, const int* out_row, int entries, int max_tiles,
+                               int units, int width, hipStream_t stream) {
+    MLLM_REQUIRE(mllm_experts_supported(width, units, MLLM_BF16), "experts_down: no kernel for width %d with %d units", width, units);
+    MLLM_REQUIRE(hidden && W && out && tiles && n_tiles && out_row && ((uintptr_t)tiles & 15) == 0, "experts_down: a missing operand");
+    MLLM_REQUIRE(entries >= 0 && max_tiles >= 0 && (long long)max_tiles * ceil_div(width, 64) < (1LL << 30) && (long long)entries * units * 2 < (1LL << 32),
+                 "experts_down: bad sizes");
+    if (entries == 0) return 0;
+    const stream::ExpertTiles<false> group{(const int4*)tiles, n_tiles, nullptr, out_row, nullptr, GateUnit{1.0f, 1.0f, 0.0f}, 0};
+    // wide tiles where they fill the rounds of blocks as well as narrow ones do (the costs of a tile of K: dispatch)
+    const long tiles_m = ceil_div(entries, EXPERT_TILE);
+    const float wide = (float)((tiles_m * ceil_div(width, 128) + 255) / 256) * 0.45f, narrow = (float)((tiles_m * ceil_div(width, 64) + 255) / 256) * 0.30f;
+    if (wide <= narrow)
+        stream::launch_grouped<float, EXPERT_TILE, 128, 2, 2, 3>((const bf16_t*)hidden, (const bf16_t*)W, out, entries, max_tiles, width, units, group, stream);
+    else
+        stream::launch_grouped<float, EXPERT_TILE, 64, 2, 2, 3>((const bf16_t*)hidden, (const bf16_t*)W, out, entries, max_tiles, width, units, group, stream);
+    return mllm_check_launch("experts_down");
+}
+
+// ------------------------------------------------------------------------------------------------
 // The product cut along K without an allocation (no_alloc.h): the partial products go to a fixed
 // array of the library instead of memory the caller brings.
 // ------------------------------------------------------------------------------------------------

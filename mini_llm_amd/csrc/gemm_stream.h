@@ -34,6 +34,8 @@
 //    out of thousands).
 #pragma once
 
+#include "gate_unit.h"
+
 #include <type_traits>
 #include <utility>
 
@@ -110,13 +112,34 @@ __device__ __forceinline__ void put4<bf16_t>(bf16_t* at, f32x4 v) {
     *reinterpret_cast<bf16x4*>(at) = o;
 }
 
+// Which rows and which matrix a block's tile takes. The whole product: rows of A in order, one matrix.
+struct Whole {
+    static constexpr bool GROUPED = false, GATED = false;
+};
+// A product over rows grouped by expert, each group with a matrix of its own: the groups' entries lie behind each other in one list, and
+// `tiles` names the tiles of it that hold an expert's entries: (expert, first entry, the end of the expert's entries, unused). Entry i
+// reads row a_row[i] of A (null: row i) and goes to row out_row[i] of out (null: row i). W holds every expert's rows behind each other.
+// GATED: an expert's rows of W are, for every 32 units, 32 gate rows and 32 up rows; out [.., N / 2] is the gate unit of the two sums,
+// weight[i] multiplying the sums (weigh_input) or the unit.
+template <bool GATED_>
+struct ExpertTiles {
+    static constexpr bool GROUPED = true, GATED = GATED_;
+    const int4* tiles;
+    const int* n_tiles;
+    const int* a_row;
+    const int* out_row;
+    const float* weight;
+    GateUnit unit;
+    int weigh_input;
+};
+
 // grid: one row of blocks, placed by 'places' (tiles and blocks along K). More than one block along K: each block takes k_per_block of K (a multiple
 // of 64) and leaves a partial product in matrix 'block_k' of `out` (float, no bias / epilogue / residual).
 // WAVES_K = 2: two waves share a tile of outputs and take half of every tile of K each; their sums meet in LDS at the end.
-template <typename OutT, int BM, int BN, int WAVES_M, int WAVES_N, int WAVES_K, int STAGES>
+template <typename OutT, int BM, int BN, int WAVES_M, int WAVES_N, int WAVES_K, int STAGES, typename Group>
 __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, const float* __restrict__ bias, const float* __restrict__ residual,
-    OutT* __restrict__ out, int M, int N, int K, int epilogue, CacheScatter scatter, int k_per_block, XcdTiles places) {
+    OutT* __restrict__ out, int M, int N, int K, int epilogue, CacheScatter scatter, int k_per_block, XcdTiles places, Group group) {
     constexpr int NW = WAVES_M * WAVES_N * WAVES_K;
     constexpr int WM = BM / WAVES_M, WN = BN / WAVES_N, FM = WM / 32, FN = WN / 32;
     constexpr int BK = 64, KS = BK / 16 / WAVES_K;           // steps of 16 along K a wave takes of a tile
@@ -129,8 +152,12 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
     static_assert(LPW * (STAGES - 1) < 64, "the loads in flight must fit the counter");
     constexpr int STAGE_BYTES = (BM + BN) * 128;
     constexpr int OUT_VEC = 16 / (int)sizeof(OutT);          // columns in a 16-byte piece of the output
-    constexpr int SLAB_ROW = WN * (int)sizeof(OutT) + 16;    // a row of a wave's tile in LDS, padded by one piece
-    constexpr int PIECES = WN / OUT_VEC;
+    constexpr bool GROUPED = Group::GROUPED, GATED = Group::GATED;
+    static_assert(!GROUPED || WAVES_K == 1, "a grouped product's tiles are taken whole");
+    static_assert(!GATED || FN % 2 == 0, "a wave holds gate and up columns of the same units");
+    constexpr int WO = GATED ? WN / 2 : WN;                  // columns of the output a wave's tile makes
+    constexpr int SLAB_ROW = WO * (int)sizeof(OutT) + 16;    // a row of a wave's tile in LDS, padded by one piece
+    constexpr int PIECES = WO / OUT_VEC;
     constexpr int SHARED_SUMS = WAVES_K == 1 ? 0 : NW * FN * OWN * 4096;  // what the waves that share a tile hand each other
     extern __shared__ __attribute__((aligned(1024))) unsigned char lds[];
 
@@ -140,11 +167,24 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
     // Blocks go round the eight XCDs in turn, each with an L2 of its own: the blocks of one XCD take the tiles of one
     // rectangle of the output, so that the rows of A and of W an XCD reads are few and each is fetched into its L2 once.
     const int xcd = blockIdx.x % 8, in_xcd = blockIdx.x / 8;
-    const int block_k = in_xcd / (places.wide * places.high), in_rectangle = in_xcd % (places.wide * places.high);
-    const int tile_m = (xcd / places.across) * places.high + in_rectangle / places.wide;
-    const int tile_n = (xcd % places.across) * places.wide + in_rectangle % places.wide;
-    const int m0 = tile_m * BM, n0 = tile_n * BN;
-    if (m0 >= M || n0 >= N) return;  // (the rectangles cover more than the matrix; the whole block leaves)
+    int block_k = 0, m0, n0, m_end = M, w_first_tile = 0;
+    if constexpr (GROUPED) {
+        // the tiles in the order of their experts, an eighth of them to each XCD: an expert's matrix goes to one or two L2 caches
+        const int across = (N + BN - 1) / BN, total = *group.n_tiles * across, share = (total + 7) / 8, at = xcd * share + in_xcd;
+        if (in_xcd >= share || at >= total) return;  // (the grid is sized for the most tiles there can be)
+        const int4 tile = group.tiles[at / across];
+        m0 = tile.y;
+        m_end = tile.z;
+        n0 = (at % across) * BN;
+        w_first_tile = tile.x * ((N + 15) / 16);
+    } else {
+        block_k = in_xcd / (places.wide * places.high);
+        const int in_rectangle = in_xcd % (places.wide * places.high);
+        m0 = ((xcd / places.across) * places.high + in_rectangle / places.wide) * BM;
+        n0 = ((xcd % places.across) * places.wide + in_rectangle % places.wide) * BN;
+        if (m0 >= M || n0 >= N) return;  // (the rectangles cover more than the matrix; the whole block leaves)
+    }
+    const int n_out = GATED ? N / 2 : N;
     const int k_begin = block_k * k_per_block, k_end = min(K, k_begin + k_per_block);
     const int k_steps = K / 32, n_tiles = (k_end - k_begin) / BK;
     const int w_row_tiles = (N + 15) / 16;
@@ -160,13 +200,15 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
         if (i < A_LPW) {
             // eight rows of 128 bytes: eight lanes take the eight pieces of a row (a whole cache line), turned by the row
             const int in_tile = q * 8 + lane / 8, piece = (lane % 8) ^ ((in_tile >> 1) & 7);
-            const int row = min(m0 + in_tile, M - 1);  // beyond the last row: that row again, never stored
+            int row = min(m0 + in_tile, m_end - 1);  // beyond the last row: that row again, never stored
+            if constexpr (GROUPED)
+                if (group.a_row) row = group.a_row[row];
             base[i] = reinterpret_cast<const unsigned char*>(A + k_begin);
             lane_offset[i] = ((unsigned)row * (unsigned)K + piece * 8) * 2;
         } else {
             const int qw = q - A_LOADS, rt = qw / 2, kc = qw % 2;
             const int row_tile = min(n0 / 16 + rt, w_row_tiles - 1);
-            base[i] = reinterpret_cast<const unsigned char*>(W + packed_offset<bf16_t>(row_tile, k_begin / 32 + kc, k_steps, 0));
+            base[i] = reinterpret_cast<const unsigned char*>(W + packed_offset<bf16_t>(w_first_tile + row_tile, k_begin / 32 + kc, k_steps, 0));
             lane_offset[i] = lane * 16;
         }
     }
@@ -187,11 +229,11 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
     constexpr int ROWS_A_STEP = PIECES > 32 ? 1 : PIECES > 16 ? 2 : PIECES > 8 ? 4 : PIECES > 4 ? 8 : 16;
     constexpr int ROW_STEPS = 32 / ROWS_A_STEP;
     static_assert(ROWS_A_STEP * PIECES <= WAVE, "a step's pieces fit a wave");
-    const int n_wave = n0 + wave_n * WN, own0 = wave_k * OWN;
+    const int n_wave = GATED ? (n0 + wave_n * WN) / 2 : n0 + wave_n * WN, own0 = wave_k * OWN;
     const int lane_row = lane / PIECES, lane_piece = lane % PIECES;
     const int m_lane = m0 + wave_m * WM + own0 * 32 + lane_row, n_lane = n_wave + lane_piece * OUT_VEC;
     // rows from the lane's first one to the end of the matrix; none for a lane that idles or whose columns lie outside
-    const int rows_left = lane_row < ROWS_A_STEP && n_lane < N ? M - m_lane : 0;
+    const int rows_left = lane_row < ROWS_A_STEP && n_lane < n_out ? m_end - m_lane : 0;
 
     // What the epilogue adds is asked for now and arrives while the products run: asked for where it is used, every
     // block would wait for it at the end, with nothing left to hide the trip behind.
@@ -203,7 +245,7 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
             const int n = n_wave + j * 32 + 8 * g + 4 * (lane / 32);  // N is a multiple of 8: four columns are inside or outside together
             early_bias[j][g] = bias && n < N ? *reinterpret_cast<const f32x4*>(bias + n) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
         }
-    constexpr bool WITH_RESIDUAL = sizeof(OutT) == 4, CAN_SCATTER = sizeof(OutT) == 2;
+    constexpr bool WITH_RESIDUAL = sizeof(OutT) == 4 && !GROUPED, CAN_SCATTER = sizeof(OutT) == 2 && !GROUPED;
     f32x4 early_residual[WITH_RESIDUAL ? OWN : 1][WITH_RESIDUAL ? ROW_STEPS : 1];
     if constexpr (WITH_RESIDUAL) {
         const float* residual_lane = residual + (size_t)m_lane * N + n_lane;
@@ -226,6 +268,22 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
                     early_slot[i][r] = row < rows_left ? scatter.slots[m_lane + row] : -1;
                 }
         }
+    }
+
+    // a grouped product: the weights of the rows a lane's sums belong to, and the rows of out its pieces go to
+    float early_weight[GATED ? FM : 1];
+    int early_row[GROUPED && !GATED ? OWN : 1][GROUPED && !GATED ? ROW_STEPS : 1];
+    if constexpr (GATED) {
+#pragma unroll
+        for (int i = 0; i < FM; i++) early_weight[i] = group.weight[min(m0 + wave_m * WM + i * 32 + lane % 32, m_end - 1)];
+    } else if constexpr (GROUPED) {
+#pragma unroll
+        for (int i = 0; i < OWN; i++)
+#pragma unroll
+            for (int r = 0; r < ROW_STEPS; r++) {
+                const int entry = min(m_lane + i * 32 + r * ROWS_A_STEP, m_end - 1);
+                early_row[i][r] = group.out_row ? group.out_row[entry] : entry;
+            }
     }
 
     f32x16 acc[FN][FM];
@@ -376,7 +434,7 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
         constexpr bool SCATTERED = WHERE != 0;
         // where a lane's piece goes: q columns to out [M, q_width], key and value columns into the cache page at the
         // row's slot (a piece lies inside one head: the head size is a multiple of 8)
-        const int row_stride = SCATTERED ? scatter.q_width : N;
+        const int row_stride = SCATTERED ? scatter.q_width : n_out;
         OutT* out_lane = out + (size_t)m_lane * row_stride + n_lane;
         // A piece in the cache lies at page * (bytes of a page) + ((head << page_shift) + offset) * (bytes of a row) + the
         // piece's place in the row: all but page and offset is the lane's own constant.
@@ -394,6 +452,18 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
         }
 #pragma unroll
         for (int i = 0; i < OWN; i++) {
+            if constexpr (GATED) {
+                const float in_weight = group.weigh_input ? early_weight[i] : 1.0f, out_weight = group.weigh_input ? 1.0f : early_weight[i];
+#pragma unroll
+                for (int j = 0; j < FN; j += 2)
+#pragma unroll
+                    for (int g = 0; g < 4; g++) {
+                        f32x4 value;
+#pragma unroll
+                        for (int e = 0; e < 4; e++) value[e] = gated(acc[j][i][4 * g + e] * in_weight, acc[j + 1][i][4 * g + e] * in_weight, group.unit) * out_weight;
+                        put4<OutT>(reinterpret_cast<OutT*>(slab_write) + (j / 2) * 32 + 8 * g, value);
+                    }
+            } else {
 #pragma unroll
             for (int j = 0; j < FN; j++)
 #pragma unroll
@@ -411,6 +481,7 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
                     }
                     put4<OutT>(reinterpret_cast<OutT*>(slab_write) + j * 32 + 8 * g, value);
                 }
+            }
             asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
 #pragma unroll
             for (int r = 0; r < ROW_STEPS; r++) {
@@ -431,7 +502,8 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
                     sum = early_residual[i][r] + sum;   // zeros where there is no residual
                     v = *reinterpret_cast<Vec16*>(&sum);
                 }
-                *reinterpret_cast<Vec16*>(out_lane + (size_t)row * row_stride) = v;
+                if constexpr (GROUPED && !GATED) *reinterpret_cast<Vec16*>(out + (size_t)early_row[i][r] * row_stride + n_lane) = v;
+                else *reinterpret_cast<Vec16*>(out_lane + (size_t)row * row_stride) = v;
             }
             asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         }
@@ -464,14 +536,30 @@ void launch(const bf16_t* a, const bf16_t* w, const float* bias, const float* re
     static bool raised = false;  // per instantiation: the limit on dynamic LDS is a property of the kernel
     if (!raised && LDS_BYTES > 64 * 1024) {
         // (if this fails the launch below fails too, and the entry point reports that)
-        raised = hipFuncSetAttribute((const void*)gemm_stream_kernel<OutT, BM, BN, WAVES_M, WAVES_N, WAVES_K, STAGES>,
+        raised = hipFuncSetAttribute((const void*)gemm_stream_kernel<OutT, BM, BN, WAVES_M, WAVES_N, WAVES_K, STAGES, Whole>,
                                      hipFuncAttributeMaxDynamicSharedMemorySize, LDS_BYTES) == hipSuccess;
     }
     const int k_per_block = k_blocks == 1 ? K : ceil_div(ceil_div(K, k_blocks), 64) * 64;
     const XcdTiles places = place_tiles(ceil_div(M, BM), ceil_div(N, BN), BM, BN);
     mllm_count_kernel(MLLM_K_GEMM_STREAM);
-    gemm_stream_kernel<OutT, BM, BN, WAVES_M, WAVES_N, WAVES_K, STAGES><<<8 * places.wide * places.high * k_blocks, 64 * NW, LDS_BYTES, stream>>>(
-        a, w, bias, residual, o, M, N, K, epilogue, scatter, k_per_block, places);
+    gemm_stream_kernel<OutT, BM, BN, WAVES_M, WAVES_N, WAVES_K, STAGES, Whole><<<8 * places.wide * places.high * k_blocks, 64 * NW, LDS_BYTES, stream>>>(
+        a, w, bias, residual, o, M, N, K, epilogue, scatter, k_per_block, places, Whole{});
+}
+
+// The same loop over rows grouped by expert. entries: how many there are; max_tiles: how many tiles of BM they can make at most.
+template <typename OutT, int BM, int BN, int WAVES_M, int WAVES_N, int STAGES, typename Group>
+void launch_grouped(const bf16_t* a, const bf16_t* w, OutT* o, int entries, int max_tiles, int N, int K, const Group& group, hipStream_t stream) {
+    constexpr int NW = WAVES_M * WAVES_N, SLAB_BYTES = NW * 32 * (BN / WAVES_N * (int)sizeof(OutT) + 16);
+    constexpr int LDS_BYTES = STAGES * (BM + BN) * 128 > SLAB_BYTES ? STAGES * (BM + BN) * 128 : SLAB_BYTES;
+    static_assert(LDS_BYTES <= 160 * 1024, "a block's LDS");
+    static bool raised = false;
+    if (!raised && LDS_BYTES > 64 * 1024)
+        raised = hipFuncSetAttribute((const void*)gemm_stream_kernel<OutT, BM, BN, WAVES_M, WAVES_N, 1, STAGES, Group>,
+                                     hipFuncAttributeMaxDynamicSharedMemorySize, LDS_BYTES) == hipSuccess;
+    const int blocks = ceil_div(max_tiles * ceil_div(N, BN), 8) * 8;
+    mllm_count_kernel(MLLM_K_GEMM_STREAM);
+    gemm_stream_kernel<OutT, BM, BN, WAVES_M, WAVES_N, 1, STAGES, Group><<<blocks, 64 * NW, LDS_BYTES, stream>>>(
+        a, w, nullptr, nullptr, o, entries, N, K, MLLM_EPI_NONE, CacheScatter{}, K, XcdTiles{1, 1, 1}, group);
 }
 
 // Whether the product takes this kernel: bfloat16 with a packed W, whole tiles of K, whole 16-byte pieces of output

@@ -6,70 +6,139 @@
 // expert, which is zero for the experts the router did not pick, so the down product's sum over all hidden units is the weighted sum
 // over the picked experts. Nothing is planned on the host and no row's result depends on the other rows of the batch.
 #include "common.h"
+#include "gate_unit.h"
 
 #include <math.h>
 
 namespace {
 
-constexpr int ROUTE_MAX_EXPERTS = 1024;
+constexpr int ROUTE_MAX_EXPERTS = 1024, ROUTE_FEW_EXPERTS = 64;
 
 // (value, index) a is picked before b: the larger value, among equals the smaller index.
 __device__ __forceinline__ bool picked_before(float a, int ia, float b, int ib) { return a > b || (a == b && ia < ib); }
 
-// One wave a row. logits: the router's 32-bit sums z [row, n_experts] (rows `stride` apart). Scores s = softmax over all n_experts, or with
-// `sigmoid` 1 / (1 + e^-z);
-// choice c = s + correction (null: none). The experts form n_groups equal groups of neighbours; a group's rank goes by the largest c
-// in it, and only experts of the best `keep` groups can be picked (the others count as minus infinity). The `top` experts of largest
-// c are picked; weights[row, e] = s_e / (sum of the picked experts' s + floor), without `renormalise` s_e itself, for them and 0 for all
-// others.
-__global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ logits, int stride, const float* __restrict__ correction,
-                                                     float* __restrict__ weights, int weights_stride, int n_experts, int top, int n_groups, int keep,
-                                                     float floor, int sigmoid, int renormalise) {
-    __shared__ float score[ROUTE_MAX_EXPERTS], choice[ROUTE_MAX_EXPERTS], group_best[ROUTE_MAX_EXPERTS];
-    const int lane = threadIdx.x, row = blockIdx.x;
-    const float* z = logits + (size_t)row * stride;
+// What a router does with a row's sums: scores s = softmax over all n_experts, or with `sigmoid` 1 / (1 + e^-z); choice c = s + correction
+// (null: none). The experts form n_groups equal groups of neighbours; a group's rank goes by the largest c in it, and only experts of
+// the best `keep` groups can be picked (the others count as minus infinity). The `top` experts of largest c are picked; a picked
+// expert's weight is s_e / (sum of the picked experts' s + floor), without `renormalise` s_e itself.
+struct Choice {
+    const float* correction;
+    int n_experts, top, n_groups, keep;
+    float floor;
+    int sigmoid, renormalise;
+};
+// Where it goes, each optional: weights [row, n_experts] (rows `stride` apart, 0 for the experts that were not picked); picks and
+// pick_weights [row, top], the picked experts in the order of their choice scores (-1 where sums that are no numbers left none to pick).
+struct Routed {
+    float* weights;
+    int stride;
+    int* picks;
+    float* pick_weights;
+};
+
+// One wave; `score` holds the row's sums.
+__device__ void route_row(const Choice& how, const Routed& to, size_t row, float* score, float* choice, float* group_best, int lane) {
+    const int n_experts = how.n_experts;
+    if (to.picks)
+        for (int k = lane; k < how.top; k += WAVE) to.picks[row * how.top + k] = -1;
     float largest = -INFINITY;
-    for (int e = lane; e < n_experts; e += WAVE) largest = fmaxf(largest, z[e]);
+    for (int e = lane; e < n_experts; e += WAVE) largest = fmaxf(largest, score[e]);
     largest = wave_max(largest);
     float total = 0.0f;
     for (int e = lane; e < n_experts; e += WAVE) {
-        const float p = sigmoid ? 1.0f / (1.0f + expf(-z[e])) : expf(z[e] - largest);
+        const float z = score[e], p = how.sigmoid ? 1.0f / (1.0f + expf(-z)) : expf(z - largest);
         score[e] = p;
         total += p;
     }
-    total = sigmoid ? 1.0f : wave_sum(total);
+    total = how.sigmoid ? 1.0f : wave_sum(total);
     for (int e = lane; e < n_experts; e += WAVE) {
         const float s = score[e] / total;
         score[e] = s;
-        choice[e] = s + (correction ? correction[e] : 0.0f);
+        choice[e] = s + (how.correction ? how.correction[e] : 0.0f);
     }
-    __syncthreads();
-    const int size = n_experts / n_groups;
-    for (int g = lane; g < n_groups; g += WAVE) {
-        float best = -INFINITY;
-        for (int e = g * size; e < (g + 1) * size; e++) best = fmaxf(best, choice[e]);
-        group_best[g] = best;
+    __builtin_amdgcn_wave_barrier();
+    __threadfence_block();
+    if (how.n_groups > 1) {
+        const int size = n_experts / how.n_groups;
+        for (int g = lane; g < how.n_groups; g += WAVE) {
+            float best = -INFINITY;
+            for (int e = g * size; e < (g + 1) * size; e++) best = fmaxf(best, choice[e]);
+            group_best[g] = best;
+        }
+        __builtin_amdgcn_wave_barrier();
+        __threadfence_block();
+        for (int g = lane; g < how.n_groups; g += WAVE) {   // a group is kept if fewer than `keep` groups come before it
+            const float mine = group_best[g];
+            int before = 0;
+            for (int o = 0; o < how.n_groups; o++) before += picked_before(group_best[o], o, mine, g) ? 1 : 0;
+            if (before >= how.keep)
+                for (int e = g * size; e < (g + 1) * size; e++) choice[e] = -INFINITY;
+        }
+        __builtin_amdgcn_wave_barrier();
+        __threadfence_block();
     }
-    __syncthreads();
-    for (int g = lane; g < n_groups; g += WAVE) {   // a group is kept if fewer than `keep` groups come before it
-        const float mine = group_best[g];
-        int before = 0;
-        for (int o = 0; o < n_groups; o++) before += picked_before(group_best[o], o, mine, g) ? 1 : 0;
-        if (before >= keep)
-            for (int e = g * size; e < (g + 1) * size; e++) choice[e] = -INFINITY;
-    }
-    __syncthreads();
     float picked_sum = 0.0f;
     for (int e = lane; e < n_experts; e += WAVE) {
         const float mine = choice[e];
         int before = 0;
         for (int o = 0; o < n_experts; o++) before += picked_before(choice[o], o, mine, e) ? 1 : 0;
-        const bool picked = before < top && mine > -INFINITY;
+        const bool picked = before < how.top && mine > -INFINITY;
         picked_sum += picked ? score[e] : 0.0f;
-        group_best[e] = picked ? 1.0f : 0.0f;   // every lane reads and writes its own experts' entries only from here on
+        group_best[e] = picked ? (float)before : -1.0f;   // every lane reads and writes its own experts' entries only from here on
     }
-    picked_sum = renormalise ? wave_sum(picked_sum) + floor : 1.0f;
-    for (int e = lane; e < n_experts; e += WAVE) weights[(size_t)row * weights_stride + e] = group_best[e] != 0.0f ? score[e] / picked_sum : 0.0f;
+    picked_sum = how.renormalise ? wave_sum(picked_sum) + how.floor : 1.0f;
+    for (int e = lane; e < n_experts; e += WAVE) {
+        const int place = (int)group_best[e];
+        const float weight = place >= 0 ? score[e] / picked_sum : 0.0f;
+        if (to.weights) to.weights[row * to.stride + e] = weight;
+        if (to.picks && place >= 0) {
+            to.picks[row * how.top + place] = e;
+            to.pick_weights[row * how.top + place] = weight;
+        }
+    }
+}
+
+// One wave a row. logits: the router's 32-bit sums [row, n_experts] (rows `stride` apart).
+__global__ __launch_bounds__(WAVE) void route_kernel(const float* __restrict__ logits, int stride, Choice how, Routed to) {
+    __shared__ float score[ROUTE_MAX_EXPERTS], choice[ROUTE_MAX_EXPERTS], group_best[ROUTE_MAX_EXPERTS];
+    const int lane = threadIdx.x;
+    const size_t row = blockIdx.x;
+    for (int e = lane; e < how.n_experts; e += WAVE) score[e] = logits[row * stride + e];
+    route_row(how, to, row, score, choice, group_best, lane);
+}
+
+// The router's product and its choice in one: four waves share a row's experts, a wave an expert at a time (16-byte pieces of x and of
+// the expert's row of the router's matrix [n_experts, K], sums in 32-bit), then the first wave chooses. For routers of few outputs: the
+// matrix is read once a row.
+template <typename T>
+__global__ __launch_bounds__(256) void route_rows_kernel(const T* __restrict__ x, const T* __restrict__ router, int K, Choice how, Routed to) {
+    __shared__ float score[ROUTE_FEW_EXPERTS], choice[ROUTE_FEW_EXPERTS], group_best[ROUTE_FEW_EXPERTS];
+    constexpr int VEC = 16 / (int)sizeof(T);
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
+    const size_t row = blockIdx.x;
+    const T* x_row = x + row * K;
+    for (int e0 = wave; e0 < how.n_experts; e0 += 8) {   // two experts of a wave at a time
+        const int e1 = min(e0 + 4, how.n_experts - 1);
+        float sum0 = 0.0f, sum1 = 0.0f;
+        for (int k = lane * VEC; k < K; k += WAVE * VEC) {
+            const Vec16 xs = *reinterpret_cast<const Vec16*>(x_row + k), a = *reinterpret_cast<const Vec16*>(router + (size_t)e0 * K + k),
+                        b = *reinterpret_cast<const Vec16*>(router + (size_t)e1 * K + k);
+            const T *xe = reinterpret_cast<const T*>(&xs), *ae = reinterpret_cast<const T*>(&a), *be = reinterpret_cast<const T*>(&b);
+#pragma unroll
+            for (int j = 0; j < VEC; j++) {
+                sum0 = __builtin_fmaf(to_float(xe[j]), to_float(ae[j]), sum0);
+                sum1 = __builtin_fmaf(to_float(xe[j]), to_float(be[j]), sum1);
+            }
+        }
+        sum0 = wave_total(sum0);
+        sum1 = wave_total(sum1);
+        if (lane == 0) {
+            score[e0] = sum0;
+            if (e0 + 4 < how.n_experts) score[e0 + 4] = sum1;
+        }
+    }
+    __syncthreads();
+    if (wave == 0) route_row(how, to, row, score, choice, group_best, lane);
 }
 
 // up: [rows, n_routed * ff + shared] hidden units before their activation, expert by expert, then `shared` units of an expert that
@@ -142,17 +211,6 @@ __global__ __launch_bounds__(256) void gate_unit_kernel(const T* __restrict__ bo
         const float u = fminf(fmaxf(to_float(*u_at), -limit), limit);
         *out_at = from_float<T>(g / (1.0f + expf(-alpha * g)) * (u + shift));
     }
-}
-
-// The gate unit of feed-forwards with clamped halves: gate * sigmoid(alpha * gate) * (up + shift), gate = min(g, limit), up = clamp(u,
-// -limit, limit).
-struct GateUnit {
-    float limit, alpha, shift;
-};
-__device__ __forceinline__ float gated(float g, float u, const GateUnit& unit) {
-    g = fminf(g, unit.limit);
-    u = fminf(fmaxf(u, -unit.limit), unit.limit);
-    return g / (1.0f + expf(-unit.alpha * g)) * (u + unit.shift);
 }
 
 // both: [rows, n_experts * 2 * ff], per expert its gate sums and then its up sums. out [rows, n_experts * ff] = the gate unit, times the
@@ -232,16 +290,51 @@ void launch_gate_unit(const void* both, void* out, int rows, int inner, float li
 
 }  // namespace
 
-MLLM_API int mllm_route(const float* logits, int stride, const float* correction, float* weights, int weights_stride, int n_rows, int n_experts, int top,
-                        int n_groups, int keep, float floor, int sigmoid, int renormalise, hipStream_t stream) {
-    MLLM_REQUIRE(n_rows >= 0 && n_experts > 0 && n_experts <= ROUTE_MAX_EXPERTS, "route: %d experts (the kernel takes up to %d)", n_experts, ROUTE_MAX_EXPERTS);
-    MLLM_REQUIRE(n_groups >= 1 && n_experts % n_groups == 0 && keep >= 1 && keep <= n_groups, "route: %d experts in %d groups of which %d are kept", n_experts, n_groups, keep);
-    MLLM_REQUIRE(top >= 1 && top <= keep * (n_experts / n_groups), "route: %d experts to pick among %d groups of %d", top, keep, n_experts / n_groups);
-    MLLM_REQUIRE(stride >= n_experts && weights_stride >= n_experts && logits != nullptr && weights != nullptr, "route: rows are too short or missing");
+namespace {
+int check_choice(int n_rows, const Choice& how, const Routed& to) {
+    MLLM_REQUIRE(n_rows >= 0 && how.n_experts > 0 && how.n_experts <= ROUTE_MAX_EXPERTS, "route: %d experts (the kernel takes up to %d)", how.n_experts, ROUTE_MAX_EXPERTS);
+    MLLM_REQUIRE(how.n_groups >= 1 && how.n_experts % how.n_groups == 0 && how.keep >= 1 && how.keep <= how.n_groups, "route: %d experts in %d groups of which %d are kept",
+                 how.n_experts, how.n_groups, how.keep);
+    MLLM_REQUIRE(how.top >= 1 && how.top <= how.keep * (how.n_experts / how.n_groups), "route: %d experts to pick among %d groups of %d", how.top, how.keep,
+                 how.n_experts / how.n_groups);
+    MLLM_REQUIRE((to.weights != nullptr || to.picks != nullptr) && (to.picks == nullptr) == (to.pick_weights == nullptr), "route: nowhere to leave the choice");
+    MLLM_REQUIRE(to.weights == nullptr || to.stride >= how.n_experts, "route: the weights' rows are too short");
+    return 0;
+}
+}  // namespace
+
+MLLM_API int mllm_route(const float* logits, int stride, const float* correction, float* weights, int weights_stride, int* picks, float* pick_weights, int n_rows,
+                        int n_experts, int top, int n_groups, int keep, float floor, int sigmoid, int renormalise, hipStream_t stream) {
+    const Choice how{correction, n_experts, top, n_groups, keep, floor, sigmoid, renormalise};
+    const Routed to{weights, weights_stride, picks, pick_weights};
+    if (int status = check_choice(n_rows, how, to)) return status;
+    MLLM_REQUIRE(stride >= n_experts && logits != nullptr, "route: rows are too short or missing");
     if (n_rows == 0) return 0;
     mllm_count_kernel(MLLM_K_ROUTE);
-    route_kernel<<<n_rows, WAVE, 0, stream>>>(logits, stride, correction, weights, weights_stride, n_experts, top, n_groups, keep, floor, sigmoid, renormalise);
+    route_kernel<<<n_rows, WAVE, 0, stream>>>(logits, stride, how, to);
     return mllm_check_launch("route");
+}
+
+// Whether the router's product rides in the choice's kernel (mllm_route_rows): few outputs, rows of whole 16-byte pieces.
+MLLM_API int mllm_route_rows_supported(int n_experts, int K, int dtype) {
+    const int vec = dtype == MLLM_F32 ? 4 : 8;
+    return n_experts >= 1 && n_experts <= ROUTE_FEW_EXPERTS && K >= vec && K % vec == 0;
+}
+
+MLLM_API int mllm_route_rows(const void* x, const void* router, int K, const float* correction, float* weights, int weights_stride, int* picks,
+                             float* pick_weights, int n_rows, int n_experts, int top, int n_groups, int keep, float floor, int sigmoid, int renormalise,
+                             int dtype, hipStream_t stream) {
+    const Choice how{correction, n_experts, top, n_groups, keep, floor, sigmoid, renormalise};
+    const Routed to{weights, weights_stride, picks, pick_weights};
+    if (int status = check_choice(n_rows, how, to)) return status;
+    MLLM_REQUIRE(dtype == MLLM_F32 || dtype == MLLM_BF16, "route_rows: unknown dtype %d", dtype);
+    MLLM_REQUIRE(mllm_route_rows_supported(n_experts, K, dtype), "route_rows: no kernel for %d outputs over rows of %d", n_experts, K);
+    MLLM_REQUIRE(((uintptr_t)x & 15) == 0 && ((uintptr_t)router & 15) == 0 && x && router, "route_rows: rows and matrix must start on 16 bytes");
+    if (n_rows == 0) return 0;
+    mllm_count_kernel(MLLM_K_ROUTE);
+    if (dtype == MLLM_F32) route_rows_kernel<float><<<n_rows, 256, 0, stream>>>((const float*)x, (const float*)router, K, how, to);
+    else route_rows_kernel<bf16_t><<<n_rows, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)router, K, how, to);
+    return mllm_check_launch("route_rows");
 }
 
 MLLM_API int mllm_expert_unit(const void* up, void* out, const float* weights, int weights_stride, int n_rows, int n_routed, int ff, int shared, const void* h,

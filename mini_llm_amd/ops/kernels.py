@@ -1332,27 +1332,109 @@ def gate_unit(both, limit: float | None = None, alpha: float = 1.0, shift: float
 ROUTE_MAX_EXPERTS = 1024
 
 
-def route(logits, n_experts: int, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0, score: str = "softmax",
-          renormalise: bool = True):
-    """A router's choice, row by row. ``logits``: float32 rows whose first ``n_experts`` columns are the router's sums (rows may be
-    strided). Scores are their softmax over all experts or, with ``score`` "sigmoid", each one's own sigmoid; the choice goes by score + correction (float32 [n_experts]; None: by the score)
-    among the experts of the ``keep`` best of ``n_groups`` equal groups of neighbours (a group counts by its best choice score); the ``top``
-    best are picked. Returns float32 [rows, n_experts]: a picked expert's score over (the sum of the picked scores + floor), without
-    ``renormalise`` its score itself, zero for the rest."""
-    _require(score in ("softmax", "sigmoid"), "scores are a softmax or sigmoids")
-    _require(isinstance(logits, torch.Tensor) and logits.is_cuda and logits.dim() == 2 and logits.dtype == torch.float32 and logits.stride(1) == 1
-             and logits.shape[1] >= n_experts, "the router's sums must be float32 GPU rows with contiguous columns")
+@dataclass
+class Picks:
+    """What a router picked for every row: ``experts`` int32 [rows, top] (in the order of their choice scores; -1 where sums that are no
+    numbers left none to pick) and ``weights`` float32 [rows, top]."""
+
+    experts: torch.Tensor
+    weights: torch.Tensor
+
+
+def _choice(n, device, n_experts, top, correction, n_groups, keep, score, dense, picks):
     _require(1 <= n_experts <= ROUTE_MAX_EXPERTS, f"the router kernel takes up to {ROUTE_MAX_EXPERTS} experts")
     _require(n_groups >= 1 and n_experts % n_groups == 0 and 1 <= keep <= n_groups, "the experts do not divide into the groups")
     _require(1 <= top <= keep * (n_experts // n_groups), "more experts to pick than the kept groups hold")
+    _require(score in ("softmax", "sigmoid"), "scores are a softmax or sigmoids")
     if correction is not None:
         _device_tensor(correction, "correction", torch.float32, 1)
         _require(correction.shape[0] == n_experts, "one correction an expert")
+    weights = torch.empty((n, n_experts), dtype=torch.float32, device=device) if dense else None
+    picked = Picks(torch.empty((n, top), dtype=torch.int32, device=device), torch.empty((n, top), dtype=torch.float32, device=device)) if picks else None
+    return weights, picked
+
+
+def route(logits, n_experts: int, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0, score: str = "softmax",
+          renormalise: bool = True, picks: bool = False):
+    """A router's choice, row by row. ``logits``: float32 rows whose first ``n_experts`` columns are the router's sums (rows may be
+    strided). Scores are their softmax over all experts or, with ``score`` "sigmoid", each one's own sigmoid; the choice goes by score +
+    correction (float32 [n_experts]; None: by the score) among the experts of the ``keep`` best of ``n_groups`` equal groups of neighbours (a
+    group counts by its best choice score); the ``top`` best are picked. Returns float32 [rows, n_experts]: a picked expert's score over (the
+    sum of the picked scores + floor), without ``renormalise`` its score itself, zero for the rest; or with ``picks`` the same as ``Picks``."""
+    _require(isinstance(logits, torch.Tensor) and logits.is_cuda and logits.dim() == 2 and logits.dtype == torch.float32 and logits.stride(1) == 1
+             and logits.shape[1] >= n_experts, "the router's sums must be float32 GPU rows with contiguous columns")
     n = logits.shape[0]
-    weights = torch.empty((n, n_experts), dtype=torch.float32, device=logits.device)
-    check(library().mllm_route(_ptr(logits), logits.stride(0), _ptr(correction), _ptr(weights), n_experts, n, n_experts, int(top), int(n_groups), int(keep),
-                               float(floor), int(score == "sigmoid"), int(bool(renormalise)), _stream()))
-    return weights
+    weights, picked = _choice(n, logits.device, n_experts, top, correction, n_groups, keep, score, not picks, picks)
+    check(library().mllm_route(_ptr(logits), logits.stride(0), _ptr(correction), _ptr(weights), n_experts, _ptr(picked.experts if picks else None),
+                               _ptr(picked.weights if picks else None), n, n_experts, int(top), int(n_groups), int(keep), float(floor),
+                               int(score == "sigmoid"), int(bool(renormalise)), _stream()))
+    return picked if picks else weights
+
+
+def route_rows_supported(n_experts: int, width: int, dtype) -> bool:
+    """Whether ``route_rows`` takes a router of so many outputs over rows of ``width`` elements."""
+    return bool(library().mllm_route_rows_supported(int(n_experts), int(width), _code(dtype)))
+
+
+def route_rows(x, router, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0, score: str = "softmax",
+               renormalise: bool = True, picks: bool = False):
+    """``route`` with the router's product inside: x [rows, width] and the router's matrix [n_experts, width] (row-major), both of one element
+    type; sums in 32-bit. For routers of few outputs (``route_rows_supported``)."""
+    _device_tensor(x, "x", dim=2)
+    _device_tensor(router, "router", x.dtype, 2)
+    n, width = x.shape
+    n_experts = router.shape[0]
+    _require(router.shape[1] == width, "x and the router's matrix differ in width")
+    _require(route_rows_supported(n_experts, width, x.dtype), f"no kernel routes {n_experts} experts over rows of {width}")
+    weights, picked = _choice(n, x.device, n_experts, top, correction, n_groups, keep, score, not picks, picks)
+    check(library().mllm_route_rows(_ptr(x), _ptr(router), width, _ptr(correction), _ptr(weights), n_experts, _ptr(picked.experts if picks else None),
+                                    _ptr(picked.weights if picks else None), n, n_experts, int(top), int(n_groups), int(keep), float(floor),
+                                    int(score == "sigmoid"), int(bool(renormalise)), _code(x.dtype), _stream()))
+    return picked if picks else weights
+
+
+def grouped_experts_supported(width: int, units: int, dtype) -> bool:
+    """Whether ``grouped_experts`` takes experts of so many (padded) hidden units over rows of ``width`` elements."""
+    return bool(library().mllm_experts_supported(int(width), int(units), _code(dtype)))
+
+
+def grouped_experts(x, picks: Picks, up: PackedMatrix, down: PackedMatrix, n_experts: int, units: int, *, limit: float | None = None, alpha: float = 1.0,
+                    shift: float = 0.0, weigh_input: bool = False):
+    """The picked experts of every row, and no others: float32 [top, rows, width], whose plane k is the k-th pick's expert, W_down unit(W_gate
+    h, W_up h) with the gate unit of ``gate_unit`` and the pick's weight on the unit or (``weigh_input``) on both sums. x: bfloat16 [rows, width]. ``up``
+    [n_experts * 2 * units, width]: per expert, for every 32 units, 32 gate rows and 32 up rows; ``down`` [n_experts * width, units]: the experts'
+    matrices behind each other; ``units`` a multiple of 64 (zero rows and columns fill an expert up). Few rows find their experts inside the
+    products; more rows are sorted by expert on the device first. A pick of -1 leaves its place undefined."""
+    _device_tensor(x, "x", torch.bfloat16, 2)
+    n, width = x.shape
+    _device_tensor(picks.experts, "picks", torch.int32, 2)
+    _device_tensor(picks.weights, "the picks' weights", torch.float32, 2)
+    top = picks.experts.shape[1]
+    _require(tuple(picks.experts.shape) == (n, top) and tuple(picks.weights.shape) == (n, top), "picks and rows differ")
+    _require(limit is None or limit > 0, "the limit must be positive")
+    for matrix, name, shape in ((up, "up", (n_experts * 2 * units, width)), (down, "down", (n_experts * width, units))):
+        _require(isinstance(matrix, PackedMatrix) and matrix.dtype == torch.bfloat16 and tuple(matrix.shape) == shape, f"{name} must be packed, bfloat16, {shape}")
+    _require(grouped_experts_supported(width, units, x.dtype), f"no kernel for experts of {units} units over rows of {width}")
+    lib = library()
+    out = torch.empty((top, n, width), dtype=torch.float32, device=x.device)
+    entries = n * top
+    hidden = torch.empty((entries, units), dtype=torch.bfloat16, device=x.device)
+    unit = (float("inf") if limit is None else float(limit), float(alpha), float(shift), int(bool(weigh_input)))
+    if n <= int(lib.mllm_experts_few_rows()):
+        check(lib.mllm_experts_few_up(_ptr(x), _ptr(up.data), _ptr(hidden), _ptr(picks.experts), _ptr(picks.weights), n, top, int(n_experts), int(units), width, *unit, _stream()))
+        check(lib.mllm_experts_few_down(_ptr(hidden), _ptr(down.data), _ptr(out), _ptr(picks.experts), n, top, int(n_experts), int(units), width, _stream()))
+        return out
+    tile = int(lib.mllm_expert_tile_rows())
+    max_tiles = entries // tile + min(n_experts, entries)
+    # one piece of memory for the lists: tiles first (they start on 16 bytes), then rows, places, weights and the number of tiles
+    lists = torch.empty((4 * max_tiles + 3 * entries + 1,), dtype=torch.int32, device=x.device)
+    tiles, rows, places = lists[: 4 * max_tiles], lists[4 * max_tiles : 4 * max_tiles + entries], lists[4 * max_tiles + entries : 4 * max_tiles + 2 * entries]
+    weights, n_tiles = lists[4 * max_tiles + 2 * entries : 4 * max_tiles + 3 * entries], lists[4 * max_tiles + 3 * entries :]
+    check(lib.mllm_expert_lists(_ptr(picks.experts), _ptr(picks.weights), n, top, int(n_experts), tile, _ptr(rows), _ptr(places), _ptr(weights), _ptr(tiles), _ptr(n_tiles),
+                                _stream()))
+    check(lib.mllm_experts_up(_ptr(x), _ptr(up.data), _ptr(hidden), _ptr(tiles), _ptr(n_tiles), _ptr(rows), _ptr(weights), entries, max_tiles, int(units), width, *unit, _stream()))
+    check(lib.mllm_experts_down(_ptr(hidden), _ptr(down.data), _ptr(out), _ptr(tiles), _ptr(n_tiles), _ptr(places), entries, max_tiles, int(units), width, _stream()))
+    return out
 
 
 def expert_unit(up, weights, n_routed: int, ff: int, shared: int = 0, *, h=None, n_identity: int = 0, carried_out=None):

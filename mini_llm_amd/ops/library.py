@@ -54,7 +54,17 @@ _SIGNATURES = {
     "mllm_map_rows": [P, c_int, c_int, c_int, c_int, P, P, c_float, P, c_int, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                       c_int, P, c_int, c_int, P],
     "mllm_turn_heads": [P, c_int, P, c_int, P, c_int, c_int, c_float, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_route": [P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, P],
+    "mllm_route": [P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, P],
+    "mllm_route_rows_supported": [c_int, c_int, c_int],
+    "mllm_route_rows": [P, P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, P],
+    "mllm_expert_tile_rows": [],
+    "mllm_experts_few_rows": [],
+    "mllm_experts_supported": [c_int, c_int, c_int],
+    "mllm_expert_lists": [P, P, c_int, c_int, c_int, c_int, P, P, P, P, P, P],
+    "mllm_experts_up": [P, P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, P],
+    "mllm_experts_down": [P, P, P, P, P, P, c_int, c_int, c_int, c_int, P],
+    "mllm_experts_few_up": [P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, P],
+    "mllm_experts_few_down": [P, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P],
     "mllm_gated_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_int, P],
     "mllm_gated_scan": [P, c_int, c_int, c_int, c_int, P, c_longlong, P, P, P, c_int, c_int, c_int, c_int, c_float, c_int, P, c_longlong, c_int, P],

@@ -19,7 +19,10 @@ down matrices laid side by side: ``kernels.expert_unit`` between the two multipl
 row, zero where the router did not pick it, so the down product's sum is the weighted sum over the picked experts; the share of the
 experts that hand h on rides in as that product's residual operand. A row's result is a function of the row alone, nothing is planned
 on the host, and a captured step replays it. The price is the arithmetic of the experts that were not picked: E / top times the needed
-work in the two products, which few rows (decoding) do not notice, since they read every expert's matrices anyway."""
+work in the two products, which few rows (decoding) do not notice, since they read every expert's matrices anyway.
+
+Experts with a gate unit run grouped instead where the kernels take the sizes (bfloat16, a width that is a multiple of 64): each expert for
+the rows that picked it alone (``kernels.grouped_experts``), planned on the device."""
 
 from __future__ import annotations
 
@@ -55,7 +58,8 @@ class RoutedExperts(FeedForward):
         self.n_outputs = total
         self.score, self.renormalise, self.weigh_input = score, bool(renormalise), weigh == "input"
         self.gated, self.limit, self.alpha, self.shift = unit == "clamped_gate", limit, float(alpha), float(shift)
-        self.router = self.correction = self.up = self.down = self._router_rows = None
+        self.router = self.correction = self.up = self.down = self._router_rows = self._small_router = None
+        self.grouped, self.units = False, ff
         self.shared_units = 0   # the shared expert's hidden units and the zeros that fill the up matrix to whole blocks
         self._down_product = BranchProduct()
         self.sums_later = False   # True: a call without a residual may return kernels.BranchRows (the block that adds the branch takes its sums)
@@ -81,6 +85,8 @@ class RoutedExperts(FeedForward):
         router = fuse_rows([tensors["router"]])
         self._router_rows = router
         self.router = kernels.pack_matrix(router) if router.is_cuda else router
+        if router.is_cuda and kernels.route_rows_supported(self.n_outputs, self.width, router.dtype):
+            self._small_router = tensors["router"].contiguous()
         self.correction = tensors.get("correction")
         if self.gated:
             self._bind_gated(tensors, names)
@@ -97,16 +103,50 @@ class RoutedExperts(FeedForward):
         self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
 
     def _bind_gated(self, tensors, names):
-        up = torch.cat([tensors[name + part] for name in names for part in ("gate", "up")], dim=0).contiguous()
-        down = torch.cat([tensors[name + "down"] for name in names], dim=1).contiguous()
-        self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
+        """Grouped (the experts run for the rows that picked them: ``kernels.grouped_experts``) where the sizes allow, else all experts as one
+        up and one down product with zeros for the units that were not picked."""
+        sample = tensors[names[0] + "up"]
+        self.units = -(-self.ff // 64) * 64
+        self.grouped = sample.is_cuda and kernels.grouped_experts_supported(self.width, self.units, sample.dtype)
+        if not self.grouped:
+            up = torch.cat([tensors[name + part] for name in names for part in ("gate", "up")], dim=0).contiguous()
+            down = torch.cat([tensors[name + "down"] for name in names], dim=1).contiguous()
+            self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
+            return
+        E, units, width = self.n_experts, self.units, self.width
+        up = torch.zeros((E, units // 32, 2, 32, width), dtype=sample.dtype, device=sample.device)   # 32 gate rows and 32 up rows in turn
+        down = torch.zeros((E, width, units), dtype=sample.dtype, device=sample.device)
+        for e, name in enumerate(names):
+            for half, part in enumerate(("gate", "up")):
+                padded = torch.zeros((units, width), dtype=sample.dtype, device=sample.device)
+                padded[: self.ff] = tensors[name + part]
+                up[e, :, half] = padded.view(units // 32, 32, width)
+            down[e, :, : self.ff] = tensors[name + "down"]
+        self.up, self.down = kernels.pack_matrix(up.view(E * 2 * units, width)), kernels.pack_matrix(down.view(E * width, units))
 
-    def _forward_gated(self, x, weights, residual):
-        units = kernels.gated_expert_unit(kernels.linear(x, self.up), weights, self.n_experts, self.ff, limit=self.limit, alpha=self.alpha, shift=self.shift,
-                                          weigh_input=self.weigh_input)
-        if residual is None and self.sums_later:
-            return self._down_product.later(units, self.down)
-        return self._down_product(units, self.down, residual)
+    def _forward_gated(self, x, carried, residual):
+        unit = dict(limit=self.limit, alpha=self.alpha, shift=self.shift, weigh_input=self.weigh_input)
+        if not self.grouped:
+            units = kernels.gated_expert_unit(kernels.linear(x, self.up), self._route(x, carried), self.n_experts, self.ff, **unit)
+            if residual is None and self.sums_later:
+                return self._down_product.later(units, self.down)
+            return self._down_product(units, self.down, residual)
+        planes = kernels.grouped_experts(x, self._route(x, carried, picks=True), self.up, self.down, self.n_experts, self.units, **unit)
+        if residual is not None:
+            return kernels.settle(kernels.PendingRows(residual, planes, None))
+        if self.sums_later:
+            return kernels.BranchRows(planes, None)
+        return planes[0] if self.top == 1 else planes   # several picks: partial sums, as a product cut along K leaves them
+
+    def _route(self, x, carried=None, picks: bool = False):
+        """The router's sums (its product inside the choice's kernel where that takes it, or its own, or what another product carried along)
+        and its choice."""
+        how = dict(correction=self.correction, n_groups=self.n_groups, keep=self.keep, floor=self.floor, score=self.score, renormalise=self.renormalise,
+                   picks=picks)
+        if carried is None and self._small_router is not None:
+            return kernels.route_rows(x, self._small_router, self.top, **how)
+        logits = carried if carried is not None else kernels.linear(x, self.router, out_dtype=torch.float32)
+        return kernels.route(logits, self.n_outputs, self.top, **how)
 
     def rows_to_carry(self):
         """The router's matrix (and no bias), for a block that lets another product over the same input rows carry it along; ``forward`` is
@@ -114,11 +154,9 @@ class RoutedExperts(FeedForward):
         return self._router_rows, None
 
     def forward(self, x, residual, carried=None):
-        logits = carried if carried is not None else kernels.linear(x, self.router, out_dtype=torch.float32)
-        weights = kernels.route(logits, self.n_outputs, self.top, correction=self.correction, n_groups=self.n_groups, keep=self.keep, floor=self.floor,
-                                score=self.score, renormalise=self.renormalise)
         if self.gated:
-            return self._forward_gated(x, weights, residual)
+            return self._forward_gated(x, carried, residual)
+        weights = self._route(x, carried)
         if self.up is None:   # nothing but experts that hand their input on
             raise ValueError("a routed feed-forward needs at least one expert with matrices")
         if residual is None and self.sums_later:

@@ -28,6 +28,26 @@ def sharpen(config, weights, factor=3.0):
     return weights
 
 
+def settle_routers(config, weights, seed=1):
+    """Routers without a close call, for bfloat16 runs: every token has a level of its own in as many columns of the stream as there are experts
+    at most, evenly spaced and in a random order, which nothing else writes to; router output e reads column e. The picks and their
+    weights then differ from token to token, but no rounding of the router's input changes one."""
+    most = max(entry["mlp"]["router"]["experts"] for entry in config["layers"] if entry["mlp"] is not None)
+    rng = np.random.default_rng(seed)
+    levels = np.linspace(-2.0, 2.0, most) if most > 1 else np.array([0.5])
+    weights["embed"][:, :most] = np.stack([rng.permutation(levels) for _ in range(config["vocab"])])
+    weights["bigram"][:, :most] = 0.0
+    for index, entry in enumerate(config["layers"]):
+        weights[f"l{index}.mix.o"][:most] = 0.0
+        if entry["mlp"] is not None:
+            router = weights[f"l{index}.mlp.router"]
+            router[:] = 0.0
+            for e in range(router.shape[0]):
+                router[e, e] = 1.5
+                weights[f"l{index}.mlp.e{e}.down"][:most] = 0.0
+    return {name: plain_gpt2.round_to_bf16(np.asarray(value, dtype=np.float32)) for name, value in weights.items()}
+
+
 @pytest.fixture(scope="module")
 def goletar_dirs(tmp_path_factory):
     out = {}
@@ -35,6 +55,9 @@ def goletar_dirs(tmp_path_factory):
         weights = sharpen(config, plain.random_weights(config, 60 + seed))
         folder = plain.write_model_dir(tmp_path_factory.mktemp(f"goletar_{name}"), config, weights)
         out[name] = (folder, copy.deepcopy(config), weights)
+        weights = settle_routers(config, sharpen(config, plain.random_weights(config, 60 + seed)))
+        folder = plain.write_model_dir(tmp_path_factory.mktemp(f"goletar_{name}_settled"), config, weights)
+        out[name, "bfloat16"] = (folder, copy.deepcopy(config), weights)
     return out
 
 
@@ -55,13 +78,11 @@ TOLERANCE = {"float32": dict(atol=3e-4, rtol=2e-4)}   # sums in another order th
 
 def check(got, config, weights, requests, dtype):
     """32-bit: every logit of every position within the tolerance (one position in a hundred may be up to five times off: a router whose
-    two candidates lie within rounding of each other picks the other one). bfloat16: the engine rounds at other places than the plain
-    implementation does when it rounds what a bfloat16 run stores, so the two are not compared with each other but each with exact
-    arithmetic, position by position (root mean square over a position's logits): the engine's distance may be three times the plain
-    bfloat16 run's at nine positions in ten, and one and a half times in the median. Where two experts' scores lie within a bfloat16 rounding
-    of the router's input, either run may pick either, which moves that position's logits by an expert's whole share, and, through keys and
-    states, those behind it a little; so the bound is on quantiles. A wrong key, page or slot moves the logits of every position behind it by
-    tens of times the noise, and shows at once in the 32-bit run of the same trace."""
+    two candidates lie within rounding of each other picks the other one). bfloat16 (weights of ``settle_routers``): the engine rounds at
+    other places than the plain implementation does when it rounds what a bfloat16 run stores, so the two are not compared with each other
+    but each with exact arithmetic, position by position (root mean square over a position's logits): the engine's distance may be three
+    times the plain bfloat16 run's at 98 positions in a hundred, and one and a half times in the median and over all positions together. A
+    wrong key, page or slot moves the logits of every position behind it by tens of times the noise."""
     exact = plain_logits(config, weights, requests, False)
     if dtype == "float32":
         atol, rtol = TOLERANCE[dtype]["atol"], TOLERANCE[dtype]["rtol"]
@@ -78,15 +99,15 @@ def check(got, config, weights, requests, dtype):
         error.append(np.sqrt(((np.stack([got[name][p] for p in range(len(rows))]).astype(np.float64) - rows) ** 2).mean(axis=1)))
     noise, error = np.concatenate(noise), np.concatenate(error)
     ratio = error / (noise + 0.05 * np.median(noise) + 1e-3)
-    assert np.quantile(ratio, 0.9) <= 3.0 and np.median(ratio) <= 1.5, (np.quantile(ratio, 0.9), np.median(ratio), ratio.max(), int(ratio.argmax()))
-    assert np.median(error) <= 1.5 * np.median(noise) + 1e-3, (np.median(error), np.median(noise))
+    assert np.quantile(ratio, 0.98) <= 3.0 and np.median(ratio) <= 1.5, (np.quantile(ratio, 0.98), np.median(ratio), ratio.max(), int(ratio.argmax()))
+    assert np.sqrt((error**2).mean()) <= 1.5 * np.sqrt((noise**2).mean()) + 1e-3, "rms error against rms noise"
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("mode", list(MODES))
 @pytest.mark.parametrize("name", list(CASES))
 def test_replay_matches_plain(goletar_dirs, tmp_path, name, mode, dtype):
-    folder, config, weights = goletar_dirs[name]
+    folder, config, weights = goletar_dirs[name if dtype == "float32" else (name, dtype)]
     requests = requests_for(config, LENGTHS[name])
     collector = MODES[mode](requests)
     for page_size in ((None, 16) if mode == "mixed" and dtype == "float32" else (None,)):
@@ -186,7 +207,7 @@ def test_the_sink_and_the_heads_gates_show(tmp_path):
     for name, value in (("l0.mix.sink", -30.0), ("l0.mix.g", 0.0)):
         changed = dict(weights)
         changed[name] = np.full_like(weights[name], value)
-        assert np.abs(plain.forward(config, plain.as_float64(changed), requests["r0"]) - base).max(axis=1).min() > 1e-2, name
+        assert np.median(np.abs(plain.forward(config, plain.as_float64(changed), requests["r0"]) - base).max(axis=1)) > 5e-2, name
 
 
 def test_a_state_that_hardly_fades(tmp_path):
@@ -267,7 +288,7 @@ def test_every_constant_of_the_design_shows(tmp_path):
 def test_generation_through_the_engine_and_its_scheduler(goletar_dirs, name, dtype):
     from mini_llm_amd.engine.engine import Engine, EngineOptions
 
-    folder, config, weights = goletar_dirs[name]
+    folder, config, weights = goletar_dirs[name if dtype == "float32" else (name, dtype)]
     prompts = [random_tokens(9, 5, config["vocab"]), random_tokens(10, 70, config["vocab"]), [3], random_tokens(11, 31, config["vocab"]), random_tokens(13, 66, config["vocab"])]
     # few pages: the requests do not all fit at once, so pages and slots are given back and used again
     with Engine(folder, EngineOptions(dtype=dtype, max_sessions=4, max_length=256, max_tokens=256)) as engine:
@@ -324,7 +345,7 @@ def test_captured_steps_match_eager_ones_over_many_replays(goletar_dirs, dtype):
     from mini_llm_amd.engine import StepEntry
     from mini_llm_amd.engine.engine import Engine, EngineOptions
 
-    folder, config, _ = goletar_dirs["mixed"]
+    folder, config, _ = goletar_dirs["mixed" if dtype == "float32" else ("mixed", dtype)]
     rng = np.random.default_rng(1)
     logits = {}
     plan = []

@@ -13,20 +13,45 @@ namespace {
 constexpr int MAX_EXPERTS = 1024;
 
 // The lists, a block an expert, without an atomic that could order them: entries of an expert in the order of their rows, experts behind
-// each other. Every block counts all experts' entries (so that it knows where its own begin) and places its own.
-__global__ __launch_bounds__(256) void expert_lists_kernel(const int* __restrict__ picks, const float* __restrict__ pick_weights, int n_rows, int top, int n_experts,
-                                                           int tile_rows, int* __restrict__ a_row, int* __restrict__ out_row, float* __restrict__ weight,
-                                                           int4* __restrict__ tiles, int* __restrict__ n_tiles) {
+// each other. Every block counts all experts' entries (so that it knows where its own begin) and places its own: wave w counts a
+// contiguous share of the entries, 64 at a time by ballots (of up to 64 experts: lane e keeps expert e's count; of more: by LDS counters,
+// which so many addresses seldom make wait for each other), and places its share behind those of the waves before it.
+constexpr int LIST_WAVES = 16;
+
+__global__ __launch_bounds__(64 * LIST_WAVES) void expert_lists_kernel(const int* __restrict__ picks, const float* __restrict__ pick_weights, int n_rows, int top,
+                                                                       int n_experts, int tile_rows, int* __restrict__ a_row, int* __restrict__ out_row,
+                                                                       float* __restrict__ weight, int4* __restrict__ tiles, int* __restrict__ n_tiles) {
     __shared__ int counts[MAX_EXPERTS];
-    __shared__ int wave_counts[4], start, first_tile;
+    __shared__ int mine_before[LIST_WAVES], start, first_tile;
     const int expert = blockIdx.x, tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
-    const int entries = n_rows * top;
-    for (int e = tid; e < n_experts; e += 256) counts[e] = 0;
+    const int entries = n_rows * top, chunks = (entries + WAVE - 1) / WAVE;
+    const int share = (chunks + LIST_WAVES - 1) / LIST_WAVES, chunk0 = min(chunks, wave * share), chunk1 = min(chunks, chunk0 + share);
+    for (int e = tid; e < n_experts; e += 64 * LIST_WAVES) counts[e] = 0;
     __syncthreads();
-    for (int p = tid; p < entries; p += 256) {
-        const int e = picks[p];
-        if (e >= 0 && e < n_experts) atomicAdd(&counts[e], 1);
+    int mine = 0, of_lane = 0;
+    constexpr int AHEAD = 4;
+    for (int c0 = chunk0; c0 < chunk1; c0 += AHEAD) {
+        int pick[AHEAD];
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++) {
+            const int p = (c0 + u) * WAVE + lane;
+            pick[u] = c0 + u < chunk1 && p < entries ? picks[p] : -1;
+        }
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++) {
+            mine += __popcll(__ballot(pick[u] == expert));
+            if (n_experts <= WAVE) {
+                for (int e = 0; e < n_experts; e++) {
+                    const int n = __popcll(__ballot(pick[u] == e));
+                    of_lane += lane == e ? n : 0;
+                }
+            } else if (pick[u] >= 0 && pick[u] < n_experts) {
+                atomicAdd(&counts[pick[u]], 1);
+            }
+        }
     }
+    if (n_experts <= WAVE && lane < n_experts && of_lane > 0) atomicAdd(&counts[lane], of_lane);
+    if (lane == 0) mine_before[wave] = mine;
     __syncthreads();
     if (wave == 0) {
         int before = 0, tiles_before = 0;
@@ -45,42 +70,55 @@ __global__ __launch_bounds__(256) void expert_lists_kernel(const int* __restrict
         }
     }
     __syncthreads();
-    const int mine = counts[expert], my_tiles = (mine + tile_rows - 1) / tile_rows, first = start;
-    for (int t = tid; t < my_tiles; t += 256) tiles[first_tile + t] = make_int4(expert, first + t * tile_rows, first + mine, 0);
+    const int total = counts[expert], my_tiles = (total + tile_rows - 1) / tile_rows, first = start;
+    for (int t = tid; t < my_tiles; t += 64 * LIST_WAVES) tiles[first_tile + t] = make_int4(expert, first + t * tile_rows, first + total, 0);
     if (expert == n_experts - 1 && tid == 0) *n_tiles = first_tile + my_tiles;
+    if (mine == 0) return;   // (uniform over the wave)
     int placed = first;
-    for (int p0 = 0; p0 < entries; p0 += 256) {   // (the same number of turns for every thread)
-        const int p = p0 + tid;
-        const bool here = p < entries && picks[p] == expert;
-        const unsigned long long ballot = __ballot(here);
-        if (lane == 0) wave_counts[wave] = __popcll(ballot);
-        __syncthreads();
-        int at = placed + __popcll(ballot & ((1ull << lane) - 1));
-        for (int w = 0; w < wave; w++) at += wave_counts[w];
-        placed += wave_counts[0] + wave_counts[1] + wave_counts[2] + wave_counts[3];
-        __syncthreads();
-        if (here) {
-            const int row = p / top;
-            a_row[at] = row;
-            out_row[at] = (p - row * top) * n_rows + row;
-            weight[at] = pick_weights[p];
+    for (int w = 0; w < wave; w++) placed += mine_before[w];
+    for (int c0 = chunk0; c0 < chunk1; c0 += AHEAD) {
+        int pick[AHEAD];
+        float its_weight[AHEAD];
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++) {
+            const int p = (c0 + u) * WAVE + lane, inside = min(p, entries - 1);
+            pick[u] = picks[inside];
+            its_weight[u] = pick_weights[inside];
+            if (c0 + u >= chunk1 || p >= entries) pick[u] = -1;
+        }
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++) {
+            const unsigned long long ballot = __ballot(pick[u] == expert);
+            if (pick[u] == expert) {
+                const int at = placed + __popcll(ballot & ((1ull << lane) - 1)), p = (c0 + u) * WAVE + lane, row = p / top;
+                a_row[at] = row;
+                out_row[at] = (p - row * top) * n_rows + row;
+                weight[at] = its_weight[u];
+            }
+            placed += __popcll(ballot);
         }
     }
 }
 
 constexpr int FEW_ROWS = 64;
 
-// This block's expert: the entries that picked it, in LDS (a row picks an expert at most once, so there are at most FEW_ROWS). Returns
-// how many; called by all threads.
-__device__ __forceinline__ int gather_entries(const int* __restrict__ picks, int entries, int expert, int* list, int* count) {
+// This block's expert: the entries that picked it, and their weights, in LDS (a row picks an expert at most once, so there are at most
+// FEW_ROWS). Returns how many; called by all threads.
+__device__ __forceinline__ int gather_entries(const int* __restrict__ picks, const float* __restrict__ pick_weights, int entries, int expert, int* list,
+                                              float* weights, int* count) {
     if (threadIdx.x < WAVE) {
         int found = 0;
         for (int p0 = 0; p0 < entries; p0 += WAVE) {
-            const int p = p0 + threadIdx.x;
-            const bool here = p < entries && picks[p] == expert;
+            const int p = p0 + threadIdx.x, inside = min(p, entries - 1);
+            const int pick = picks[inside];
+            const float weight = pick_weights ? pick_weights[inside] : 0.0f;
+            const bool here = p < entries && pick == expert;
             const unsigned long long ballot = __ballot(here);
             const int at = found + __popcll(ballot & ((1ull << threadIdx.x) - 1));
-            if (here && at < FEW_ROWS) list[at] = p;
+            if (here && at < FEW_ROWS) {
+                list[at] = p;
+                weights[at] = weight;
+            }
             found += __popcll(ballot);
         }
         if (threadIdx.x == 0) *count = min(found, FEW_ROWS);
@@ -99,9 +137,10 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const bf16_
     constexpr int UNROLL = MT == 4 ? 4 : 8;
     __shared__ float sums[KSPLIT][2 * MT * 4][WAVE];
     __shared__ int list[FEW_ROWS], count;
+    __shared__ float weights[FEW_ROWS];
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, row16 = lane % 16, quad = lane / 16;
     const int expert = blockIdx.y, u0 = blockIdx.x * 16;
-    const int n = gather_entries(picks, n_rows * top, expert, list, &count);
+    const int n = gather_entries(picks, pick_weights, n_rows * top, expert, list, weights, &count);
     if (n == 0) return;   // nobody picked this expert (uniform over the block)
     const int steps = width / 32;   // a multiple of two: the width is one of 64
     const int gate_tile = expert * (2 * units / 16) + u0 / 32 * 4 + u0 / 16 % 2;   // 32 gate rows, 32 up rows in turn
@@ -151,7 +190,7 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const bf16_
             u += sums[w][(MT + i) * 4 + r][l];
         }
         const int p = list[entry];
-        const float weight = pick_weights[p];
+        const float weight = weights[entry];
         const float value = weigh_input ? gated(g * weight, u * weight, unit) : gated(g, u, unit) * weight;
         hidden[(size_t)p * units + u0 + unit_at] = static_cast<bf16_t>(value);
     }
@@ -164,9 +203,10 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const bf1
     constexpr int UNROLL = MT == 4 ? 4 : 8;
     __shared__ float sums[KSPLIT][MT * 4][WAVE];
     __shared__ int list[FEW_ROWS], count;
+    __shared__ float weights[FEW_ROWS];
     const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, row16 = lane % 16, quad = lane / 16;
     const int expert = blockIdx.y, n0 = blockIdx.x * 16;
-    const int n = gather_entries(picks, n_rows * top, expert, list, &count);
+    const int n = gather_entries(picks, nullptr, n_rows * top, expert, list, weights, &count);
     if (n == 0) return;
     const int steps = units / 32, tile = expert * (width / 16) + blockIdx.x;
     const bf16_t* h_row[MT];
@@ -224,7 +264,7 @@ MLLM_API int mllm_expert_lists(const int* picks, const float* pick_weights, int 
     MLLM_REQUIRE(n_rows >= 0 && top >= 1 && n_experts >= 1 && n_experts <= MAX_EXPERTS && tile_rows >= 1 && (long long)n_rows * top < (1LL << 30), "expert_lists: bad sizes");
     MLLM_REQUIRE(picks && pick_weights && a_row && out_row && weight && tiles && n_tiles && ((uintptr_t)tiles & 15) == 0, "expert_lists: a missing operand");
     mllm_count_kernel(MLLM_K_EXPERT_LISTS);
-    expert_lists_kernel<<<n_experts, 256, 0, stream>>>(picks, pick_weights, n_rows, top, n_experts, tile_rows, a_row, out_row, weight, (int4*)tiles, n_tiles);
+    expert_lists_kernel<<<n_experts, 64 * LIST_WAVES, 0, stream>>>(picks, pick_weights, n_rows, top, n_experts, tile_rows, a_row, out_row, weight, (int4*)tiles, n_tiles);
     return mllm_check_launch("expert_lists");
 }
 

@@ -132,17 +132,93 @@ __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(const XT* __rest
     }
     const int row = row0 + lane32;
     if (row >= n_rows) return;
+    float head_factor = 1.0f;
+    if (gate && gate_per_head) head_factor = 1.0f / (1.0f + expf(-load_as_float(gate, (size_t)row * gate_row_stride + head, gate_code)));
+    // a lane holds four neighbouring columns at a time: one store where four elements start on their own size's border
+    const size_t out_at = (size_t)row * out_row_stride + (size_t)head * out_head_stride;
+    const bool fours = N % 4 == 0 && out_row_stride % 4 == 0 && out_head_stride % 4 == 0 && ((size_t)out & 15) == 0;
 #pragma unroll
-    for (int v = 0; v < 16; v++) {
-        const int n = n0 + 8 * (v / 4) + 4 * half + (v % 4);
-        if (n >= N) continue;
-        float value = acc[v];
-        if (gate) {
-            const float g = load_as_float(gate, (size_t)row * gate_row_stride + (gate_per_head ? (size_t)head : (size_t)head * N + n), gate_code);
-            value *= 1.0f / (1.0f + expf(-g));
+    for (int g4 = 0; g4 < 4; g4++) {
+        const int n = n0 + 8 * g4 + 4 * half;
+        float value[4];
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            value[e] = acc[4 * g4 + e] * head_factor;
+            if (gate && !gate_per_head && n + e < N) {
+                const float g = load_as_float(gate, (size_t)row * gate_row_stride + (size_t)head * N + n + e, gate_code);
+                value[e] *= 1.0f / (1.0f + expf(-g));
+            }
         }
-        store_from_float(out, (size_t)row * out_row_stride + (size_t)head * out_head_stride + n, out_code, value);
+        if (fours) {
+            if (n >= N) continue;
+            if (out_code == MLLM_F32) {
+                *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(out) + out_at + n) = f32x4{value[0], value[1], value[2], value[3]};
+            } else {
+                bf16x4 rounded;
+#pragma unroll
+                for (int e = 0; e < 4; e++) rounded[e] = static_cast<bf16_t>(value[e]);
+                *reinterpret_cast<bf16x4*>(reinterpret_cast<bf16_t*>(out) + out_at + n) = rounded;
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; e++)
+                if (n + e < N) store_from_float(out, out_at + n + e, out_code, value[e]);
+        }
     }
+}
+
+// The same for few rows (decoding): a block takes 16 columns of a head for 16 rows, its waves share the steps of 32 along K, so that a
+// wave waits for memory once, and their sums meet in LDS. The gate is asked for with the first operands.
+constexpr int HEADS_FEW_WAVES = 4, HEADS_FEW_ROWS = 64;
+
+template <typename XT>
+__global__ __launch_bounds__(64 * HEADS_FEW_WAVES) void heads_few_kernel(const XT* __restrict__ x, int x_row_stride, int x_head_stride, const bf16_t* __restrict__ w,
+                                                                         const void* __restrict__ gate, int gate_code, int gate_row_stride, int gate_per_head,
+                                                                         void* __restrict__ out, int out_code, int out_row_stride, int out_head_stride, int n_rows,
+                                                                         int N, int K) {
+    __shared__ float sums[HEADS_FEW_WAVES][4][WAVE];
+    const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, row16 = lane % 16, quad = lane / 16;
+    const int head = blockIdx.y, n0 = blockIdx.x * 16, row0 = blockIdx.z * 16;
+    // a thread finishes one output: row row0 + lane % 16, column n0 + 4 * (lane / 16) + wave
+    const int row = row0 + row16, n = n0 + 4 * quad + wave;
+    const bool mine = row < n_rows && n < N;
+    float g = 0.0f;
+    if (gate && mine) g = load_as_float(gate, (size_t)row * gate_row_stride + (gate_per_head ? (size_t)head : (size_t)head * N + n), gate_code);
+    const bf16_t* w_row = w + ((size_t)head * N + min(n0 + row16, N - 1)) * K + 8 * quad;
+    const XT* x_row = x + (size_t)min(row, n_rows - 1) * x_row_stride + (size_t)head * x_head_stride + 8 * quad;
+    f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    const int steps = K / 32;
+    constexpr int AHEAD = 4;
+    for (int step0 = wave; step0 < steps; step0 += HEADS_FEW_WAVES * AHEAD) {
+        bf16x8 a[AHEAD], b[AHEAD];
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++) {
+            const int k = min(step0 + u * HEADS_FEW_WAVES, steps - 1) * 32;   // beyond the end: the last step again, not used
+            a[u] = *reinterpret_cast<const bf16x8*>(w_row + k);
+            if constexpr (sizeof(XT) == 2) {
+                b[u] = *reinterpret_cast<const bf16x8*>(x_row + k);
+            } else {
+                const f32x4 lo = *reinterpret_cast<const f32x4*>(x_row + k), hi = *reinterpret_cast<const f32x4*>(x_row + k + 4);
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    b[u][e] = static_cast<bf16_t>(lo[e]);
+                    b[u][4 + e] = static_cast<bf16_t>(hi[e]);
+                }
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < AHEAD; u++)
+            if (step0 + u * HEADS_FEW_WAVES < steps) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u], b[u], acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; r++) sums[wave][r][lane] = acc[r];
+    __syncthreads();
+    if (!mine) return;
+    float value = 0.0f;
+#pragma unroll
+    for (int w4 = 0; w4 < HEADS_FEW_WAVES; w4++) value += sums[w4][wave][lane];   // acc[r] of a lane: column 4 * (lane / 16) + r, row lane % 16
+    if (gate) value *= 1.0f / (1.0f + expf(-g));
+    store_from_float(out, (size_t)row * out_row_stride + (size_t)head * out_head_stride + n, out_code, value);
 }
 
 constexpr int LATENT_ROWS = 4;   // rows of the batch a block takes, a wave each
@@ -598,6 +674,18 @@ MLLM_API int mllm_heads_linear(const void* x, int x_dtype, int x_row_stride, int
     const size_t x_element = x_dtype == MLLM_F32 ? 4 : 2;
     if (w_dtype == MLLM_BF16 && K % 16 == 0 && (size_t)x % 16 == 0 && (x_row_stride * x_element) % 16 == 0 && (x_head_stride * x_element) % 16 == 0 &&
         (size_t)w % 16 == 0) {
+        if (n_rows <= HEADS_FEW_ROWS && K % 32 == 0) {
+            dim3 grid(ceil_div(N, 16), n_heads, ceil_div(n_rows, 16));
+            if (x_dtype == MLLM_F32)
+                heads_few_kernel<float><<<grid, 64 * HEADS_FEW_WAVES, 0, stream>>>((const float*)x, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype,
+                                                                                   gate_row_stride, gate_per_head, out, out_dtype, out_row_stride, out_head_stride,
+                                                                                   n_rows, N, K);
+            else
+                heads_few_kernel<bf16_t><<<grid, 64 * HEADS_FEW_WAVES, 0, stream>>>((const bf16_t*)x, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype,
+                                                                                    gate_row_stride, gate_per_head, out, out_dtype, out_row_stride, out_head_stride,
+                                                                                    n_rows, N, K);
+            return mllm_check_launch("heads_linear");
+        }
         dim3 tiles(ceil_div(n_rows, 32), n_heads, ceil_div(N, 128));
         if (x_dtype == MLLM_F32)
             heads_linear_mfma_kernel<float><<<tiles, 256, 0, stream>>>((const float*)x, x_row_stride, x_head_stride, (const bf16_t*)w, gate, gate_dtype,

@@ -439,149 +439,211 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
     }
 }
 
-// The same attention on the matrix cores, for bfloat16 caches whose rows are DK x 16 elements with a latent of up to 32 x RT.
-// A wave takes 32 (token, head) pairs of one request's portion, neighbours in (token, head) order: they all read the same cached
-// rows, so a tile of 32 keys serves 32 pairs in one product. S^T = C Q'^T (a lane's 16-byte piece of its key's row is the
-// operand as it lies in memory; the folded queries, rounded to bfloat16 with the scale folded in, stay in registers for the
-// whole kernel), the statistics per pair in the lane that owns the pair's column, then O^T += C_latent^T P^T with the weights
-// rounded to bfloat16 and the latent elements gathered two at a time (a lane's 32-bit load gives an element to each of two
-// output tiles). Sums, scores and statistics are 32-bit. Runs of keys and the sink as in the kernel above.
-template <int DK, int RT>
-__global__ __launch_bounds__(64) void latent_attention_mfma_kernel(
+// The same attention on the matrix cores, for bfloat16 caches whose rows are DK x 16 elements with a latent of up to 256.
+// A block takes 32 (token, head) pairs of one request's portion, neighbours in (token, head) order: they all read the same cached
+// rows, so a tile of keys serves 32 pairs in one product. Its four waves take 128 keys at a time: each makes the scores of 32 of them,
+// S^T = C Q'^T (a lane's 16-byte piece of its key's row is the operand as it lies in memory; the folded queries, rounded to bfloat16
+// with the scale folded in, lie in LDS for the whole kernel); the maxima meet in LDS, the weights go there rounded to bfloat16; and
+// each sums 64 latent elements over all 128, O^T += C_latent^T P^T, the latent's elements gathered two at a time (a lane's 32-bit load
+// gives an element to each of two output tiles). So a wave holds the sums of 64 elements alone (with all of them in one wave, sums and
+// operands fill a SIMD's registers and nothing hides the trips to memory: 109 us where this takes 48, for 2 x 1,024 tokens of 12 heads over
+// rows of 288 elements).
+// A tile's keys are asked for while the tile before it is summed. Sums, scores and statistics are 32-bit. Runs of keys and the sink as
+// in the kernel above.
+constexpr int LATENT_WAVES = 4, LATENT_KEYS = 32 * LATENT_WAVES;
+constexpr float LOG2_E = 1.44269504088896340736f;
+
+// e^(x - base) as a power of two (base finite)
+__device__ __forceinline__ float exp_from(float x, float base) { return __builtin_amdgcn_exp2f(__builtin_fmaf(x, LOG2_E, -base * LOG2_E)); }
+
+template <int DK>
+__global__ __launch_bounds__(64 * LATENT_WAVES, 2) void latent_attention_mfma_kernel(
     const float* __restrict__ q, const bf16_t* __restrict__ pages, const float* __restrict__ sinks, float* __restrict__ out, float* __restrict__ parts,
     const int* __restrict__ q_starts, const int* __restrict__ context_lens, const int* __restrict__ block_tables, int max_blocks,
     int n_heads, int R, int page_size, float scale, int run_length) {
     constexpr int D = 16 * DK;
-    const int lane = threadIdx.x, lane32 = lane % 32, half = lane / 32;
+    constexpr int Q_ROW = D * 2 + 16, P_ROW = LATENT_KEYS * 2 + 16;   // bytes of a pair's folded query and of its weights in LDS, padded by a piece
+    __shared__ __attribute__((aligned(16))) unsigned char queries[32 * Q_ROW];
+    __shared__ __attribute__((aligned(16))) unsigned char weights[32 * P_ROW];
+    __shared__ __attribute__((aligned(16))) int slots[2][LATENT_KEYS];   // where the tile's keys lie; two tiles in turn
+    __shared__ float exchanged[LATENT_WAVES][32];
+    const int lane = threadIdx.x % WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE), lane32 = lane % 32, half = lane / 32;
     const int request = blockIdx.y, run = blockIdx.z, n_runs = gridDim.z;
     const int context = context_lens[request];
     if (context < 0) return;   // a padding request
     const int q_first = q_starts[request], q_len = q_starts[request + 1] - q_first;
-    const int pair0 = blockIdx.x * 32, n_pairs = q_len * n_heads;
+    const int pair0 = (gridDim.x - 1 - blockIdx.x) * 32, n_pairs = q_len * n_heads;   // (a portion's last pairs, which have the most keys, go first)
     if (pair0 >= n_pairs) return;
     const int pair = pair0 + lane32;
     const bool pair_valid = pair < n_pairs;
-    const int token = min(pair / n_heads, q_len - 1), head = pair_valid ? pair % n_heads : 0;
-    const int row = q_first + token, position = context + token;
-    const int wave_last_position = context + min(q_len - 1, (pair0 + 31) / n_heads);
+    const int position = context + min(pair / n_heads, q_len - 1);
     const int* table = block_tables + (size_t)request * max_blocks;
+    const int first_key = run * run_length, block_last_position = context + min(q_len - 1, (pair0 + 31) / n_heads);
+    const int last_key = run == n_runs - 1 ? block_last_position : min(block_last_position, first_key + run_length - 1);
 
-    bf16x8 q_op[DK];
-    {
-        const float* q_row = q + ((size_t)row * n_heads + head) * D + 8 * half;
-        const float factor = pair_valid ? scale : 0.0f;
-#pragma unroll
-        for (int ks = 0; ks < DK; ks++) {
-            const f32x4 lo = *reinterpret_cast<const f32x4*>(q_row + 16 * ks), hi = *reinterpret_cast<const f32x4*>(q_row + 16 * ks + 4);
-#pragma unroll
-            for (int e = 0; e < 4; e++) {
-                q_op[ks][e] = static_cast<bf16_t>(lo[e] * factor);
-                q_op[ks][4 + e] = static_cast<bf16_t>(hi[e] * factor);
-            }
-        }
-    }
-    f32x16 o[RT];
-#pragma unroll
-    for (int i = 0; i < RT; i++)
-#pragma unroll
-        for (int v = 0; v < 16; v++) o[i][v] = 0.0f;
-    float top = -INFINITY, weight = 0.0f;
-
-    const int first_key = run * run_length;
-    const int last_key = run == n_runs - 1 ? wave_last_position : min(wave_last_position, first_key + run_length - 1);
-    for (int kt = first_key; kt <= last_key; kt += 32) {
-        const int key = min(kt + lane32, last_key);
-        const int slot = table[key / page_size] * page_size + key % page_size;
+    // this wave's key of a tile (lanes of both halves: the same), from a clamped place
+    auto slot_of = [&](int kt) {
+        const int key = max(min(kt + 32 * wave + lane32, last_key), 0);
+        return table[key / page_size] * page_size + key % page_size;
+    };
+    bf16x8 k_op[DK];
+    auto ask_keys = [&](int slot) {
         const bf16_t* k_row = pages + (size_t)slot * D + 8 * half;
-        bf16x8 k_op[DK];
 #pragma unroll
         for (int ks = 0; ks < DK; ks++) k_op[ks] = *reinterpret_cast<const bf16x8*>(k_row + 16 * ks);
+    };
+    int slot = 0, next_slot = 0;
+    if (first_key <= last_key) {   // (uniform over the block, as the loop below is)
+        slot = slot_of(first_key);
+        next_slot = slot_of(first_key + LATENT_KEYS);
+        ask_keys(slot);
+    }
+    // pairs are (token, head) in order, as q's rows are: the block's queries lie behind each other
+    for (int i = threadIdx.x; i < 32 * (D / 8); i += 64 * LATENT_WAVES) {
+        const int p = i / (D / 8), piece = i % (D / 8);
+        const float factor = pair0 + p < n_pairs ? scale : 0.0f;
+        const float* from = q + ((size_t)q_first * n_heads + min(pair0 + p, n_pairs - 1)) * D + 8 * piece;
+        const f32x4 lo = *reinterpret_cast<const f32x4*>(from), hi = *reinterpret_cast<const f32x4*>(from + 4);
+        bf16x8 rounded;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            rounded[e] = static_cast<bf16_t>(lo[e] * factor);
+            rounded[4 + e] = static_cast<bf16_t>(hi[e] * factor);
+        }
+        *reinterpret_cast<bf16x8*>(queries + p * Q_ROW + piece * 16) = rounded;
+    }
+    __syncthreads();
+    const unsigned char* q_row = queries + lane32 * Q_ROW + half * 16;
+    unsigned char* my_weights = weights + lane32 * P_ROW;
+    const bool sums_here = 64 * wave < R;   // this wave's 64 latent elements (uniform over the wave)
+    const int latent = min(64 * wave + 2 * lane32, D - 2);
+
+    f32x16 o[2];
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int v = 0; v < 16; v++) o[i][v] = 0.0f;
+    float top = -INFINITY, weight = 0.0f;   // the pair's maximum over all keys so far, and its weights' sum over this wave's keys
+
+    int turn = 0;
+    for (int kt = first_key; kt <= last_key; kt += LATENT_KEYS, turn ^= 1) {
         f32x16 s;
 #pragma unroll
         for (int v = 0; v < 16; v++) s[v] = 0.0f;
 #pragma unroll
-        for (int ks = 0; ks < DK; ks++) s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(k_op[ks], q_op[ks], s, 0, 0, 0);
+        for (int ks = 0; ks < DK; ks++)
+            s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(k_op[ks], *reinterpret_cast<const bf16x8*>(q_row + 32 * ks), s, 0, 0, 0);
         float tile_top = -INFINITY;
 #pragma unroll
         for (int v = 0; v < 16; v++) {
-            const int at = kt + 8 * (v / 4) + 4 * half + (v % 4);
+            const int at = kt + 32 * wave + 8 * (v / 4) + 4 * half + (v % 4);
             s[v] = pair_valid && at <= position && at <= last_key ? s[v] : -INFINITY;
             tile_top = fmaxf(tile_top, s[v]);
         }
         tile_top = fmaxf(tile_top, __shfl_xor(tile_top, 32, WAVE));
-        const float new_top = fmaxf(top, tile_top);
-        const float safe_top = new_top == -INFINITY ? 0.0f : new_top;   // a pair none of whose keys has come yet
-        const float rescale = expf(top - safe_top);
-        top = new_top;
-        weight *= rescale;
-#pragma unroll
-        for (int i = 0; i < RT; i++)
-#pragma unroll
-            for (int v = 0; v < 16; v++) o[i][v] *= rescale;
-#pragma unroll
-        for (int v = 0; v < 16; v++) {
-            s[v] = expf(s[v] - safe_top);
-            weight += s[v];
+        if (half == 0) {
+            exchanged[wave][lane32] = tile_top;
+            slots[turn][32 * wave + lane32] = slot;
         }
+        __syncthreads();
+        // the latent elements of all 128 keys: key 16 * slab + 8 * half + e of the tile, in the order of the operand
+        uint32_t word[LATENT_KEYS / 16][8];
+        if (sums_here) {
 #pragma unroll
-        for (int slab = 0; slab < 2; slab++) {   // 16 keys each: the lane's score registers 8 * slab .. + 7
-            bf16x8 p;
+            for (int slab = 0; slab < LATENT_KEYS / 16; slab++) {
+                const int4 a = *reinterpret_cast<const int4*>(&slots[turn][16 * slab + 8 * half]), b = *reinterpret_cast<const int4*>(&slots[turn][16 * slab + 8 * half + 4]);
+                const int at[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
 #pragma unroll
-            for (int e = 0; e < 8; e++) p[e] = static_cast<bf16_t>(s[8 * slab + e]);
-            // the keys those registers belong to: 16 * slab + 4 * half + 0..3 and eight further on; their cached rows
-            const bf16_t* rows_at[8];
+                for (int e = 0; e < 8; e++) word[slab][e] = *reinterpret_cast<const uint32_t*>(pages + (size_t)at[e] * D + latent);
+            }
+        }
+        ask_keys(next_slot);   // the next tile's keys (behind the last tile: the last key's row, not used)
+        slot = next_slot;
+        next_slot = slot_of(kt + 2 * LATENT_KEYS);
+        float new_top = top;
 #pragma unroll
-            for (int e = 0; e < 8; e++) rows_at[e] = pages + (size_t)__shfl(slot, 16 * slab + 4 * half + (e % 4) + 8 * (e / 4), WAVE) * D;
+        for (int w = 0; w < LATENT_WAVES; w++) new_top = fmaxf(new_top, exchanged[w][lane32]);
+        const float safe_top = new_top == -INFINITY ? 0.0f : new_top;   // a pair none of whose keys has come yet
+        if (__any(new_top != top)) {
+            const float rescale = exp_from(top, safe_top);
+            weight *= rescale;
 #pragma unroll
-            for (int t = 0; t < RT / 2; t++) {
-                const int d = min(64 * t + 2 * lane32, D - 2);
-                uint32_t word[8];
+            for (int i = 0; i < 2; i++)
 #pragma unroll
-                for (int e = 0; e < 8; e++) word[e] = *reinterpret_cast<const uint32_t*>(rows_at[e] + d);
+                for (int v = 0; v < 16; v++) o[i][v] *= rescale;
+        }
+        top = new_top;
+#pragma unroll
+        for (int g = 0; g < 4; g++) {
+            bf16x4 p;
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const float value = exp_from(s[4 * g + e], safe_top);
+                weight += value;
+                p[e] = static_cast<bf16_t>(value);
+            }
+            *reinterpret_cast<bf16x4*>(my_weights + (32 * wave + 8 * g + 4 * half) * 2) = p;
+        }
+        __syncthreads();
+        if (sums_here) {
+#pragma unroll
+            for (int slab = 0; slab < LATENT_KEYS / 16; slab++) {
+                const bf16x8 p = *reinterpret_cast<const bf16x8*>(my_weights + (16 * slab + 8 * half) * 2);
                 Vec16 even, odd;
 #pragma unroll
                 for (int j = 0; j < 4; j++) {
-                    even.w[j] = (word[2 * j] & 0xffffu) | (word[2 * j + 1] << 16);
-                    odd.w[j] = (word[2 * j] >> 16) | (word[2 * j + 1] & 0xffff0000u);
+                    const uint32_t first = word[slab][2 * j], second = word[slab][2 * j + 1];
+                    even.w[j] = (first & 0xffffu) | (second << 16);
+                    odd.w[j] = (first >> 16) | (second & 0xffff0000u);
                 }
-                o[2 * t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(&even), p, o[2 * t], 0, 0, 0);
-                o[2 * t + 1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(&odd), p, o[2 * t + 1], 0, 0, 0);
+                o[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(&even), p, o[0], 0, 0, 0);
+                o[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8*>(&odd), p, o[1], 0, 0, 0);
             }
         }
     }
     weight += __shfl_xor(weight, 32, WAVE);
+    __syncthreads();   // (the maxima of the last tile have been read)
+    if (half == 0) exchanged[wave][lane32] = weight;
+    __syncthreads();
+    weight = 0.0f;
+#pragma unroll
+    for (int w = 0; w < LATENT_WAVES; w++) weight += exchanged[w][lane32];
     if (!pair_valid) return;
-    const size_t item = (size_t)row * n_heads + head;
-    if (n_runs == 1) {
-        float inverse;
+    const size_t item = (size_t)q_first * n_heads + pair;
+    float factor = 1.0f;
+    float* to = parts + (item * n_runs + run) * (R + 2);
+    if (n_runs == 1) {   // the finished sums: the sink joins the denominator once, measured from the larger of the two
+        to = out + item * R;
         if (sinks) {
-            const float sink = sinks[head], highest = fmaxf(top, sink);
-            const float shrink = expf(top - highest);
-            inverse = shrink / (weight * shrink + expf(sink - highest));
+            const float sink = sinks[pair % n_heads], highest = fmaxf(top, sink), shrink = expf(top - highest);
+            factor = shrink / (weight * shrink + expf(sink - highest));
         } else {
-            inverse = 1.0f / weight;
+            factor = 1.0f / weight;
         }
-        float* out_row = out + item * R;
-#pragma unroll
-        for (int i = 0; i < RT; i++)
-#pragma unroll
-            for (int v = 0; v < 16; v++) {
-                const int d = 64 * (i / 2) + 2 * (8 * (v / 4) + 4 * half + (v % 4)) + (i % 2);
-                if (d < R) out_row[d] = o[i][v] * inverse;
-            }
-        return;
+    } else if (wave == 0 && half == 0) {
+        to[R] = top;   // -inf and 0 for a run without keys
+        to[R + 1] = weight;
     }
-    float* mine = parts + (item * n_runs + run) * (R + 2);
+    if (!sums_here) return;
+    // o[i][v] is latent element 64 * wave + 2 * (8 * (v / 4) + 4 * half + v % 4) + i: eight neighbours at a time
+    const bool fours = n_runs == 1 && R % 4 == 0;
 #pragma unroll
-    for (int i = 0; i < RT; i++)
+    for (int g = 0; g < 4; g++) {
+        const int d0 = 64 * wave + 16 * g + 8 * half;
+        float value[8];
 #pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const int d = 64 * (i / 2) + 2 * (8 * (v / 4) + 4 * half + (v % 4)) + (i % 2);
-            if (d < R) mine[d] = o[i][v];
+        for (int e = 0; e < 4; e++) {
+            value[2 * e] = o[0][4 * g + e] * factor;
+            value[2 * e + 1] = o[1][4 * g + e] * factor;
         }
-    if (half == 0) {
-        mine[R] = top;
-        mine[R + 1] = weight;
+        if (fours) {
+            if (d0 < R) *reinterpret_cast<f32x4*>(to + d0) = f32x4{value[0], value[1], value[2], value[3]};
+            if (d0 + 4 < R) *reinterpret_cast<f32x4*>(to + d0 + 4) = f32x4{value[4], value[5], value[6], value[7]};
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; e++)
+                if (d0 + e < R) to[d0 + e] = value[e];
+        }
     }
 }
 
@@ -590,21 +652,10 @@ struct LatentMfmaArgs {
     const int* block_tables; int max_blocks, n_heads, R, page_size; float scale; int run_length; dim3 grid; hipStream_t stream;
 };
 
-template <int DK, int RT>
-void launch_latent_mfma(const LatentMfmaArgs& a) {
-    latent_attention_mfma_kernel<DK, RT><<<a.grid, 64, 0, a.stream>>>(a.q, a.pages, a.sinks, a.out, a.parts, a.q_starts, a.context_lens, a.block_tables,
-                                                                      a.max_blocks, a.n_heads, a.R, a.page_size, a.scale, a.run_length);
-}
-
 template <int DK>
-bool launch_latent_mfma_rt(const LatentMfmaArgs& a) {
-    if (a.R <= 64) launch_latent_mfma<DK, 2>(a);
-    else if constexpr (DK >= 6) {
-        if (a.R <= 128) launch_latent_mfma<DK, 4>(a);
-        else if constexpr (DK >= 12) launch_latent_mfma<DK, 8>(a);
-        else return false;
-    } else return false;
-    return true;
+void launch_latent_mfma(const LatentMfmaArgs& a) {
+    latent_attention_mfma_kernel<DK><<<a.grid, 64 * LATENT_WAVES, 0, a.stream>>>(a.q, a.pages, a.sinks, a.out, a.parts, a.q_starts, a.context_lens, a.block_tables,
+                                                                                 a.max_blocks, a.n_heads, a.R, a.page_size, a.scale, a.run_length);
 }
 
 template <typename KernelT>
@@ -759,23 +810,21 @@ MLLM_API int mllm_latent_attention_mfma(const float* q, const void* pages, const
                                         int run_length, hipStream_t stream) {
     MLLM_REQUIRE(n_rows >= 0 && n_requests >= 0 && n_heads > 0 && max_blocks > 0 && page_size > 0 && max_pairs > 0, "latent_attention_mfma: bad sizes");
     MLLM_REQUIRE(mllm_latent_attention_mfma_supported(R, D, MLLM_BF16), "latent_attention_mfma: no kernel for rows of %d elements with a latent of %d", D, R);
-    MLLM_REQUIRE(n_runs >= 1 && n_runs <= MERGE_MAX_RUNS && n_requests <= 65535 && run_length >= 1 && (n_runs == 1 || run_length % 32 == 0), "latent_attention_mfma: bad runs");
+    MLLM_REQUIRE(n_runs >= 1 && n_runs <= MERGE_MAX_RUNS && n_requests <= 65535 && run_length >= 1 && (n_runs == 1 || run_length % 64 == 0), "latent_attention_mfma: bad runs");
     MLLM_REQUIRE(n_runs == 1 || parts != nullptr, "latent_attention_mfma: runs need room for their sums");
     if (n_rows == 0 || n_requests == 0) return 0;
     if (n_runs == 1) run_length = 1 << 30;
     LatentMfmaArgs a{q, (const bf16_t*)pages, sinks, out, parts, q_starts, context_lens, block_tables, max_blocks, n_heads, R, page_size, scale, run_length,
                      dim3(ceil_div(max_pairs, 32), n_requests, n_runs), stream};
     mllm_count_kernel(MLLM_K_LATENT_ATTENTION);
-    bool launched = false;
     switch (D / 16) {
-        case 2: launched = launch_latent_mfma_rt<2>(a); break;
-        case 4: launched = launch_latent_mfma_rt<4>(a); break;
-        case 6: launched = launch_latent_mfma_rt<6>(a); break;
-        case 8: launched = launch_latent_mfma_rt<8>(a); break;
-        case 12: launched = launch_latent_mfma_rt<12>(a); break;
-        case 18: launched = launch_latent_mfma_rt<18>(a); break;
+        case 2: launch_latent_mfma<2>(a); break;
+        case 4: launch_latent_mfma<4>(a); break;
+        case 6: launch_latent_mfma<6>(a); break;
+        case 8: launch_latent_mfma<8>(a); break;
+        case 12: launch_latent_mfma<12>(a); break;
+        case 18: launch_latent_mfma<18>(a); break;
     }
-    MLLM_REQUIRE(launched, "latent_attention_mfma: no kernel for rows of %d elements with a latent of %d", D, R);
     int status = mllm_check_launch("latent_attention_mfma");
     if (status || n_runs == 1) return status;
     const long long items = (long long)n_rows * n_heads;

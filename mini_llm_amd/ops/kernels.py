@@ -1024,6 +1024,8 @@ def heads_linear(x, weight, out, *, n_heads, k, x_head_stride, n_out=None, gate=
 
 
 LATENT_RUN_MIN = 64        # cached rows a run of a token's keys should at least hold: a tile of the kernel
+LATENT_TARGET_BLOCKS = 256   # blocks (four waves that share the keys of 32 pairs) the matrix-core kernel's launch should have before keys are left whole
+LATENT_BLOCK_RUN_MIN = 128   # and the cached rows its runs are multiples of there: what a block takes at a time
 LATENT_TARGET_WAVES = 2048   # waves a launch should have before a token's keys are left whole (eight to a compute unit)
 
 
@@ -1046,7 +1048,7 @@ def latent_attention(q_full, pages, sinks, token_request, positions, block_table
     rank]. Few rows with many keys are cut into runs of keys (``max_len``: the longest sequence of the batch).
     With ``q_starts`` ([requests + 1]: each request's rows are consecutive), ``context_lens`` ([requests]: the position of a
     request's first row; negative: a padding request) and ``max_q_len``, a bfloat16 cache of a row size the matrix-core kernel
-    takes runs through that kernel (32 (token, head) pairs of a request to a wave)."""
+    takes runs through that kernel (32 (token, head) pairs of a request to a block)."""
     _device_tensor(q_full, "q_full", torch.float32, 3)
     _device_tensor(pages, "pages", dim=4)
     n, n_heads, row_size = q_full.shape
@@ -1072,9 +1074,9 @@ def latent_attention(q_full, pages, sinks, token_request, positions, block_table
         n_requests = context_lens.shape[0]
         _require(q_starts.shape[0] == n_requests + 1 and block_tables.shape[0] >= n_requests, "q_starts, context_lens and block tables do not match")
         max_pairs = max(1, min(int(max_q_len), n)) * n_heads
-        waves = n_requests * -(-max_pairs // 32)
-        n_runs = max(1, min(LATENT_TARGET_WAVES // 2 // waves, longest // LATENT_RUN_MIN, 256))
-        run_length = -(-(-(-longest // n_runs)) // 64) * 64 if n_runs > 1 else reach
+        blocks = n_requests * -(-max_pairs // 32)
+        n_runs = max(1, min(LATENT_TARGET_BLOCKS // blocks, longest // LATENT_BLOCK_RUN_MIN, 256))
+        run_length = -(-(-(-longest // n_runs)) // LATENT_BLOCK_RUN_MIN) * LATENT_BLOCK_RUN_MIN if n_runs > 1 else reach
         parts = torch.empty((n, n_heads, n_runs, rank + 2), dtype=torch.float32, device=q_full.device) if n_runs > 1 else None
         if n_runs == 1:   # rows that belong to no request (padding) are reached by no wave; with runs the merge writes every row
             out.zero_()

@@ -46,6 +46,12 @@ CASES = {
         latent(heads=6, dim=48, rot_dim=32, vdim=64, kv_rank=160, scale=0.11, base=20000.0, mlp=moe(experts=12, top=3, ff=96)),
         latent(heads=8, dim=64, rot_dim=32, vdim=40, kv_rank=256, scale=0.1, base=300.0, mlp=moe(experts=4, top=1, ff=192)),
     ], width=192, vocab=211, buckets=1021, mul_prev=257, mul_cur=65),
+    # latents wider than the matrix-core kernel takes, one of them in whole sixteens and one not
+    "large": model([
+        latent(heads=3, dim=32, rot_dim=32, vdim=48, kv_rank=320, scale=0.12, base=5000.0, mlp=moe(experts=4, top=2, ff=128)),
+        mingru(width=520, mlp=None),
+        latent(heads=2, dim=40, rot_dim=38, vdim=72, kv_rank=300, scale=0.1, mlp=None),
+    ], width=128, vocab=90),
     # one kind of mixer alone: no pages at all; and no state but the previous token
     "recurrent": model([mingru(width=96), mingru(width=40, mlp=None)], width=64, vocab=61, mul_prev=0, mul_cur=1),
     "attending": model([latent(), latent(heads=2, dim=32, rot_dim=2, vdim=48, kv_rank=96, scale=0.2)], width=80, vocab=130, mul_prev=1, mul_cur=0),

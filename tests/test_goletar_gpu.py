@@ -71,6 +71,7 @@ def plain_logits(config, weights, requests, bf16):
 
 
 LENGTHS = {"mixed": [5, 130, 64, 65, 1, 200, 33], "odd": [67, 2, 130, 31], "wide": [3, 150, 64, 17, 129, 260], "recurrent": [150, 1, 70, 3, 97],
+           "large": [3, 140, 66],
            "attending": [66, 2, 140, 20]}
 MODES = {"whole": replay.whole, "tail": replay.prefill_then_decode, "chunked": replay.chunked, "mixed": replay.mixed}
 TOLERANCE = {"float32": dict(atol=3e-4, rtol=2e-4)}   # sums in another order than numpy's

@@ -459,6 +459,7 @@ __device__ __forceinline__ float exp_from(float x, float base) { return __builti
 template <int DK>
 __global__ __launch_bounds__(64 * LATENT_WAVES, 2) void latent_attention_mfma_kernel(
     const float* __restrict__ q, const bf16_t* __restrict__ pages, const float* __restrict__ sinks, float* __restrict__ out, float* __restrict__ parts,
+    const int* __restrict__ token_request, int n_rows,
     const int* __restrict__ q_starts, const int* __restrict__ context_lens, const int* __restrict__ block_tables, int max_blocks,
     int n_heads, int R, int page_size, float scale, int run_length) {
     constexpr int D = 16 * DK;
@@ -469,6 +470,16 @@ __global__ __launch_bounds__(64 * LATENT_WAVES, 2) void latent_attention_mfma_ke
     __shared__ float exchanged[LATENT_WAVES][32];
     const int lane = threadIdx.x % WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE), lane32 = lane % 32, half = lane / 32;
     const int request = blockIdx.y, run = blockIdx.z, n_runs = gridDim.z;
+    // rows that belong to no request are zero (with several runs the merge sees to it): the first blocks look 64 rows a wave over for them
+    if (n_runs == 1 && request == 0) {
+        for (int row0 = (blockIdx.x * LATENT_WAVES + wave) * WAVE; row0 < n_rows; row0 += gridDim.x * LATENT_WAVES * WAVE) {
+            unsigned long long nobodys = __ballot(row0 + lane < n_rows && token_request[min(row0 + lane, n_rows - 1)] < 0);
+            for (; nobodys; nobodys &= nobodys - 1) {
+                float* row = out + (size_t)(row0 + __builtin_ctzll(nobodys)) * n_heads * R;
+                for (int i = lane; i < n_heads * R; i += WAVE) row[i] = 0.0f;
+            }
+        }
+    }
     const int context = context_lens[request];
     if (context < 0) return;   // a padding request
     const int q_first = q_starts[request], q_len = q_starts[request + 1] - q_first;
@@ -648,13 +659,13 @@ __global__ __launch_bounds__(64 * LATENT_WAVES, 2) void latent_attention_mfma_ke
 }
 
 struct LatentMfmaArgs {
-    const float* q; const bf16_t* pages; const float* sinks; float* out; float* parts; const int* q_starts; const int* context_lens;
-    const int* block_tables; int max_blocks, n_heads, R, page_size; float scale; int run_length; dim3 grid; hipStream_t stream;
+    const float* q; const bf16_t* pages; const float* sinks; float* out; float* parts; const int* token_request; int n_rows;
+    const int* q_starts; const int* context_lens; const int* block_tables; int max_blocks, n_heads, R, page_size; float scale; int run_length; dim3 grid; hipStream_t stream;
 };
 
 template <int DK>
 void launch_latent_mfma(const LatentMfmaArgs& a) {
-    latent_attention_mfma_kernel<DK><<<a.grid, 64 * LATENT_WAVES, 0, a.stream>>>(a.q, a.pages, a.sinks, a.out, a.parts, a.q_starts, a.context_lens, a.block_tables,
+    latent_attention_mfma_kernel<DK><<<a.grid, 64 * LATENT_WAVES, 0, a.stream>>>(a.q, a.pages, a.sinks, a.out, a.parts, a.token_request, a.n_rows, a.q_starts, a.context_lens, a.block_tables,
                                                                                  a.max_blocks, a.n_heads, a.R, a.page_size, a.scale, a.run_length);
 }
 
@@ -812,9 +823,10 @@ MLLM_API int mllm_latent_attention_mfma(const float* q, const void* pages, const
     MLLM_REQUIRE(mllm_latent_attention_mfma_supported(R, D, MLLM_BF16), "latent_attention_mfma: no kernel for rows of %d elements with a latent of %d", D, R);
     MLLM_REQUIRE(n_runs >= 1 && n_runs <= MERGE_MAX_RUNS && n_requests <= 65535 && run_length >= 1 && (n_runs == 1 || run_length % 64 == 0), "latent_attention_mfma: bad runs");
     MLLM_REQUIRE(n_runs == 1 || parts != nullptr, "latent_attention_mfma: runs need room for their sums");
+    MLLM_REQUIRE(token_request != nullptr || n_rows == 0, "latent_attention_mfma: no token_request");
     if (n_rows == 0 || n_requests == 0) return 0;
     if (n_runs == 1) run_length = 1 << 30;
-    LatentMfmaArgs a{q, (const bf16_t*)pages, sinks, out, parts, q_starts, context_lens, block_tables, max_blocks, n_heads, R, page_size, scale, run_length,
+    LatentMfmaArgs a{q, (const bf16_t*)pages, sinks, out, parts, token_request, n_rows, q_starts, context_lens, block_tables, max_blocks, n_heads, R, page_size, scale, run_length,
                      dim3(ceil_div(max_pairs, 32), n_requests, n_runs), stream};
     mllm_count_kernel(MLLM_K_LATENT_ATTENTION);
     switch (D / 16) {

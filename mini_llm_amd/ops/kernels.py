@@ -1078,8 +1078,7 @@ def latent_attention(q_full, pages, sinks, token_request, positions, block_table
         n_runs = max(1, min(LATENT_TARGET_BLOCKS // blocks, longest // LATENT_BLOCK_RUN_MIN, 256))
         run_length = -(-(-(-longest // n_runs)) // LATENT_BLOCK_RUN_MIN) * LATENT_BLOCK_RUN_MIN if n_runs > 1 else reach
         parts = torch.empty((n, n_heads, n_runs, rank + 2), dtype=torch.float32, device=q_full.device) if n_runs > 1 else None
-        if n_runs == 1:   # rows that belong to no request (padding) are reached by no wave; with runs the merge writes every row
-            out.zero_()
+        _require(n_requests >= 1, "rows of no request")
         check(lib.mllm_latent_attention_mfma(_ptr(q_full), _ptr(pages), _ptr(sinks), _ptr(out), _ptr(parts), _ptr(token_request), _ptr(q_starts),
                                              _ptr(context_lens), _ptr(block_tables), block_tables.shape[1], n, n_requests, max_pairs, n_heads,
                                              int(rank), row_size, page_size, float(scale), n_runs, run_length, _stream()))

@@ -104,6 +104,88 @@ def test_latent_rows_of_neighbouring_pairs(dtype, heads, dim, rot, rot_dims, ran
     assert (np.delete(kept, [s for s in slots if s >= 0], axis=0) == 7).all()
 
 
+@pytest.mark.parametrize("sink", [True, False])
+@pytest.mark.parametrize("heads,rank,rot,page_size", [(3, 24, 8, 16), (6, 64, 32, 64), (2, 100, 20, 32), (17, 160, 32, 64), (5, 256, 32, 64), (1, 61, 3, 8)])
+def test_latent_attention_on_the_matrix_cores(heads, rank, rot, page_size, sink):
+    # A batch of portions at any depth, single tokens among them, and rows of no request behind; every row's query makes one key stand out:
+    # its sequence's first, the last it sees, or one beside the borders of pages and of the 32 and 128 keys a wave and a block take at a
+    # time. One key further on, which the row must not see, would stand out still more.
+    k = kernels()
+    rng = np.random.default_rng(rank)
+    contexts, portions = [0, 130, 1000, 31, 700, 127], [150, 2, 1, 97, 33, 129]
+    row_size, pad = k.latent_row_size(rank + rot), 5
+    assert k.library().mllm_latent_attention_mfma_supported(rank, row_size, 1)
+    lengths = [c + n for c, n in zip(contexts, portions)]
+    n_blocks = [-(-n // page_size) for n in lengths]
+    order = rng.permutation(sum(n_blocks) + 2)
+    pages = torch.zeros((len(order), 1, page_size, row_size), dtype=torch.bfloat16)
+    tables, cached, at = np.full((len(lengths) + 1, max(n_blocks) + 1), -1, dtype=np.int32), [], 0
+    for r, n in enumerate(lengths):
+        rows = rounded(rng.normal(0, 1, (n, row_size)), torch.bfloat16)
+        rows[:, rank + rot :] = 0
+        cached.append(rows)
+        for b in range(n_blocks[r]):
+            tables[r, b] = order[at]
+            chunk = rows[b * page_size : (b + 1) * page_size]
+            pages[order[at], 0, : len(chunk)] = torch.tensor(chunk).to(torch.bfloat16)
+            at += 1
+    total = sum(portions)
+    starts = np.concatenate([[0], np.cumsum(portions), [total + pad]])
+    owner, positions = np.full(total + pad, -1), np.zeros(total + pad, dtype=int)
+    q = rng.normal(0, 0.1, (total + pad, heads, row_size))
+    borders = (0, 31, 32, 63, 64, 127, 128, 255, 256, 999)
+    for r, (c, n) in enumerate(zip(contexts, portions)):
+        for i in range(n):
+            row, position = starts[r] + i, c + i
+            owner[row], positions[row] = r, position
+            seen = [b for b in borders if b <= position] + [position]
+            hot = seen[int(rng.integers(len(seen)))] if i % 3 else position
+            q[row] += cached[r][hot] * 20.0 / np.linalg.norm(cached[r][hot])
+            if position + 1 < lengths[r]:
+                q[row] += cached[r][position + 1] * 40.0 / np.linalg.norm(cached[r][position + 1])
+    q[:, :, rank + rot :] = 0
+    q = rounded(q, torch.bfloat16)
+    sinks, scale = rng.normal(0, 1, heads), 0.5
+    for max_len, longest in ((max(lengths), max(portions)), (8 * max(lengths), total)):   # bounds as they are, and as a captured step gives them
+        got = k.latent_attention(gpu(q), pages.cuda(), gpu(sinks) if sink else None, ints(owner), ints(positions), ints(tables), rank, scale, max_len=max_len,
+                                 q_starts=ints(starts), context_lens=ints(contexts + [-1]), max_q_len=longest).cpu().numpy()
+        assert (got[total:] == 0).all()
+        for row in range(total):
+            keys = cached[owner[row]][: positions[row] + 1]
+            scores = q[row] @ keys.T * scale
+            weights = np.exp(scores - scores.max(axis=1, keepdims=True))
+            bottom = weights.sum(axis=1, keepdims=True) + (np.exp(sinks[:, None] - scores.max(axis=1, keepdims=True)) if sink else 0.0)
+            np.testing.assert_allclose(got[row], weights @ keys[:, :rank] / bottom, atol=4e-2, rtol=3e-2, err_msg=f"row {row} position {positions[row]}")
+
+
+@pytest.mark.parametrize("sink", [True, False])
+def test_latent_attention_of_few_rows_with_many_keys(sink):
+    # runs of keys by different blocks, put together behind them; rows of no request between and behind
+    k = kernels()
+    rng = np.random.default_rng(7)
+    heads, rank, rot, page_size, length, row_size = 4, 64, 32, 64, 3000, 96
+    cached = rounded(rng.normal(0, 1, (length, row_size)), torch.bfloat16)
+    blocks = -(-length // page_size)
+    pages = torch.zeros((blocks, 1, page_size, row_size), dtype=torch.bfloat16)
+    pages.view(-1, row_size)[:length] = torch.tensor(cached).to(torch.bfloat16)
+    tables = np.stack([np.arange(blocks)] * 3)
+    sinks = rng.normal(0, 1, heads)
+    for hot in (0, 127, 128, 1535, 1536, 2998, 2999):
+        positions = [2999, 0, 2998]
+        q = np.tile(cached[hot] * 30.0 / np.linalg.norm(cached[hot]), (3, heads, 1)) + rng.normal(0, 0.1, (3, heads, row_size))
+        q = rounded(q, torch.bfloat16)
+        got = k.latent_attention(gpu(q), pages.cuda(), gpu(sinks) if sink else None, ints([0, -1, 2]), ints(positions), ints(tables), rank, 1.0, max_len=length,
+                                 q_starts=ints([0, 1, 2, 3]), context_lens=ints([2999, -1, 2998]), max_q_len=1).cpu().numpy()
+        assert (got[1] == 0).all()
+        for row in (0, 2):
+            keys = cached[: positions[row] + 1]
+            scores = q[row] @ keys.T
+            top = np.maximum(scores.max(axis=1, keepdims=True), sinks[:, None] if sink else -np.inf)
+            weights = np.exp(scores - top)
+            want = weights @ keys[:, :rank] / (weights.sum(axis=1, keepdims=True) + (np.exp(sinks[:, None] - top) if sink else 0.0))
+            np.testing.assert_allclose(got[row], want, atol=4e-2, rtol=3e-2, err_msg=f"hot key {hot} row {row}")
+
+
 @pytest.mark.parametrize("w_dtype", DTYPES)
 @pytest.mark.parametrize("rows,heads,n,k_size", [(1, 3, 40, 16), (17, 2, 24, 64), (33, 5, 48, 21), (5, 6, 7, 512), (70, 3, 130, 32)])
 def test_heads_linear_with_a_gate_a_head(w_dtype, rows, heads, n, k_size):

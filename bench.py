@@ -337,10 +337,10 @@ DESIGN_SIZES = {   # width, layers; heads of 64; GPT-2's inner size 4 x width, t
     "medium": (1024, 24),
 }
 _KERNEL_CLASSES = {
-    "products": ("gemm", "gemm_split", "gemm_qkv_cache", "gemm_best", "heads_linear"),
-    "attention": ("attention", "attention_decode", "attention_prefill", "latent_attention"),
+    "products": ("gemm", "gemm_split", "gemm_qkv_cache", "gemm_best", "heads_linear", "experts_up", "experts_down", "experts_few_up", "experts_few_down"),
+    "attention": ("attention", "attention_decode", "attention_prefill", "latent_attention", "latent_attention_mfma"),
     "row-wise": ("layernorm", "pending_layernorm", "rms_norm", "head_norm", "latent_rows", "silu_mul", "pending_sum", "add", "cache_write", "embed",
-                 "projection_rows", "head_gate", "gated_norm", "short_conv", "map_rows", "map_difference", "turn_heads", "gate_unit", "route", "expert_unit", "gated_expert_unit",
+                 "projection_rows", "head_gate", "gated_norm", "short_conv", "map_rows", "map_difference", "turn_heads", "gate_unit", "route", "route_rows", "expert_unit", "expert_lists",
                  "branch_join"),
     "recurrence": ("recurrence", "gated_scan"),
     "layer kernels": ("decode_attention_half", "decode_mlp_half"),

@@ -3,7 +3,8 @@
 //
 // A router leaves picks [rows, top] (expert ids, -1 for none) and their weights. Entry p = row * top + k is row `row` with its k-th
 // pick. An expert's matrices: the gate and up rows of the up matrix in turns of 32, [2 * units, width], and the down matrix [width,
-// units], both packed, one expert behind the other; units a multiple of 64 (zero rows and columns fill it up). The down product of a
+// units], both packed, one expert behind the other; units a multiple of 64 (zero rows and columns fill it up), the down matrix's rows
+// whole sixteens. The down product of a
 // row's k-th pick goes to plane k of out [top, rows, width]: whoever reads the branch adds the planes up, in that order.
 #include "common.h"
 #include "gate_unit.h"
@@ -127,14 +128,26 @@ __device__ __forceinline__ int gather_entries(const int* __restrict__ picks, con
     return *count;
 }
 
+// A step of K of one 16 x 16 tile of sums: 32 of bfloat16, 16 of float (the true 32-bit product), from 16 bytes a lane of either operand.
+template <typename T>
+__device__ __forceinline__ void multiply(const Vec16& w, const Vec16& x, f32x4& acc) {
+    if constexpr (sizeof(T) == 2) {
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(&w), *reinterpret_cast<const bf16x8*>(&x), acc, 0, 0, 0);
+    } else {
+#pragma unroll
+        for (int c = 0; c < 4; c++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32((*reinterpret_cast<const f32x4*>(&w))[c], (*reinterpret_cast<const f32x4*>(&x))[c], acc, 0, 0, 0);
+    }
+}
+
 // hidden[p, units] = the gate unit of entry p's row with its expert's matrices. A block takes 16 units of an expert: its gate and up rows
 // stream from memory once, straight into matrix-core operands (out^T = W . x^T, W the 16-row operand), for up to MT times 16 rows at a
-// time; the waves take the steps of 32 along the width in turns and their sums meet in LDS, where the gate unit is.
-template <int MT, int KSPLIT>
-__global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ W, bf16_t* __restrict__ hidden,
+// time; the waves take the steps along the width in turns and their sums meet in LDS, where the gate unit is. Rows of x are whole 16-byte
+// pieces; a piece beyond their end is the last one again, and meets the zeros that fill the packed matrix.
+template <typename T, int MT, int KSPLIT>
+__global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const T* __restrict__ x, const T* __restrict__ W, T* __restrict__ hidden,
                                                                      const int* __restrict__ picks, const float* __restrict__ pick_weights, int n_rows, int top,
                                                                      int units, int width, GateUnit unit, int weigh_input) {
-    constexpr int UNROLL = MT == 4 ? 4 : 8;
+    constexpr int UNROLL = MT == 4 ? 4 : 8, VEC = 16 / (int)sizeof(T), KSTEP = 4 * VEC;
     __shared__ float sums[KSPLIT][2 * MT * 4][WAVE];
     __shared__ int list[FEW_ROWS], count;
     __shared__ float weights[FEW_ROWS];
@@ -142,31 +155,31 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const bf16_
     const int expert = blockIdx.y, u0 = blockIdx.x * 16;
     const int n = gather_entries(picks, pick_weights, n_rows * top, expert, list, weights, &count);
     if (n == 0) return;   // nobody picked this expert (uniform over the block)
-    const int steps = width / 32;   // a multiple of two: the width is one of 64
+    const int steps = packed_k_steps<T>(width);
     const int gate_tile = expert * (2 * units / 16) + u0 / 32 * 4 + u0 / 16 % 2;   // 32 gate rows, 32 up rows in turn
-    const bf16_t* x_row[MT];
+    const T* x_row[MT];
 #pragma unroll
-    for (int i = 0; i < MT; i++) x_row[i] = x + (size_t)(list[min(i * 16 + row16, n - 1)] / top) * width + quad * 8;   // beyond the last: never stored
+    for (int i = 0; i < MT; i++) x_row[i] = x + (size_t)(list[min(i * 16 + row16, n - 1)] / top) * width;   // beyond the last: never stored
     f32x4 gate[MT], up[MT];
 #pragma unroll
     for (int i = 0; i < MT; i++) gate[i] = up[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     for (int step0 = wave * UNROLL; step0 < steps; step0 += KSPLIT * UNROLL) {
-        bf16x8 g_op[UNROLL], u_op[UNROLL], x_op[UNROLL][MT];
+        Vec16 g_op[UNROLL], u_op[UNROLL], x_op[UNROLL][MT];
 #pragma unroll
         for (int u = 0; u < UNROLL; u++) {
             const int step = min(step0 + u, steps - 1);   // beyond the end: the last step again, not used
-            g_op[u] = *reinterpret_cast<const bf16x8*>(W + packed_offset<bf16_t>(gate_tile, step, steps, lane));
-            u_op[u] = *reinterpret_cast<const bf16x8*>(W + packed_offset<bf16_t>(gate_tile + 2, step, steps, lane));
+            g_op[u] = *reinterpret_cast<const Vec16*>(W + packed_offset<T>(gate_tile, step, steps, lane));
+            u_op[u] = *reinterpret_cast<const Vec16*>(W + packed_offset<T>(gate_tile + 2, step, steps, lane));
 #pragma unroll
-            for (int i = 0; i < MT; i++) x_op[u][i] = *reinterpret_cast<const bf16x8*>(x_row[i] + step * 32);
+            for (int i = 0; i < MT; i++) x_op[u][i] = *reinterpret_cast<const Vec16*>(x_row[i] + min(step * KSTEP + quad * VEC, width - VEC));
         }
 #pragma unroll
         for (int u = 0; u < UNROLL; u++) {
             if (step0 + u >= steps) break;
 #pragma unroll
             for (int i = 0; i < MT; i++) {
-                gate[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(g_op[u], x_op[u][i], gate[i], 0, 0, 0);
-                up[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u_op[u], x_op[u][i], up[i], 0, 0, 0);
+                multiply<T>(g_op[u], x_op[u][i], gate[i]);
+                multiply<T>(u_op[u], x_op[u][i], up[i]);
             }
         }
     }
@@ -189,18 +202,17 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_up_kernel(const bf16_
             g += sums[w][i * 4 + r][l];
             u += sums[w][(MT + i) * 4 + r][l];
         }
-        const int p = list[entry];
         const float weight = weights[entry];
         const float value = weigh_input ? gated(g * weight, u * weight, unit) : gated(g, u, unit) * weight;
-        hidden[(size_t)p * units + u0 + unit_at] = static_cast<bf16_t>(value);
+        hidden[(size_t)list[entry] * units + u0 + unit_at] = from_float<T>(value);
     }
 }
 
 // out[k, row, :] = hidden[row * top + k, units] . its expert's down matrix^T, 32-bit; a block takes 16 columns of an expert.
-template <int MT, int KSPLIT>
-__global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const bf16_t* __restrict__ hidden, const bf16_t* __restrict__ W, float* __restrict__ out,
+template <typename T, int MT, int KSPLIT>
+__global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const T* __restrict__ hidden, const T* __restrict__ W, float* __restrict__ out,
                                                                        const int* __restrict__ picks, int n_rows, int top, int units, int width) {
-    constexpr int UNROLL = MT == 4 ? 4 : 8;
+    constexpr int UNROLL = MT == 4 ? 4 : 8, VEC = 16 / (int)sizeof(T), KSTEP = 4 * VEC;
     __shared__ float sums[KSPLIT][MT * 4][WAVE];
     __shared__ int list[FEW_ROWS], count;
     __shared__ float weights[FEW_ROWS];
@@ -208,27 +220,27 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const bf1
     const int expert = blockIdx.y, n0 = blockIdx.x * 16;
     const int n = gather_entries(picks, nullptr, n_rows * top, expert, list, weights, &count);
     if (n == 0) return;
-    const int steps = units / 32, tile = expert * (width / 16) + blockIdx.x;
-    const bf16_t* h_row[MT];
+    const int steps = units / KSTEP, tile = expert * ((width + 15) / 16) + blockIdx.x;   // (the units are whole steps)
+    const T* h_row[MT];
 #pragma unroll
-    for (int i = 0; i < MT; i++) h_row[i] = hidden + (size_t)list[min(i * 16 + row16, n - 1)] * units + quad * 8;
+    for (int i = 0; i < MT; i++) h_row[i] = hidden + (size_t)list[min(i * 16 + row16, n - 1)] * units + quad * VEC;
     f32x4 acc[MT];
 #pragma unroll
     for (int i = 0; i < MT; i++) acc[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     for (int step0 = wave * UNROLL; step0 < steps; step0 += KSPLIT * UNROLL) {
-        bf16x8 w_op[UNROLL], h_op[UNROLL][MT];
+        Vec16 w_op[UNROLL], h_op[UNROLL][MT];
 #pragma unroll
         for (int u = 0; u < UNROLL; u++) {
             const int step = min(step0 + u, steps - 1);
-            w_op[u] = *reinterpret_cast<const bf16x8*>(W + packed_offset<bf16_t>(tile, step, steps, lane));
+            w_op[u] = *reinterpret_cast<const Vec16*>(W + packed_offset<T>(tile, step, steps, lane));
 #pragma unroll
-            for (int i = 0; i < MT; i++) h_op[u][i] = *reinterpret_cast<const bf16x8*>(h_row[i] + step * 32);
+            for (int i = 0; i < MT; i++) h_op[u][i] = *reinterpret_cast<const Vec16*>(h_row[i] + step * KSTEP);
         }
 #pragma unroll
         for (int u = 0; u < UNROLL; u++) {
             if (step0 + u >= steps) break;
 #pragma unroll
-            for (int i = 0; i < MT; i++) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w_op[u], h_op[u][i], acc[i], 0, 0, 0);
+            for (int i = 0; i < MT; i++) multiply<T>(w_op[u], h_op[u][i], acc[i]);
         }
     }
 #pragma unroll
@@ -239,6 +251,7 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const bf1
     for (int index = threadIdx.x; index < n * 16; index += 64 * KSPLIT) {
         const int entry = index / 16, column = index % 16, i = entry / 16;
         const int l = (column / 4) * 16 + entry % 16, r = column % 4;
+        if (n0 + column >= width) continue;
         float value = 0.0f;
 #pragma unroll
         for (int w = 0; w < KSPLIT; w++) value += sums[w][i * 4 + r][l];
@@ -247,15 +260,16 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_few_down_kernel(const bf1
     }
 }
 
-bool few_sizes(int n_rows, int top, int n_experts, int units, int width) {
-    return n_rows >= 0 && n_rows <= FEW_ROWS && top >= 1 && n_experts >= 1 && n_experts <= MAX_EXPERTS && top <= n_experts && units >= 64 && units % 64 == 0 &&
-           width >= 64 && width % 64 == 0;
+bool few_sizes(int n_rows, int top, int n_experts, int units, int width, int dtype) {
+    const int vec = dtype == MLLM_F32 ? 4 : 8;
+    return (dtype == MLLM_F32 || dtype == MLLM_BF16) && n_rows >= 0 && n_rows <= FEW_ROWS && top >= 1 && n_experts >= 1 && n_experts <= MAX_EXPERTS && top <= n_experts &&
+           units >= 64 && units % 64 == 0 && width >= vec && width % vec == 0;
 }
 
 }  // namespace
 
-// Rows up to which the products of few rows take the experts.
-MLLM_API int mllm_experts_few_rows() { return FEW_ROWS; }
+// Rows up to which the products of few rows take the experts (0: rows of this width are not whole 16-byte pieces).
+MLLM_API int mllm_experts_few_rows(int width, int dtype) { return few_sizes(0, 1, 1, 64, width, dtype) ? FEW_ROWS : 0; }
 
 // picks, pick_weights [n_rows, top] -> the lists: a_row, out_row, weight [n_rows * top] (as many entries as picks that name an expert), tiles [up to
 // n_rows * top / tile_rows + min(n_experts, n_rows * top)] of four integers each, n_tiles [1].
@@ -268,41 +282,49 @@ MLLM_API int mllm_expert_lists(const int* picks, const float* pick_weights, int 
     return mllm_check_launch("expert_lists");
 }
 
-#define MLLM_FEW_CASES(KERNEL, GRID, STEPS, ...)                                                       \
+// STEPS: the steps of K; four waves share them, eight where they are many
+#define MLLM_FEW_CASES(KERNEL, T, GRID, STEPS, ...)                                                    \
     do {                                                                                               \
         if ((STEPS) <= 32) {                                                                           \
-            if (n_rows <= 16) KERNEL<1, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                     \
-            else if (n_rows <= 32) KERNEL<2, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                \
-            else KERNEL<4, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                                  \
+            if (n_rows <= 16) KERNEL<T, 1, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                  \
+            else if (n_rows <= 32) KERNEL<T, 2, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);             \
+            else KERNEL<T, 4, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);                               \
         } else {                                                                                       \
-            if (n_rows <= 16) KERNEL<1, 8><<<GRID, 512, 0, stream>>>(__VA_ARGS__);                     \
-            else if (n_rows <= 32) KERNEL<2, 8><<<GRID, 512, 0, stream>>>(__VA_ARGS__);                \
-            else KERNEL<4, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);   /* (its sums take 32 KB of LDS as it is) */ \
+            if (n_rows <= 16) KERNEL<T, 1, 8><<<GRID, 512, 0, stream>>>(__VA_ARGS__);                  \
+            else if (n_rows <= 32) KERNEL<T, 2, 8><<<GRID, 512, 0, stream>>>(__VA_ARGS__);             \
+            else KERNEL<T, 4, 4><<<GRID, 256, 0, stream>>>(__VA_ARGS__);   /* (its sums take 32 KB of LDS as it is) */ \
         }                                                                                              \
     } while (0)
 
 // x [n_rows, width], hidden [n_rows * top, units] (rows of picks that name no expert are left alone), W packed [n_experts * 2 * units, width].
 MLLM_API int mllm_experts_few_up(const void* x, const void* W, void* hidden, const int* picks, const float* pick_weights, int n_rows, int top, int n_experts, int units,
-                                 int width, float limit, float alpha, float shift, int weigh_input, hipStream_t stream) {
-    MLLM_REQUIRE(few_sizes(n_rows, top, n_experts, units, width), "experts_few_up: no kernel for %d rows, %d of %d experts, %d units, width %d", n_rows, top, n_experts, units, width);
+                                 int width, float limit, float alpha, float shift, int weigh_input, int dtype, hipStream_t stream) {
+    MLLM_REQUIRE(few_sizes(n_rows, top, n_experts, units, width, dtype), "experts_few_up: no kernel for %d rows, %d of %d experts, %d units, width %d", n_rows, top, n_experts, units, width);
     MLLM_REQUIRE(x && W && hidden && picks && pick_weights && limit > 0.0f && ((uintptr_t)x & 15) == 0, "experts_few_up: a missing operand");
     if (n_rows == 0) return 0;
     mllm_count_kernel(MLLM_K_EXPERTS_FEW);
     const dim3 grid(units / 16, n_experts);
     const GateUnit unit{limit, alpha, shift};
-    MLLM_FEW_CASES(experts_few_up_kernel, grid, width / 32, (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)hidden, picks, pick_weights, n_rows, top, units, width, unit,
-                   weigh_input);
+    if (dtype == MLLM_F32)
+        MLLM_FEW_CASES(experts_few_up_kernel, float, grid, packed_k_steps<float>(width), (const float*)x, (const float*)W, (float*)hidden, picks, pick_weights, n_rows, top,
+                       units, width, unit, weigh_input);
+    else
+        MLLM_FEW_CASES(experts_few_up_kernel, bf16_t, grid, packed_k_steps<bf16_t>(width), (const bf16_t*)x, (const bf16_t*)W, (bf16_t*)hidden, picks, pick_weights, n_rows,
+                       top, units, width, unit, weigh_input);
     return mllm_check_launch("experts_few_up");
 }
 
-// out [top, n_rows, width] (rows of picks that name no expert are left alone), W packed [n_experts * width, units].
-MLLM_API int mllm_experts_few_down(const void* hidden, const void* W, float* out, const int* picks, int n_rows, int top, int n_experts, int units, int width,
+// out [top, n_rows, width] (rows of picks that name no expert are left alone), W packed, every expert's [width, units] filled up to whole sixteens of rows.
+MLLM_API int mllm_experts_few_down(const void* hidden, const void* W, float* out, const int* picks, int n_rows, int top, int n_experts, int units, int width, int dtype,
                                    hipStream_t stream) {
-    MLLM_REQUIRE(few_sizes(n_rows, top, n_experts, units, width), "experts_few_down: no kernel for %d rows, %d of %d experts, %d units, width %d", n_rows, top, n_experts, units, width);
+    MLLM_REQUIRE(few_sizes(n_rows, top, n_experts, units, width, dtype), "experts_few_down: no kernel for %d rows, %d of %d experts, %d units, width %d", n_rows, top, n_experts, units, width);
     MLLM_REQUIRE(hidden && W && out && picks && ((uintptr_t)hidden & 15) == 0, "experts_few_down: a missing operand");
     if (n_rows == 0) return 0;
     mllm_count_kernel(MLLM_K_EXPERTS_FEW);
-    const dim3 grid(width / 16, n_experts);
-    MLLM_FEW_CASES(experts_few_down_kernel, grid, units / 32, (const bf16_t*)hidden, (const bf16_t*)W, out, picks, n_rows, top, units, width);
+    const dim3 grid(ceil_div(width, 16), n_experts);
+    if (dtype == MLLM_F32)
+        MLLM_FEW_CASES(experts_few_down_kernel, float, grid, units / 16, (const float*)hidden, (const float*)W, out, picks, n_rows, top, units, width);
+    else
+        MLLM_FEW_CASES(experts_few_down_kernel, bf16_t, grid, units / 32, (const bf16_t*)hidden, (const bf16_t*)W, out, picks, n_rows, top, units, width);
     return mllm_check_launch("experts_few_down");
 }

@@ -80,14 +80,15 @@ __device__ __forceinline__ Vec16 mask_piece(Vec16 v, bool valid) {
 // Tiles of A and W go memory -> registers -> LDS; the loads run two tiles ahead of the products
 // (two register sets used in turn), so that one block per compute unit still hides the memory
 // latency: these products are small enough that the grid often is no more than that.
+// Group: the whole product, or one over rows grouped by expert (gemm_stream.h's ExpertTiles; a one-dimensional grid).
 // BEST: the block leaves no sums but, per row, the best (sum, column) of each of its waves (BestOfColumns).
-template <typename T, typename OutT, int BM, int BN, int WAVES_M, int WAVES_N, bool ALIGNED, bool PACKED, bool BEST = false>
+template <typename T, typename OutT, int BM, int BN, int WAVES_M, int WAVES_N, bool ALIGNED, bool PACKED, bool BEST = false, typename Group = stream::Whole>
 __global__ __launch_bounds__(64 * WAVES_M * WAVES_N) void gemm_kernel(const T* __restrict__ A, const T* __restrict__ W,
                                                    const float* __restrict__ bias,
                                                    const float* __restrict__ residual,
                                                    OutT* __restrict__ out, int M, int N, int K,
                                                    int epilogue, CacheScatter scatter, int k_per_block,
-                                                   BestOfColumns best_out = BestOfColumns{}) {
+                                                   BestOfColumns best_out = BestOfColumns{}, Group group = Group{}) {
     constexpr int BK = Tile<T>::BK, VEC = Tile<T>::VEC, PAD = Tile<T>::PAD;
     constexpr int LDK = BK + PAD;
     constexpr int TM = BM / WAVES_M / 32, TN = BN / WAVES_N / 32;
@@ -103,7 +104,15 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N) void gemm_kernel(const T* _
 
     const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
     const int wave_m = wave / WAVES_N, wave_n = wave % WAVES_N;
-    const int m0 = blockIdx.y * BM, n0 = blockIdx.x * BN;
+    int m0 = blockIdx.y * BM, n0 = blockIdx.x * BN, m_end = M, w_first_tile = 0;
+    if constexpr (Group::GROUPED) {
+        stream::GroupTile tile;
+        if (!stream::group_tile(group, N, BN, tile)) return;  // (the whole block leaves)
+        m0 = tile.m0;
+        m_end = tile.m_end;
+        n0 = tile.n0;
+        w_first_tile = tile.expert * w_row_tiles;
+    }
     const int half = lane / 32, lane32 = lane % 32;
     // The block's part of K: all of it, or, when several blocks share the tile (gridDim.z), a run
     // of k_per_block (a multiple of two LDS tiles), whose sums go to matrix blockIdx.z of `out`
@@ -137,13 +146,24 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N) void gemm_kernel(const T* _
             }
     }
 
+    int a_rows[Group::GROUPED ? A_PIECES : 1];  // a grouped product: the row of A that each of this thread's pieces comes from
+    if constexpr (Group::GROUPED) {
+#pragma unroll
+        for (int i = 0; i < A_PIECES; i++) {
+            const int entry = min(m0 + (tid + i * THREADS) / VPR, m_end - 1);  // beyond the last: that row again, never stored
+            a_rows[i] = group.a_row ? group.a_row[entry] : entry;
+        }
+    }
     Vec16 a_regs[2][A_PIECES], w_regs[2][W_PIECES];
     bool a_valid[2][A_PIECES], w_valid[2][W_PIECES];
     auto fetch = [&](int set, int k0) {
 #pragma unroll
         for (int i = 0; i < A_PIECES; i++) {
             int piece = tid + i * THREADS;
-            if (BM * VPR % THREADS == 0 || piece < BM * VPR) a_regs[set][i] = load_piece<T, ALIGNED>(A, m0 + piece / VPR, M, k0 + (piece % VPR) * VEC, K, k_end, a_valid[set][i]);
+            if (BM * VPR % THREADS == 0 || piece < BM * VPR) {
+                if constexpr (Group::GROUPED) a_regs[set][i] = load_piece<T, ALIGNED>(A, a_rows[i], a_rows[i] + 1, k0 + (piece % VPR) * VEC, K, k_end, a_valid[set][i]);
+                else a_regs[set][i] = load_piece<T, ALIGNED>(A, m0 + piece / VPR, M, k0 + (piece % VPR) * VEC, K, k_end, a_valid[set][i]);
+            }
         }
 #pragma unroll
         for (int i = 0; i < W_PIECES; i++) {
@@ -153,7 +173,7 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N) void gemm_kernel(const T* _
                     // 64 consecutive pieces are one chunk: 1 KiB of contiguous memory
                     int chunk = piece / 64, row_tile = n0 / 16 + chunk / CHUNKS_K, k_step = k0 / KC + chunk % CHUNKS_K;
                     w_valid[set][i] = row_tile < w_row_tiles && k_step * KC < k_end;  // k_end is K or a multiple of the chunk
-                    w_regs[set][i] = *reinterpret_cast<const Vec16*>(W + packed_offset<T>(min(row_tile, w_row_tiles - 1), min(k_step, w_k_steps - 1), w_k_steps, piece % 64));
+                    w_regs[set][i] = *reinterpret_cast<const Vec16*>(W + packed_offset<T>(w_first_tile + min(row_tile, w_row_tiles - 1), min(k_step, w_k_steps - 1), w_k_steps, piece % 64));
                 } else {
                     w_regs[set][i] = load_piece<T, ALIGNED>(W, n0 + piece / VPR, N, k0 + (piece % VPR) * VEC, K, k_end, w_valid[set][i]);
                 }
@@ -248,6 +268,32 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N) void gemm_kernel(const T* _
     }
 
     // A lane holds column lane%32 and rows 8*(v/4) + 4*(lane/32) + v%4 of each 32x32 tile.
+    if constexpr (Group::GROUPED) {
+        static_assert(!Group::GATED || TN % 2 == 0, "a wave holds gate and up columns of the same units");
+        constexpr int STEP = Group::GATED ? 2 : 1;
+#pragma unroll
+        for (int i = 0; i < TM; i++)
+#pragma unroll
+            for (int v = 0; v < 16; v++) {
+                const int entry = m0 + wave_m * TM * 32 + i * 32 + 8 * (v / 4) + 4 * half + (v % 4);
+                if (entry >= m_end) continue;
+                const int row = Group::GATED ? entry : (group.out_row ? group.out_row[entry] : entry);
+                const float weight = Group::GATED ? group.weight[entry] : 1.0f;
+                const float in_weight = group.weigh_input ? weight : 1.0f, out_weight = group.weigh_input ? 1.0f : weight;
+#pragma unroll
+                for (int j = 0; j < TN; j += STEP) {
+                    const int column = n0 + wave_n * TN * 32 + j * 32;   // of W's rows
+                    if constexpr (Group::GATED) {
+                        if (column < N)   // (N is a multiple of 64, the pair's columns lie inside together)
+                            out[(size_t)row * (N / 2) + column / 2 + lane32] =
+                                from_float<OutT>(gated(acc[i][j][v] * in_weight, acc[i][j + 1][v] * in_weight, group.unit) * out_weight);
+                    } else if (column + lane32 < N) {
+                        out[(size_t)row * N + column + lane32] = from_float<OutT>(acc[i][j][v]);
+                    }
+                }
+            }
+        return;
+    }
     if constexpr (BEST) {
         // Per row the best of this block's columns. The sums go to LDS as a [BM, BN] matrix (the tiles' memory: every
         // wave has left the loop behind the last barrier); then the THREADS / BM threads next to each other that share
@@ -807,41 +853,68 @@ constexpr int EXPERT_TILE = 128;   // entries a tile of the lists holds
 
 MLLM_API int mllm_expert_tile_rows() { return EXPERT_TILE; }
 
-// Whether the two products of experts run grouped: bfloat16, whole tiles of K in both (the width and an expert's padded units).
-MLLM_API int mllm_experts_supported(int width, int units, int dtype) {
-    return dtype == MLLM_BF16 && width >= 64 && width % 64 == 0 && units >= 64 && units % 64 == 0;
+namespace {
+
+template <typename T, typename OutT, bool ALIGNED, typename Group>
+void launch_tiled_experts(const void* a, const void* w, void* o, int entries, int max_tiles, int N, int K, const Group& group, hipStream_t stream) {
+    constexpr int BN = 128, PAIR = 2 * Tile<T>::BK;
+    mllm_count_kernel(MLLM_K_GEMM_TILED);
+    gemm_kernel<T, OutT, EXPERT_TILE, BN, 4, 2, ALIGNED, true, false, Group><<<ceil_div(max_tiles * ceil_div(N, BN), 8) * 8, 512, 0, stream>>>(
+        (const T*)a, (const T*)w, nullptr, nullptr, (OutT*)o, entries, N, K, 0, CacheScatter{}, ceil_div(K, PAIR) * PAIR, BestOfColumns{}, group);
 }
 
+int check_experts(const char* what, int entries, int max_tiles, int units, int width, int dtype) {
+    MLLM_REQUIRE(dtype == MLLM_F32 || dtype == MLLM_BF16, "%s: unknown dtype %d", what, dtype);
+    MLLM_REQUIRE(width >= 1 && units >= 64 && units % 64 == 0, "%s: no kernel for width %d with %d units", what, width, units);
+    const long long widest = width > units ? width : units;
+    MLLM_REQUIRE(entries >= 0 && max_tiles >= 0 && (long long)max_tiles * ceil_div((int)(2 * widest), 64) < (1LL << 30) && entries * widest * 4 < (1LL << 32),
+                 "%s: %d entries of %lld are more than the kernels take", what, entries, widest);
+    return 0;
+}
+
+}  // namespace
+
 // hidden [entries, units]: the gate unit of row a_row[i] of x [.., width] with its expert's matrices, W [n_experts * 2 * units, width] packed, an
-// expert's rows 32 gate rows and 32 up rows in turn. tiles / n_tiles / max_tiles: see ExpertTiles.
+// expert's rows 32 gate rows and 32 up rows in turn; units a multiple of 64. tiles / n_tiles / max_tiles: see ExpertTiles.
 MLLM_API int mllm_experts_up(const void* x, const void* W, void* hidden, const int* tiles, const int* n_tiles, const int* a_row, const float* weight, int entries,
-                             int max_tiles, int units, int width, float limit, float alpha, float shift, int weigh_input, hipStream_t stream) {
-    MLLM_REQUIRE(mllm_experts_supported(width, units, MLLM_BF16), "experts_up: no kernel for width %d with %d units", width, units);
+                             int max_tiles, int units, int width, float limit, float alpha, float shift, int weigh_input, int dtype, hipStream_t stream) {
+    if (int status = check_experts("experts_up", entries, max_tiles, units, width, dtype)) return status;
     MLLM_REQUIRE(x && W && hidden && tiles && n_tiles && a_row && weight && limit > 0.0f && ((uintptr_t)tiles & 15) == 0, "experts_up: a missing operand");
-    MLLM_REQUIRE(entries >= 0 && max_tiles >= 0 && (long long)max_tiles * ceil_div(2 * units, 128) < (1LL << 30) && (long long)entries * width * 2 < (1LL << 32),
-                 "experts_up: bad sizes");
     if (entries == 0) return 0;
     const stream::ExpertTiles<true> group{(const int4*)tiles, n_tiles, a_row, nullptr, weight, GateUnit{limit, alpha, shift}, weigh_input};
-    stream::launch_grouped<bf16_t, EXPERT_TILE, 128, 2, 2, 3>((const bf16_t*)x, (const bf16_t*)W, (bf16_t*)hidden, entries, max_tiles, 2 * units, width, group, stream);
+    if (dtype == MLLM_F32) {
+        if (width % 4 == 0) launch_tiled_experts<float, float, true>(x, W, hidden, entries, max_tiles, 2 * units, width, group, stream);
+        else launch_tiled_experts<float, float, false>(x, W, hidden, entries, max_tiles, 2 * units, width, group, stream);
+    } else if (width % 64 == 0) {
+        stream::launch_grouped<bf16_t, EXPERT_TILE, 128, 2, 2, 3>((const bf16_t*)x, (const bf16_t*)W, (bf16_t*)hidden, entries, max_tiles, 2 * units, width, group, stream);
+    } else if (width % 8 == 0) {
+        launch_tiled_experts<bf16_t, bf16_t, true>(x, W, hidden, entries, max_tiles, 2 * units, width, group, stream);
+    } else {
+        launch_tiled_experts<bf16_t, bf16_t, false>(x, W, hidden, entries, max_tiles, 2 * units, width, group, stream);
+    }
     return mllm_check_launch("experts_up");
 }
 
-// out row out_row[i] = hidden row i . its expert's down matrix^T, 32-bit; W [n_experts * width, units] packed.
+// out row out_row[i] = hidden row i . its expert's down matrix^T, 32-bit; W packed, every expert's [width, units] filled up to whole sixteens of rows.
 MLLM_API int mllm_experts_down(const void* hidden, const void* W, float* out, const int* tiles, const int* n_tiles, const int* out_row, int entries, int max_tiles,
-                               int units, int width, hipStream_t stream) {
-    MLLM_REQUIRE(mllm_experts_supported(width, units, MLLM_BF16), "experts_down: no kernel for width %d with %d units", width, units);
+                               int units, int width, int dtype, hipStream_t stream) {
+    if (int status = check_experts("experts_down", entries, max_tiles, units, width, dtype)) return status;
     MLLM_REQUIRE(hidden && W && out && tiles && n_tiles && out_row && ((uintptr_t)tiles & 15) == 0, "experts_down: a missing operand");
-    MLLM_REQUIRE(entries >= 0 && max_tiles >= 0 && (long long)max_tiles * ceil_div(width, 64) < (1LL << 30) && (long long)entries * units * 2 < (1LL << 32),
-                 "experts_down: bad sizes");
     if (entries == 0) return 0;
     const stream::ExpertTiles<false> group{(const int4*)tiles, n_tiles, nullptr, out_row, nullptr, GateUnit{1.0f, 1.0f, 0.0f}, 0};
-    // wide tiles where they fill the rounds of blocks as well as narrow ones do (the costs of a tile of K: dispatch)
-    const long tiles_m = ceil_div(entries, EXPERT_TILE);
-    const float wide = (float)((tiles_m * ceil_div(width, 128) + 255) / 256) * 0.45f, narrow = (float)((tiles_m * ceil_div(width, 64) + 255) / 256) * 0.30f;
-    if (wide <= narrow)
-        stream::launch_grouped<float, EXPERT_TILE, 128, 2, 2, 3>((const bf16_t*)hidden, (const bf16_t*)W, out, entries, max_tiles, width, units, group, stream);
-    else
-        stream::launch_grouped<float, EXPERT_TILE, 64, 2, 2, 3>((const bf16_t*)hidden, (const bf16_t*)W, out, entries, max_tiles, width, units, group, stream);
+    if (dtype == MLLM_F32) {
+        launch_tiled_experts<float, float, true>(hidden, W, out, entries, max_tiles, width, units, group, stream);
+    } else if (width % 8 != 0) {
+        launch_tiled_experts<bf16_t, float, true>(hidden, W, out, entries, max_tiles, width, units, group, stream);
+    } else {
+        // wide tiles where they fill the rounds of blocks as well as narrow ones do (the costs of a tile of K: dispatch)
+        const long tiles_m = ceil_div(entries, EXPERT_TILE);
+        const float wide = (float)((tiles_m * ceil_div(width, 128) + 255) / 256) * 0.45f, narrow = (float)((tiles_m * ceil_div(width, 64) + 255) / 256) * 0.30f;
+        if (wide <= narrow)
+            stream::launch_grouped<float, EXPERT_TILE, 128, 2, 2, 3>((const bf16_t*)hidden, (const bf16_t*)W, out, entries, max_tiles, width, units, group, stream);
+        else
+            stream::launch_grouped<float, EXPERT_TILE, 64, 2, 2, 3>((const bf16_t*)hidden, (const bf16_t*)W, out, entries, max_tiles, width, units, group, stream);
+    }
     return mllm_check_launch("experts_down");
 }
 

@@ -133,6 +133,21 @@ struct ExpertTiles {
     int weigh_input;
 };
 
+// The tile of this block, an eighth of the tiles to each XCD in the order of their experts: an expert's matrix goes to one or two L2 caches.
+// False: the grid, which is sized for the most tiles there can be, has a block too many.
+struct GroupTile {
+    int expert, m0, m_end, n0;
+};
+template <typename Group>
+__device__ __forceinline__ bool group_tile(const Group& group, int N, int BN, GroupTile& out) {
+    const int xcd = blockIdx.x % 8, in_xcd = blockIdx.x / 8;
+    const int across = (N + BN - 1) / BN, total = *group.n_tiles * across, share = (total + 7) / 8, at = xcd * share + in_xcd;
+    if (in_xcd >= share || at >= total) return false;
+    const int4 tile = group.tiles[at / across];
+    out = GroupTile{tile.x, tile.y, tile.z, (at % across) * BN};
+    return true;
+}
+
 // grid: one row of blocks, placed by 'places' (tiles and blocks along K). More than one block along K: each block takes k_per_block of K (a multiple
 // of 64) and leaves a partial product in matrix 'block_k' of `out` (float, no bias / epilogue / residual).
 // WAVES_K = 2: two waves share a tile of outputs and take half of every tile of K each; their sums meet in LDS at the end.
@@ -169,14 +184,12 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
     const int xcd = blockIdx.x % 8, in_xcd = blockIdx.x / 8;
     int block_k = 0, m0, n0, m_end = M, w_first_tile = 0;
     if constexpr (GROUPED) {
-        // the tiles in the order of their experts, an eighth of them to each XCD: an expert's matrix goes to one or two L2 caches
-        const int across = (N + BN - 1) / BN, total = *group.n_tiles * across, share = (total + 7) / 8, at = xcd * share + in_xcd;
-        if (in_xcd >= share || at >= total) return;  // (the grid is sized for the most tiles there can be)
-        const int4 tile = group.tiles[at / across];
-        m0 = tile.y;
-        m_end = tile.z;
-        n0 = (at % across) * BN;
-        w_first_tile = tile.x * ((N + 15) / 16);
+        GroupTile tile;
+        if (!group_tile(group, N, BN, tile)) return;  // (the whole block leaves)
+        m0 = tile.m0;
+        m_end = tile.m_end;
+        n0 = tile.n0;
+        w_first_tile = tile.expert * ((N + 15) / 16);
     } else {
         block_k = in_xcd / (places.wide * places.high);
         const int in_rectangle = in_xcd % (places.wide * places.high);

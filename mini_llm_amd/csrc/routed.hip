@@ -182,10 +182,9 @@ __global__ __launch_bounds__(256) void expert_unit_kernel(const T* __restrict__ 
     }
 }
 
-// both: [rows, 2 * inner], a gate half and an up half. out = g * sigmoid(alpha * g) * (u + shift) with g = min(gate, limit) and u =
-// clamp(up, -limit, limit) (limit infinite: unclamped). PIECES: a thread takes 16 bytes of each half.
+// both: [rows, 2 * inner], a gate half and an up half; out = their gate unit (gate_unit.h). PIECES: a thread takes 16 bytes of each half.
 template <typename T, bool PIECES>
-__global__ __launch_bounds__(256) void gate_unit_kernel(const T* __restrict__ both, T* __restrict__ out, int inner, float limit, float alpha, float shift) {
+__global__ __launch_bounds__(256) void gate_unit_kernel(const T* __restrict__ both, T* __restrict__ out, int inner, GateUnit unit) {
     constexpr int VEC = PIECES ? 16 / (int)sizeof(T) : 1;
     const int j = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
     if (j >= inner) return;
@@ -201,62 +200,11 @@ __global__ __launch_bounds__(256) void gate_unit_kernel(const T* __restrict__ bo
         T* re = reinterpret_cast<T*>(&result);
 #pragma unroll
         for (int e = 0; e < VEC; e++) {
-            const float g = fminf(to_float(ge[e]), limit);
-            const float u = fminf(fmaxf(to_float(ue[e]), -limit), limit);
-            re[e] = from_float<T>(g / (1.0f + expf(-alpha * g)) * (u + shift));
+            re[e] = from_float<T>(gated(to_float(ge[e]), to_float(ue[e]), unit));
         }
         *reinterpret_cast<Vec16*>(out_at) = result;
     } else {
-        const float g = fminf(to_float(*g_at), limit);
-        const float u = fminf(fmaxf(to_float(*u_at), -limit), limit);
-        *out_at = from_float<T>(g / (1.0f + expf(-alpha * g)) * (u + shift));
-    }
-}
-
-// both: [rows, n_experts * 2 * ff], per expert its gate sums and then its up sums. out [rows, n_experts * ff] = the gate unit, times the
-// row's weight for the expert; with `weigh_input` the weight multiplies both sums instead (a product of w h is w times the product of
-// h). An expert of weight zero gives zeros. PIECES: a thread takes 16 bytes of units (ff is a multiple of that many).
-template <typename T, bool PIECES>
-__global__ __launch_bounds__(256) void gated_expert_unit_kernel(const T* __restrict__ both, T* __restrict__ out, const float* __restrict__ weights,
-                                                                int weights_stride, int n_experts, int ff, GateUnit unit, int weigh_input) {
-    constexpr int VEC = PIECES ? 16 / (int)sizeof(T) : 1;
-    const int inner = n_experts * ff;
-    const int j = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
-    if (j >= inner) return;
-    const size_t row = blockIdx.y;
-    const int expert = j / ff;
-    const float weight = weights[row * weights_stride + expert];
-    const float in_weight = weigh_input ? weight : 1.0f, out_weight = weigh_input ? 1.0f : weight;
-    const T* g_at = both + row * 2 * inner + (size_t)expert * 2 * ff + (j - expert * ff);
-    const T* u_at = g_at + ff;
-    T* out_at = out + row * inner + j;
-    if constexpr (PIECES) {
-        Vec16 result = {};
-        if (weight != 0.0f) {
-            const Vec16 gs = *reinterpret_cast<const Vec16*>(g_at), us = *reinterpret_cast<const Vec16*>(u_at);
-            const T* ge = reinterpret_cast<const T*>(&gs);
-            const T* ue = reinterpret_cast<const T*>(&us);
-            T* re = reinterpret_cast<T*>(&result);
-#pragma unroll
-            for (int e = 0; e < VEC; e++) re[e] = from_float<T>(gated(to_float(ge[e]) * in_weight, to_float(ue[e]) * in_weight, unit) * out_weight);
-        }
-        *reinterpret_cast<Vec16*>(out_at) = result;
-    } else {
-        *out_at = from_float<T>(weight != 0.0f ? gated(to_float(*g_at) * in_weight, to_float(*u_at) * in_weight, unit) * out_weight : 0.0f);
-    }
-}
-
-template <typename T>
-void launch_gated_expert_unit(const void* both, void* out, const float* weights, int weights_stride, int rows, int n_experts, int ff, GateUnit unit,
-                              int weigh_input, hipStream_t stream) {
-    constexpr int VEC = 16 / (int)sizeof(T);
-    const int inner = n_experts * ff;
-    if (ff % VEC == 0 && ((uintptr_t)both & 15) == 0 && ((uintptr_t)out & 15) == 0) {
-        dim3 grid(ceil_div(inner / VEC, 256), rows);
-        gated_expert_unit_kernel<T, true><<<grid, 256, 0, stream>>>((const T*)both, (T*)out, weights, weights_stride, n_experts, ff, unit, weigh_input);
-    } else {
-        dim3 grid(ceil_div(inner, 256), rows);
-        gated_expert_unit_kernel<T, false><<<grid, 256, 0, stream>>>((const T*)both, (T*)out, weights, weights_stride, n_experts, ff, unit, weigh_input);
+        *out_at = from_float<T>(gated(to_float(*g_at), to_float(*u_at), unit));
     }
 }
 
@@ -277,14 +225,14 @@ void launch_expert_unit(const void* up, void* out, const float* weights, int wei
 }
 
 template <typename T>
-void launch_gate_unit(const void* both, void* out, int rows, int inner, float limit, float alpha, float shift, hipStream_t stream) {
+void launch_gate_unit(const void* both, void* out, int rows, int inner, GateUnit unit, hipStream_t stream) {
     constexpr int VEC = 16 / (int)sizeof(T);
     if (inner % VEC == 0 && ((uintptr_t)both & 15) == 0 && ((uintptr_t)out & 15) == 0) {
         dim3 grid(ceil_div(inner / VEC, 256), rows);
-        gate_unit_kernel<T, true><<<grid, 256, 0, stream>>>((const T*)both, (T*)out, inner, limit, alpha, shift);
+        gate_unit_kernel<T, true><<<grid, 256, 0, stream>>>((const T*)both, (T*)out, inner, unit);
     } else {
         dim3 grid(ceil_div(inner, 256), rows);
-        gate_unit_kernel<T, false><<<grid, 256, 0, stream>>>((const T*)both, (T*)out, inner, limit, alpha, shift);
+        gate_unit_kernel<T, false><<<grid, 256, 0, stream>>>((const T*)both, (T*)out, inner, unit);
     }
 }
 
@@ -360,26 +308,6 @@ MLLM_API int mllm_expert_unit(const void* up, void* out, const float* weights, i
     return mllm_check_launch("expert_unit");
 }
 
-MLLM_API int mllm_gated_expert_unit(const void* both, void* out, const float* weights, int weights_stride, int n_rows, int n_experts, int ff, float limit,
-                                    float alpha, float shift, int weigh_input, int dtype, hipStream_t stream) {
-    MLLM_REQUIRE(n_rows >= 0 && n_experts > 0 && ff > 0 && limit > 0.0f, "gated_expert_unit: bad sizes or limit");
-    MLLM_REQUIRE(weights_stride >= n_experts && both != nullptr && out != nullptr && weights != nullptr, "gated_expert_unit: a missing operand or short weights");
-    MLLM_REQUIRE(dtype == MLLM_F32 || dtype == MLLM_BF16, "gated_expert_unit: unknown dtype %d", dtype);
-    if (n_rows == 0) return 0;
-    mllm_count_kernel(MLLM_K_EXPERT_UNIT);
-    const GateUnit unit{limit, alpha, shift};
-    const size_t inner = (size_t)n_experts * ff, element = dtype == MLLM_F32 ? 4 : 2;
-    for (int row0 = 0; row0 < n_rows; row0 += 65535) {   // the grid's second dimension holds 65,535 rows
-        const int rows = n_rows - row0 < 65535 ? n_rows - row0 : 65535;
-        const char* in_at = (const char*)both + (size_t)row0 * 2 * inner * element;
-        char* out_at = (char*)out + (size_t)row0 * inner * element;
-        const float* weights_at = weights + (size_t)row0 * weights_stride;
-        if (dtype == MLLM_F32) launch_gated_expert_unit<float>(in_at, out_at, weights_at, weights_stride, rows, n_experts, ff, unit, weigh_input, stream);
-        else launch_gated_expert_unit<bf16_t>(in_at, out_at, weights_at, weights_stride, rows, n_experts, ff, unit, weigh_input, stream);
-    }
-    return mllm_check_launch("gated_expert_unit");
-}
-
 MLLM_API int mllm_gate_unit(const void* both, void* out, int n_rows, int inner, float limit, float alpha, float shift, int dtype, hipStream_t stream) {
     MLLM_REQUIRE(n_rows >= 0 && inner > 0, "gate_unit: bad sizes");
     MLLM_REQUIRE(limit > 0.0f, "gate_unit: the limit must be positive (infinite: none)");
@@ -391,8 +319,8 @@ MLLM_API int mllm_gate_unit(const void* both, void* out, int n_rows, int inner, 
         const int rows = n_rows - row0 < 65535 ? n_rows - row0 : 65535;
         const char* in_at = (const char*)both + (size_t)row0 * 2 * inner * element;
         char* out_at = (char*)out + (size_t)row0 * inner * element;
-        if (dtype == MLLM_F32) launch_gate_unit<float>(in_at, out_at, rows, inner, limit, alpha, shift, stream);
-        else launch_gate_unit<bf16_t>(in_at, out_at, rows, inner, limit, alpha, shift, stream);
+        if (dtype == MLLM_F32) launch_gate_unit<float>(in_at, out_at, rows, inner, GateUnit{limit, alpha, shift}, stream);
+        else launch_gate_unit<bf16_t>(in_at, out_at, rows, inner, GateUnit{limit, alpha, shift}, stream);
     }
     return mllm_check_launch("gate_unit");
 }

@@ -1394,36 +1394,42 @@ def route_rows(x, router, top: int, *, correction=None, n_groups: int = 1, keep:
     return picked if picks else weights
 
 
-def grouped_experts_supported(width: int, units: int, dtype) -> bool:
-    """Whether ``grouped_experts`` takes experts of so many (padded) hidden units over rows of ``width`` elements."""
-    return bool(library().mllm_experts_supported(int(width), int(units), _code(dtype)))
+EXPERT_UNITS = 64   # an expert's hidden units are filled up to a multiple of this with zeros
+
+
+def expert_down_rows(width: int) -> int:
+    """Rows an expert's down matrix is filled up to (whole row tiles of the packed layout, so that every expert starts with one)."""
+    return -(-int(width) // 16) * 16
 
 
 def grouped_experts(x, picks: Picks, up: PackedMatrix, down: PackedMatrix, n_experts: int, units: int, *, limit: float | None = None, alpha: float = 1.0,
                     shift: float = 0.0, weigh_input: bool = False):
     """The picked experts of every row, and no others: float32 [top, rows, width], whose plane k is the k-th pick's expert, W_down unit(W_gate
-    h, W_up h) with the gate unit of ``gate_unit`` and the pick's weight on the unit or (``weigh_input``) on both sums. x: bfloat16 [rows, width]. ``up``
-    [n_experts * 2 * units, width]: per expert, for every 32 units, 32 gate rows and 32 up rows; ``down`` [n_experts * width, units]: the experts'
-    matrices behind each other; ``units`` a multiple of 64 (zero rows and columns fill an expert up). Few rows find their experts inside the
-    products; more rows are sorted by expert on the device first. A pick of -1 leaves its place undefined."""
-    _device_tensor(x, "x", torch.bfloat16, 2)
+    h, W_up h) with the gate unit of ``gate_unit`` and the pick's weight on the unit or (``weigh_input``) on both sums. x: [rows, width]. ``up``
+    [n_experts * 2 * units, width]: per expert, for every 32 units, 32 gate rows and 32 up rows; ``down`` [n_experts * expert_down_rows(width),
+    units]: the experts' matrices behind each other, each filled up with zero rows; ``units`` a multiple of EXPERT_UNITS (zero rows and columns
+    fill an expert up). Few rows find their experts inside the products; more rows are sorted by expert on the device first. A pick of -1
+    leaves its place undefined."""
+    _device_tensor(x, "x", dim=2)
+    code = _code(x.dtype)
     n, width = x.shape
     _device_tensor(picks.experts, "picks", torch.int32, 2)
     _device_tensor(picks.weights, "the picks' weights", torch.float32, 2)
     top = picks.experts.shape[1]
     _require(tuple(picks.experts.shape) == (n, top) and tuple(picks.weights.shape) == (n, top), "picks and rows differ")
     _require(limit is None or limit > 0, "the limit must be positive")
-    for matrix, name, shape in ((up, "up", (n_experts * 2 * units, width)), (down, "down", (n_experts * width, units))):
-        _require(isinstance(matrix, PackedMatrix) and matrix.dtype == torch.bfloat16 and tuple(matrix.shape) == shape, f"{name} must be packed, bfloat16, {shape}")
-    _require(grouped_experts_supported(width, units, x.dtype), f"no kernel for experts of {units} units over rows of {width}")
+    _require(units >= EXPERT_UNITS and units % EXPERT_UNITS == 0, f"an expert's units are a multiple of {EXPERT_UNITS}")
+    for matrix, name, shape in ((up, "up", (n_experts * 2 * units, width)), (down, "down", (n_experts * expert_down_rows(width), units))):
+        _require(isinstance(matrix, PackedMatrix) and matrix.dtype == x.dtype and tuple(matrix.shape) == shape, f"{name} must be packed, of x's type, {shape}")
     lib = library()
     out = torch.empty((top, n, width), dtype=torch.float32, device=x.device)
     entries = n * top
-    hidden = torch.empty((entries, units), dtype=torch.bfloat16, device=x.device)
+    hidden = torch.empty((entries, units), dtype=x.dtype, device=x.device)
     unit = (float("inf") if limit is None else float(limit), float(alpha), float(shift), int(bool(weigh_input)))
-    if n <= int(lib.mllm_experts_few_rows()):
-        check(lib.mllm_experts_few_up(_ptr(x), _ptr(up.data), _ptr(hidden), _ptr(picks.experts), _ptr(picks.weights), n, top, int(n_experts), int(units), width, *unit, _stream()))
-        check(lib.mllm_experts_few_down(_ptr(hidden), _ptr(down.data), _ptr(out), _ptr(picks.experts), n, top, int(n_experts), int(units), width, _stream()))
+    if n <= int(lib.mllm_experts_few_rows(width, code)):
+        check(lib.mllm_experts_few_up(_ptr(x), _ptr(up.data), _ptr(hidden), _ptr(picks.experts), _ptr(picks.weights), n, top, int(n_experts), int(units), width, *unit, code,
+                                      _stream()))
+        check(lib.mllm_experts_few_down(_ptr(hidden), _ptr(down.data), _ptr(out), _ptr(picks.experts), n, top, int(n_experts), int(units), width, code, _stream()))
         return out
     tile = int(lib.mllm_expert_tile_rows())
     max_tiles = entries // tile + min(n_experts, entries)
@@ -1433,8 +1439,9 @@ def grouped_experts(x, picks: Picks, up: PackedMatrix, down: PackedMatrix, n_exp
     weights, n_tiles = lists[4 * max_tiles + 2 * entries : 4 * max_tiles + 3 * entries], lists[4 * max_tiles + 3 * entries :]
     check(lib.mllm_expert_lists(_ptr(picks.experts), _ptr(picks.weights), n, top, int(n_experts), tile, _ptr(rows), _ptr(places), _ptr(weights), _ptr(tiles), _ptr(n_tiles),
                                 _stream()))
-    check(lib.mllm_experts_up(_ptr(x), _ptr(up.data), _ptr(hidden), _ptr(tiles), _ptr(n_tiles), _ptr(rows), _ptr(weights), entries, max_tiles, int(units), width, *unit, _stream()))
-    check(lib.mllm_experts_down(_ptr(hidden), _ptr(down.data), _ptr(out), _ptr(tiles), _ptr(n_tiles), _ptr(places), entries, max_tiles, int(units), width, _stream()))
+    check(lib.mllm_experts_up(_ptr(x), _ptr(up.data), _ptr(hidden), _ptr(tiles), _ptr(n_tiles), _ptr(rows), _ptr(weights), entries, max_tiles, int(units), width, *unit, code,
+                              _stream()))
+    check(lib.mllm_experts_down(_ptr(hidden), _ptr(down.data), _ptr(out), _ptr(tiles), _ptr(n_tiles), _ptr(places), entries, max_tiles, int(units), width, code, _stream()))
     return out
 
 
@@ -1461,23 +1468,6 @@ def expert_unit(up, weights, n_routed: int, ff: int, shared: int = 0, *, h=None,
     check(library().mllm_expert_unit(_ptr(up), _ptr(out), _ptr(weights), weights.stride(0), n, int(n_routed), int(ff), int(shared), _ptr(h if n_identity else None),
                                      _ptr(carried), int(n_identity), int(width), _code(up.dtype), _stream()))
     return out, carried
-
-
-def gated_expert_unit(both, weights, n_experts: int, ff: int, *, limit: float | None = None, alpha: float = 1.0, shift: float = 0.0, weigh_input: bool = False):
-    """``expert_unit`` for experts with a gate unit (``gate_unit``): ``both`` [rows, n_experts * 2 * ff], per expert the sums of its gate and
-    of its up matrix -> [rows, n_experts * ff], the unit times the row's weight for the expert, or with ``weigh_input`` the unit of the
-    sums times that weight (the experts of weight * h instead of weight * the experts of h). Experts of weight zero give zeros."""
-    _device_tensor(both, "both", dim=2)
-    n = both.shape[0]
-    _require(both.shape[1] == 2 * n_experts * ff, "the hidden units do not match the experts")
-    _require(limit is None or limit > 0, "the limit must be positive")
-    _require(isinstance(weights, torch.Tensor) and weights.is_cuda and weights.dim() == 2 and weights.dtype == torch.float32 and weights.stride(1) == 1
-             and weights.shape[0] == n and weights.shape[1] >= n_experts, "the weights must be float32 GPU rows, one column an expert")
-    out = torch.empty((n, n_experts * ff), dtype=both.dtype, device=both.device)
-    check(library().mllm_gated_expert_unit(_ptr(both), _ptr(out), _ptr(weights), weights.stride(0), n, int(n_experts), int(ff),
-                                           float("inf") if limit is None else float(limit), float(alpha), float(shift), int(bool(weigh_input)), _code(both.dtype),
-                                           _stream()))
-    return out
 
 
 def gated_scan(rows, z_at: int, x_at: int, g_at: int, width: int, state, q_starts, state_slots, out_dtype, *, shift: float, max_q_len: int | None = None):

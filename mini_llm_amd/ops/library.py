@@ -58,15 +58,13 @@ _SIGNATURES = {
     "mllm_route_rows_supported": [c_int, c_int, c_int],
     "mllm_route_rows": [P, P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, P],
     "mllm_expert_tile_rows": [],
-    "mllm_experts_few_rows": [],
-    "mllm_experts_supported": [c_int, c_int, c_int],
+    "mllm_experts_few_rows": [c_int, c_int],
     "mllm_expert_lists": [P, P, c_int, c_int, c_int, c_int, P, P, P, P, P, P],
-    "mllm_experts_up": [P, P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, P],
-    "mllm_experts_down": [P, P, P, P, P, P, c_int, c_int, c_int, c_int, P],
-    "mllm_experts_few_up": [P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, P],
-    "mllm_experts_few_down": [P, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
+    "mllm_experts_up": [P, P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_int, P],
+    "mllm_experts_down": [P, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
+    "mllm_experts_few_up": [P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_int, P],
+    "mllm_experts_few_down": [P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_int, P, P, c_int, c_int, c_int, P],
-    "mllm_gated_expert_unit": [P, P, P, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_int, c_int, P],
     "mllm_gated_scan": [P, c_int, c_int, c_int, c_int, P, c_longlong, P, P, P, c_int, c_int, c_int, c_int, c_float, c_int, P, c_longlong, c_int, P],
     "mllm_gated_scan_chunk_rows": [],
     "mllm_gate_unit": [P, P, c_int, c_int, c_float, c_float, c_float, c_int, P],

@@ -14,15 +14,15 @@ Other designs' forms: ``score`` "sigmoid" takes s = sigmoid(z), each expert's ow
 relu; ``weigh`` "input" multiplies an expert's input by its weight instead of its output (the same thing only for linear experts): the
 gate unit then takes the weight times the sums.
 
-All experts run as ONE up product over their matrices laid behind each other (the shared expert's last) and ONE down product over their
+Experts of the plain form: all run as ONE up product over their matrices laid behind each other (the shared expert's last) and ONE down product over their
 down matrices laid side by side: ``kernels.expert_unit`` between the two multiplies every hidden unit by its expert's weight for the
 row, zero where the router did not pick it, so the down product's sum is the weighted sum over the picked experts; the share of the
 experts that hand h on rides in as that product's residual operand. A row's result is a function of the row alone, nothing is planned
 on the host, and a captured step replays it. The price is the arithmetic of the experts that were not picked: E / top times the needed
 work in the two products, which few rows (decoding) do not notice, since they read every expert's matrices anyway.
 
-Experts with a gate unit run grouped instead where the kernels take the sizes (bfloat16, a width that is a multiple of 64): each expert for
-the rows that picked it alone (``kernels.grouped_experts``), planned on the device."""
+Experts with a gate unit run grouped instead: each expert for the rows that picked it alone (``kernels.grouped_experts``), planned on the
+device."""
 
 from __future__ import annotations
 
@@ -59,7 +59,7 @@ class RoutedExperts(FeedForward):
         self.score, self.renormalise, self.weigh_input = score, bool(renormalise), weigh == "input"
         self.gated, self.limit, self.alpha, self.shift = unit == "clamped_gate", limit, float(alpha), float(shift)
         self.router = self.correction = self.up = self.down = self._router_rows = self._small_router = None
-        self.grouped, self.units = False, ff
+        self.units = ff
         self.shared_units = 0   # the shared expert's hidden units and the zeros that fill the up matrix to whole blocks
         self._down_product = BranchProduct()
         self.sums_later = False   # True: a call without a residual may return kernels.BranchRows (the block that adds the branch takes its sums)
@@ -103,37 +103,30 @@ class RoutedExperts(FeedForward):
         self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
 
     def _bind_gated(self, tensors, names):
-        """Grouped (the experts run for the rows that picked them: ``kernels.grouped_experts``) where the sizes allow, else all experts as one
-        up and one down product with zeros for the units that were not picked."""
+        """The layout ``kernels.grouped_experts`` reads: 32 gate rows and 32 up rows in turn, units and the down matrices' rows filled up with zeros."""
         sample = tensors[names[0] + "up"]
-        self.units = -(-self.ff // 64) * 64
-        self.grouped = sample.is_cuda and kernels.grouped_experts_supported(self.width, self.units, sample.dtype)
-        if not self.grouped:
-            up = torch.cat([tensors[name + part] for name in names for part in ("gate", "up")], dim=0).contiguous()
-            down = torch.cat([tensors[name + "down"] for name in names], dim=1).contiguous()
-            self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
-            return
-        E, units, width = self.n_experts, self.units, self.width
-        up = torch.zeros((E, units // 32, 2, 32, width), dtype=sample.dtype, device=sample.device)   # 32 gate rows and 32 up rows in turn
-        down = torch.zeros((E, width, units), dtype=sample.dtype, device=sample.device)
+        E, width, rows = self.n_experts, self.width, kernels.expert_down_rows(self.width)
+        units = self.units = -(-self.ff // kernels.EXPERT_UNITS) * kernels.EXPERT_UNITS
+        up = torch.zeros((E, units // 32, 2, 32, width), dtype=sample.dtype, device=sample.device)
+        down = torch.zeros((E, rows, units), dtype=sample.dtype, device=sample.device)
         for e, name in enumerate(names):
             for half, part in enumerate(("gate", "up")):
                 padded = torch.zeros((units, width), dtype=sample.dtype, device=sample.device)
                 padded[: self.ff] = tensors[name + part]
                 up[e, :, half] = padded.view(units // 32, 32, width)
-            down[e, :, : self.ff] = tensors[name + "down"]
-        self.up, self.down = kernels.pack_matrix(up.view(E * 2 * units, width)), kernels.pack_matrix(down.view(E * width, units))
+            down[e, :width, : self.ff] = tensors[name + "down"]
+        up, down = up.view(E * 2 * units, width), down.view(E * rows, units)
+        self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
 
     def _forward_gated(self, x, carried, residual):
-        unit = dict(limit=self.limit, alpha=self.alpha, shift=self.shift, weigh_input=self.weigh_input)
-        if not self.grouped:
-            units = kernels.gated_expert_unit(kernels.linear(x, self.up), self._route(x, carried), self.n_experts, self.ff, **unit)
-            if residual is None and self.sums_later:
-                return self._down_product.later(units, self.down)
-            return self._down_product(units, self.down, residual)
-        planes = kernels.grouped_experts(x, self._route(x, carried, picks=True), self.up, self.down, self.n_experts, self.units, **unit)
+        planes = kernels.grouped_experts(x, self._route(x, carried, picks=True), self.up, self.down, self.n_experts, self.units, limit=self.limit, alpha=self.alpha,
+                                         shift=self.shift, weigh_input=self.weigh_input)
         if residual is not None:
-            return kernels.settle(kernels.PendingRows(residual, planes, None))
+            if self.width % 4 == 0:
+                return kernels.settle(kernels.PendingRows(residual, planes, None))
+            for plane in planes:   # rows that are no whole pieces of 16 bytes: plane by plane
+                residual = kernels.add(residual, plane)
+            return residual
         if self.sums_later:
             return kernels.BranchRows(planes, None)
         return planes[0] if self.top == 1 else planes   # several picks: partial sums, as a product cut along K leaves them

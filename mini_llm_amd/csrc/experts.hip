@@ -4,8 +4,8 @@
 // A router leaves picks [rows, top] (expert ids, -1 for none) and their weights. Entry p = row * top + k is row `row` with its k-th
 // pick. An expert's matrices: the gate and up rows of the up matrix in turns of 32, [2 * units, width], and the down matrix [width,
 // units], both packed, one expert behind the other; units a multiple of 64 (zero rows and columns fill it up), the down matrix's rows
-// whole sixteens. The down product of a
-// row's k-th pick goes to plane k of out [top, rows, width]: whoever reads the branch adds the planes up, in that order.
+// whole sixteens. The down product of a row's k-th pick goes to plane k of out [top, rows, width]: whoever reads the branch adds the
+// planes up, in that order.
 #include "common.h"
 #include "gate_unit.h"
 

@@ -31,7 +31,7 @@ class RotaryEncoding(PositionEncoding):
     """Rotation of the first ``dims`` elements of a head by an angle that grows with the position: pair i turns by p * f_i with
     f_i = base^(-2i / dims). ``pairing`` says which elements make pair i: "half" pairs element i with element i + dims / 2,
     "neighbours" pairs element 2i with element 2i + 1, (u, v) -> (u cos a - v sin a, v cos a + u sin a). It has no tensors; the
-    mixer that holds it applies it to its queries and keys (``stage`` "mixer") with ``frequencies`` and ``magnitude``.
+    mixer that holds it applies it to its queries and keys (``stage`` "mixer") with ``frequencies64`` and ``magnitude``.
 
     ``scaling`` stretches the slow pairs for sequences longer than ``original`` positions, in one of two ways (``kind``):
 
@@ -83,22 +83,14 @@ class RotaryEncoding(PositionEncoding):
                     values[i] = (1.0 - s) * f / factor + s * f
         elif self.scaling:
             raise ValueError(f"unknown kind of scaling {kind!r}: yarn or wavelength")
-        self.values = values   # float64 on the host; ``frequencies`` rounds them to 32-bit on the device, ``frequencies64`` does not
+        self.values = values   # float64 on the host
         self._on_device = {}
 
-    def frequencies(self, device):
+    def frequencies64(self, device):
+        """The pairs' frequencies on the device, in 64-bit, as the kernels take their angles."""
         import torch
 
         key = str(device)
-        if key not in self._on_device:
-            self._on_device[key] = torch.tensor(self.values or [0.0], dtype=torch.float64).to(torch.float32).to(device)
-        return self._on_device[key]
-
-    def frequencies64(self, device):
-        """The same numbers unrounded, for a kernel that takes its angles in 64-bit."""
-        import torch
-
-        key = (str(device), 64)
         if key not in self._on_device:
             self._on_device[key] = torch.tensor(self.values or [0.0], dtype=torch.float64).to(device)
         return self._on_device[key]

@@ -162,18 +162,19 @@ class CacheManager:
         entry.reserved = max(entry.reserved, n_new)
 
     def commit(self, request_id, n_new: int) -> None:
-        """The step has stored ``n_new`` tokens: the length grows, and pages that a window has
-        passed (no later query can read them) go back to their pool."""
+        """The step has stored ``n_new`` tokens: the length grows, and pages that a window or the
+        end of a chunk has passed (no later query can read them) go back to their pool."""
         entry = self._entry(request_id)
         if n_new > entry.reserved:
             raise CacheError(f"request {request_id!r} commits {n_new} tokens but reserved {entry.reserved}")
         entry.length += n_new
         entry.reserved = 0
         for group, pool, table in zip(self.groups, self.pools, entry.tables):
-            if group.window is None:
+            if group.window is None and group.chunk is None:
                 continue
-            keep_from = first_needed_block(entry.length, group.window, self.page_size)
-            passed = [b for b in range(min(keep_from, len(table))) if table[b] != NO_PAGE]
+            keep_from = first_needed_block(entry.length, group.window, self.page_size, group.chunk)
+            kept_first = blocks_for(group.keep_first, self.page_size)
+            passed = [b for b in range(kept_first, min(keep_from, len(table))) if table[b] != NO_PAGE]
             pool.give([table[b] for b in passed])
             for b in passed:
                 table[b] = NO_PAGE
@@ -249,6 +250,6 @@ class CacheManager:
             for group, table in zip(self.groups, entry.tables):
                 if len(table) < blocks_for(entry.length, self.page_size):
                     raise AssertionError(f"request {entry.request_id!r}: table shorter than its length")
-                first = first_needed_block(entry.length, group.window, self.page_size)
-                if any(p == NO_PAGE for p in table[first:]):
+                first = first_needed_block(entry.length, group.window, self.page_size, group.chunk)
+                if any(p == NO_PAGE for p in table[first:] + table[: blocks_for(group.keep_first, self.page_size)]):
                     raise AssertionError(f"request {entry.request_id!r}: a page inside the window is missing")

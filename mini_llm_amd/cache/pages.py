@@ -46,8 +46,10 @@ def blocks_for(length: int, page_size: int) -> int:
     return (length + page_size - 1) // page_size
 
 
-def first_needed_block(next_position: int, window: int | None, page_size: int) -> int:
-    """The first block a query at ``next_position`` (or any later one) can still read."""
+def first_needed_block(next_position: int, window: int | None, page_size: int, chunk: int | None = None) -> int:
+    """The first block a query at ``next_position`` (or any later one) can still read (blocks that hold kept first keys aside)."""
+    if chunk is not None:
+        return next_position // chunk * chunk // page_size
     if window is None:
         return 0
     return max(0, next_position - window + 1) // page_size

@@ -1,5 +1,6 @@
 from .base import ConfigError, ModelConfig, read_config_json
 from .dizizen import DizizenConfig
+from .gevulorn import GevulornConfig
 from .gimozen import GimozenConfig
 from .goletar import GoletarConfig
 from .gpt2 import GPT2Config
@@ -19,6 +20,7 @@ __all__ = [
     "Architecture",
     "ConfigError",
     "DizizenConfig",
+    "GevulornConfig",
     "GimozenConfig",
     "GoletarConfig",
     "GPT2Config",

@@ -3,7 +3,7 @@
 // Pages of one cache layer: [num_pages, n_kv_heads, page_size, head_size], so the rows of one
 // head inside a page lie together. A request's block table names its pages in order. A token at
 // position p attends to the cached keys max(0, p - window + 1) .. p of its request (window 0 =
-// all; or, with chunks, to the keys of its own chunk up to p), which after cache_write include the tokens of its own step: decoding and prompt
+// all; with kept first keys also to those, however far back; or, with chunks, to the keys of its own chunk up to p), which after cache_write include the tokens of its own step: decoding and prompt
 // portions are the same kernel.
 #include "common.h"
 #include "key_sweep.h"
@@ -39,12 +39,15 @@ constexpr int MAX_HEAD = 256;
 // behind the scale. sinks [n_heads]: exp(sink_h) joins the softmax's denominator of head h, once, with no key and no value.
 // chunk > 0: the sequence is cut into chunks of so many positions, counted from position 0, and a query sees only the keys of its own
 // chunk (up to itself): its first key is the chunk's start instead of a window's.
+// keep > 0 (with a window): the first so many keys of a sequence stay visible to every query behind them, with whatever lies between
+// them and the window passed over (the pages of that gap may have been given back).
 // wide_out: the results leave as 32-bit floats whatever the pages' type (`out` is then a float array and `out_stride` counts floats):
 // for a mixer that goes on computing with them before anything is rounded.
 struct ScoreOptions {
     float softcap;
     const float* sinks;
     int chunk;
+    int keep;
     int wide_out;
 };
 
@@ -91,6 +94,7 @@ __global__ __launch_bounds__(256) void attention_general_kernel(
     const int kv_head = head / (n_heads / n_kv_heads);
     const int position = positions[token];
     const int first_key = first_visible_key(position, window, options.chunk);
+    const int keep = min(options.keep, first_key);   // keys 0 .. keep - 1 count beside first_key .. position
     const int* table = block_tables + (size_t)request * max_blocks;
 
     float* my_q = q_shared[wave];
@@ -105,9 +109,10 @@ __global__ __launch_bounds__(256) void attention_general_kernel(
     for (int r = 0; r < REGS; r++) o[r] = 0.0f;
     float running_max = -INFINITY, running_sum = 0.0f;
 
-    for (int tile = (first_key / WAVE) * WAVE; tile <= position; tile += WAVE) {
+    const int first_tile = (first_key / WAVE) * WAVE;
+    for (int tile = keep > 0 ? 0 : first_tile; tile <= position;) {
         int key = tile + lane;
-        bool valid = key >= first_key && key <= position;
+        bool valid = key <= position && (key >= first_key || key < keep);
         int row = 0;
         float score = -INFINITY;
         if (valid) {
@@ -125,8 +130,10 @@ __global__ __launch_bounds__(256) void attention_general_kernel(
         running_max = new_max;
 #pragma unroll
         for (int r = 0; r < REGS; r++) o[r] *= rescale;
-        int first = max(first_key - tile, 0), last = min(WAVE - 1, position - tile);
-        for (int j = first; j <= last; j++) {
+        unsigned long long seen = __ballot(valid);
+        while (seen) {
+            const int j = __builtin_ctzll(seen);
+            seen &= seen - 1;
             float pj = __shfl(p, j, WAVE);
             int row_j = __shfl(row, j, WAVE);
             const T* v_row = v_pages + (size_t)row_j * head_size;
@@ -136,6 +143,8 @@ __global__ __launch_bounds__(256) void attention_general_kernel(
                 if (d < head_size) o[r] += pj * to_float(v_row[d]);
             }
         }
+        tile += WAVE;
+        if (tile >= keep && tile < first_tile) tile = first_tile;   // over the gap
     }
     if (options.sinks) running_sum += expf(options.sinks[head] - running_max);
     float inverse = 1.0f / running_sum;
@@ -175,14 +184,15 @@ MLLM_API int mllm_attention(const void* q, int q_stride, const void* k_pages, co
                             void* out, int out_stride, const int* token_request,
                             const int* positions, const int* block_tables, int max_blocks,
                             int n_tokens, int n_heads, int n_kv_heads, int head_size, int page_size,
-                            int window, float scale, int dtype, float softcap, const float* sinks, int chunk, int wide_out, hipStream_t stream) {
+                            int window, float scale, int dtype, float softcap, const float* sinks, int chunk, int keep, int wide_out, hipStream_t stream) {
     MLLM_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && max_blocks > 0, "attention: bad sizes");
-    const ScoreOptions options = {softcap, sinks, chunk, wide_out};
+    const ScoreOptions options = {softcap, sinks, chunk, keep, wide_out};
     MLLM_REQUIRE(n_heads % n_kv_heads == 0, "attention: %d heads do not divide into %d key/value heads",
                  n_heads, n_kv_heads);
     MLLM_REQUIRE(head_size > 0 && head_size <= MAX_HEAD,
                  "attention: head size %d is not in 1..%d", head_size, MAX_HEAD);
     MLLM_REQUIRE(page_size > 0 && window >= 0 && chunk >= 0, "attention: bad page size, window or chunk");
+    MLLM_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "attention: first keys are kept beside a window");
     MLLM_REQUIRE(q_stride >= n_heads * head_size && out_stride >= n_heads * head_size,
                  "attention: rows are too short for the heads");
     if (n_tokens == 0) return 0;
@@ -219,13 +229,14 @@ constexpr int DECODE_MAX_SPLITS = 16;
 
 // A block per (token, head); its waves (blockDim.x / 64 of them, a power of two up to 16) split
 // the token's keys evenly among themselves, and their partial results meet in LDS.
-// TOGETHER: how a wave starts (see there); the host chooses.
+// TOGETHER: how a wave starts (see there); the host chooses. KEPT: a window with kept first keys (ScoreOptions): the keys are counted
+// without the gap between the two, and the sweep adds it where it looks a key up.
 // parts (gridDim.z) > 1: few tokens with many keys, where a block per (token, head) would leave most of the chip idle.
 // The token's keys are cut into so many runs, a block each. A block leaves its unnormalised sums with their maximum and
 // weight in `parts_out` ([token, head, part, HD + 2] floats) and counts itself in arrivals[token, head] (zero before the
 // launch); the block that is through last puts the runs together, out = sum_p o_p e^(m_p - M) / sum_p l_p e^(m_p - M),
 // and the count is zero again behind it (it wraps), so the same counters serve the next launch.
-template <typename T, int HD, bool TOGETHER>
+template <typename T, int HD, bool TOGETHER, bool KEPT = false>
 __global__ __launch_bounds__(1024) void attention_decode_kernel(
     const T* __restrict__ q, int q_stride, const T* __restrict__ k_pages,
     const T* __restrict__ v_pages, T* __restrict__ out, int out_stride,
@@ -255,6 +266,13 @@ __global__ __launch_bounds__(1024) void attention_decode_kernel(
     constexpr int KPI = KeySweep<T, HD>::KPI;
     int first_key = first_visible_key(position, window, options.chunk);
     int last_key = position + 1;  // exclusive
+    int kept = 0, gap = 0;
+    if constexpr (KEPT) {   // from here on key numbers leave the gap out: 0 .. kept - 1, then the window's
+        kept = min(options.keep, first_key);
+        gap = first_key - kept;
+        first_key = 0;
+        last_key -= gap;
+    }
     if (n_parts > 1) {  // this block's run of the keys, in whole rounds of the sweep
         const int run = (((last_key - first_key + n_parts - 1) / n_parts + KPI - 1) / KPI) * KPI;
         first_key = min(first_key + part * run, last_key);
@@ -270,9 +288,10 @@ __global__ __launch_bounds__(1024) void attention_decode_kernel(
     const int kv_head = head / (n_heads / n_kv_heads);
     const int* table = block_tables + (size_t)request * max_blocks;
 
-    KeySweep<T, HD> sweep;
+    KeySweep<T, HD, KEPT> sweep;
     sweep.init();
     sweep.cap = options.softcap;
+    if constexpr (KEPT) sweep.gap_from = kept, sweep.gap = gap;
     if (begin < end && !TOGETHER) {
         // the plain order: the query, then round by round the pages, their rows, the softmax
         float qf[VEC];
@@ -293,7 +312,7 @@ __global__ __launch_bounds__(1024) void attention_decode_kernel(
         const typename Chunk<T>::Raw raw = *reinterpret_cast<const typename Chunk<T>::Raw*>(q + (size_t)token * q_stride + head * HD + sub * VEC);
         int page[UNROLL];
         sweep.look_up(page, table, page_shift, begin, end, spare_key, lane);
-        typename KeySweep<T, HD>::Fetched f;
+        typename KeySweep<T, HD, KEPT>::Fetched f;
         sweep.fetch_rows(f, page, k_pages, v_pages, kv_head, n_kv_heads, page_shift, begin, end, spare_key, lane);
         float qf[VEC];
 #pragma unroll
@@ -394,13 +413,17 @@ int dispatch_decode(int head_size, const void* q, int q_stride, const void* k_pa
     // order is 5 % faster.
     const int reach = max_blocks << page_shift;
     const int keys_per_round = (sizeof(T) == 2 ? 4096 : 2048) / head_size;  // KeySweep's KPI
-    const int seen = options.chunk > 0 ? options.chunk : window;   // the most keys a token sees, if a mask bounds them
+    const int seen = options.chunk > 0 ? options.chunk : (window > 0 ? window + options.keep : 0);   // the most keys a token sees, if a mask bounds them
     const int rounds = ceil_div(ceil_div(seen > 0 && seen < reach ? seen : reach, n_splits * n_parts), keys_per_round);
     const bool together = sizeof(T) == 2 || rounds <= 12;
 #define MLLM_DECODE_CASE(HD)                                                                                   \
     case HD:                                                                                                   \
         mllm_count_kernel(MLLM_K_ATTENTION_DECODE);                                                            \
-        if (together)                                                                                          \
+        if (options.keep > 0)                                                                                  \
+            attention_decode_kernel<T, HD, true, true><<<grid, block, 0, stream>>>(                            \
+                (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, (T*)out, out_stride, token_request,   \
+                positions, block_tables, max_blocks, n_heads, n_kv_heads, page_shift, window, scale, out_packed, parts, arrivals, options);  \
+        else if (together)                                                                                     \
             attention_decode_kernel<T, HD, true><<<grid, block, 0, stream>>>(                                  \
                 (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, (T*)out, out_stride, token_request,   \
                 positions, block_tables, max_blocks, n_heads, n_kv_heads, page_shift, window, scale, out_packed, parts, arrivals, options);  \
@@ -434,14 +457,15 @@ MLLM_API int mllm_attention_decode(const void* q, int q_stride, const void* k_pa
                                    const int* block_tables, int max_blocks, int n_tokens, int n_heads,
                                    int n_kv_heads, int head_size, int page_size, int window, float scale,
                                    int n_splits, int dtype, int out_packed, int n_parts, float* parts, int* arrivals,
-                                   float softcap, const float* sinks, int chunk, int wide_out, hipStream_t stream) {
-    const ScoreOptions options = {softcap, sinks, chunk, wide_out};
+                                   float softcap, const float* sinks, int chunk, int keep, int wide_out, hipStream_t stream) {
+    const ScoreOptions options = {softcap, sinks, chunk, keep, wide_out};
     MLLM_REQUIRE(!(wide_out && out_packed), "attention_decode: rows in the packed layout leave in the pages' type");
     MLLM_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && max_blocks > 0, "attention_decode: bad sizes");
     MLLM_REQUIRE(n_heads % n_kv_heads == 0, "attention_decode: %d heads do not divide into %d key/value heads", n_heads, n_kv_heads);
     MLLM_REQUIRE(mllm_attention_decode_supported(head_size, page_size, dtype),
                  "attention_decode: head size %d is not one of 16, 32, 64, 128, 256, or page size %d is no power of two", head_size, page_size);
     MLLM_REQUIRE(window >= 0 && chunk >= 0, "attention_decode: bad window or chunk");
+    MLLM_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "attention_decode: first keys are kept beside a window");
     MLLM_REQUIRE(n_splits >= 1 && n_splits <= DECODE_MAX_SPLITS && (n_splits & (n_splits - 1)) == 0,
                  "attention_decode: %d splits is not a power of two in 1..%d", n_splits, DECODE_MAX_SPLITS);
     MLLM_REQUIRE(q_stride >= n_heads * head_size && out_stride >= n_heads * head_size, "attention_decode: rows are too short for the heads");
@@ -569,8 +593,9 @@ __global__ __launch_bounds__(64 * QG * KS) void attention_prefill_kernel(
     const int block_last_position = context + min(tile_q0 + 32 * QG, q_len) - 1;
     const int block_first_key = first_visible_key(context + tile_q0, window, options.chunk);
     const bool masked_from = window > 0 || options.chunk > 0;   // the queries' first keys are not key 0
+    const int keep = options.keep;
     // the pages this block walks, copied to LDS once: a tile's loads then do not wait for a lookup in memory
-    const int first_page = block_first_key >> page_shift, last_page = block_last_position >> page_shift;
+    const int first_page = keep > 0 ? 0 : block_first_key >> page_shift, last_page = block_last_position >> page_shift;
     const bool table_in_lds = last_page - first_page < PF_TABLE;
     if (table_in_lds)
         for (int i = tid; i <= last_page - first_page; i += THREADS) table_lds[i] = table[first_page + i];
@@ -596,8 +621,8 @@ __global__ __launch_bounds__(64 * QG * KS) void attention_prefill_kernel(
                 int key = k_base + row + e;
                 // pages before a window may be gone, keys beyond the last query are not stored yet:
                 // the load goes to a clamped key and column, the result is zeroed afterwards
-                bool valid = key >= block_first_key && key <= block_last_position && c * VEC < head_size;
-                int safe_key = min(max(key, block_first_key), block_last_position);
+                bool valid = (key >= block_first_key || key < keep) && key <= block_last_position && c * VEC < head_size;
+                int safe_key = min(key < keep ? key : max(key, block_first_key), block_last_position);
                 int page = table_in_lds ? table_lds[(safe_key >> page_shift) - first_page] : table[safe_key >> page_shift];
                 size_t at = ((((size_t)page * n_kv_heads + kv_head) << page_shift) + (safe_key & page_mask)) * head_size + min(c * VEC, head_size - VEC);
                 k_regs[i][e] = *reinterpret_cast<const Vec16*>(k_pages + at);
@@ -643,16 +668,22 @@ __global__ __launch_bounds__(64 * QG * KS) void attention_prefill_kernel(
     const T* const k_tile = k_tiles + key_split * L::K_ELEMS;
     const T* const v_tile = v_tiles + key_split * L::V_ELEMS;
     const int first_base = (block_first_key / PF_KEYS) * PF_KEYS;
-    fetch(first_base);
-    for (int k_base = first_base; k_base <= block_last_position; k_base += SPAN) {
+    // the next keys: with kept first keys, those that lie between them and the window of the block's first query are passed over
+    auto next_base = [&](int base) {
+        const int next = base + SPAN;
+        return next >= keep && next < first_base ? first_base : next;
+    };
+    const int start_base = keep > 0 ? 0 : first_base;
+    fetch(start_base);
+    for (int k_base = start_base; k_base <= block_last_position; k_base = next_base(k_base)) {
         __syncthreads();  // the previous tiles have been consumed
         stage();
         __syncthreads();
-        fetch(k_base + SPAN);  // unconditional: beyond the last key it reads a clamped address and is masked away
+        fetch(next_base(k_base));  // unconditional: beyond the last key it reads a clamped address and is masked away
         const int k0 = k_base + key_split * PF_KEYS;
         // a wave whose queries all lie before its tile, or whose windows have all passed it, has nothing to add
         if (!wave_active || k0 > wave_last_position) continue;
-        if (masked_from && k0 + PF_KEYS - 1 < first_visible_key(wave_first_position, window, options.chunk)) continue;
+        if (masked_from && k0 >= keep && k0 + PF_KEYS - 1 < first_visible_key(wave_first_position, window, options.chunk)) continue;
 
         // ---- S^T = K . Q^T : two 32-key tiles ----
         f32x16 s_acc[2];
@@ -694,7 +725,7 @@ __global__ __launch_bounds__(64 * QG * KS) void attention_prefill_kernel(
 #pragma unroll
                 for (int v = 0; v < 16; v++) {
                     int key = k0 + j * 32 + 8 * (v / 4) + 4 * half + (v % 4);
-                    bool allowed = q_valid && key <= q_position && key >= first_allowed;
+                    bool allowed = q_valid && key <= q_position && (key >= first_allowed || key < keep);
                     float s = options.softcap > 0.0f ? capped_score<!HALF>(s_acc[j][v] * scale, options.softcap) * (HALF ? LOG2E : 1.0f) : s_acc[j][v] * score_scale;
                     s = allowed ? s : -INFINITY;
                     s_acc[j][v] = s;
@@ -851,8 +882,8 @@ MLLM_API int mllm_attention_prefill(const void* q, int q_stride, const void* k_p
                                     int out_stride, const int* q_starts, const int* context_lens,
                                     const int* block_tables, int max_blocks, int n_requests, int max_q_len,
                                     int max_len, int n_heads, int n_kv_heads, int head_size, int page_size, int window,
-                                    float scale, int dtype, float softcap, const float* sinks, int chunk, int wide_out, hipStream_t stream) {
-    const ScoreOptions options = {softcap, sinks, chunk, wide_out};
+                                    float scale, int dtype, float softcap, const float* sinks, int chunk, int keep, int wide_out, hipStream_t stream) {
+    const ScoreOptions options = {softcap, sinks, chunk, keep, wide_out};
     // max_len: the longest sequence after this step, or a bound on it (0 or less: what the block tables can hold); it only
     // decides how many waves share a block's keys
     MLLM_REQUIRE(n_requests >= 0 && max_q_len >= 0 && n_heads > 0 && n_kv_heads > 0 && max_blocks > 0, "attention_prefill: bad sizes");
@@ -860,6 +891,7 @@ MLLM_API int mllm_attention_prefill(const void* q, int q_stride, const void* k_p
     MLLM_REQUIRE(mllm_attention_prefill_supported(head_size, page_size),
                  "attention_prefill: head size %d is not a multiple of 16 in 16..128, or page size %d is no power of two", head_size, page_size);
     MLLM_REQUIRE(window >= 0 && chunk >= 0, "attention_prefill: bad window or chunk");
+    MLLM_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "attention_prefill: first keys are kept beside a window");
     MLLM_REQUIRE(q_stride >= n_heads * head_size && out_stride >= n_heads * head_size, "attention_prefill: rows are too short for the heads");
     MLLM_REQUIRE(n_requests <= 65535 && n_heads <= 65535, "attention_prefill: too many requests or heads for one launch");
     if (n_requests == 0 || max_q_len == 0) return 0;

@@ -207,14 +207,19 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
     const int block_last_position = context + min(tile_q0 + QUERIES, q_len) - 1;
     const int block_first_key = first_visible_key(context + tile_q0, window, options.chunk);
     const int first_base = (block_first_key / KEYS) * KEYS;
-    const int n_tiles = (block_last_position - first_base) / KEYS + 1;
+    // with kept first keys: the tiles that hold them come first, the tiles between them and the window are passed over
+    const int kept_tiles = min((options.keep + KEYS - 1) / KEYS, first_base / KEYS);
+    const int n_tiles = kept_tiles + (block_last_position - first_base) / KEYS + 1;
     const int n_mine = n_tiles > wave ? (n_tiles - wave + SPLITS - 1) / SPLITS : 0;  // tiles wave, wave + SPLITS, ...
 
     // One half (keys or values) of this wave's i-th tile, into place i % 2. A lane asks for piece (slot ^ turn) of its
     // row, and the load puts it in the row's slot. Beyond the wave's last tile the last one is asked for again (never
     // used), so that the count of loads in flight is the same in every step.
     unsigned char* const wave_lds = lds + wave * L::WAVE_BYTES;
-    auto tile_base = [&](int i) { return first_base + (wave + SPLITS * min(i, n_mine - 1)) * KEYS; };
+    auto tile_base = [&](int i) {
+        const int tile = wave + SPLITS * min(i, n_mine - 1);
+        return tile < kept_tiles ? tile * KEYS : first_base + (tile - kept_tiles) * KEYS;
+    };
     // a lane's place among the rows of a whole tile, in bytes: the same for every tile, so an address is a base all lanes
     // share plus this (worked out anew for every load it was a sixth of the loop's vector instructions)
     unsigned k_lane[L::LOADS], v_lane[L::LOADS];
@@ -317,7 +322,7 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
 
     auto tile = [&](int i, f32x16 (&s_acc)[QSUB], f32x16 (&s_next)[QSUB]) {
         const int page_next = table[tile_base(i + 4) >> page_shift];
-        const int k0 = first_base + (wave + SPLITS * i) * KEYS;
+        const int k0 = tile_base(i);
         const unsigned char* v_tile = wave_lds + 2 * L::TILE_BYTES + (i % 2) * L::TILE_BYTES;
         const unsigned char* k_next = wave_lds + ((i + 1) % 2) * L::TILE_BYTES;
         bf16x8 p[QSUB][2];  // the probabilities of a sub-tile of queries, as the second product's operand: keys 0-15 and 16-31 of the tile
@@ -347,12 +352,22 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
             } else {
                 const int first_allowed = q_position[qs] < 0 ? 0 : first_visible_key(q_position[qs], window, options.chunk);
                 const int key0 = k0 + 4 * half;
+                if (k0 < options.keep) {   // a tile that holds kept keys (the same for all lanes)
 #pragma unroll
-                for (int v = 0; v < 16; v++) {
-                    const int key = key0 + 8 * (v / 4) + (v % 4);
-                    const bool allowed = (key <= q_position[qs]) & (key >= first_allowed);
-                    s_acc[qs][v] = allowed ? s_acc[qs][v] : -INFINITY;
-                    tile_max = fmaxf(tile_max, s_acc[qs][v]);
+                    for (int v = 0; v < 16; v++) {
+                        const int key = key0 + 8 * (v / 4) + (v % 4);
+                        const bool allowed = (key <= q_position[qs]) & ((key >= first_allowed) | (key < options.keep));
+                        s_acc[qs][v] = allowed ? s_acc[qs][v] : -INFINITY;
+                        tile_max = fmaxf(tile_max, s_acc[qs][v]);
+                    }
+                } else {
+#pragma unroll
+                    for (int v = 0; v < 16; v++) {
+                        const int key = key0 + 8 * (v / 4) + (v % 4);
+                        const bool allowed = (key <= q_position[qs]) & (key >= first_allowed);
+                        s_acc[qs][v] = allowed ? s_acc[qs][v] : -INFINITY;
+                        tile_max = fmaxf(tile_max, s_acc[qs][v]);
+                    }
                 }
             }
             tile_max = fmaxf(tile_max, __shfl_xor(tile_max, 32, WAVE)) * score_scale;
@@ -559,7 +574,7 @@ void launch(const void* q, int q_stride, const void* k_pages, const void* v_page
         // unit of its own at once (eight waves' tiles leave room for one block a unit): a long context with few queries.
         // Measured, heads of 64: 512 queries on 7,680 cached keys 38.2 against 46.7 us with four waves; but two prompts of 1,024
         // tokens (384 blocks: a second round) 19.1 against 15.9 us, one of 4,096 64.8 against 57 us.
-        const int reach = options.chunk > 0 ? min(max_len, options.chunk + 64) : (window > 0 ? min(max_len, window + 64) : max_len);
+        const int reach = options.chunk > 0 ? min(max_len, options.chunk + 64) : (window > 0 ? min(max_len, window + options.keep + 64) : max_len);
         const long blocks = (long)n_heads * n_requests * ceil_div(max_q_len, wide ? 64 : 32);
         bool eight = false;
         if constexpr (HD * sizeof(T) <= 128) {  // (eight waves' tiles of rows of 256 bytes do not fit a compute unit's LDS)

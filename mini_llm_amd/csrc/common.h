@@ -16,6 +16,7 @@ enum MllmEpilogue : int {
     MLLM_EPI_NONE = 0,       // (+ bias)
     MLLM_EPI_GELU_TANH = 1,  // gelu_new(+ bias)
     MLLM_EPI_GELU_ERF = 2,   // gelu(+ bias)
+    MLLM_EPI_SQUARED_RELU = 3,   // max(+ bias, 0)^2
 };
 
 typedef __bf16 bf16_t;
@@ -70,7 +71,7 @@ enum MllmKernel : int {
     MLLM_K_LATENT_ROWS, MLLM_K_SILU_MUL, MLLM_K_HEADS_LINEAR, MLLM_K_LATENT_ATTENTION, MLLM_K_LATENT_MERGE, MLLM_K_PROJECTION_ROWS,
     MLLM_K_HEAD_GATE, MLLM_K_GATED_NORM, MLLM_K_SHORT_CONV, MLLM_K_RECURRENCE, MLLM_K_MAP_ROWS,
     MLLM_K_MAP_DIFFERENCE, MLLM_K_TURN_HEADS, MLLM_K_GATE_UNIT, MLLM_K_ROUTE, MLLM_K_EXPERT_UNIT, MLLM_K_BRANCH_JOIN,
-    MLLM_K_GATED_SCAN, MLLM_K_EXPERT_LISTS, MLLM_K_EXPERTS_FEW, MLLM_K_KINDS
+    MLLM_K_GATED_SCAN, MLLM_K_EXPERT_LISTS, MLLM_K_EXPERTS_FEW, MLLM_K_JOIN_NORMS, MLLM_K_SOFT_CAP, MLLM_K_CHANNEL_MEMORY, MLLM_K_KINDS
 };
 void mllm_count_kernel(MllmKernel kind);
 
@@ -217,10 +218,16 @@ __device__ __forceinline__ float gelu_erf_for_bf16(float x) {
     return 0.5f * x * (1.0f + copysignf(erf_abs, x));
 }
 
+__device__ __forceinline__ float squared_relu(float x) {
+    const float positive = fmaxf(x, 0.0f);
+    return positive * positive;
+}
+
 template <int EPI>
 __device__ __forceinline__ float apply_activation(float x) {
     if constexpr (EPI == MLLM_EPI_GELU_TANH) return gelu_tanh(x);
     if constexpr (EPI == MLLM_EPI_GELU_ERF) return gelu_erf(x);
+    if constexpr (EPI == MLLM_EPI_SQUARED_RELU) return squared_relu(x);
     return x;
 }
 

@@ -105,7 +105,7 @@ __global__ __launch_bounds__(256) void turn_heads_pieces_kernel(const float* __r
 // A wave per (row, item); a row's items are its n_heads * maps queries, then (where the layer keeps keys and values of its own: k_at
 // >= 0) its n_kv_heads * maps keys and its n_kv_heads values. `rows` are the 32-bit sums of the product that made them, [.. | q | k |
 // v | ..] at columns q_at, k_at, v_at: q as [n_heads, maps, dim], k as [n_kv_heads, maps, dim], v as [n_kv_heads, vdim].
-// A query or key: RMS norm over its dim elements (gain [dim], shared by all heads and maps; null: no norm), then of its first
+// A query or key: RMS norm over its dim elements (gain [dim], shared by all heads and maps; null: no norm or, with `unit`, one without a gain), then of its first
 // rot_dims elements i and i + rot_dims / 2 turned as a pair by position x frequencies[i]. Queries go to q_out [row, n_kv_heads, maps, R,
 // head_size], keys to head g * maps + m of the row's slot in k_pages, a value to heads g * maps + 0 .. maps - 1 of v_pages, zeros
 // beyond dim / vdim up to head_size. Padding rows (slot < 0) store nothing.
@@ -116,7 +116,7 @@ __global__ __launch_bounds__(64 * MAP_WAVES) void map_rows_kernel(
     const float* __restrict__ rows, int stride, int q_at, int k_at, int v_at, const float* __restrict__ q_gain, const float* __restrict__ k_gain,
     float eps, const double* __restrict__ frequencies, int rot_dims, const int* __restrict__ positions, const int* __restrict__ slots,
     T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages, int n_rows, int n_heads, int n_kv_heads, int maps, int dim,
-    int vdim, int head_size, int page_size, const double* __restrict__ v_frequencies, int v_rot_dims, int v_neighbours) {
+    int vdim, int head_size, int page_size, const double* __restrict__ v_frequencies, int v_rot_dims, int v_neighbours, int unit) {
     const int lane = threadIdx.x % WAVE;
     const int n_q = n_heads * maps, n_k = k_at >= 0 ? n_kv_heads * maps : 0, n_v = k_at >= 0 ? n_kv_heads : 0;
     const int per_row = n_q + n_k + n_v;
@@ -156,7 +156,7 @@ __global__ __launch_bounds__(64 * MAP_WAVES) void map_rows_kernel(
         out = k_pages + (((size_t)(slot / page_size) * n_k + head * maps + map) * page_size + slot % page_size) * head_size;
     }
     float factor = 1.0f;
-    if (gain) {
+    if (gain || unit) {
         float squares = 0.0f;
         for (int d = lane; d < dim; d += WAVE) squares += in[d] * in[d];
         factor = 1.0f / sqrtf(wave_sum(squares) / (float)dim + eps);
@@ -228,6 +228,69 @@ __global__ __launch_bounds__(256) void rotate_rows_pieces_kernel(
     store_four(out + d, made);
 }
 
+// map_rows_kernel for heads of one map whose queries and keys are normed, four neighbouring elements a lane: LPH lanes (a power of two, LPH
+// * 4 >= head_size) take a query, key or value head, so a wave takes 64 / LPH of them. A lane asks for its four elements and, where they
+// are the first halves of turning pairs, for the second halves and both gains, all at once; the squares' sum goes over the head's lanes by
+// shuffles; the lane of a pair's first element makes both. Sizes and places as for rotate_rows_pieces_kernel; values stay as they are.
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void norm_rows_pieces_kernel(
+    const float* __restrict__ rows, int stride, int q_at, int k_at, int v_at, const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
+    const double* __restrict__ frequencies, int rot_dims, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
+    T* __restrict__ k_pages, T* __restrict__ v_pages, int n_rows, int n_heads, int n_kv_heads, int dim, int vdim, int head_size, int page_size) {
+    const int n_kept = k_at >= 0 ? n_kv_heads : 0;
+    const int per_row = n_heads + 2 * n_kept;
+    const long long index = ((long long)blockIdx.x * blockDim.x + threadIdx.x) / LPH;
+    const bool live = index < (long long)n_rows * per_row;   // (a wave's lanes stay together up to the shuffles)
+    const int row = live ? (int)(index / per_row) : 0, item = live ? (int)(index % per_row) : 0;
+    const int d = (threadIdx.x % LPH) * 4;
+    const bool is_q = item < n_heads, is_k = !is_q && item < n_heads + n_kept;
+    const int g = is_q ? item : item - n_heads - (is_k ? 0 : n_kept);
+    const int size = is_q || is_k ? dim : vdim, half = rot_dims / 2;
+    const float* in = rows + (size_t)row * stride + (is_q ? q_at : (is_k ? k_at : v_at)) + (size_t)g * size;
+    const float* gain = is_q ? q_gain : k_gain;
+    const bool turns = (is_q || is_k) && d < half;
+    const int at = min(d, size - 4), partner_at = turns ? d + half : at;
+    f32x4 own = *reinterpret_cast<const f32x4*>(in + at), partner = *reinterpret_cast<const f32x4*>(in + partner_at);
+    f32x4 own_gain = {1.0f, 1.0f, 1.0f, 1.0f}, partner_gain = {1.0f, 1.0f, 1.0f, 1.0f};
+    if (gain && (is_q || is_k)) {
+        own_gain = *reinterpret_cast<const f32x4*>(gain + at);
+        partner_gain = *reinterpret_cast<const f32x4*>(gain + partner_at);
+    }
+    const int position = positions[row];
+    const int slot = is_q ? 0 : slots[row];
+    float squares = 0.0f;
+    if (d < size) {
+#pragma unroll
+        for (int e = 0; e < 4; e++) squares += own[e] * own[e];
+    }
+    squares = lanes_sum<LPH>(squares);
+    if (!live || slot < 0 || d >= head_size) return;
+    T* out;
+    if (is_q) out = q_out + ((size_t)row * n_heads + item) * head_size;
+    else out = (is_k ? k_pages : v_pages) + (((size_t)(slot / page_size) * n_kept + g) * page_size + slot % page_size) * head_size;
+    if (!is_q && !is_k) {
+        store_four(out + d, d < size ? own : f32x4{0.0f, 0.0f, 0.0f, 0.0f});
+        return;
+    }
+    const float factor = 1.0f / sqrtf(squares / (float)dim + eps);
+#pragma unroll
+    for (int e = 0; e < 4; e++) own[e] *= factor * own_gain[e], partner[e] *= factor * partner_gain[e];
+    if (d < rot_dims) {
+        if (!turns) return;
+        f32x4 a, b;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            float x, y;
+            turned(own[e], partner[e], position, frequencies[d + e], x, y);
+            a[e] = x, b[e] = y;
+        }
+        store_four(out + d, a);
+        store_four(out + d + half, b);
+        return;
+    }
+    store_four(out + d, d < size ? own : f32x4{0.0f, 0.0f, 0.0f, 0.0f});
+}
+
 // A wave per (row, head): with a1 and a2 the results of the head's two maps (attention heads (g * 2 + 0) * R + r and (g * 2 + 1) * R + r
 // of `maps_out`, heads of head_size of which the first vdim count), x = a1 - lambda a2, out = x / sqrt(mean(x^2) + eps) * scale *
 // sigmoid(gate) -> out [row, head * vdim ..]. gate: 32-bit rows (null: no gate), the head's vdim elements at column head * vdim. The
@@ -267,7 +330,7 @@ __global__ __launch_bounds__(64 * MAP_WAVES) void map_difference_kernel(
 MLLM_API int mllm_map_rows(const float* rows, int stride, int q_at, int k_at, int v_at, const float* q_gain, const float* k_gain, float eps,
                            const double* frequencies, int rot_dims, const int* positions, const int* slots, void* q_out, void* k_pages,
                            void* v_pages, int n_rows, int n_heads, int n_kv_heads, int maps, int dim, int vdim, int head_size, int page_size,
-                           int dtype, const double* v_frequencies, int v_rot_dims, int v_neighbours, hipStream_t stream) {
+                           int dtype, const double* v_frequencies, int v_rot_dims, int v_neighbours, int unit, hipStream_t stream) {
     MLLM_REQUIRE(n_rows >= 0 && n_heads > 0 && n_kv_heads > 0 && maps > 0 && dim > 0 && vdim > 0 && page_size > 0, "map_rows: bad sizes");
     MLLM_REQUIRE(n_heads % n_kv_heads == 0, "map_rows: %d heads do not divide into %d key/value heads", n_heads, n_kv_heads);
     MLLM_REQUIRE(head_size >= dim && head_size >= vdim, "map_rows: heads of %d do not hold %d / %d elements", head_size, dim, vdim);
@@ -282,11 +345,36 @@ MLLM_API int mllm_map_rows(const float* rows, int stride, int q_at, int k_at, in
     const long long items = (long long)n_rows * (n_heads * maps + (k_at >= 0 ? n_kv_heads * (maps + 1) : 0));
     const int blocks = (int)((items + MAP_WAVES - 1) / MAP_WAVES);
     mllm_count_kernel(MLLM_K_MAP_ROWS);
-    // one map a head and no norm, everything in whole fours: four elements a thread
+    // one map a head, everything in whole fours: four elements a thread
     const bool values_fit = v_frequencies == nullptr || v_rot_dims == 0 || (v_neighbours == 0 && v_rot_dims % 8 == 0);
-    if (maps == 1 && q_gain == nullptr && k_gain == nullptr && rot_dims % 8 == 0 && dim % 4 == 0 && vdim % 4 == 0 && head_size % 4 == 0 && stride % 4 == 0 &&
+    const bool normed = q_gain != nullptr || k_gain != nullptr || unit;
+    const bool norms_fit = !normed || (head_size <= 256 && (v_frequencies == nullptr || v_rot_dims == 0) && (unit || (q_gain != nullptr && (k_gain != nullptr || k_at < 0))) &&
+                                       ((uintptr_t)q_gain & 15) == 0 && ((uintptr_t)k_gain & 15) == 0);
+    if (maps == 1 && norms_fit && rot_dims % 8 == 0 && dim % 4 == 0 && vdim % 4 == 0 && head_size % 4 == 0 && stride % 4 == 0 &&
         q_at % 4 == 0 && (k_at < 0 || (k_at % 4 == 0 && v_at % 4 == 0)) && ((uintptr_t)rows & 15) == 0 && ((uintptr_t)q_out & 15) == 0 &&
         (k_at < 0 || (((uintptr_t)k_pages & 15) == 0 && ((uintptr_t)v_pages & 15) == 0)) && values_fit) {
+        if (normed) {
+            int lanes = 4;
+            while (lanes * 4 < head_size) lanes *= 2;
+            const long long all = (long long)n_rows * (n_heads + (k_at >= 0 ? 2 * n_kv_heads : 0)) * lanes;
+            const int norm_blocks = (int)((all + 255) / 256);
+#define NORM_ROWS(T, LPH) norm_rows_pieces_kernel<T, LPH><<<norm_blocks, 256, 0, stream>>>(rows, stride, q_at, k_at, v_at, q_gain, k_gain, eps, frequencies, rot_dims, \
+                              positions, slots, (T*)q_out, (T*)k_pages, (T*)v_pages, n_rows, n_heads, n_kv_heads, dim, vdim, head_size, page_size)
+#define NORM_ROWS_OF(T)                                                                     \
+    do {                                                                                    \
+        if (lanes == 4) NORM_ROWS(T, 4);                                                    \
+        else if (lanes == 8) NORM_ROWS(T, 8);                                               \
+        else if (lanes == 16) NORM_ROWS(T, 16);                                             \
+        else if (lanes == 32) NORM_ROWS(T, 32);                                             \
+        else NORM_ROWS(T, 64);                                                              \
+    } while (0)
+            if (dtype == MLLM_F32) NORM_ROWS_OF(float);
+            else if (dtype == MLLM_BF16) NORM_ROWS_OF(bf16_t);
+            else MLLM_REQUIRE(false, "map_rows: unknown dtype %d", dtype);
+#undef NORM_ROWS_OF
+#undef NORM_ROWS
+            return mllm_check_launch("map_rows");
+        }
         const long long threads = (long long)n_rows * (n_heads + (k_at >= 0 ? 2 * n_kv_heads : 0)) * (head_size / 4);
         const int piece_blocks = (int)((threads + 255) / 256);
         const double* vf = v_rot_dims > 0 ? v_frequencies : nullptr;
@@ -299,7 +387,7 @@ MLLM_API int mllm_map_rows(const float* rows, int stride, int q_at, int k_at, in
         return mllm_check_launch("map_rows");
     }
 #define MAP_ROWS_ARGS(T) rows, stride, q_at, k_at, v_at, q_gain, k_gain, eps, frequencies, rot_dims, positions, slots, (T*)q_out, (T*)k_pages, \
-                         (T*)v_pages, n_rows, n_heads, n_kv_heads, maps, dim, vdim, head_size, page_size, v_frequencies, v_rot_dims, v_neighbours
+                         (T*)v_pages, n_rows, n_heads, n_kv_heads, maps, dim, vdim, head_size, page_size, v_frequencies, v_rot_dims, v_neighbours, unit
     if (dtype == MLLM_F32) map_rows_kernel<float><<<blocks, 64 * MAP_WAVES, 0, stream>>>(MAP_ROWS_ARGS(float));
     else if (dtype == MLLM_BF16) map_rows_kernel<bf16_t><<<blocks, 64 * MAP_WAVES, 0, stream>>>(MAP_ROWS_ARGS(bf16_t));
     else MLLM_REQUIRE(false, "map_rows: unknown dtype %d", dtype);

@@ -391,6 +391,7 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N) void gemm_kernel(const T* _
                 float value = acc[i][j][v] + b;
                 if (epilogue == MLLM_EPI_GELU_TANH) value = sizeof(OutT) == 2 ? gelu_tanh_for_bf16(value) : gelu_tanh(value);
                 else if (epilogue == MLLM_EPI_GELU_ERF) value = sizeof(OutT) == 2 ? gelu_erf_for_bf16(value) : gelu_erf(value);
+                else if (epilogue == MLLM_EPI_SQUARED_RELU) value = squared_relu(value);
                 size_t at = (size_t)row * N + col;
                 if (residual) value = early_residual[i][j][v] + value;
                 out[at] = from_float<OutT>(value);
@@ -540,6 +541,7 @@ __global__ __launch_bounds__(64 * KSPLIT) void gemm_skinny_kernel(
         if (bias) value += EARLY ? early_bias[j] : bias[col];
         if (epilogue == MLLM_EPI_GELU_TANH) value = sizeof(OutT) == 2 ? gelu_tanh_for_bf16(value) : gelu_tanh(value);
         else if (epilogue == MLLM_EPI_GELU_ERF) value = sizeof(OutT) == 2 ? gelu_erf_for_bf16(value) : gelu_erf(value);
+        else if (epilogue == MLLM_EPI_SQUARED_RELU) value = squared_relu(value);
         if (scatter.enabled) {
             if (col < scatter.q_width) {
                 out[(size_t)token * scatter.q_width + col] = from_float<OutT>(value);
@@ -713,7 +715,7 @@ MLLM_API int mllm_gemm(const void* A, const void* W, int w_packed, const float* 
                        void* out, int M, int N, int K, int in_dtype, int out_dtype, int epilogue,
                        int x_packed, int out_packed, hipStream_t stream) {
     MLLM_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm: bad sizes M=%d N=%d K=%d", M, N, K);
-    MLLM_REQUIRE(epilogue >= 0 && epilogue <= 2, "gemm: unknown epilogue %d", epilogue);
+    MLLM_REQUIRE(epilogue >= 0 && epilogue <= 3, "gemm: unknown epilogue %d", epilogue);
     MLLM_REQUIRE(ceil_div(M, 32) <= 65535, "gemm: M=%d has too many row tiles", M);
     MLLM_REQUIRE((!x_packed && !out_packed) || mllm_gemm_takes_packed_rows(M, N, K, in_dtype),
                  "gemm: rows in the packed layout are for the kernel for few rows, which M=%d N=%d K=%d do not take", M, N, K);

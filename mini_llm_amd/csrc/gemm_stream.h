@@ -491,6 +491,9 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
                     } else if constexpr (KIND == MLLM_EPI_GELU_ERF) {
 #pragma unroll
                         for (int e = 0; e < 4; e++) value[e] = sizeof(OutT) == 2 ? gelu_erf_for_bf16(value[e]) : gelu_erf(value[e]);
+                    } else if constexpr (KIND == MLLM_EPI_SQUARED_RELU) {
+#pragma unroll
+                        for (int e = 0; e < 4; e++) value[e] = squared_relu(value[e]);
                     }
                     put4<OutT>(reinterpret_cast<OutT*>(slab_write) + j * 32 + 8 * g, value);
                 }
@@ -533,6 +536,7 @@ __global__ __launch_bounds__(64 * WAVES_M * WAVES_N * WAVES_K) void gemm_stream_
     }
     if (epilogue == MLLM_EPI_GELU_TANH) leave(integral_constant<int, MLLM_EPI_GELU_TANH>{}, integral_constant<int, 0>{});
     else if (epilogue == MLLM_EPI_GELU_ERF) leave(integral_constant<int, MLLM_EPI_GELU_ERF>{}, integral_constant<int, 0>{});
+    else if (epilogue == MLLM_EPI_SQUARED_RELU) leave(integral_constant<int, MLLM_EPI_SQUARED_RELU>{}, integral_constant<int, 0>{});
     else leave(integral_constant<int, MLLM_EPI_NONE>{}, integral_constant<int, 0>{});
 }
 

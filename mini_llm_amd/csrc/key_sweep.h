@@ -34,7 +34,8 @@ __device__ __forceinline__ float sweep_exp(float x) {
     else return expf(x);
 }
 
-template <typename T, int HD>
+// GAPS: keys are numbered without a stretch the request does not look at: number n from `gap_from` on is key n + gap.
+template <typename T, int HD, bool GAPS = false>
 struct KeySweep {
     static constexpr int VEC = Chunk<T>::VEC;
     static constexpr int LPR = HD / VEC;      // lanes that share a row
@@ -47,6 +48,7 @@ struct KeySweep {
     float o[VEC];         // this lane's share of sum p * v, dimensions sub * VEC ..
     float running_max;    // the same in every lane
     float running_sum;    // this lane's share until merge_groups()
+    int gap_from, gap;    // (GAPS) set by the caller behind init()
     float cap;            // > 0: a score s counts as cap tanh(s / cap) (a caller that wants it sets it behind init())
 
     __device__ __forceinline__ void init() {
@@ -55,6 +57,12 @@ struct KeySweep {
         running_max = -INFINITY;
         running_sum = 0.0f;
         cap = 0.0f;
+        gap_from = gap = 0;
+    }
+
+    __device__ __forceinline__ int real_key(int number) const {
+        if constexpr (GAPS) return number + (number >= gap_from ? gap : 0);
+        else return number;
     }
 
     // KPI keys as loaded: converted where they are used.
@@ -71,7 +79,7 @@ struct KeySweep {
 #pragma unroll
         for (int u = 0; u < UNROLL; u++) {
             int key = base + u * RPI + group;
-            page[u] = table[(key < end ? key : spare_key) >> page_shift];
+            page[u] = table[real_key(key < end ? key : spare_key) >> page_shift];
         }
     }
 
@@ -86,7 +94,7 @@ struct KeySweep {
 #pragma unroll
         for (int u = 0; u < UNROLL; u++) {
             int key = base + u * RPI + group;
-            int safe_key = key < end ? key : spare_key;
+            int safe_key = real_key(key < end ? key : spare_key);
             size_t row = ((((size_t)page[u] * n_kv_heads + kv_head) << page_shift) + (safe_key & page_mask));
             if constexpr (KEYS) f.kf[u] = *reinterpret_cast<const Raw*>(k_pages + row * HD + sub * VEC);
             if constexpr (VALUES) f.vf[u] = *reinterpret_cast<const Raw*>(v_pages + row * HD + sub * VEC);

@@ -122,11 +122,13 @@ __global__ __launch_bounds__(256) void head_gate_kernel(const T* __restrict__ x,
 }
 
 // A wave per (row, group of `group` neighbouring elements): out = x / sqrt(mean over the group of x^2 + eps) * weight *
-// sigmoid(gate) * scale. weight [width] and gate [rows, width] may each be null.
+// sigmoid(gate) * scale (silu: gate * sigmoid(gate) * scale). weight [width] (shared_weight: [group], the same for all groups) and gate
+// [rows, width] may each be null.
 template <typename T>
 __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict__ x, int x_stride, const float* __restrict__ weight,
                                                          const float* __restrict__ gate, int gate_stride, float eps, float scale,
-                                                         T* __restrict__ out, int out_stride, int n_rows, int width, int group) {
+                                                         T* __restrict__ out, int out_stride, int n_rows, int width, int group, int silu,
+                                                         int shared_weight) {
     const int lane = threadIdx.x % WAVE;
     const int groups = width / group;
     const long long item = (long long)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
@@ -140,7 +142,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict
         for (int r = 0; r < 4; r++) {
             const int d = min(lane + r * WAVE, group - 1);
             xs[r] = in[d];
-            ws[r] = weight ? weight[first + d] : 1.0f;
+            ws[r] = weight ? weight[(shared_weight ? 0 : first) + d] : 1.0f;
             gs[r] = gate ? gate[(size_t)row * gate_stride + first + d] : 0.0f;
         }
         float squares = 0.0f;
@@ -150,7 +152,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict
 #pragma unroll
         for (int r = 0; r < 4; r++) {
             const int d = lane + r * WAVE;
-            if (d < group) out[(size_t)row * out_stride + first + d] = from_float<T>(xs[r] * factor * ws[r] * (gate ? sigmoid_f(gs[r]) : 1.0f));
+            if (d < group) out[(size_t)row * out_stride + first + d] = from_float<T>(xs[r] * factor * ws[r] * (gate ? sigmoid_f(gs[r]) * (silu ? gs[r] : 1.0f) : 1.0f));
         }
         return;
     }
@@ -159,8 +161,11 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict
     const float factor = scale / sqrtf(wave_sum(squares) / (float)group + eps);
     for (int d = lane; d < group; d += WAVE) {
         float value = in[d] * factor;
-        if (weight) value *= weight[first + d];
-        if (gate) value *= sigmoid_f(gate[(size_t)row * gate_stride + first + d]);
+        if (weight) value *= weight[(shared_weight ? 0 : first) + d];
+        if (gate) {
+            const float g = gate[(size_t)row * gate_stride + first + d];
+            value *= sigmoid_f(g) * (silu ? g : 1.0f);
+        }
         out[(size_t)row * out_stride + first + d] = from_float<T>(value);
     }
 }
@@ -170,7 +175,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict
 template <typename T>
 __global__ __launch_bounds__(256) void gated_norm_wide_kernel(const float* __restrict__ x, int x_stride, const float* __restrict__ weight,
                                                               const float* __restrict__ gate, int gate_stride, float eps, float scale,
-                                                              T* __restrict__ out, int out_stride, int width, int group) {
+                                                              T* __restrict__ out, int out_stride, int width, int group, int silu, int shared_weight) {
     __shared__ float scratch[16];
     const int groups = width / group;
     const int row = blockIdx.x / groups, first = (blockIdx.x % groups) * group;
@@ -182,7 +187,7 @@ __global__ __launch_bounds__(256) void gated_norm_wide_kernel(const float* __res
         for (int r = 0; r < REGS; r++) {
             const int d = min((int)threadIdx.x + r * 256, group - 1);
             xs[r] = in[d];
-            ws[r] = weight ? weight[first + d] : 1.0f;
+            ws[r] = weight ? weight[(shared_weight ? 0 : first) + d] : 1.0f;
             gs[r] = gate ? gate[(size_t)row * gate_stride + first + d] : 0.0f;
         }
         float squares = 0.0f;
@@ -192,7 +197,7 @@ __global__ __launch_bounds__(256) void gated_norm_wide_kernel(const float* __res
 #pragma unroll
         for (int r = 0; r < REGS; r++) {
             const int d = threadIdx.x + r * 256;
-            if (d < group) out[(size_t)row * out_stride + first + d] = from_float<T>(xs[r] * factor * ws[r] * (gate ? sigmoid_f(gs[r]) : 1.0f));
+            if (d < group) out[(size_t)row * out_stride + first + d] = from_float<T>(xs[r] * factor * ws[r] * (gate ? sigmoid_f(gs[r]) * (silu ? gs[r] : 1.0f) : 1.0f));
         }
         return;
     }
@@ -201,8 +206,11 @@ __global__ __launch_bounds__(256) void gated_norm_wide_kernel(const float* __res
     const float factor = scale / sqrtf(block_sum(squares, scratch) / (float)group + eps);
     for (int d = threadIdx.x; d < group; d += 256) {
         float value = in[d] * factor;
-        if (weight) value *= weight[first + d];
-        if (gate) value *= sigmoid_f(gate[(size_t)row * gate_stride + first + d]);
+        if (weight) value *= weight[(shared_weight ? 0 : first) + d];
+        if (gate) {
+            const float g = gate[(size_t)row * gate_stride + first + d];
+            value *= sigmoid_f(g) * (silu ? g : 1.0f);
+        }
         out[(size_t)row * out_stride + first + d] = from_float<T>(value);
     }
 }
@@ -296,7 +304,7 @@ MLLM_API int mllm_head_gate(const void* x, int x_stride, const float* gate, int 
 }
 
 MLLM_API int mllm_gated_norm(const float* x, int x_stride, const float* weight, const float* gate, int gate_stride, float eps, float scale, void* out,
-                             int out_stride, int n_rows, int width, int group, int dtype, hipStream_t stream) {
+                             int out_stride, int n_rows, int width, int group, int silu, int shared_weight, int dtype, hipStream_t stream) {
     MLLM_REQUIRE(n_rows >= 0 && width > 0 && group > 0 && width % group == 0, "gated_norm: %d elements do not divide into groups of %d", width, group);
     MLLM_REQUIRE(x_stride >= width && out_stride >= width && (gate == nullptr || gate_stride >= width), "gated_norm: rows are too short");
     MLLM_REQUIRE(x != nullptr && out != nullptr, "gated_norm: a missing operand");
@@ -306,13 +314,13 @@ MLLM_API int mllm_gated_norm(const float* x, int x_stride, const float* weight, 
     mllm_count_kernel(MLLM_K_GATED_NORM);
     if (group > 4 * WAVE) {   // wide groups: a block each
         MLLM_REQUIRE(items <= 0x7fffffffLL, "gated_norm: too many groups for one launch");
-        if (dtype == MLLM_F32) gated_norm_wide_kernel<float><<<(int)items, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (float*)out, out_stride, width, group);
-        else if (dtype == MLLM_BF16) gated_norm_wide_kernel<bf16_t><<<(int)items, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (bf16_t*)out, out_stride, width, group);
+        if (dtype == MLLM_F32) gated_norm_wide_kernel<float><<<(int)items, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (float*)out, out_stride, width, group, silu, shared_weight);
+        else if (dtype == MLLM_BF16) gated_norm_wide_kernel<bf16_t><<<(int)items, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (bf16_t*)out, out_stride, width, group, silu, shared_weight);
         else MLLM_REQUIRE(false, "gated_norm: unknown dtype %d", dtype);
         return mllm_check_launch("gated_norm");
     }
-    if (dtype == MLLM_F32) gated_norm_kernel<float><<<blocks, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (float*)out, out_stride, n_rows, width, group);
-    else if (dtype == MLLM_BF16) gated_norm_kernel<bf16_t><<<blocks, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (bf16_t*)out, out_stride, n_rows, width, group);
+    if (dtype == MLLM_F32) gated_norm_kernel<float><<<blocks, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (float*)out, out_stride, n_rows, width, group, silu, shared_weight);
+    else if (dtype == MLLM_BF16) gated_norm_kernel<bf16_t><<<blocks, 256, 0, stream>>>(x, x_stride, weight, gate, gate_stride, eps, scale, (bf16_t*)out, out_stride, n_rows, width, group, silu, shared_weight);
     else MLLM_REQUIRE(false, "gated_norm: unknown dtype %d", dtype);
     return mllm_check_launch("gated_norm");
 }

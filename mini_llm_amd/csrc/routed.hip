@@ -20,15 +20,17 @@ __device__ __forceinline__ bool picked_before(float a, int ia, float b, int ib) 
 // What a router does with a row's sums: scores s = softmax over all n_experts, or with `sigmoid` 1 / (1 + e^-z); choice c = s + correction
 // (null: none). The experts form n_groups equal groups of neighbours; a group's rank goes by the largest c in it, and only experts of
 // the best `keep` groups can be picked (the others count as minus infinity). The `top` experts of largest c are picked; a picked
-// expert's weight is s_e / (sum of the picked experts' s + floor), without `renormalise` s_e itself.
+// expert's weight is s_e / (sum of the picked experts' s + floor), without `renormalise` s_e itself. (Softmax scores without a correction
+// are compared by the sums themselves: the same order, also where scores vanish in 32 bits.)
 struct Choice {
     const float* correction;
     int n_experts, top, n_groups, keep;
     float floor;
     int sigmoid, renormalise;
+    int always;   // so many experts n_experts, n_experts + 1, ... that every row uses stand behind its own picks, with weight 1
 };
 // Where it goes, each optional: weights [row, n_experts] (rows `stride` apart, 0 for the experts that were not picked); picks and
-// pick_weights [row, top], the picked experts in the order of their choice scores (-1 where sums that are no numbers left none to pick).
+// pick_weights [row, top + always], the picked experts in the order of their choice scores (-1 where sums that are no numbers left none to pick).
 struct Routed {
     float* weights;
     int stride;
@@ -39,8 +41,12 @@ struct Routed {
 // One wave; `score` holds the row's sums.
 __device__ void route_row(const Choice& how, const Routed& to, size_t row, float* score, float* choice, float* group_best, int lane) {
     const int n_experts = how.n_experts;
+    const int places = how.top + how.always;
     if (to.picks)
-        for (int k = lane; k < how.top; k += WAVE) to.picks[row * how.top + k] = -1;
+        for (int k = lane; k < places; k += WAVE) {
+            to.picks[row * places + k] = k < how.top ? -1 : n_experts + k - how.top;
+            if (k >= how.top) to.pick_weights[row * places + k] = 1.0f;
+        }
     float largest = -INFINITY;
     for (int e = lane; e < n_experts; e += WAVE) largest = fmaxf(largest, score[e]);
     largest = wave_max(largest);
@@ -48,13 +54,14 @@ __device__ void route_row(const Choice& how, const Routed& to, size_t row, float
     for (int e = lane; e < n_experts; e += WAVE) {
         const float z = score[e], p = how.sigmoid ? 1.0f / (1.0f + expf(-z)) : expf(z - largest);
         score[e] = p;
+        choice[e] = z;
         total += p;
     }
     total = how.sigmoid ? 1.0f : wave_sum(total);
     for (int e = lane; e < n_experts; e += WAVE) {
         const float s = score[e] / total;
         score[e] = s;
-        choice[e] = s + (how.correction ? how.correction[e] : 0.0f);
+        if (how.sigmoid || how.correction) choice[e] = s + (how.correction ? how.correction[e] : 0.0f);
     }
     __builtin_amdgcn_wave_barrier();
     __threadfence_block();
@@ -92,8 +99,8 @@ __device__ void route_row(const Choice& how, const Routed& to, size_t row, float
         const float weight = place >= 0 ? score[e] / picked_sum : 0.0f;
         if (to.weights) to.weights[row * to.stride + e] = weight;
         if (to.picks && place >= 0) {
-            to.picks[row * how.top + place] = e;
-            to.pick_weights[row * how.top + place] = weight;
+            to.picks[row * places + place] = e;
+            to.pick_weights[row * places + place] = weight;
         }
     }
 }
@@ -246,14 +253,15 @@ int check_choice(int n_rows, const Choice& how, const Routed& to) {
     MLLM_REQUIRE(how.top >= 1 && how.top <= how.keep * (how.n_experts / how.n_groups), "route: %d experts to pick among %d groups of %d", how.top, how.keep,
                  how.n_experts / how.n_groups);
     MLLM_REQUIRE((to.weights != nullptr || to.picks != nullptr) && (to.picks == nullptr) == (to.pick_weights == nullptr), "route: nowhere to leave the choice");
+    MLLM_REQUIRE(how.always >= 0 && (how.always == 0 || to.picks != nullptr) && how.n_experts + how.always <= ROUTE_MAX_EXPERTS, "route: %d experts behind the picks", how.always);
     MLLM_REQUIRE(to.weights == nullptr || to.stride >= how.n_experts, "route: the weights' rows are too short");
     return 0;
 }
 }  // namespace
 
 MLLM_API int mllm_route(const float* logits, int stride, const float* correction, float* weights, int weights_stride, int* picks, float* pick_weights, int n_rows,
-                        int n_experts, int top, int n_groups, int keep, float floor, int sigmoid, int renormalise, hipStream_t stream) {
-    const Choice how{correction, n_experts, top, n_groups, keep, floor, sigmoid, renormalise};
+                        int n_experts, int top, int n_groups, int keep, float floor, int sigmoid, int renormalise, int always, hipStream_t stream) {
+    const Choice how{correction, n_experts, top, n_groups, keep, floor, sigmoid, renormalise, always};
     const Routed to{weights, weights_stride, picks, pick_weights};
     if (int status = check_choice(n_rows, how, to)) return status;
     MLLM_REQUIRE(stride >= n_experts && logits != nullptr, "route: rows are too short or missing");
@@ -271,8 +279,8 @@ MLLM_API int mllm_route_rows_supported(int n_experts, int K, int dtype) {
 
 MLLM_API int mllm_route_rows(const void* x, const void* router, int K, const float* correction, float* weights, int weights_stride, int* picks,
                              float* pick_weights, int n_rows, int n_experts, int top, int n_groups, int keep, float floor, int sigmoid, int renormalise,
-                             int dtype, hipStream_t stream) {
-    const Choice how{correction, n_experts, top, n_groups, keep, floor, sigmoid, renormalise};
+                             int always, int dtype, hipStream_t stream) {
+    const Choice how{correction, n_experts, top, n_groups, keep, floor, sigmoid, renormalise, always};
     const Routed to{weights, weights_stride, picks, pick_weights};
     if (int status = check_choice(n_rows, how, to)) return status;
     MLLM_REQUIRE(dtype == MLLM_F32 || dtype == MLLM_BF16, "route_rows: unknown dtype %d", dtype);

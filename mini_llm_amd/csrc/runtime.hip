@@ -34,7 +34,7 @@ static const char* const g_kernel_names[MLLM_K_KINDS] = {
     "rms_norm", "head_norm", "latent_rows", "silu_mul", "heads_linear", "latent_attention", "latent_merge", "projection_rows",
     "head_gate", "gated_norm", "short_conv", "recurrence", "map_rows", "map_difference", "turn_heads", "gate_unit", "route",
     "expert_unit", "branch_join", "gated_scan",
-    "expert_lists", "experts_few",
+    "expert_lists", "experts_few", "join_norms", "soft_cap", "channel_memory",
 };
 
 void mllm_count_kernel(MllmKernel kind) { g_launches[kind].fetch_add(1, std::memory_order_relaxed); }

@@ -9,8 +9,9 @@ from __future__ import annotations
 from dataclasses import dataclass
 
 from ..ops import kernels
-from ..parts.base import Norm, Part, PositionEncoding
+from ..parts.base import Ahead, Norm, Part, PositionEncoding
 from ..parts.embedding import TokenEmbedding
+from ..weights.spec import VECTOR, Normal, TensorSpec
 
 
 EMBEDDING_STATE = "embedding"   # the state layer of an embedding that keeps state (mixers' are named by their cache layer)
@@ -21,6 +22,7 @@ class LayerCall:
     block: int               # index into Model.blocks
     cache: int               # cache layer (and state layer) this call uses
     write_cache: bool = True
+    step: int | None = None  # the row of the model's step vectors that joins the stream right before this call
 
 
 @dataclass(frozen=True)
@@ -34,6 +36,8 @@ class CacheGroupSpec:
     head_size: int
     window: int | None
     planes: int = 2   # 1: the layers keep one row per token that serves as key and value (no value pages)
+    keep_first: int = 0          # beside a window: the first so many keys stay
+    chunk: int | None = None     # only keys of the current chunk of so many positions are read
 
 
 @dataclass
@@ -63,16 +67,38 @@ class TokenChoice:
     draws: DrawParameters | None = None
 
 
+class StepVectors(Part):
+    """A table [steps, width] of vectors that join the stream at places of the schedule (``LayerCall.step``): what tells the passes of a
+    loop over the same layers apart. Kept in 32-bit, as the stream is."""
+
+    def __init__(self, steps: int, width: int, tensor_name: str = "weight"):
+        self.steps, self.width = steps, width
+        self._tensor_name = tensor_name
+        self.weight = None
+
+    def tensor_specs(self):
+        return {self._tensor_name: TensorSpec((self.steps, self.width), VECTOR, Normal(0.3))}
+
+    def bind(self, tensors):
+        self.weight = tensors[self._tensor_name]
+
+    def vector(self, step: int):
+        return self.weight[step]
+
+
 class Model(Part):
     def __init__(self, config, precision, *, embedding: TokenEmbedding, position_encoding: PositionEncoding | None,
-                 blocks: list, schedule: list, final_norm: Norm, head, names: dict):
+                 blocks: list, schedule: list, final_norm: Norm, head, names: dict, step_vectors: StepVectors | None = None):
         self.config, self.precision = config, precision
         self.embedding, self.position_encoding = embedding, position_encoding
         self.blocks, self.schedule = list(blocks), list(schedule)
         self.final_norm, self.head = final_norm, head
-        self._names = names  # prefixes: embedding, position_encoding, block (format with {i}), final_norm
+        self._names = names  # prefixes: embedding, position_encoding, block (format with {i}), final_norm, head, step_vectors
+        self.step_vectors = step_vectors
         written = set()
         for call in self.schedule:
+            if call.step is not None and (step_vectors is None or not 0 <= call.step < step_vectors.steps):
+                raise ValueError(f"a layer call names step vector {call.step}, and the model has {0 if step_vectors is None else step_vectors.steps}")
             if not 0 <= call.block < len(self.blocks):
                 raise ValueError(f"the schedule names layer {call.block}, but there are {len(self.blocks)}")
             if call.write_cache:
@@ -90,6 +116,8 @@ class Model(Part):
         for i, block in enumerate(self.blocks):
             out[self._names["block"].format(i=i)] = block
         out[self._names["final_norm"]] = self.final_norm
+        if self.step_vectors is not None:
+            out[self._names["step_vectors"]] = self.step_vectors
         if "head" in self._names:   # a head with a matrix of its own (a tied head has no tensors)
             out[self._names["head"]] = self.head
         return out
@@ -126,15 +154,17 @@ class Model(Part):
             need = self.blocks[call.block].mixer_part().kv_need()
             if need is None:
                 continue
-            layers = groups.setdefault((need.n_kv_heads, need.head_size, need.window, need.planes), [])
+            layers = groups.setdefault((need.n_kv_heads, need.head_size, need.window, need.planes, need.keep_first, need.chunk), [])
             if call.write_cache:
                 layers.append(call.cache)
             elif call.cache not in layers:
                 raise ValueError(f"a layer call reads cache layer {call.cache}, whose pages have another shape or window")
-        return [
-            CacheGroupSpec(f"{'window' + str(key[2]) if key[2] else 'full'}_h{key[0]}x{key[1]}{'' if key[3] == 2 else 'p' + str(key[3])}", tuple(layers), *key)
-            for key, layers in groups.items()
-        ]
+        specs = []
+        for key, layers in groups.items():
+            n_kv_heads, head_size, window, planes, keep_first, chunk = key
+            reach = f"window{window}" + (f"+{keep_first}" if keep_first else "") if window else (f"chunk{chunk}" if chunk else "full")
+            specs.append(CacheGroupSpec(f"{reach}_h{n_kv_heads}x{head_size}{'' if planes == 2 else 'p' + str(planes)}", tuple(layers), *key))
+        return specs
 
     def state_needs(self) -> dict:
         """state layer id -> StateNeed, for the mixers that keep state of fixed size, and for an embedding that does."""
@@ -149,12 +179,24 @@ class Model(Part):
         return out
 
     def _layers(self, hidden, batch, cache, observer=None):
-        """The schedule over the rows of ``batch``; the stream comes back as the last layer leaves it."""
+        """The schedule over the rows of ``batch``; the stream comes back as the last layer leaves it. A layer is told what comes ahead of
+        the next one (``Ahead``) and may do it in its own last kernel; it is not told of a vector that joins the stream behind it while an
+        observer looks on, which is shown the stream as the layer alone leaves it."""
+        told = None
         for index, call in enumerate(self.schedule):
             block = self.blocks[call.block]
+            vector = None if call.step is None else self.step_vectors.vector(call.step)
+            if vector is not None and not (isinstance(hidden, kernels.ReadyRows) and hidden.joined is not None and hidden.joined is told.vector):
+                hidden = kernels.PendingRows(kernels.settle(hidden), None, vector)
             if not block.takes_pending:
                 hidden = kernels.settle(hidden)
-            hidden = block.forward(hidden, cache.layer_context(batch, call))
+            ctx = cache.layer_context(batch, call)
+            following = self.schedule[index + 1] if index + 1 < len(self.schedule) else None
+            told = None
+            if following is not None and (following.step is None or observer is None):
+                told = ctx.ahead = Ahead(None if following.step is None else self.step_vectors.vector(following.step),
+                                         self.blocks[following.block].first_norms())
+            hidden = block.forward(hidden, ctx)
             if observer is not None:
                 observer(index, kernels.settle(hidden))
         return hidden

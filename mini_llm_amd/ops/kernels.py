@@ -15,7 +15,7 @@ from .library import check, library
 
 F32, BF16 = 0, 1
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16}
-EPILOGUES = {None: 0, "none": 0, "gelu_new": 1, "gelu": 2}
+EPILOGUES = {None: 0, "none": 0, "gelu_new": 1, "gelu": 2, "squared_relu": 3}
 
 
 class OperandError(ValueError):
@@ -429,9 +429,10 @@ def _arrivals(k_pages, rows: int, n_heads: int):
 
 
 def paged_attention(q, k_pages, v_pages, token_request, positions, block_tables, n_heads, n_kv_heads, head_size, scale, window=0, max_q_len=None, max_len=None, q_starts=None, context_lens=None, out=None,
-                    short_rows=None, short_requests=None, packed_out=False, first_row=0, softcap: float = 0.0, sinks=None, chunk: int = 0, wide_out: bool = False):
+                    short_rows=None, short_requests=None, packed_out=False, first_row=0, softcap: float = 0.0, sinks=None, chunk: int = 0, keep_first: int = 0, wide_out: bool = False):
     """Causal attention of each row of q over its request's cached keys (max(0, p-window+1)..p; with ``chunk`` > 0 the keys of
     the row's own chunk of so many positions, chunks counted from position 0: floor(p / chunk) * chunk .. p).
+    ``keep_first`` > 0 (with a window): the first so many keys of a sequence stay visible, however far back they are.
     ``softcap`` > 0: a scaled score s counts as softcap * tanh(s / softcap). ``sinks`` (float32 [n_heads]): exp(sink_h) joins
     the denominator of head h's softmax, once, with no key and no value. ``wide_out``: the result is float32 whatever the pages' type
     is (for a mixer that goes on computing with the heads' results before anything is rounded); not together with ``packed_out``.
@@ -476,7 +477,9 @@ def paged_attention(q, k_pages, v_pages, token_request, positions, block_tables,
         _device_tensor(sinks, "sinks", torch.float32, 1)
         _require(sinks.shape[0] == n_heads, "one sink a head")
     softcap, chunk = float(softcap or 0.0), int(chunk or 0)
+    keep_first = int(keep_first or 0) if window else 0
     _require(chunk >= 0 and not (chunk and window), "the keys a row sees are bounded by a window or by chunks, not both")
+    _require(keep_first >= 0, "kept first keys are a number of them")
     rows_aligned = q.data_ptr() % 16 == 0 and (q.stride(0) * q.element_size()) % 16 == 0  # 16-byte loads of q
     if (short_rows is not None and short_requests is not None and 0 < short_rows < n and max_q_len is not None
             and max_q_len > DECODE_MAX_Q_LEN and q_starts is not None and context_lens is not None and rows_aligned
@@ -484,7 +487,7 @@ def paged_attention(q, k_pages, v_pages, token_request, positions, block_tables,
             and lib.mllm_attention_prefill_supported(head_size, page_size)):
         _require(0 < short_requests < context_lens.shape[0], "short_requests does not cut the batch in two")
         common = dict(n_heads=n_heads, n_kv_heads=n_kv_heads, head_size=head_size, scale=scale, window=window, max_len=max_len, first_row=first_row,
-                      softcap=softcap, sinks=sinks, chunk=chunk, wide_out=wide_out)
+                      softcap=softcap, sinks=sinks, chunk=chunk, keep_first=keep_first, wide_out=wide_out)
         paged_attention(q[:short_rows], k_pages, v_pages, token_request, positions, block_tables, max_q_len=DECODE_MAX_Q_LEN,
                         q_starts=q_starts[: short_requests + 1], context_lens=context_lens[:short_requests],
                         out=out[:short_rows], **common)
@@ -499,7 +502,7 @@ def paged_attention(q, k_pages, v_pages, token_request, positions, block_tables,
         # per 64 keys of reach
         reach = block_tables.shape[1] * page_size if max_len is None else max(1, min(max_len, block_tables.shape[1] * page_size))
         if window or chunk:
-            reach = min(reach, int(window or chunk))
+            reach = min(reach, int(window or chunk) + keep_first)
         # few tokens with many keys: a token's keys in several runs, a block each, so that the blocks are about as many
         # as the chip has compute units, and a second small kernel that puts the runs together
         n_parts, units = 1, _compute_units(q.device)
@@ -521,7 +524,7 @@ def paged_attention(q, k_pages, v_pages, token_request, positions, block_tables,
         check(lib.mllm_attention_decode(_ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), width if packed_out else out.stride(0),
                                         _ptr(token_request), _ptr(positions), _ptr(block_tables), block_tables.shape[1], n, n_heads, n_kv_heads,
                                         head_size, page_size, int(window), float(scale), n_splits, _code(q.dtype), int(packed_out),
-                                        n_parts, _ptr(parts), _ptr(arrivals), softcap, _ptr(sinks), chunk, int(wide_out), _stream()))
+                                        n_parts, _ptr(parts), _ptr(arrivals), softcap, _ptr(sinks), chunk, keep_first, int(wide_out), _stream()))
         return result
     if (max_q_len is not None and max_q_len > DECODE_MAX_Q_LEN and q_starts is not None and context_lens is not None
             and rows_aligned and lib.mllm_attention_prefill_supported(head_size, page_size)):
@@ -530,9 +533,9 @@ def paged_attention(q, k_pages, v_pages, token_request, positions, block_tables,
         n_requests = context_lens.shape[0]
         _require(q_starts.shape[0] == n_requests + 1, "q_starts must have one entry more than context_lens")
         _require(block_tables.shape[0] >= n_requests, "fewer block tables than requests")
-        check(lib.mllm_attention_prefill(_ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(q_starts), _ptr(context_lens), _ptr(block_tables), block_tables.shape[1], n_requests, int(max_q_len), int(max_len or 0), n_heads, n_kv_heads, head_size, page_size, int(window), float(scale), _code(q.dtype), softcap, _ptr(sinks), chunk, int(wide_out), _stream()))
+        check(lib.mllm_attention_prefill(_ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(q_starts), _ptr(context_lens), _ptr(block_tables), block_tables.shape[1], n_requests, int(max_q_len), int(max_len or 0), n_heads, n_kv_heads, head_size, page_size, int(window), float(scale), _code(q.dtype), softcap, _ptr(sinks), chunk, keep_first, int(wide_out), _stream()))
         return out
-    check(lib.mllm_attention(_ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(token_request), _ptr(positions), _ptr(block_tables), block_tables.shape[1], n, n_heads, n_kv_heads, head_size, page_size, int(window), float(scale), _code(q.dtype), softcap, _ptr(sinks), chunk, int(wide_out), _stream()))
+    check(lib.mllm_attention(_ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(token_request), _ptr(positions), _ptr(block_tables), block_tables.shape[1], n, n_heads, n_kv_heads, head_size, page_size, int(window), float(scale), _code(q.dtype), softcap, _ptr(sinks), chunk, keep_first, int(wide_out), _stream()))
     return out
 
 
@@ -777,11 +780,15 @@ class NormedRows:
 class ReadyRows:
     """Rows of the residual stream in float32 (``stream``) and, made ahead of time by the kernel that wrote them, the rows that the
     norm ``norm`` (a part) makes of them, in the element type the next products read (``rows``). A layer whose last norm sits on a
-    branch's output hands these to the layer whose first norm is ``norm``; any other reader takes ``stream``."""
+    branch's output hands these to the layer whose first norm is ``norm``; any other reader takes ``stream``. ``rows_2``: what the second
+    norm of a layer that norms the same rows twice makes of them. ``joined``: the vector that has already joined the stream on behalf of
+    whoever asked for it (parts.base.Ahead)."""
 
     stream: torch.Tensor
     rows: torch.Tensor
     norm: object
+    rows_2: torch.Tensor | None = None
+    joined: object = None
 
     @property
     def shape(self):
@@ -1150,22 +1157,24 @@ def head_gate(x, gate, out, n_heads, head_size, scale: float = 1.0):
     return out
 
 
-def gated_norm(x, weight, gate, eps, out, group: int | None = None, scale: float = 1.0):
-    """out = x / sqrt(mean(x^2) + eps) * weight * sigmoid(gate) * scale, the mean taken over each group of ``group`` neighbouring
-    elements (None: the whole row). x: float32 [rows, width]; weight: float32 [width] or None; gate: float32 [rows, width] (strided) or
+def gated_norm(x, weight, gate, eps, out, group: int | None = None, scale: float = 1.0, silu: bool = False):
+    """out = x / sqrt(mean(x^2) + eps) * weight * sigmoid(gate) * scale (``silu``: gate * sigmoid(gate) in the gate's place), the mean taken over each group of ``group`` neighbouring
+    elements (None: the whole row). x: float32 [rows, width]; weight: float32 [width], or [group] for all groups, or None; gate: float32 [rows, width] (strided) or
     None; out: [rows, >= width] (strided), any element type."""
     width = x.shape[1]
     _rows_f32(x, "x", width)
     group = width if group is None else int(group)
+    shared = False
     if weight is not None:
         _device_tensor(weight, "weight", torch.float32, 1)
-        _require(weight.shape[0] == width, "the gain vector does not match the rows")
+        shared = weight.shape[0] == group != width
+        _require(weight.shape[0] in (width, group), "the gain vector does not match the rows")
     if gate is not None:
         _rows_f32(gate, "gate", width)
         _require(gate.shape[0] == x.shape[0], "the gate does not match the rows")
     _require(out.is_cuda and out.dim() == 2 and out.stride(1) == 1 and out.shape[0] == x.shape[0] and out.shape[1] >= width, "out does not match the rows")
     check(library().mllm_gated_norm(_ptr(x), x.stride(0), _ptr(weight), _ptr(gate), 0 if gate is None else gate.stride(0), float(eps), float(scale), _ptr(out),
-                                    out.stride(0), x.shape[0], width, group, _code(out.dtype), _stream()))
+                                    out.stride(0), x.shape[0], width, group, int(bool(silu)), int(shared), _code(out.dtype), _stream()))
     return out
 
 
@@ -1245,11 +1254,11 @@ def recurrence(q, k, v, state, q_starts, state_slots, n_heads, dim, vdim, *, gat
 
 # -- attention whose heads hold several maps over one value (differential attention) -----------------------------------------
 def map_rows(rows, q_at: int, k_at: int | None, v_at: int | None, q_gain, k_gain, eps, frequencies, rot_dims, positions, slots, k_pages, v_pages,
-             n_heads, n_kv_heads, maps, dim, vdim, *, v_frequencies=None, v_rot_dims: int = 0, v_pairing: str = "half"):
+             n_heads, n_kv_heads, maps, dim, vdim, *, v_frequencies=None, v_rot_dims: int = 0, v_pairing: str = "half", unit: bool = False):
     """The row-wise work between the fused projection of a mixer with ``maps`` maps a head and its attention. ``rows``: the float32
     sums of that product, the queries [n_heads, maps, dim] at column ``q_at``, the keys [n_kv_heads, maps, dim] at ``k_at`` and the values
     [n_kv_heads, vdim] at ``v_at`` (both None: the layer reads keys and values another layer keeps, and only its queries are made).
-    Every query and key is RMS-normed over its ``dim`` elements (gains [dim], shared by heads and maps; None: no norm), then of its
+    Every query and key is RMS-normed over its ``dim`` elements (gains [dim], shared by heads and maps; None: no norm or, with ``unit``, one without gains), then of its
     first ``rot_dims`` elements i and i + rot_dims / 2 are turned as a pair by position * frequencies[i] (float64; the angle is taken in
     64-bit). Returns the queries as [rows, n_heads * maps * head_size] in the pages' type, laid out for the paged attention kernels run with
     n_heads * maps heads over n_kv_heads * maps key/value heads: query head g R + r (R = n_heads / n_kv_heads) of map m is their head (g *
@@ -1291,7 +1300,7 @@ def map_rows(rows, q_at: int, k_at: int | None, v_at: int | None, q_gain, k_gain
     check(library().mllm_map_rows(_ptr(rows), rows.stride(0), int(q_at), int(k_at) if keeps else -1, int(v_at) if keeps else -1, _ptr(q_gain), _ptr(k_gain),
                                   float(eps), _ptr(frequencies if rot_dims else None), int(rot_dims), _ptr(positions), _ptr(slots if keeps else None), _ptr(out),
                                   _ptr(k_pages), _ptr(v_pages), n, n_heads, n_kv_heads, int(maps), dim, vdim, head_size, page_size, _code(k_pages.dtype),
-                                  _ptr(v_frequencies), int(v_rot_dims), int(v_pairing == "neighbours"), _stream()))
+                                  _ptr(v_frequencies), int(v_rot_dims), int(v_pairing == "neighbours"), int(bool(unit)), _stream()))
     return out
 
 
@@ -1342,7 +1351,7 @@ class Picks:
     weights: torch.Tensor
 
 
-def _choice(n, device, n_experts, top, correction, n_groups, keep, score, dense, picks):
+def _choice(n, device, n_experts, top, correction, n_groups, keep, score, dense, picks, always):
     _require(1 <= n_experts <= ROUTE_MAX_EXPERTS, f"the router kernel takes up to {ROUTE_MAX_EXPERTS} experts")
     _require(n_groups >= 1 and n_experts % n_groups == 0 and 1 <= keep <= n_groups, "the experts do not divide into the groups")
     _require(1 <= top <= keep * (n_experts // n_groups), "more experts to pick than the kept groups hold")
@@ -1350,25 +1359,28 @@ def _choice(n, device, n_experts, top, correction, n_groups, keep, score, dense,
     if correction is not None:
         _device_tensor(correction, "correction", torch.float32, 1)
         _require(correction.shape[0] == n_experts, "one correction an expert")
+    _require(always >= 0 and (picks or always == 0), "experts that every row uses are named among the picks")
     weights = torch.empty((n, n_experts), dtype=torch.float32, device=device) if dense else None
-    picked = Picks(torch.empty((n, top), dtype=torch.int32, device=device), torch.empty((n, top), dtype=torch.float32, device=device)) if picks else None
+    places = top + always
+    picked = Picks(torch.empty((n, places), dtype=torch.int32, device=device), torch.empty((n, places), dtype=torch.float32, device=device)) if picks else None
     return weights, picked
 
 
 def route(logits, n_experts: int, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0, score: str = "softmax",
-          renormalise: bool = True, picks: bool = False):
+          renormalise: bool = True, picks: bool = False, always: int = 0):
     """A router's choice, row by row. ``logits``: float32 rows whose first ``n_experts`` columns are the router's sums (rows may be
     strided). Scores are their softmax over all experts or, with ``score`` "sigmoid", each one's own sigmoid; the choice goes by score +
     correction (float32 [n_experts]; None: by the score) among the experts of the ``keep`` best of ``n_groups`` equal groups of neighbours (a
     group counts by its best choice score); the ``top`` best are picked. Returns float32 [rows, n_experts]: a picked expert's score over (the
-    sum of the picked scores + floor), without ``renormalise`` its score itself, zero for the rest; or with ``picks`` the same as ``Picks``."""
+    sum of the picked scores + floor), without ``renormalise`` its score itself, zero for the rest; or with ``picks`` the same as ``Picks``, and behind every row's own picks the ``always`` experts n_experts, n_experts +
+    1, ... with weight 1. Softmax scores without a correction are compared by their sums (the same order, also where scores vanish)."""
     _require(isinstance(logits, torch.Tensor) and logits.is_cuda and logits.dim() == 2 and logits.dtype == torch.float32 and logits.stride(1) == 1
              and logits.shape[1] >= n_experts, "the router's sums must be float32 GPU rows with contiguous columns")
     n = logits.shape[0]
-    weights, picked = _choice(n, logits.device, n_experts, top, correction, n_groups, keep, score, not picks, picks)
+    weights, picked = _choice(n, logits.device, n_experts, top, correction, n_groups, keep, score, not picks, picks, int(always))
     check(library().mllm_route(_ptr(logits), logits.stride(0), _ptr(correction), _ptr(weights), n_experts, _ptr(picked.experts if picks else None),
                                _ptr(picked.weights if picks else None), n, n_experts, int(top), int(n_groups), int(keep), float(floor),
-                               int(score == "sigmoid"), int(bool(renormalise)), _stream()))
+                               int(score == "sigmoid"), int(bool(renormalise)), int(always), _stream()))
     return picked if picks else weights
 
 
@@ -1378,7 +1390,7 @@ def route_rows_supported(n_experts: int, width: int, dtype) -> bool:
 
 
 def route_rows(x, router, top: int, *, correction=None, n_groups: int = 1, keep: int = 1, floor: float = 0.0, score: str = "softmax",
-               renormalise: bool = True, picks: bool = False):
+               renormalise: bool = True, picks: bool = False, always: int = 0):
     """``route`` with the router's product inside: x [rows, width] and the router's matrix [n_experts, width] (row-major), both of one element
     type; sums in 32-bit. For routers of few outputs (``route_rows_supported``)."""
     _device_tensor(x, "x", dim=2)
@@ -1387,10 +1399,10 @@ def route_rows(x, router, top: int, *, correction=None, n_groups: int = 1, keep:
     n_experts = router.shape[0]
     _require(router.shape[1] == width, "x and the router's matrix differ in width")
     _require(route_rows_supported(n_experts, width, x.dtype), f"no kernel routes {n_experts} experts over rows of {width}")
-    weights, picked = _choice(n, x.device, n_experts, top, correction, n_groups, keep, score, not picks, picks)
+    weights, picked = _choice(n, x.device, n_experts, top, correction, n_groups, keep, score, not picks, picks, int(always))
     check(library().mllm_route_rows(_ptr(x), _ptr(router), width, _ptr(correction), _ptr(weights), n_experts, _ptr(picked.experts if picks else None),
                                     _ptr(picked.weights if picks else None), n, n_experts, int(top), int(n_groups), int(keep), float(floor),
-                                    int(score == "sigmoid"), int(bool(renormalise)), _code(x.dtype), _stream()))
+                                    int(score == "sigmoid"), int(bool(renormalise)), int(always), _code(x.dtype), _stream()))
     return picked if picks else weights
 
 
@@ -1543,6 +1555,120 @@ def branch_join(stream, a, b=None, *, a_bias=None, b_bias=None, scale_a=None, sc
                                      _ptr(gates), gates_stride, int(gate_a_at), int(gate_b_at), float(mult), _ptr(out), _ptr(next_weight), int(bool(one_plus)),
                                      float(eps), _ptr(rows), 0 if rows is None else _code(rows.dtype), n, width, _stream()))
     return out if rows is None else (out, rows)
+
+
+@dataclass(frozen=True)
+class RowNorm:
+    """A norm over rows as a kernel runs it behind a sum: (h - mean) / sqrt(variance + eps) * gain + offset (``centred``: a layer norm), or h /
+    sqrt(mean(h^2) + eps) * gain; ``one_plus``: 1 + gain in the gain's place; ``offset`` None: none."""
+
+    gain: torch.Tensor
+    offset: torch.Tensor | None
+    eps: float
+    centred: bool
+    one_plus: bool = False
+
+
+def shared_row_norms(norms) -> bool:
+    """Whether one kernel can run these norms (RowNorm or None) over the same rows: of one kind, with one eps."""
+    return bool(norms) and all(n is not None and (n.eps, n.centred, n.one_plus, n.offset is None) ==
+                               (norms[0].eps, norms[0].centred, norms[0].one_plus, norms[0].offset is None) for n in norms)
+
+
+def join_norms(stream, branches=(), *, vector=None, norms=(), out_dtype=None):
+    """stream + the branches + vector, float32 [rows, width], and what up to two norms of the same kind (RowNorm) make of that sum, in
+    ``out_dtype``: (sum, [normed rows of each norm]). ``branches``: up to two, each float32 [rows, width] or [n, rows, width], the partial
+    products of a product cut along K (added up here), or BranchRows with a bias; None is left out. ``vector``: float32 [width]. Without
+    branches and vector the sum is the stream itself and is not written again."""
+    _device_tensor(stream, "stream", torch.float32, 2)
+    n, width = stream.shape
+    given = []
+    for branch in branches:
+        if branch is None:
+            continue
+        rows, bias = (branch.rows, branch.bias) if isinstance(branch, BranchRows) else (branch, None)
+        _device_tensor(rows, "a branch", torch.float32)
+        _require(rows.dim() in (2, 3) and tuple(rows.shape[-2:]) == (n, width), "a branch must have the stream's shape")
+        if bias is not None:
+            _device_tensor(bias, "a branch's bias", torch.float32, 1)
+            _require(bias.shape[0] == width, "a branch's bias does not match the row width")
+        given.append((rows, rows.shape[0] if rows.dim() == 3 else 1, rows.stride(0) if rows.dim() == 3 else 0, bias))
+    _require(len(given) <= 2 and len(norms) <= 2, "two branches and two norms at most")
+    _require(not norms or (shared_row_norms(norms) and out_dtype is not None), "the norms must be of one kind, with one eps, and need an element type")
+    vectors = [vector] + [v for norm in norms for v in (norm.gain, norm.offset)]
+    for v in vectors:
+        if v is not None:
+            _device_tensor(v, "a vector of the join", torch.float32, 1)
+            _require(v.shape[0] == width, "a vector of the join does not match the row width")
+    summed = bool(given) or vector is not None
+    total = torch.empty_like(stream) if summed else stream
+    rows = [torch.empty((n, width), dtype=out_dtype, device=stream.device) for _ in norms]
+    if not summed and not norms:
+        return total, rows
+    (a, n_a, a_stride, a_bias), (b, n_b, b_stride, b_bias) = (given + [(None, 0, 0, None)] * 2)[:2]
+    first, second = (list(norms) + [None, None])[:2]
+    check(library().mllm_join_norms(_ptr(stream), _ptr(a), n_a, a_stride, _ptr(a_bias), _ptr(b), n_b, b_stride, _ptr(b_bias), _ptr(vector), _ptr(total if summed else None),
+                                    _ptr(first.gain if first else None), _ptr(first.offset if first else None), _ptr(rows[0] if first else None),
+                                    _ptr(second.gain if second else None), _ptr(second.offset if second else None), _ptr(rows[1] if second else None),
+                                    int(bool(first and first.centred)), int(bool(first and first.one_plus)), float(first.eps) if first else 1.0,
+                                    0 if first is None else _code(out_dtype), n, width, _stream()))
+    return total, rows
+
+
+def soft_cap(x, cap: float, out=None):
+    """cap * tanh(x / cap) of float32 rows (``out``: may be x itself)."""
+    _device_tensor(x, "x", torch.float32)
+    _require(cap > 0, "the cap must be positive")
+    if out is None:
+        out = torch.empty_like(x)
+    _device_tensor(out, "out", torch.float32)
+    _require(out.shape == x.shape, "out has the wrong shape")
+    check(library().mllm_soft_cap(_ptr(x), _ptr(out), x.numel(), float(cap), _stream()))
+    return out
+
+
+def channel_memory(rows, q_at: int, k_at: int, v_at: int, g_at: int, low_at: int, decay_up, decay_bias, state, q_starts, state_slots, n_heads, dim, vdim, *,
+                   tau: float, q_scale: float, gain, eps: float, out_dtype, max_q_len: int | None = None):
+    """A matrix per head and request whose rows (key channels) each fade at a pace of their own (gated linear attention): S <- diag(alpha) S + k
+    v^T, o = S^T q, alpha = sigmoid(z)^(1 / tau), z = decay_up^T low + decay_bias; every head's o then divided by its root mean square (eps
+    inside the root), times ``gain`` (float32 [vdim]), times silu(g). ``rows``: the float32 sums of a fused product (rows may be strided) with q, k
+    [n_heads * dim] at columns ``q_at``, ``k_at`` (q is multiplied by ``q_scale``), v and g [n_heads * vdim] at ``v_at``, ``g_at``, and low [rank] at
+    ``low_at``; ``decay_up`` float32 [rank, n_heads * dim], ``decay_bias`` float32 [n_heads * dim]. ``state``: float32 [slots, n_heads * dim * vdim],
+    moved on in place; request r's rows are q_starts[r] .. q_starts[r + 1], its slot state_slots[r] (negative: passed by, its rows of the
+    result are undefined). All in 32-bit up to the result, [rows, n_heads * vdim] of ``out_dtype``. ``max_q_len``: the longest portion of the
+    batch, or a bound on it; above RECURRENCE_ROW_BY_ROW the portions run chunk by chunk."""
+    _require(isinstance(rows, torch.Tensor) and rows.is_cuda and rows.dim() == 2 and rows.dtype == torch.float32 and rows.stride(1) == 1,
+             "the rows must be float32 GPU rows with contiguous columns")
+    n, width = rows.shape
+    _device_tensor(decay_up, "decay_up", torch.float32, 2)
+    _device_tensor(decay_bias, "decay_bias", torch.float32, 1)
+    _device_tensor(gain, "gain", torch.float32, 1)
+    rank, qw, vw = decay_up.shape[0], n_heads * dim, n_heads * vdim
+    _require(decay_up.shape[1] == qw and decay_bias.shape[0] == qw and gain.shape[0] == vdim, "decays or gains do not match the heads")
+    _require(all(0 <= at and at + size <= width for at, size in ((q_at, qw), (k_at, qw), (v_at, vw), (g_at, vw), (low_at, rank))), "columns lie beyond the rows")
+    _require(state.is_cuda and state.dim() == 2 and state.dtype == torch.float32 and state.stride(1) == 1 and state.shape[1] >= qw * vdim,
+             "the state must be float32 rows on the GPU that hold the matrices")
+    _device_tensor(q_starts, "q_starts", torch.int32, 1)
+    _device_tensor(state_slots, "state_slots", torch.int32, 1)
+    n_requests = state_slots.shape[0]
+    _require(q_starts.shape[0] >= n_requests + 1, "q_starts must have one entry more than there are requests")
+    _require(tau > 0 and eps > 0, "tau and eps must be positive")
+    lib = library()
+    longest = n if max_q_len is None else max(1, min(int(max_q_len), max(n, 1)))
+    chunk = int(lib.mllm_channel_memory_chunk_rows(int(dim), int(vdim))) if longest > RECURRENCE_ROW_BY_ROW else 0
+    out = torch.empty((n, vw), dtype=out_dtype, device=rows.device)
+    records = sums = None
+    if chunk:
+        records = torch.empty(((n // chunk + n_requests + 1) * n_heads * (dim * vdim + dim),), dtype=torch.float32, device=rows.device)
+    elif not lib.mllm_channel_memory_norms(int(dim), int(vdim)):   # heads so large that no block holds all of a row's values
+        sums = torch.empty((n, vw), dtype=torch.float32, device=rows.device)
+    check(lib.mllm_channel_memory(_ptr(rows), rows.stride(0), int(q_at), int(k_at), int(v_at), int(g_at), int(low_at), _ptr(decay_up), _ptr(decay_bias), rank,
+                                  1.0 / float(tau), float(q_scale), _ptr(gain), float(eps), _ptr(state), state.stride(0), _ptr(q_starts), _ptr(state_slots),
+                                  _ptr(out), _ptr(sums), n, n_requests, n_heads, dim, vdim, longest, _ptr(records), 0 if records is None else records.numel(),
+                                  chunk, _code(out_dtype), _stream()))
+    if sums is not None:
+        gated_norm(sums, gain, rows[:, g_at : g_at + vw], eps, out, group=vdim, silu=True)
+    return out
 
 
 def map_difference(maps_out, gate, lam: float, eps: float, n_heads, n_kv_heads, vdim, head_size, scale: float = 1.0, out=None, out_dtype=None):

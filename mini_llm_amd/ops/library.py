@@ -29,10 +29,10 @@ _SIGNATURES = {
     "mllm_probe_read": [P, c_longlong, P, c_int, P],
     "mllm_probe_mfma": [P, c_int, c_int, c_int, P],
     "mllm_cache_write": [P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_attention": [P, c_int, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_float, P, c_int, c_int, P],
-    "mllm_attention_decode": [P, c_int, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, P, P, c_float, P, c_int, c_int, P],
+    "mllm_attention": [P, c_int, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_float, P, c_int, c_int, c_int, P],
+    "mllm_attention_decode": [P, c_int, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, P, P, c_float, P, c_int, c_int, c_int, P],
     "mllm_attention_decode_supported": [c_int, c_int, c_int],
-    "mllm_attention_prefill": [P, c_int, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_float, P, c_int, c_int, P],
+    "mllm_attention_prefill": [P, c_int, P, P, P, c_int, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_float, P, c_int, c_int, c_int, P],
     "mllm_attention_prefill_supported": [c_int, c_int],
     "mllm_sample": [P, c_int, c_int, P, P, P, P, P, P, P, P],
     "mllm_gemm_best_per_row": [c_int, c_int, c_int, c_int],
@@ -52,11 +52,11 @@ _SIGNATURES = {
     "mllm_latent_rows": [P, c_int, P, c_int, P, c_float, P, c_float, c_int, c_int, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_silu_mul": [P, P, c_int, c_int, c_int, P],
     "mllm_map_rows": [P, c_int, c_int, c_int, c_int, P, P, c_float, P, c_int, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                      c_int, P, c_int, c_int, P],
+                      c_int, P, c_int, c_int, c_int, P],
     "mllm_turn_heads": [P, c_int, P, c_int, P, c_int, c_int, c_float, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_route": [P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, P],
+    "mllm_route": [P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, P],
     "mllm_route_rows_supported": [c_int, c_int, c_int],
-    "mllm_route_rows": [P, P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, P],
+    "mllm_route_rows": [P, P, c_int, P, P, c_int, P, P, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, P],
     "mllm_expert_tile_rows": [],
     "mllm_experts_few_rows": [c_int, c_int],
     "mllm_expert_lists": [P, P, c_int, c_int, c_int, c_int, P, P, P, P, P, P],
@@ -70,6 +70,12 @@ _SIGNATURES = {
     "mllm_gate_unit": [P, P, c_int, c_int, c_float, c_float, c_float, c_int, P],
     "mllm_branch_join": [P, P, c_int, c_longlong, P, P, c_int, c_longlong, P, P, P, P, c_int, c_int, c_int, c_float, P, P, c_int, c_float, P, c_int,
                          c_int, c_int, P],
+    "mllm_join_norms": [P, P, c_int, c_longlong, P, P, c_int, c_longlong, P, P, P, P, P, P, P, P, P, c_int, c_int, c_float, c_int, c_int, c_int, P],
+    "mllm_soft_cap": [P, P, c_longlong, c_float, P],
+    "mllm_channel_memory_chunk_rows": [c_int, c_int],
+    "mllm_channel_memory_norms": [c_int, c_int],
+    "mllm_channel_memory": [P, c_int, c_int, c_int, c_int, c_int, c_int, P, P, c_int, c_float, c_float, P, c_float, P, c_longlong, P, P, P, P, c_int, c_int,
+                            c_int, c_int, c_int, c_int, P, c_longlong, c_int, c_int, P],
     "mllm_map_difference": [P, c_int, P, c_int, P, c_int, c_float, c_float, c_float, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_heads_linear": [P, c_int, c_int, c_int, P, c_int, P, c_int, c_int, c_int, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_latent_attention_supported": [c_int, c_int, c_int],
@@ -81,7 +87,7 @@ _SIGNATURES = {
     "mllm_projection_rows": [P, c_int, P, c_int, P, c_int, P, c_int, P, P, P, c_float, P, c_int, P, P, P, P, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                              c_int, c_int, P],
     "mllm_head_gate": [P, c_int, P, c_int, c_float, P, c_int, c_int, c_int, c_int, c_int, P],
-    "mllm_gated_norm": [P, c_int, P, P, c_int, c_float, c_float, P, c_int, c_int, c_int, c_int, c_int, P],
+    "mllm_gated_norm": [P, c_int, P, P, c_int, c_float, c_float, P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_short_conv": [P, c_int, P, c_int, P, c_longlong, P, P, P, P, c_int, c_int, c_int, c_int, c_int, P],
     "mllm_recurrence_supported": [c_int, c_int],
     "mllm_recurrence": [c_int, P, c_int, P, c_int, P, c_int, P, P, c_int, c_float, P, c_float, P, c_longlong, c_longlong, c_longlong, P, P, P, c_int, c_int,

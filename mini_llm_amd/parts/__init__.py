@@ -7,7 +7,7 @@ from .base import (
 from .block import BranchNormBlock, ParallelBlock, PostNormBlock, PreNormBlock, SandwichNormBlock
 from .differential_attention import DifferentialAttention
 from .embedding import LinearHead, PairEmbedding, TiedHead, TokenEmbedding
-from .feedforward import ClampedGatedMLP, DenseMLP, GatedMLP
+from .feedforward import ClampedGatedMLP, DenseMLP, GatedMLP, PlainMLP
 from .latent_attention import LatentAttention
 from .linear import Linear
 from .norms import LayerNorm, RMSNorm
@@ -15,7 +15,7 @@ from .positions import LearnedPositions, RotaryEncoding
 from .projection_attention import ProjectionNormAttention
 from .rotary_attention import RotaryAttention
 from .routed import RoutedExperts
-from .recurrent import DecayedLinearAttention, MatrixMemoryMixer, MinGRUMixer, ParallelMixer
+from .recurrent import DecayedLinearAttention, GatedLinearAttention, MatrixMemoryMixer, MinGRUMixer, ParallelMixer
 
 __all__ = [
     "BLOCKS", "FEED_FORWARDS", "MIXERS", "NORMS", "POSITION_ENCODINGS",
@@ -23,5 +23,5 @@ __all__ = [
     "make_part", "register_part",
     "CausalSelfAttention", "PreNormBlock", "TiedHead", "TokenEmbedding", "DenseMLP", "Linear", "LayerNorm", "LearnedPositions",
     "NormedHeadAttention", "LatentAttention", "BranchNormBlock", "ProjectionNormAttention", "DecayedLinearAttention",
-    "MatrixMemoryMixer", "ParallelMixer", "PostNormBlock", "SandwichNormBlock", "DifferentialAttention", "LinearHead", "GatedMLP", "RMSNorm", "RotaryEncoding", "ClampedGatedMLP", "ParallelBlock", "RotaryAttention", "RoutedExperts", "PairEmbedding", "MinGRUMixer",
+    "MatrixMemoryMixer", "ParallelMixer", "PostNormBlock", "SandwichNormBlock", "DifferentialAttention", "LinearHead", "GatedMLP", "RMSNorm", "RotaryEncoding", "ClampedGatedMLP", "ParallelBlock", "RotaryAttention", "RoutedExperts", "PairEmbedding", "MinGRUMixer", "PlainMLP", "GatedLinearAttention",
 ]

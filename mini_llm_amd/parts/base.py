@@ -54,12 +54,20 @@ class Part:
 @dataclass(frozen=True)
 class KVNeed:
     """Keys and values that grow with the sequence, kept in pages. ``window`` None: every key
-    is kept; an integer w: only the last w keys are ever read, older pages are given back."""
+    is kept; an integer w: only the last w keys are ever read, older pages are given back
+    (``keep_first``: but the first so many keys stay). ``chunk`` c: only keys of the query's own
+    chunk of c positions are ever read, the pages of earlier chunks are given back."""
 
     n_kv_heads: int
     head_size: int
     window: int | None = None
     planes: int = 2   # 2: keys and values; 1: one row per token that serves as both (a latent cache): no value pages are kept
+    keep_first: int = 0
+    chunk: int | None = None
+
+    def __post_init__(self):
+        if self.keep_first < 0 or (self.keep_first and self.window is None) or (self.chunk is not None and (self.chunk < 1 or self.window is not None)):
+            raise ValueError("first keys are kept beside a window, and keys are bounded by a window or by chunks, not both")
 
 
 @dataclass(frozen=True)
@@ -81,9 +89,24 @@ class LayerContext:
     write_cache: bool = True      # False: the layer reads a cache another layer call has written
     state: object = None          # [num_slots, *StateNeed.shape] of the call's state layer
     extra: dict = field(default_factory=dict)
+    ahead: "Ahead | None" = None  # what will be done to the stream behind this layer call (None: unknown, or left to whoever does it)
+
+
+@dataclass(frozen=True)
+class Ahead:
+    """What happens to the stream between this layer call and the branches of the next one: ``vector`` (float32 [width], or None) is
+    added to every row, then the layer norms ``norms`` read it (empty: unknown). A block that does either in its own last kernel
+    returns kernels.ReadyRows; one that looks at neither may ignore both, and the model adds the vector itself."""
+
+    vector: object = None
+    norms: tuple = ()
 
 
 class Norm(Part):
+    def row_norm(self):
+        """What a kernel needs to run this norm behind a sum of its own (kernels.RowNorm), or None: it has to be called."""
+        return None
+
     # True if ``forward`` also takes rows whose last sums are pending (ops.kernels.PendingRows)
     takes_pending = False
 
@@ -170,6 +193,10 @@ class Block(Part):
     # True if ``forward`` takes and may return rows whose last sums are pending
     # (ops.kernels.PendingRows); a block that says False always gets plain float32 rows.
     takes_pending = False
+
+    def first_norms(self) -> tuple:
+        """The norms that read the stream as it reaches this layer (for the layer before, which may run them: Ahead.norms)."""
+        return ()
 
     def forward(self, hidden, ctx: LayerContext):
         """hidden: [rows, width] float32 residual stream -> the same after this layer."""

@@ -152,12 +152,20 @@ class ParallelBlock(Block):
     stored matrices ``rg1``, ``rg2`` [width, width] and biases ``rg1.b``, ``rg2.b`` (else 1); both gates come from one product over the two
     matrices laid behind each other, in 32-bit: the mixer's own first product where it can carry them (``Mixer.carries_rows``). The sum is one kernel (``kernels.branch_join``: it also adds up the partial products of a
     branch whose last product was cut along K), which norms the sum for the layer that follows where that layer's first norm is known
-    (``hand_to``): the layer then returns kernels.ReadyRows, and a layer that is handed rows made by its own ``norm_1`` does not run it."""
+    (``hand_to``): the layer then returns kernels.ReadyRows, and a layer that is handed rows made by its own ``norm_1`` does not run it.
+
+``norm_2``: the feed-forward reads a norm of its own, x <- x + mixer(norm_1(x)) + feed_forward(norm_2(x)), both norms of the same x (then
+without layer scale, gates and ``mult``). The sum, what the model says comes ahead of the next layer (``LayerContext.ahead``: a vector that
+joins the stream, the next layer's norms) and both of that layer's norms are then one kernel, ``kernels.join_norms``."""
 
     takes_pending = True   # takes plain rows, pending rows or the ReadyRows of the layer before
 
     def __init__(self, norm_1: Norm, mixer: Mixer, feed_forward: FeedForward | None, width: int, compute_dtype, *, mult: float = 1.0,
-                 layer_scale: bool = False, gated: bool = False, names=("norm1", "mix.", "mlp.")):
+                 layer_scale: bool = False, gated: bool = False, norm_2: Norm | None = None, names=("norm1", "mix.", "mlp.", "norm2")):
+        if norm_2 is not None and (feed_forward is None or layer_scale or gated or mult != 1.0):
+            raise ValueError("a second norm goes with a feed-forward, and not with layer scale, gates or a multiplier")
+        self.norm_2 = norm_2
+        self._joins_norms = not (layer_scale or gated or mult != 1.0)   # the sum is a plain one: join_norms takes it
         self.norm_1, self.mixer, self.feed_forward = norm_1, mixer, feed_forward
         self.width, self.compute_dtype, self.mult, self.layer_scale, self.gated = width, compute_dtype, float(mult), bool(layer_scale), bool(gated)
         self._names = names
@@ -169,7 +177,7 @@ class ParallelBlock(Block):
                 part.sums_later = True
 
     def children(self):
-        parts = dict(zip(self._names, (self.norm_1, self.mixer, self.feed_forward)))
+        parts = dict(zip(self._names, (self.norm_1, self.mixer, self.feed_forward, self.norm_2)))
         return {name: part for name, part in parts.items() if part is not None}
 
     def mixer_part(self):
@@ -177,6 +185,9 @@ class ParallelBlock(Block):
 
     def hand_to(self, norm: Norm | None):
         self._following = norm
+
+    def first_norms(self):
+        return (self.norm_1,) if self.norm_2 is None else (self.norm_1, self.norm_2)
 
     def _branches(self):
         return ("1", "2") if self.feed_forward is not None else ("1",)
@@ -217,7 +228,7 @@ class ParallelBlock(Block):
         """A feed-forward whose first small product reads the layer's input rows (a router) sends it along in the mixer's too."""
         rider = getattr(self.feed_forward, "rows_to_carry", None)
         self._feed_forward_rides = False
-        if rider is not None and self.mixer.carries_rows:
+        if rider is not None and self.mixer.carries_rows and self.norm_2 is None:
             rows = rider()
             if rows is not None:
                 self.mixer.carry_rows("feed_forward", *rows)
@@ -234,6 +245,8 @@ class ParallelBlock(Block):
         else:
             self._ride_feed_forward()
         self.norm_1.bind_named(tensors, prefix + self._names[0])
+        if self.norm_2 is not None:
+            self.norm_2.bind_named(tensors, prefix + self._names[3])
         self.mixer.bind_named(tensors, prefix + self._names[1])
 
     def forward(self, hidden, ctx: LayerContext):
@@ -241,11 +254,22 @@ class ParallelBlock(Block):
 
         from ..ops import kernels
 
+        rows_2 = None
         if isinstance(hidden, kernels.ReadyRows) and hidden.norm is self.norm_1:
-            stream, rows = hidden.stream, hidden.rows
+            stream, rows, rows_2 = hidden.stream, hidden.rows, hidden.rows_2
+        elif self._joins_norms and self.norm_2 is not None and kernels.shared_row_norms([norm.row_norm() for norm in self.first_norms()]):
+            vector = None
+            if isinstance(hidden, kernels.PendingRows) and hidden.partials is None:   # a vector that joins the stream on its way in
+                hidden, vector = hidden.base, hidden.bias
+            stream, (rows, rows_2) = kernels.join_norms(kernels.settle(hidden), vector=vector, norms=[norm.row_norm() for norm in self.first_norms()],
+                                                        out_dtype=self.compute_dtype)
         else:
             stream = kernels.settle(hidden)
             rows = self.norm_1.forward(stream, self.compute_dtype)
+        if self.norm_2 is None:
+            rows_2 = rows
+        elif rows_2 is None:
+            rows_2 = self.norm_2.forward(stream, self.compute_dtype)
         gates = kernels.linear(rows, self.gates, self.gates_bias, out_dtype=torch.float32) if self.gated and self.gates is not None else None
         first = self.mixer.forward(rows, None, ctx)
         carried = ctx.extra.pop("carried", {})
@@ -253,7 +277,9 @@ class ParallelBlock(Block):
             gates = carried["gates"]
         second = None
         if self.feed_forward is not None:
-            second = self.feed_forward.forward(rows, None, carried=carried["feed_forward"]) if self._feed_forward_rides else self.feed_forward.forward(rows, None)
+            second = self.feed_forward.forward(rows, None, carried=carried["feed_forward"]) if self._feed_forward_rides else self.feed_forward.forward(rows_2, None)
+        if self._joins_norms and self._following is None:
+            return self._joined(stream, first, second, ctx.ahead)
         following = self._following
         ahead = {}
         if following is not None and hasattr(following, "one_plus") and getattr(following, "out_scale", 1.0) == 1.0:
@@ -261,6 +287,18 @@ class ParallelBlock(Block):
         joined = kernels.branch_join(stream, first, second, scale_a=self.scale_1, scale_b=self.scale_2, gates=gates, gate_a_at=0, gate_b_at=self.width,
                                      mult=self.mult, **ahead)
         return kernels.ReadyRows(joined[0], joined[1], following) if ahead else joined
+
+    def _joined(self, stream, first, second, ahead):
+        from ..ops import kernels
+
+        if ahead is None:
+            return kernels.join_norms(stream, [first, second])[0]
+        norms = [norm.row_norm() for norm in ahead.norms]
+        if not norms or len(norms) > 2 or not kernels.shared_row_norms(norms):
+            norms = []
+        total, rows = kernels.join_norms(stream, [first, second], vector=ahead.vector, norms=norms, out_dtype=self.compute_dtype)
+        return kernels.ReadyRows(total, rows[0] if rows else None, ahead.norms[0] if rows else None, rows_2=rows[1] if len(rows) > 1 else None,
+                                 joined=ahead.vector)
 
 
 register_part("block", "pre_norm", PreNormBlock)

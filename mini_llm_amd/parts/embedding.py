@@ -90,10 +90,12 @@ class TiedHead(Part):
 
 
 class LinearHead(Part):
-    """logits = x . W^T with a matrix of its own, [vocab, width], no bias."""
+    """logits = x . W^T with a matrix of its own, [vocab, width], no bias. ``softcap``: a logit z then counts as softcap tanh(z / softcap)."""
 
-    def __init__(self, vocab_size: int, width: int, tensor_name: str = "weight"):
-        self.vocab_size, self.width = vocab_size, width
+    def __init__(self, vocab_size: int, width: int, tensor_name: str = "weight", softcap: float | None = None):
+        if softcap is not None and not softcap > 0:
+            raise ValueError(f"the cap must be positive, not {softcap}")
+        self.vocab_size, self.width, self.softcap = vocab_size, width, softcap
         self._tensor_name = tensor_name
         self.weight = None
 
@@ -106,10 +108,11 @@ class LinearHead(Part):
     def forward(self, x):
         import torch
 
-        return kernels.linear(x, self.weight, out_dtype=torch.float32)
+        logits = kernels.linear(x, self.weight, out_dtype=torch.float32)
+        return logits if self.softcap is None else kernels.soft_cap(logits, self.softcap, out=logits)
 
     def forward_best(self, x):
-        """See TiedHead.forward_best."""
+        """See TiedHead.forward_best. (A cap does not change which logit is the largest: the pairs hold what goes into it.)"""
         if not kernels.best_per_row(x.shape[0], self.weight, x.dtype):
             return None
         return kernels.linear_best(x, self.weight)

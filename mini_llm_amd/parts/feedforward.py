@@ -120,6 +120,37 @@ class ClampedGatedMLP(FeedForward):
         return self._down_product(inner, self.down, residual, bias=self.down_bias)
 
 
+class PlainMLP(FeedForward):
+    """down(act(up x)), no biases, both matrices stored [out, in] under their bare names; the activation (``ops.kernels.EPILOGUES``:
+    "squared_relu", "gelu", "gelu_new") is fused into the up product."""
+
+    def __init__(self, width: int, inner: int, activation: str, names=("up", "down")):
+        if activation not in kernels.EPILOGUES:
+            raise ValueError(f"activation {activation!r} is not one of {', '.join(str(name) for name in kernels.EPILOGUES)}")
+        self.width, self.inner, self.activation = width, inner, activation
+        self._names = names
+        self.up = self.down = None
+        self._down_product = BranchProduct()
+        self.sums_later = False   # True: a call without a residual may return kernels.BranchRows (the block that adds the branch takes its sums)
+
+    def tensor_specs(self):
+        from ..weights.spec import MATRIX, Normal, TensorSpec
+
+        up, down = self._names
+        return {up: TensorSpec((self.inner, self.width), MATRIX, Normal(self.width ** -0.5)),
+                down: TensorSpec((self.width, self.inner), MATRIX, Normal(self.inner ** -0.5))}
+
+    def bind(self, tensors):
+        self.up, self.down = (tensors[name] for name in self._names)
+
+    def forward(self, x, residual):
+        inner = kernels.linear(x, self.up, activation=self.activation)
+        if residual is None and self.sums_later:
+            return self._down_product.later(inner, self.down)
+        return self._down_product(inner, self.down, residual)
+
+
 register_part("feed_forward", "dense_mlp", DenseMLP)
+register_part("feed_forward", "plain_mlp", PlainMLP)
 register_part("feed_forward", "clamped_gated_mlp", ClampedGatedMLP)
 register_part("feed_forward", "gated_mlp", GatedMLP)

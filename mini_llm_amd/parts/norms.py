@@ -9,18 +9,28 @@ from .base import Norm, register_part
 
 
 class LayerNorm(Norm):
+    """``tensor_names``: the gain's and the offset's names behind the part's prefix ("" where the part's own name is the tensor's)."""
+
     takes_pending = True
 
-    def __init__(self, width: int, eps: float):
+    def __init__(self, width: int, eps: float, tensor_names=("weight", "bias")):
         self.width, self.eps = width, eps
+        self._tensor_names = tuple(tensor_names)
         self.weight = None
         self.bias = None
 
     def tensor_specs(self):
+        gain, offset = self._tensor_names
         return {
-            "weight": TensorSpec((self.width,), VECTOR, Normal(0.05, mean=1.0)),
-            "bias": TensorSpec((self.width,), VECTOR, Normal(0.02)),
+            gain: TensorSpec((self.width,), VECTOR, Normal(0.05, mean=1.0)),
+            offset: TensorSpec((self.width,), VECTOR, Normal(0.02)),
         }
+
+    def bind(self, tensors):
+        self.weight, self.bias = (tensors[name] for name in self._tensor_names)
+
+    def row_norm(self):
+        return kernels.RowNorm(self.weight, self.bias, self.eps, centred=True)
 
     def forward(self, x, out_dtype, row_index=None):
         return kernels.layernorm(x, self.weight, self.bias, self.eps, out_dtype=out_dtype, row_index=row_index)
@@ -58,6 +68,9 @@ class RMSNorm(Norm):
             self.weight = self.weight.reshape(1).expand(self.width).contiguous()
         if self.out_scale != 1.0:
             self.weight = (self.weight.double() * self.out_scale).float()
+
+    def row_norm(self):
+        return kernels.RowNorm(self.weight, None, self.eps, centred=False, one_plus=self.one_plus)
 
     def forward(self, x, out_dtype, row_index=None):
         return kernels.rms_norm(x, self.weight, self.eps, one_plus=self.one_plus, out_dtype=out_dtype, row_index=row_index)

@@ -14,6 +14,10 @@ Both: one product makes everything that reads h (32-bit sums), ``kernels.recurre
 the state its slot holds (zero at admission), ``kernels.gated_norm`` norms and gates. State, gates and sums are 32-bit in every
 precision.
 
+``GatedLinearAttention`` (GLA): q = W_q h / sqrt(dim), k = W_k h, v = W_v h; a decay per key channel, alpha = sigmoid(z)^(1 / tau) with z = W_a2
+(W_a1 h) + b, W_a1 of a rank the tensors give; S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t; every head's o divided by its root mean
+square, times one gain vector of vdim for all heads, times silu(W_g h), then W_o (``kernels.channel_memory``, norm and gate inside).
+
 ``MinGRUMixer``: a vector per request; z = sigmoid(W_z h + b_z), u = W_x h + b_x, candidate c = u + shift where u >= 0 and sigmoid(u) where u
 < 0; S_t = (1 - z) S_(t-1) + z c element by element, and W_o (S_t * silu(W_g h)). The gates read the current row alone, so a portion is
 a scan (``kernels.gated_scan``).
@@ -29,7 +33,7 @@ from dataclasses import replace
 import torch
 
 from ..ops import kernels
-from ..weights.spec import TABLE, VECTOR, Normal, TensorSpec
+from ..weights.spec import TABLE, VECTOR, FreeDim, Normal, TensorSpec
 from .base import LayerContext, Mixer, StateNeed, register_part
 from .linear import BranchProduct, fuse_rows
 
@@ -141,6 +145,55 @@ class DecayedLinearAttention(Mixer):
         return self._out_product(mixed, self.o, residual)
 
 
+class GatedLinearAttention(Mixer):
+    graph_safe = True
+
+    def __init__(self, width: int, n_heads: int, dim: int, vdim: int, tau: float, eps: float):
+        if not tau > 0 or not eps > 0:
+            raise ValueError(f"tau and eps must be positive, not {tau} and {eps}")
+        self.width, self.n_heads, self.dim, self.vdim, self.tau, self.eps = width, n_heads, dim, vdim, float(tau), float(eps)
+        self.rank = FreeDim(16)
+        self.w_in = self.o = self.norm = self.decay_up = self.decay_bias = None
+        self._out_product = BranchProduct()
+        self.sums_later = False   # True: a call without a residual may return kernels.BranchRows (the block that adds the branch takes its sums)
+
+    def tensor_specs(self):
+        H, std = self.n_heads, self.width ** -0.5
+        return {"q": TensorSpec((H * self.dim, self.width), TABLE, Normal(std)),
+                "k": TensorSpec((H * self.dim, self.width), TABLE, Normal(std)),
+                "v": TensorSpec((H * self.vdim, self.width), TABLE, Normal(std)),
+                "g": TensorSpec((H * self.vdim, self.width), TABLE, Normal(std)),
+                "a1": TensorSpec((self.rank, self.width), TABLE, Normal(std)),
+                "a2": TensorSpec((H * self.dim, self.rank), VECTOR, Normal(0.25)),   # 32-bit: it makes decays of 32-bit sums
+                "a2.b": TensorSpec((H * self.dim,), VECTOR, Normal(1.0, mean=1.0)),
+                "norm": TensorSpec((self.vdim,), VECTOR, Normal(0.1, mean=1.0)),
+                "o": TensorSpec((self.width, H * self.vdim), TABLE, Normal((H * self.vdim) ** -0.5))}
+
+    def bind(self, tensors):
+        self.rank = tensors["a1"].shape[0]
+        fused = fuse_rows([tensors[name] for name in ("q", "k", "v", "g", "a1")])
+        on_gpu = fused.is_cuda
+        self.w_in = kernels.pack_matrix(fused) if on_gpu else fused
+        self.o = kernels.pack_matrix(tensors["o"].contiguous()) if on_gpu else tensors["o"]
+        self.decay_up, self.decay_bias, self.norm = tensors["a2"].t().contiguous(), tensors["a2.b"], tensors["norm"]
+
+    def state_need(self):
+        return StateNeed((self.n_heads * self.dim * self.vdim,), torch.float32)
+
+    def forward(self, x, residual, ctx: LayerContext):
+        """The branch alone (float32) when ``residual`` is None, else residual + branch."""
+        batch, H = ctx.batch, self.n_heads
+        _whole_batch(batch)
+        fused = kernels.linear(x, self.w_in, out_dtype=torch.float32)
+        qw, vw = H * self.dim, H * self.vdim
+        mixed = kernels.channel_memory(fused, 0, qw, 2 * qw, 2 * qw + vw, 2 * qw + 2 * vw, self.decay_up, self.decay_bias, ctx.state, batch.q_starts,
+                                       batch.state_slots, H, self.dim, self.vdim, tau=self.tau, q_scale=self.dim ** -0.5, gain=self.norm, eps=self.eps,
+                                       out_dtype=x.dtype, max_q_len=batch.max_q_len)
+        if residual is None and self.sums_later:
+            return self._out_product.later(mixed, self.o)
+        return self._out_product(mixed, self.o, residual)
+
+
 class MinGRUMixer(Mixer):
     graph_safe = True
 
@@ -226,5 +279,6 @@ class ParallelMixer(Mixer):
 
 register_part("mixer", "matrix_memory", MatrixMemoryMixer)
 register_part("mixer", "decayed_linear_attention", DecayedLinearAttention)
+register_part("mixer", "gated_linear_attention", GatedLinearAttention)
 register_part("mixer", "mingru", MinGRUMixer)
 register_part("mixer", "parallel", ParallelMixer)

@@ -12,7 +12,7 @@ Other designs' forms: ``score`` "sigmoid" takes s = sigmoid(z), each expert's ow
 ``correction`` False picks by the scores; ``unit`` "clamped_gate" gives an expert a gate matrix beside its up matrix (stored ``gate``, ``up``,
 ``down``) and the unit g * sigmoid(alpha g) * (u + shift), g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit), in place of the squared
 relu; ``weigh`` "input" multiplies an expert's input by its weight instead of its output (the same thing only for linear experts): the
-gate unit then takes the weight times the sums.
+gate unit then takes the weight times the sums. Without a limit, with alpha 1 and shift 0, the unit is silu(g) u.
 
 Experts of the plain form: all run as ONE up product over their matrices laid behind each other (the shared expert's last) and ONE down product over their
 down matrices laid side by side: ``kernels.expert_unit`` between the two multiplies every hidden unit by its expert's weight for the
@@ -22,7 +22,8 @@ on the host, and a captured step replays it. The price is the arithmetic of the 
 work in the two products, which few rows (decoding) do not notice, since they read every expert's matrices anyway.
 
 Experts with a gate unit run grouped instead: each expert for the rows that picked it alone (``kernels.grouped_experts``), planned on the
-device."""
+device. A shared expert of theirs (its hidden units are a sum like any other) is laid out as so many experts of the others' size as
+hold its units, which every row picks behind its own picks, with weight 1."""
 
 from __future__ import annotations
 
@@ -40,8 +41,10 @@ class RoutedExperts(FeedForward):
                  unit: str = "squared_relu", limit: float | None = None, alpha: float = 1.0, shift: float = 0.0, weigh: str = "output"):
         if score not in ("softmax", "sigmoid") or unit not in ("squared_relu", "clamped_gate") or weigh not in ("output", "input"):
             raise ValueError(f"unknown score {score!r}, unit {unit!r} or weigh {weigh!r}")
-        if unit == "clamped_gate" and (n_identity or shared_ff or n_experts < 1):
-            raise ValueError("experts with a gate unit go without shared experts and without experts that hand their input on")
+        if unit == "clamped_gate" and (n_identity or n_experts < 1):
+            raise ValueError("experts with a gate unit go without experts that hand their input on")
+        if unit == "clamped_gate" and shared_ff and weigh == "input":
+            raise ValueError("a shared expert beside experts whose input is weighed is not laid out")
         if unit != "clamped_gate" and (limit is not None or weigh == "input"):
             raise ValueError("a limit and weights on the input go with experts that have a gate unit")
         if limit is not None and not limit > 0:
@@ -59,7 +62,10 @@ class RoutedExperts(FeedForward):
         self.score, self.renormalise, self.weigh_input = score, bool(renormalise), weigh == "input"
         self.gated, self.limit, self.alpha, self.shift = unit == "clamped_gate", limit, float(alpha), float(shift)
         self.router = self.correction = self.up = self.down = self._router_rows = self._small_router = None
-        self.units = ff
+        self.units = -(-ff // kernels.EXPERT_UNITS) * kernels.EXPERT_UNITS if self.gated else ff
+        self.shared_parts = -(-self.shared_ff // self.units) if self.gated else 0   # experts the shared one is laid out as
+        if total + self.shared_parts > kernels.ROUTE_MAX_EXPERTS:
+            raise ValueError(f"{total} experts and a shared one of {self.shared_parts} times their size are more than {kernels.ROUTE_MAX_EXPERTS}")
         self.shared_units = 0   # the shared expert's hidden units and the zeros that fill the up matrix to whole blocks
         self._down_product = BranchProduct()
         self.sums_later = False   # True: a call without a residual may return kernels.BranchRows (the block that adds the branch takes its sums)
@@ -105,21 +111,22 @@ class RoutedExperts(FeedForward):
     def _bind_gated(self, tensors, names):
         """The layout ``kernels.grouped_experts`` reads: 32 gate rows and 32 up rows in turn, units and the down matrices' rows filled up with zeros."""
         sample = tensors[names[0] + "up"]
-        E, width, rows = self.n_experts, self.width, kernels.expert_down_rows(self.width)
-        units = self.units = -(-self.ff // kernels.EXPERT_UNITS) * kernels.EXPERT_UNITS
+        E, width, rows, units = self.n_experts + self.shared_parts, self.width, kernels.expert_down_rows(self.width), self.units
         up = torch.zeros((E, units // 32, 2, 32, width), dtype=sample.dtype, device=sample.device)
         down = torch.zeros((E, rows, units), dtype=sample.dtype, device=sample.device)
-        for e, name in enumerate(names):
+        places = [(e, f"e{e}.", 0, self.ff) for e in range(self.n_experts)]   # (expert, its tensors, the units it takes of them)
+        places += [(self.n_experts + i, "shared.", i * units, min(self.shared_ff, (i + 1) * units)) for i in range(self.shared_parts)]
+        for e, name, first, last in places:
             for half, part in enumerate(("gate", "up")):
                 padded = torch.zeros((units, width), dtype=sample.dtype, device=sample.device)
-                padded[: self.ff] = tensors[name + part]
+                padded[: last - first] = tensors[name + part][first:last]
                 up[e, :, half] = padded.view(units // 32, 32, width)
-            down[e, :width, : self.ff] = tensors[name + "down"]
+            down[e, :width, : last - first] = tensors[name + "down"][:, first:last]
         up, down = up.view(E * 2 * units, width), down.view(E * rows, units)
         self.up, self.down = (kernels.pack_matrix(up), kernels.pack_matrix(down)) if up.is_cuda else (up, down)
 
     def _forward_gated(self, x, carried, residual):
-        planes = kernels.grouped_experts(x, self._route(x, carried, picks=True), self.up, self.down, self.n_experts, self.units, limit=self.limit, alpha=self.alpha,
+        planes = kernels.grouped_experts(x, self._route(x, carried, picks=True), self.up, self.down, self.n_experts + self.shared_parts, self.units, limit=self.limit, alpha=self.alpha,
                                          shift=self.shift, weigh_input=self.weigh_input)
         if residual is not None:
             if self.width % 4 == 0:
@@ -129,13 +136,13 @@ class RoutedExperts(FeedForward):
             return residual
         if self.sums_later:
             return kernels.BranchRows(planes, None)
-        return planes[0] if self.top == 1 else planes   # several picks: partial sums, as a product cut along K leaves them
+        return planes[0] if planes.shape[0] == 1 else planes   # several picks: partial sums, as a product cut along K leaves them
 
     def _route(self, x, carried=None, picks: bool = False):
         """The router's sums (its product inside the choice's kernel where that takes it, or its own, or what another product carried along)
         and its choice."""
         how = dict(correction=self.correction, n_groups=self.n_groups, keep=self.keep, floor=self.floor, score=self.score, renormalise=self.renormalise,
-                   picks=picks)
+                   picks=picks, always=self.shared_parts)
         if carried is None and self._small_router is not None:
             return kernels.route_rows(x, self._small_router, self.top, **how)
         logits = carried if carried is not None else kernels.linear(x, self.router, out_dtype=torch.float32)

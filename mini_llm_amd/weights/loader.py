@@ -12,7 +12,7 @@ from pathlib import Path
 import torch
 
 from .safetensors_io import SafetensorsError, SafetensorsFile
-from .spec import INT_TABLE, MATRIX, TABLE, VECTOR, TensorSpec
+from .spec import INT_TABLE, MATRIX, TABLE, VECTOR, FreeDim, TensorSpec
 
 WEIGHTS_FILE = "model.safetensors"
 
@@ -34,6 +34,18 @@ class WeightsError(ValueError):
         super().__init__("\n".join(lines))
 
 
+def _fits(shape, wanted, settled: dict) -> bool:
+    if len(shape) != len(wanted):
+        return False
+    for have, want in zip(shape, wanted):
+        if isinstance(want, FreeDim):
+            if have < 1 or settled.setdefault(id(want), have) != have:
+                return False
+        elif have != want:
+            return False
+    return True
+
+
 def check_names(where, expected: dict, found: dict, canonical) -> dict:
     """expected: name -> TensorSpec; found: name in file -> (shape, is_float). Returns
     name -> name in file, or raises one WeightsError with all problems."""
@@ -50,10 +62,11 @@ def check_names(where, expected: dict, found: dict, canonical) -> dict:
             mapping[name] = file_name
     missing = [n for n in expected if n not in mapping]
     wrong = []
+    settled = {}   # FreeDim object -> the number the first tensor that has it brings
     for name, file_name in mapping.items():
         shape, is_float = found[file_name]
         spec = expected[name]
-        if tuple(shape) != tuple(spec.shape):
+        if not _fits(shape, spec.shape, settled):
             wrong.append((file_name, tuple(shape), tuple(spec.shape)))
         elif (spec.role == INT_TABLE) == is_float:
             other.append(f"{file_name} holds {'floats' if is_float else 'integers'}, which a {spec.role} cannot be")

@@ -10,6 +10,11 @@ VECTOR = "vector"        # bias / norm gain / norm offset: kept in 32-bit
 INT_TABLE = "int_table"  # integer table: kept as int32
 
 
+class FreeDim(int):
+    """A dimension that no configuration gives: the file's tensors do. The number itself is what a randomly drawn model takes; a file
+    may bring any other (at least 1), the same one wherever a part names the same FreeDim object."""
+
+
 @dataclass(frozen=True)
 class Normal:
     """Draw from N(mean, std)."""
@@ -20,7 +25,7 @@ class Normal:
 
 @dataclass(frozen=True)
 class TensorSpec:
-    shape: tuple  # as stored in the file
+    shape: tuple  # as stored in the file (a dimension may be a FreeDim)
     role: str
     init: Normal
     # Stored [in, out] (the Conv1D layout of GPT-2 files); kept transposed, [out, in], which is

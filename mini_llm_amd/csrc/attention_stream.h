@@ -160,7 +160,9 @@ struct Layout {
 // without a block: what the kernel waits for is the wave with the most tiles, and a tile of 32 queries takes it half as long.
 // SPLITS: four waves a block, or eight where the portions reach far back: the kernel's time is the time of the wave with
 // the most tiles (it pays every tile's chain in full), which eight waves halve; a block then has a compute unit to itself.
-template <typename T, int HD, int QUERIES, int SPLITS>
+// KEPT: a window with kept first keys (ScoreOptions). A kernel of its own: the fragments of the next tile sit in registers that nothing may copy
+// until they have landed, so the kernel without kept keys carries nothing for them.
+template <typename T, int HD, int QUERIES, int SPLITS, bool KEPT>
 __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4) ? 2 : 1) void attention_prefill_stream_kernel(
     const T* __restrict__ q, int q_stride, const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     T* __restrict__ out, int out_stride, const int* __restrict__ q_starts, const int* __restrict__ context_lens,
@@ -208,7 +210,7 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
     const int block_first_key = first_visible_key(context + tile_q0, window, options.chunk);
     const int first_base = (block_first_key / KEYS) * KEYS;
     // with kept first keys: the tiles that hold them come first, the tiles between them and the window are passed over
-    const int kept_tiles = min((options.keep + KEYS - 1) / KEYS, first_base / KEYS);
+    const int kept_tiles = KEPT ? min((options.keep + KEYS - 1) / KEYS, first_base / KEYS) : 0;
     const int n_tiles = kept_tiles + (block_last_position - first_base) / KEYS + 1;
     const int n_mine = n_tiles > wave ? (n_tiles - wave + SPLITS - 1) / SPLITS : 0;  // tiles wave, wave + SPLITS, ...
 
@@ -218,7 +220,7 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
     unsigned char* const wave_lds = lds + wave * L::WAVE_BYTES;
     auto tile_base = [&](int i) {
         const int tile = wave + SPLITS * min(i, n_mine - 1);
-        return tile < kept_tiles ? tile * KEYS : first_base + (tile - kept_tiles) * KEYS;
+        return KEPT && tile < kept_tiles ? tile * KEYS : first_base + (tile - kept_tiles) * KEYS;
     };
     // a lane's place among the rows of a whole tile, in bytes: the same for every tile, so an address is a base all lanes
     // share plus this (worked out anew for every load it was a sixth of the loop's vector instructions)
@@ -322,7 +324,7 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
 
     auto tile = [&](int i, f32x16 (&s_acc)[QSUB], f32x16 (&s_next)[QSUB]) {
         const int page_next = table[tile_base(i + 4) >> page_shift];
-        const int k0 = tile_base(i);
+        const int k0 = KEPT ? tile_base(i) : first_base + (wave + SPLITS * i) * KEYS;
         const unsigned char* v_tile = wave_lds + 2 * L::TILE_BYTES + (i % 2) * L::TILE_BYTES;
         const unsigned char* k_next = wave_lds + ((i + 1) % 2) * L::TILE_BYTES;
         bf16x8 p[QSUB][2];  // the probabilities of a sub-tile of queries, as the second product's operand: keys 0-15 and 16-31 of the tile
@@ -352,22 +354,12 @@ __global__ __launch_bounds__(64 * SPLITS, (HD * sizeof(T) <= 128 && SPLITS == 4)
             } else {
                 const int first_allowed = q_position[qs] < 0 ? 0 : first_visible_key(q_position[qs], window, options.chunk);
                 const int key0 = k0 + 4 * half;
-                if (k0 < options.keep) {   // a tile that holds kept keys (the same for all lanes)
 #pragma unroll
-                    for (int v = 0; v < 16; v++) {
-                        const int key = key0 + 8 * (v / 4) + (v % 4);
-                        const bool allowed = (key <= q_position[qs]) & ((key >= first_allowed) | (key < options.keep));
-                        s_acc[qs][v] = allowed ? s_acc[qs][v] : -INFINITY;
-                        tile_max = fmaxf(tile_max, s_acc[qs][v]);
-                    }
-                } else {
-#pragma unroll
-                    for (int v = 0; v < 16; v++) {
-                        const int key = key0 + 8 * (v / 4) + (v % 4);
-                        const bool allowed = (key <= q_position[qs]) & (key >= first_allowed);
-                        s_acc[qs][v] = allowed ? s_acc[qs][v] : -INFINITY;
-                        tile_max = fmaxf(tile_max, s_acc[qs][v]);
-                    }
+                for (int v = 0; v < 16; v++) {
+                    const int key = key0 + 8 * (v / 4) + (v % 4);
+                    const bool allowed = (key <= q_position[qs]) & ((key >= first_allowed) | (KEPT && key < options.keep));
+                    s_acc[qs][v] = allowed ? s_acc[qs][v] : -INFINITY;
+                    tile_max = fmaxf(tile_max, s_acc[qs][v]);
                 }
             }
             tile_max = fmaxf(tile_max, __shfl_xor(tile_max, 32, WAVE)) * score_scale;
@@ -537,20 +529,33 @@ inline bool takes(int head_size, int page_size, int max_q_len, float scale, int 
     return (q_stride * sizeof(T)) % 16 == 0 && (out_stride * sizeof(T)) % (4 * sizeof(T)) == 0 && ((size_t)q) % 16 == 0 && ((size_t)out) % (4 * sizeof(T)) == 0;
 }
 
-template <typename T, int HD, int QUERIES, int SPLITS>
-void launch_queries(const void* q, int q_stride, const void* k_pages, const void* v_pages, void* out, int out_stride, const int* q_starts,
+template <typename T, int HD, int QUERIES, int SPLITS, bool KEPT>
+void launch_with(const void* q, int q_stride, const void* k_pages, const void* v_pages, void* out, int out_stride, const int* q_starts,
                     const int* context_lens, const int* block_tables, int max_blocks, int n_requests, int max_q_len, int n_heads, int n_kv_heads,
                     int page_shift, int window, float scale, ScoreOptions options, hipStream_t stream) {
     constexpr int LDS_BYTES = Layout<T, HD, SPLITS>::LDS_BYTES;
     static bool raised = false;  // per instantiation: the limit on dynamic LDS is a property of the kernel
     if (!raised && LDS_BYTES > 60 * 1024)  // (if this fails the launch below fails too, and the entry point reports that)
-        raised = hipFuncSetAttribute((const void*)attention_prefill_stream_kernel<T, HD, QUERIES, SPLITS>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS_BYTES) == hipSuccess;
+        raised = hipFuncSetAttribute((const void*)attention_prefill_stream_kernel<T, HD, QUERIES, SPLITS, KEPT>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS_BYTES) == hipSuccess;
     // x: (request, head), so that with a multiple of eight heads the blocks of one head share an XCD's L2; y: tiles of queries
     dim3 grid(n_heads * n_requests, ceil_div(max_q_len, QUERIES));
     mllm_count_kernel(MLLM_K_ATTENTION_PREFILL_STREAM);
-    attention_prefill_stream_kernel<T, HD, QUERIES, SPLITS><<<grid, 64 * SPLITS, LDS_BYTES, stream>>>(
+    attention_prefill_stream_kernel<T, HD, QUERIES, SPLITS, KEPT><<<grid, 64 * SPLITS, LDS_BYTES, stream>>>(
         (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, (T*)out, out_stride, q_starts, context_lens,
         block_tables, max_blocks, n_heads, n_kv_heads, page_shift, window, scale, options);
+}
+
+template <typename T, int HD, int QUERIES, int SPLITS>
+void launch_queries(const void* q, int q_stride, const void* k_pages, const void* v_pages, void* out, int out_stride, const int* q_starts,
+                    const int* context_lens, const int* block_tables, int max_blocks, int n_requests, int max_q_len, int n_heads, int n_kv_heads,
+                    int page_shift, int window, float scale, ScoreOptions options, hipStream_t stream) {
+#define MLLM_STREAM_WITH(QUERIES, KEPT)                                                                                                        \
+    launch_with<T, HD, QUERIES, SPLITS, KEPT>(q, q_stride, k_pages, v_pages, out, out_stride, q_starts, context_lens, block_tables, max_blocks, \
+                                              n_requests, max_q_len, n_heads, n_kv_heads, page_shift, window, scale, options, stream)
+    constexpr int KEPT_QUERIES = HD * sizeof(T) > 128 ? 32 : QUERIES;   // (rows of 256 bytes with 64 queries leave no register for the second mask)
+    if (options.keep > 0) MLLM_STREAM_WITH(KEPT_QUERIES, true);
+    else MLLM_STREAM_WITH(QUERIES, false);
+#undef MLLM_STREAM_WITH
 }
 
 template <typename T, int HD>

@@ -1,6 +1,8 @@
 """Helpers for the replay tests: traces in the four ways of cutting the work, a driver for
 bin/trace_run, and the plain implementation's logits to compare with."""
 
+import gc
+import io
 import json
 import subprocess
 import sys
@@ -25,11 +27,11 @@ def tolerance(dtype: str) -> dict:
     return F32_TOL if dtype == "float32" else BF16_TOL
 
 
-def run_trace(model_dir, dtype, steps, out_dir, max_tokens, page_size=None, timeout=600, hidden_out=None):
-    """Runs bin/trace_run over the steps; returns {step: array [wanted, vocab]}."""
+def run_trace(model_dir, dtype, steps, out_dir, max_tokens, page_size=None, timeout=600, hidden_out=None, own_process=False):
+    """Runs the trace runner over the steps; returns {step: array [wanted, vocab]}. Its program is called in this process (a process
+    of its own, ``own_process``, takes seconds to start); what it makes is given back when it returns."""
     out_dir = Path(out_dir)
-    cmd = [sys.executable, str(ROOT / "bin" / "trace_run"), "--model", str(model_dir), "--dtype", dtype,
-           "--out", str(out_dir), "--max-tokens", str(max_tokens)]
+    cmd = ["--model", str(model_dir), "--dtype", dtype, "--out", str(out_dir), "--max-tokens", str(max_tokens)]
     live, most = set(), 4   # state slots: as many as requests are live at once (the runner's own default is four)
     for s in steps:
         live |= {e["id"] for e in s["entries"]}
@@ -41,10 +43,19 @@ def run_trace(model_dir, dtype, steps, out_dir, max_tokens, page_size=None, time
         cmd += ["--page-size", str(page_size)]
     if hidden_out:
         cmd += ["--hidden-out", str(hidden_out)]
-    text = "".join(json.dumps(s) + "\n" for s in steps)
-    done = subprocess.run(cmd, input=text, capture_output=True, text=True, timeout=timeout)
-    assert done.returncode == 0, f"trace_run failed ({done.returncode}):\n{done.stderr[-3000:]}"
-    assert [l for l in done.stdout.split("\n") if l.startswith("done")] == [f"done {s['step']}" for s in steps]
+    lines = [json.dumps(s) + "\n" for s in steps]
+    if own_process:
+        done = subprocess.run([sys.executable, str(ROOT / "bin" / "trace_run"), *cmd], input="".join(lines), capture_output=True, text=True, timeout=timeout)
+        assert done.returncode == 0, f"trace_run failed ({done.returncode}):\n{done.stderr[-3000:]}"
+        said = done.stdout
+    else:
+        from mini_llm_amd.cli.trace_run import main
+
+        out = io.StringIO()
+        assert main(cmd, steps=lines, out=out) == 0
+        said = out.getvalue()
+        gc.collect()   # captured steps and their runner refer to each other
+    assert [l for l in said.split("\n") if l.startswith("done")] == [f"done {s['step']}" for s in steps]
     config = json.loads((Path(model_dir) / "config.json").read_text())
     vocab = config["vocab_size"] if "vocab_size" in config else config["vocab"]
     out = {}

@@ -341,8 +341,8 @@ _KERNEL_CLASSES = {
     "attention": ("attention", "attention_decode", "attention_prefill", "latent_attention", "latent_attention_mfma"),
     "row-wise": ("layernorm", "pending_layernorm", "rms_norm", "head_norm", "latent_rows", "silu_mul", "pending_sum", "add", "cache_write", "embed",
                  "projection_rows", "head_gate", "gated_norm", "short_conv", "map_rows", "map_difference", "turn_heads", "gate_unit", "route", "route_rows", "expert_unit", "expert_lists",
-                 "branch_join"),
-    "recurrence": ("recurrence", "gated_scan"),
+                 "branch_join", "join_norms", "soft_cap"),
+    "recurrence": ("recurrence", "recurrence_chunked", "gated_scan", "channel_memory"),
     "layer kernels": ("decode_attention_half", "decode_mlp_half"),
     "choice": ("choose", "sample"),
 }
@@ -442,9 +442,30 @@ def goletar_shape(width: int, layers: int, vocab: int = 50257) -> dict:
                        for index in range(layers)]}
 
 
+def gevulorn_shape(width: int, layers: int, vocab: int = 50257) -> dict:
+    """Layers in fours: gated linear attention (width / 128 heads of 64 x 128, decays of rank 16), attention with queries and keys of unit size
+    over a window of 512 that keeps the first 64 keys, gated linear attention, attention with biases, normed queries and keys and capped
+    scores inside chunks of 512 (heads of 64, a key/value head for every four, all of a head rotated); the first and third with a dense
+    feed-forward of 4 x width (square of relu), the second and fourth with eight routed experts of 2/3 x width, two picked, and a shared one
+    of 4/3 x width (as many multiply-adds a token, for the picked experts). All layers are one pass of a loop, so that a vector joins the stream."""
+    heads, wide_heads = width // 64, max(1, width // 128)
+    dense = {"kind": "dense", "ff": 4 * width}
+    small = -(-(2 * width // 3) // 64) * 64
+    routed = {"kind": "moe", "expert": {"ff": small}, "shared": {"ff": 2 * small}, "router": {"experts": 8, "top": 2}}
+    common = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 64, "vdim": 64, "scale": 0.125}
+    memory = {"type": "gla", "mlp": dense, "mixer": {"heads": wide_heads, "dim": 64, "vdim": 128, "tau": 16.0}}
+    window = {"type": "attention", "mlp": routed, "mixer": {**common, "mask": {"size": 512, "keep_first": 64}, "rot": {"dims": 64, "base": 500000.0}}}
+    scaling = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 512}
+    chunks = {"type": "attention_2", "mlp": routed, "mixer": {**common, "mask": {"size": 512}, "softcap": 30.0, "rot": {"dims": 64, "base": 500000.0, "scaling": scaling}}}
+    pattern = [memory, window, memory, chunks]
+    return {"architecture": "Gevulorn", "vocab": vocab, "width": width, "embedding": {"scale": width ** 0.5}, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "loop": {"start": 0, "stop": layers, "times": 1}, "layers": [pattern[i % 4] for i in range(layers)]}
+
+
 def measure_design(args) -> dict:
     """Prefill and decode throughput of a design and of the framework's closest older model with as many layers of the same width
-    (random weights): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen, Goletar beside Dizizen (routed experts) and Gimozen (latent attention); and where each model's step spends its time, by class of
+    (random weights): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen, Goletar beside Dizizen (routed experts) and Gimozen (latent attention), Gevulorn
+    beside Dizizen (branches side by side, rotated attention, experts) and Ketolix (a matrix memory, windows); and where each model's step spends its time, by class of
     kernel, inside a prompt step and a decode step."""
     import numpy as np
     import torch
@@ -454,7 +475,9 @@ def measure_design(args) -> dict:
     from mini_llm_amd.engine.engine import Engine, EngineOptions
 
     width, layers = DESIGN_SIZES[args.shape]
-    if args.design == "goletar":
+    if args.design == "gevulorn":
+        raws = {"gevulorn": gevulorn_shape(width, layers), "dizizen": dizizen_shape(width, layers), "ketolix": ketolix_shape(width, layers)}
+    elif args.design == "goletar":
         raws = {"goletar": goletar_shape(width, layers), "dizizen": dizizen_shape(width, layers), "gimozen": gimozen_shape(width, layers)}
     elif args.design == "dizizen":
         raws = {"dizizen": dizizen_shape(width, layers), "gimozen": gimozen_shape(width, layers)}
@@ -725,8 +748,8 @@ def main() -> int:
     parser.add_argument("--serving", action="store_true", help="continuous batching of 64 requests on the GPT-2 medium shape through the scheduler")
     parser.add_argument("--temperature", type=float, default=0.0, help="sampling temperature of --serving (0: greedy)")
     parser.add_argument("--step-by-step", action="store_true", help="--serving reads every step's tokens before it launches the next")
-    parser.add_argument("--design", default=None, choices=("gimozen", "ketolix", "perezen", "dizizen", "goletar"), help="a design beside the closest older model with as many layers of the same width "
-                        "(--shape small|medium): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen, Goletar beside Dizizen and Gimozen; prefill and decode throughput of both, and where their steps spend the time")
+    parser.add_argument("--design", default=None, choices=("gimozen", "ketolix", "perezen", "dizizen", "goletar", "gevulorn"), help="a design beside the closest older model with as many layers of the same width "
+                        "(--shape small|medium): Gimozen beside GPT-2, Ketolix beside Gimozen, Perezen beside Ketolix, Dizizen beside Gimozen, Goletar beside Dizizen and Gimozen, Gevulorn beside Dizizen and Ketolix; prefill and decode throughput of both, and where their steps spend the time")
     parser.add_argument("--peaks", action="store_true", help="measure this machine's read bandwidth and matrix-core rate with the library's probes")
     args = parser.parse_args()
     if args.gpus != 1:

@@ -66,30 +66,34 @@ __global__ __launch_bounds__(THREADS) void memory_rows_kernel(MemoryRows op, flo
     for (int r = 0; r < R; r++) S[r] = column && i0 + r < dim ? S_at[(size_t)(i0 + r) * vdim + j] : 0.0f;
     for (int t0 = 0; t0 < rows; t0 += TB) {
         const int n_valid = min(TB, rows - t0);
-        for (int e = tid; e < n_valid * dim_pad; e += blockDim.x) {
-            const int t = e / dim_pad, i = e % dim_pad;
-            const float* row = op.rows + (size_t)(first_row + t0 + t) * op.stride;
-            float qv = 0.0f, kv = 0.0f, decay = 0.0f;
-            if (i < dim) {
-                const int channel = head * dim + i;
-                qv = row[op.q_at + channel] * op.q_scale;
-                kv = row[op.k_at + channel];
+        // an element of the values and one of the channels a thread: all of an element's loads are under way before the first is used
+        for (int e = tid; e < n_valid * max(dim_pad, VT); e += blockDim.x) {
+            const bool is_value = e < n_valid * VT, is_channel = e < n_valid * dim_pad;
+            float value = 0.0f, gate = 0.0f, gain = 0.0f;
+            if (is_value) {
+                const int t = e / VT, c = min(j0 + e % VT, vdim - 1);
+                const float* row = op.rows + (size_t)(first_row + t0 + t) * op.stride + head * vdim + c;
+                value = row[op.v_at];
+                if (NORMS) gate = row[op.g_at], gain = op.gain[c];
+            }
+            if (is_channel) {
+                const int t = e / dim_pad, i = e % dim_pad, channel = head * dim + min(i, dim - 1);
+                const float* row = op.rows + (size_t)(first_row + t0 + t) * op.stride;
+                const float qv = row[op.q_at + channel] * op.q_scale, kv = row[op.k_at + channel];
                 float z = op.bias[channel];
                 const float* low = row + op.low_at;
                 const float* up = op.up + channel;
-#pragma unroll 8
+#pragma unroll 16
                 for (int r = 0; r < op.rank; r++) z = __builtin_fmaf(low[r], up[(size_t)r * n_heads * dim], z);
-                decay = exp2_of(log2_decay(z, op.inverse_tau));
+                const bool counts = i < dim;
+                sq[e] = counts ? qv : 0.0f;
+                sk[e] = counts ? kv : 0.0f;
+                sa[e] = counts ? exp2_of(log2_decay(z, op.inverse_tau)) : 0.0f;
             }
-            sq[e] = qv;
-            sk[e] = kv;
-            sa[e] = decay;
-        }
-        for (int e = tid; e < n_valid * VT; e += blockDim.x) {
-            const int t = e / VT, c = j0 + e % VT;
-            const float* row = op.rows + (size_t)(first_row + t0 + t) * op.stride;
-            sv[e] = c < vdim ? row[op.v_at + head * vdim + c] : 0.0f;
-            if (NORMS) sg[e] = op.gain[c] * silu_of(row[op.g_at + head * vdim + c]);   // (VT is vdim then)
+            if (is_value) {
+                sv[e] = j0 + e % VT < vdim ? value : 0.0f;
+                if (NORMS) sg[e] = gain * silu_of(gate);
+            }
         }
         __syncthreads();
         if (works) {
@@ -191,12 +195,34 @@ struct Chunk {
 __device__ __forceinline__ size_t record_of(int first_row, int chunk_rows, int request) { return (size_t)(first_row / chunk_rows + request); }
 __device__ __forceinline__ f32x4 multiply_add(float a, float b, f32x4 sums) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, sums, 0, 0, 0); }
 
-// The log decays of a chunk's rows for one head into la[s * la_stride + i] (0 beyond n_valid rows and dim channels); `low` [L][16] holds 16 of
-// the rank at a time. A lane a channel, a wave every eighth row. Ends with a barrier.
+// What a thread needs of 16 of the decays' rank, asked for at once (from clamped places), early in a kernel.
 template <int L, int DPT>
-__device__ __forceinline__ void chunk_decays(const MemoryRows& op, int chunk_first, int n_valid, int head, int n_heads, float* la, int la_stride, float* low) {
+struct DecayPiece {
     using C = Chunk<L, DPT>;
-    const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE, columns = n_heads * op.dim;
+    static constexpr int LOWS = L * 16 / THREADS;
+    float w[C::CB][16], low[LOWS];
+    __device__ __forceinline__ void ask(const MemoryRows& op, int chunk_first, int n_valid, int head, int n_heads, int r0) {
+        const int tid = threadIdx.x, lane = tid % WAVE, columns = n_heads * op.dim;
+#pragma unroll
+        for (int u = 0; u < LOWS; u++) {
+            const int e = tid + u * THREADS, r = r0 + e % 16;
+            low[u] = op.rows[(size_t)(chunk_first + min(e / 16, n_valid - 1)) * op.stride + op.low_at + min(r, op.rank - 1)];
+            if (r >= op.rank) low[u] = 0.0f;
+        }
+#pragma unroll
+        for (int cb = 0; cb < C::CB; cb++)
+#pragma unroll
+            for (int r = 0; r < 16; r++) w[cb][r] = op.up[(size_t)min(r0 + r, op.rank - 1) * columns + head * op.dim + min(cb * WAVE + lane, op.dim - 1)];
+    }
+};
+
+// The log decays of a chunk's rows for one head into la[s * la_stride + i] (0 beyond n_valid rows and dim channels); `low` [L][16] holds 16 of
+// the rank at a time, `piece` brings the first. A lane a channel, a wave every eighth row. Ends with a barrier.
+template <int L, int DPT>
+__device__ __forceinline__ void chunk_decays(const MemoryRows& op, DecayPiece<L, DPT>& piece, int chunk_first, int n_valid, int head, int n_heads, float* la, int la_stride,
+                                             float* low) {
+    using C = Chunk<L, DPT>;
+    const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
     float z[C::CB][C::RPW];
 #pragma unroll
     for (int cb = 0; cb < C::CB; cb++) {
@@ -205,16 +231,12 @@ __device__ __forceinline__ void chunk_decays(const MemoryRows& op, int chunk_fir
         for (int u = 0; u < C::RPW; u++) z[cb][u] = bias;
     }
     for (int r0 = 0; r0 < op.rank; r0 += 16) {
-        float w[C::CB][16];
-#pragma unroll
-        for (int cb = 0; cb < C::CB; cb++)
-#pragma unroll
-            for (int r = 0; r < 16; r++) w[cb][r] = op.up[(size_t)min(r0 + r, op.rank - 1) * columns + head * op.dim + min(cb * WAVE + lane, op.dim - 1)];
-        if (r0 > 0) __syncthreads();
-        for (int e = tid; e < L * 16; e += THREADS) {
-            const int s = e / 16, r = r0 + e % 16;
-            low[e] = s < n_valid && r < op.rank ? op.rows[(size_t)(chunk_first + s) * op.stride + op.low_at + r] : 0.0f;
+        if (r0 > 0) {
+            piece.ask(op, chunk_first, n_valid, head, n_heads, r0);
+            __syncthreads();
         }
+#pragma unroll
+        for (int u = 0; u < DecayPiece<L, DPT>::LOWS; u++) low[tid + u * THREADS] = piece.low[u];
         __syncthreads();
 #pragma unroll
         for (int u = 0; u < C::RPW; u++) {
@@ -225,7 +247,7 @@ __device__ __forceinline__ void chunk_decays(const MemoryRows& op, int chunk_fir
 #pragma unroll
                 for (int cb = 0; cb < C::CB; cb++)
 #pragma unroll
-                    for (int e = 0; e < 4; e++) z[cb][u] = __builtin_fmaf(four[e], w[cb][r4 * 4 + e], z[cb][u]);
+                    for (int e = 0; e < 4; e++) z[cb][u] = __builtin_fmaf(four[e], piece.w[cb][r4 * 4 + e], z[cb][u]);
             }
         }
     }
@@ -269,13 +291,16 @@ __global__ __launch_bounds__(THREADS) void memory_sums_kernel(MemoryRows op, flo
         keys[s] = op.rows[(size_t)(chunk_first + row) * op.stride + op.k_at + head * dim + min(i, dim - 1)];
     }
     constexpr int VPER = L * SUM_TILE / THREADS;
+    const int column = tile * SUM_TILE + lane;
+    float values[VPER];
 #pragma unroll
-    for (int u = 0; u < VPER; u++) {
-        const int s = wave + u * WAVES, c = tile * SUM_TILE + lane;
-        const float value = op.rows[(size_t)(chunk_first + min(s, n_valid - 1)) * op.stride + op.v_at + head * vdim + min(c, vdim - 1)];
-        V[s * VS + lane] = s < n_valid && c < vdim ? value : 0.0f;
-    }
-    chunk_decays<L, DPT>(op, chunk_first, n_valid, head, n_heads, K, KS, low);
+    for (int u = 0; u < VPER; u++)
+        values[u] = op.rows[(size_t)(chunk_first + min(wave + u * WAVES, n_valid - 1)) * op.stride + op.v_at + head * vdim + min(column, vdim - 1)];
+    DecayPiece<L, DPT> piece;
+    piece.ask(op, chunk_first, n_valid, head, n_heads, 0);
+    chunk_decays<L, DPT>(op, piece, chunk_first, n_valid, head, n_heads, K, KS, low);
+#pragma unroll
+    for (int u = 0; u < VPER; u++) V[(wave + u * WAVES) * VS + lane] = wave + u * WAVES < n_valid && column < vdim ? values[u] : 0.0f;
     float la[SUB];
     if (works) {
         float sum = 0.0f;
@@ -300,10 +325,10 @@ __global__ __launch_bounds__(THREADS) void memory_sums_kernel(MemoryRows op, flo
     __syncthreads();
     // U = (faded keys)^T V: a wave 16 columns j, every second tile of 16 channels i
     const int l16 = lane % 16, quad = lane / 16, jt = wave % 4;
-    const int steps = ceil_div(n_valid, 4);
     for (int it = wave / 4; it < DPT; it += 2) {
         f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
-        for (int step = 0; step < steps; step++) {
+#pragma unroll
+        for (int step = 0; step < L / 4; step++) {   // (rows beyond the chunk's are zeros)
             const int s = step * 4 + quad;
             acc = multiply_add(K[s * KS + it * 16 + l16], V[s * VS + jt * 16 + l16], acc);
         }
@@ -316,10 +341,10 @@ __global__ __launch_bounds__(THREADS) void memory_sums_kernel(MemoryRows op, flo
     }
 }
 
-// The chunks of one (request, head) in order, 1,024 elements of the matrix a block (four a thread); four chunks asked for at a time.
+// The chunks of one (request, head) in order, 1,024 elements of the matrix a block (four a thread); eight chunks asked for at a time.
 __global__ __launch_bounds__(256) void memory_scan_kernel(const int* __restrict__ q_starts, const int* __restrict__ state_slots, float* __restrict__ records,
                                                           float* __restrict__ state, long long state_stride, int dim, int vdim, int chunk_rows) {
-    constexpr int PER = 4, AHEAD = 4;
+    constexpr int PER = 4, AHEAD = 8;
     const int request = blockIdx.x, head = blockIdx.y, n_heads = gridDim.y, tid = threadIdx.x;
     const int slot = state_slots[request];
     const int first_row = q_starts[request], rows = q_starts[request + 1] - first_row;
@@ -388,23 +413,73 @@ __global__ __launch_bounds__(THREADS) void memory_output_kernel(MemoryRows op, c
     const float* record = records + (record_of(chunk_first, L, request) * n_heads + head) * ((size_t)dim * vdim + dim);
     const int value_tiles = ceil_div(vdim, 16);
 
+    // Everything the block reads from memory is asked for here, from clamped places, and waits in registers for its turn: queries and keys, the
+    // decays' operands, the values of the first 128 columns, the state the chunk starts from and the gates (in the order of their use).
+    constexpr int QPER = L * DP / THREADS, VROWS = L / WAVES, VBLOCKS = 2, ITEMS = 2;
+    float q_mine[QPER], k_mine[QPER];
+#pragma unroll
+    for (int u = 0; u < QPER; u++) {
+        const int e = tid + u * THREADS, s = e / DP, i = e % DP;
+        const float* row = op.rows + (size_t)(chunk_first + min(s, n_valid - 1)) * op.stride + head * dim + min(i, dim - 1);
+        q_mine[u] = row[op.q_at], k_mine[u] = row[op.k_at];
+    }
+    DecayPiece<L, DPT> piece;
+    piece.ask(op, chunk_first, n_valid, head, n_heads, 0);
+    float v_mine[VBLOCKS][VROWS];   // column block * 64 + lane of every eighth row
+    auto ask_values = [&](int block, float (&mine)[VROWS]) {
+#pragma unroll
+        for (int u = 0; u < VROWS; u++)
+            mine[u] = op.rows[(size_t)(chunk_first + min(wave + u * WAVES, n_valid - 1)) * op.stride + op.v_at + head * vdim + min(block * WAVE + lane, vdim - 1)];
+    };
+    auto leave_values = [&](int block, const float (&mine)[VROWS]) {
+        const int c = block * WAVE + lane;
+        if (c >= value_tiles * 16) return;
+#pragma unroll
+        for (int u = 0; u < VROWS; u++) V[(wave + u * WAVES) * VS + c] = wave + u * WAVES < n_valid && c < vdim ? mine[u] : 0.0f;
+    };
+#pragma unroll
+    for (int block = 0; block < VBLOCKS; block++) ask_values(block, v_mine[block]);
     auto load_values = [&]() {
-        for (int e = tid; e < L * value_tiles * 16; e += THREADS) {
-            const int s = e / (value_tiles * 16), c = e % (value_tiles * 16);
-            V[s * VS + c] = s < n_valid && c < vdim ? op.rows[(size_t)(chunk_first + s) * op.stride + op.v_at + head * vdim + c] : 0.0f;
+#pragma unroll
+        for (int block = 0; block < VBLOCKS; block++) leave_values(block, v_mine[block]);
+        for (int block = VBLOCKS; block * WAVE < vdim; block++) {
+            float more[VROWS];
+            ask_values(block, more);
+            leave_values(block, more);
         }
     };
-    for (int e = tid; e < L * DP; e += THREADS) {
-        const int s = e / DP, i = e % DP;
-        const float* row = op.rows + (size_t)(chunk_first + min(s, n_valid - 1)) * op.stride + head * dim + min(i, dim - 1);
-        const float qv = row[op.q_at], kv = row[op.k_at];
-        const bool counts = s < n_valid && i < dim;
-        Q[s * QS + i] = counts ? qv * op.q_scale : 0.0f;
-        K[s * QS + i] = counts ? kv : 0.0f;
+    // outputs: 16 value columns a wave (up to ITEMS such tiles), all rows or, where there are few columns, half of them
+    const bool halves = value_tiles <= WAVES / 2 && NS >= 2;
+    constexpr int EARLY = DPT <= 4 ? ITEMS : DPT * L <= 256 ? 1 : 0;   // tiles whose states wait in registers (more of them would not fit)
+    auto ask_state = [&](int j, float (&mine)[DPT][4]) {
+#pragma unroll
+        for (int step = 0; step < DPT; step++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) mine[step][e] = record[(size_t)min(step * 16 + quad * 4 + e, dim - 1) * vdim + j];
+    };
+    float start[ITEMS][DPT][4], gates[ITEMS][NS][4], gain[ITEMS];
+#pragma unroll
+    for (int u = 0; u < ITEMS; u++) {
+        const int item = wave + u * WAVES, jt = halves ? item / 2 : item, j = min(jt * 16 + l16, vdim - 1);
+        if (jt >= value_tiles) continue;
+        if (u < EARLY) ask_state(j, start[u]);
+#pragma unroll
+        for (int t = 0; t < NS; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++)
+                gates[u][t][r] = op.rows[(size_t)(chunk_first + min(t * SUB + quad * 4 + r, n_valid - 1)) * op.stride + op.g_at + head * vdim + j];
+        gain[u] = op.gain[j];
     }
-    if (v_early) load_values();
+#pragma unroll
+    for (int u = 0; u < QPER; u++) {
+        const int e = tid + u * THREADS, s = e / DP, i = e % DP;
+        const bool counts = s < n_valid && i < dim;
+        Q[s * QS + i] = counts ? q_mine[u] * op.q_scale : 0.0f;
+        K[s * QS + i] = counts ? k_mine[u] : 0.0f;
+    }
     for (int e = tid; e < WAVES * L; e += THREADS) squares_lds[e] = 0.0f;
-    chunk_decays<L, DPT>(op, chunk_first, n_valid, head, n_heads, D, QS, A);
+    chunk_decays<L, DPT>(op, piece, chunk_first, n_valid, head, n_heads, D, QS, A);
+    if (v_early) load_values();
 
     // ---- decays inside the stretches: thread (channel i, stretch n) ----
     const int i = tid % DP, n = tid / DP;
@@ -492,9 +567,7 @@ __global__ __launch_bounds__(THREADS) void memory_output_kernel(MemoryRows op, c
         __syncthreads();
     }
 
-    // ---- outputs: 16 value columns a wave (up to two such tiles), all rows or, where there are few columns, half of them ----
-    constexpr int ITEMS = 2;
-    const bool halves = value_tiles <= WAVES / 2 && NS >= 2;
+    // ---- outputs ----
     f32x4 acc[ITEMS][NS];
 #pragma unroll
     for (int u = 0; u < ITEMS; u++) {
@@ -502,12 +575,8 @@ __global__ __launch_bounds__(THREADS) void memory_output_kernel(MemoryRows op, c
         for (int t = 0; t < NS; t++) acc[u][t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
         const int item = wave + u * WAVES, jt = halves ? item / 2 : item;
         if (jt >= value_tiles) continue;
-        const int t_first = halves && item % 2 ? NS / 2 : 0, t_last = halves && item % 2 == 0 ? NS / 2 : NS, j = min(jt * 16 + l16, vdim - 1);
-        float start[DPT][4];   // the state the chunk starts from, this lane's operands
-#pragma unroll
-        for (int step = 0; step < DPT; step++)
-#pragma unroll
-            for (int e = 0; e < 4; e++) start[step][e] = record[(size_t)min(step * 16 + quad * 4 + e, dim - 1) * vdim + j];
+        const int t_first = halves && item % 2 ? NS / 2 : 0, t_last = halves && item % 2 == 0 ? NS / 2 : NS;
+        if (u >= EARLY) ask_state(min(jt * 16 + l16, vdim - 1), start[u]);
 #pragma unroll
         for (int block = 0; block < NS; block++) {
             if (block >= t_last) continue;
@@ -534,7 +603,7 @@ __global__ __launch_bounds__(THREADS) void memory_output_kernel(MemoryRows op, c
                     for (int e = 0; e < 4; e++) qs[e] *= fade[e];
                 }
 #pragma unroll
-                for (int e = 0; e < 4; e++) acc[u][t] = multiply_add(qs[e], start[step][e], acc[u][t]);
+                for (int e = 0; e < 4; e++) acc[u][t] = multiply_add(qs[e], start[u][step][e], acc[u][t]);
             }
         }
         // (a lane's sums: rows t * 16 + 4 * quad + r of column jt * 16 + l16)
@@ -561,17 +630,13 @@ __global__ __launch_bounds__(THREADS) void memory_output_kernel(MemoryRows op, c
         const int item = wave + u * WAVES, jt = halves ? item / 2 : item, j = jt * 16 + l16;
         if (j >= vdim) continue;
         const int t_first = halves && item % 2 ? NS / 2 : 0, t_last = halves && item % 2 == 0 ? NS / 2 : NS;
-        const float gain = op.gain[j];
 #pragma unroll
         for (int t = 0; t < NS; t++) {
             if (t < t_first || t >= t_last) continue;
-            float gates[4];
-#pragma unroll
-            for (int r = 0; r < 4; r++) gates[r] = op.rows[(size_t)(chunk_first + min(t * SUB + quad * 4 + r, n_valid - 1)) * op.stride + op.g_at + head * vdim + j];
 #pragma unroll
             for (int r = 0; r < 4; r++) {
                 const int row = t * SUB + quad * 4 + r;
-                if (row < n_valid) out[(size_t)(chunk_first + row) * n_heads * vdim + head * vdim + j] = from_float<T>(acc[u][t][r] * factor_lds[row] * gain * silu_of(gates[r]));
+                if (row < n_valid) out[(size_t)(chunk_first + row) * n_heads * vdim + head * vdim + j] = from_float<T>(acc[u][t][r] * factor_lds[row] * gain[u] * silu_of(gates[u][t][r]));
             }
         }
     }
